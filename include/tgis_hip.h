@@ -62,7 +62,8 @@ int tgis_device_info(int device, int* num_cus, int64_t* hbm_bytes, char* name, i
 #define TGIS_OP_DECODE_TAIL 7
 #define TGIS_OP_SCAN 8      /* recurrent scans (tgis_wkv_scan, tgis_delta_scan) */
 #define TGIS_OP_MOE_GEMM 9  /* grouped expert GEMMs (tgis_moe_gemm) */
-#define TGIS_OP_COUNT 10
+#define TGIS_OP_HEAD_PRODUCT 10 /* small products per head (tgis_head_product) */
+#define TGIS_OP_COUNT 11
 int tgis_timing_enable(int on);
 int tgis_timing_reset(void);
 int tgis_timing_read(int op, int64_t* count, double* total_ms);
@@ -608,6 +609,54 @@ int tgis_poly_norm(const void* z, int64_t ld_z, void* y, int64_t ld_y, int64_t r
 int tgis_moe_route_grouped(const void* h, int64_t ld_h, const float* router_w, const float* correction, int n_groups,
                            int keep_groups, float renorm_eps, int32_t* idx, float* weight, int64_t T, int64_t W, int E, int k,
                            int dtype, void* stream);
+
+/* ---- several residual streams, rotated values with capped scores, latent attention without positions, minGRU, clamped experts ---- */
+/* turns[t][i] = (cos, sin) of positions[t] * inv_freq[i], i < n (fp32 angles): turns is [T][n][2] fp32. */
+int tgis_pair_turns(const int32_t* positions, const float* inv_freq, float* turns, int64_t T, int n, void* stream);
+/* tgis_rope_rows_kv_write, and the values are turned on their way into the cache: pair (2m, 2m + 1) of every value head by the
+ * angle whose (cos, sin) is v_turns[t][m] (tgis_pair_turns with n = dv / 2; dv even). */
+int tgis_rope_rows_turned_kv_write(void* proj, int64_t ld, int64_t q_col0, int64_t k_col0, int64_t v_col0, const float* inv_freq,
+                                   const int32_t* positions, const int32_t* slots, void* k_pool, void* v_pool, int64_t T, int H,
+                                   int G, int dk, int dv, int rot_dims, const float* v_turns, int dtype, void* stream);
+/* tgis_attn_varlen_win (without a gate) with capped scores (softcap > 0: s <- softcap tanh(s / softcap), after the scale; the
+ * sink is neither scaled nor capped) and / or outputs turned BACK by the reader's position: pair (2m, 2m + 1) of every head's
+ * output by minus the angle whose (cos, sin) is turns[t][m] (turns [total_q][dv / 2][2] fp32 or NULL; dv even). */
+int tgis_attn_varlen_turned(const void* q, int64_t ldq, const void* k_pool, const void* v_pool, const int32_t* block_tables,
+                            int64_t max_pages, const int32_t* ctx_lens, const int32_t* cu_seqlens_q, int64_t B, void* out,
+                            int64_t ld_out, int64_t total_q, int64_t max_q_len, int64_t max_ctx, int H, int G, int dk, int dv,
+                            float scale, int window, int keep_first, const float* sink, float softcap, const float* turns,
+                            float out_scale, void* workspace, int64_t workspace_bytes, int impl, int dtype, void* stream);
+/* From one down-projection down [T, ld]: columns q_col0 .. + q_rank divided by their root mean square times q_gain to cq [T, ld_cq];
+ * columns c_col0 .. + kv_rank likewise (c_gain) to the page slot of their token, as the key row and as the value columns of ONE
+ * kv head of width kv_rank (on long steps the columns are normed in place on the way). */
+int tgis_latent_norm_write(void* down, int64_t ld, int64_t q_col0, int64_t q_rank, const float* q_gain, void* cq, int64_t ld_cq,
+                           int64_t c_col0, int64_t kv_rank, const float* c_gain, const int32_t* slots, void* k_pool, void* v_pool,
+                           int64_t T, float eps, int dtype, void* stream);
+/* out[t][h][n] = sum_k x[t][h][k] w[h][n][k]; head h of a token starts at h * head_stride elements of its row in x and in out. */
+int tgis_head_product(const void* x, int64_t ld_x, int64_t head_stride_x, const void* w, void* out, int64_t ld_out,
+                      int64_t head_stride_out, int64_t T, int H, int N, int K, int dtype, void* stream);
+/* minGRU per (sequence, channel), tokens in order, on columns of proj [T, ld]: z = sigmoid(proj[z_col0 + c]), u = proj[x_col0 + c],
+ * cand = u + 1/2 if u >= 0 else sigmoid(u); S <- (1 - z) S + z cand; out[t][c] = S silu(proj[g_col0 + c]) out_scale.
+ * state [slots][D] fp32, read unless the step starts at position 0, written back.  max_q_len: launch shaping only. */
+int tgis_min_gru_scan(const void* proj, int64_t ld, int64_t z_col0, int64_t x_col0, int64_t g_col0, float* state,
+                      const int32_t* state_slots, const int32_t* cu_seqlens_q, const int32_t* positions, void* out,
+                      int64_t ld_out, float out_scale, int64_t B, int64_t T, int64_t max_q_len, int64_t D, int dtype, void* stream);
+/* tgis_moe_gemm over stacked [gate | up] weights with the clamped unit g = min(gate, limit), u = clamp(up, -limit, limit):
+ * g sigmoid(alpha g) (u + 1). */
+int tgis_moe_gemm_clamped(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
+                          const int32_t* tile_expert, const int32_t* n_tiles, const void* weights, int64_t expert_stride, int64_t N,
+                          int64_t K, float alpha, float limit, void* out, int64_t ld_out, int64_t capacity, int dtype, void* stream);
+/* s residual streams per token, X [T][s][W] fp32 (s <= 8): the update of the sublayer that ran and the input of the next one,
+ *   X'_b = sum_a cur.mix[a][b] X_a + cur.out[b] y   (kind 0: X' = X);   u = sum_a next.in[a] X'_a;
+ *   h = u / sqrt(mean u^2 + eps) * next.gain   (h [T, W] of `dtype`)
+ * cur = [s * s mix (from, to) | s out], next = [s in | gain], fp32.  y by kind: 1 a [T, ld_y] tensor of `dtype`; 2 the fp32 split-K
+ * slabs of tgis_dense_gemm_partial (ld_y their row stride); 3 a mixture: sum_j weight[t][j] y[pos[t][j]] over k expert rows, plus
+ * shared_gate[t] * shared[t] (shared: rows of `dtype`, or slabs if shared_slabs > 0; weight, shared, shared_gate may be NULL).
+ * ids instead of x (kind 0): every stream is table[ids[t]] * emb_scale.  x_out (may alias x, may be NULL) receives X'. */
+int tgis_hyper_update(const float* x, const int64_t* ids, const void* table, int64_t vocab, float emb_scale, float* x_out,
+                      int kind, const void* y, int64_t ld_y, int slabs, const int32_t* pos, const float* weight, int k,
+                      const void* shared, int64_t ld_shared, int shared_slabs, const float* shared_gate, const float* cur,
+                      const float* next, void* h, int64_t rows, int64_t W, int streams, float eps, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

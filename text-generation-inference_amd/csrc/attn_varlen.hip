@@ -45,7 +45,33 @@ struct AttnExt {
     const float* sink = nullptr;
     int gate_per_head = 0;
     float out_scale = 1.f;
+    //   softcap > 0: the scaled score s becomes softcap * tanh(s / softcap)
+    //   turns:      [token][dv / 2] (cos, sin) of the reader's own position: every pair of output channels (2m, 2m + 1) is turned
+    //               BACK by it where it is written, before gate and scale (the cached values were turned by their positions, so
+    //               what is left of them depends on the distance)
+    float softcap = 0.f;
+    const float* turns = nullptr;
 };
+// softcap * tanh(s / softcap); two-byte models take tanh as 1 - 2 / (1 + e^(2x)) on the hardware exponential (an absolute error
+// of about 1e-7 softcap)
+template <typename T> __device__ __forceinline__ float capped_score(float s, float cap) {
+    if (sizeof(T) == 4) return cap * tanhf(s / cap);
+    const float e = __builtin_amdgcn_exp2f(s * (2.8853900817779268f / cap));
+    return cap - 2.f * cap * __builtin_amdgcn_rcpf(1.f + e);
+}
+// channels c, c + 1 of token t (c even): turned back by the token's position
+__device__ __forceinline__ void turn_back(const AttnExt& e, int64_t t, int dv, int c, float& u, float& v) {
+    const f32x2 cs = *reinterpret_cast<const f32x2*>(e.turns + t * dv + c);
+    const float a = u * cs[0] + v * cs[1], b = v * cs[0] - u * cs[1];
+    u = a;
+    v = b;
+}
+// channel c of token t in this lane, its pair's other channel in the neighbouring lane
+__device__ __forceinline__ float turn_back_lane(const AttnExt& e, int64_t t, int dv, int c, float v) {
+    const float o = __shfl_xor(v, 1, 64);
+    const f32x2 cs = *reinterpret_cast<const f32x2*>(e.turns + t * dv + (c & ~1));
+    return (c & 1) ? v * cs[0] - o * cs[1] : v * cs[0] + o * cs[1];
+}
 __device__ __forceinline__ float sigmoid_f32(float z) { return 1.f / (1.f + expf(-z)); }
 __device__ __forceinline__ int first_visible(const AttnExt& e, int pos) {
     if (e.window > 0) return max(pos - e.window + 1, 0);
@@ -159,14 +185,21 @@ __global__ __launch_bounds__(256) void qk_norm_kv_write_kernel(
     for (int d = lane; d < dk; d += 64) dst[d] = (T)(ldf(p + d) * rinv * w[d]);
 }
 
-// Values: blended if asked, then written channel-major.  A workgroup takes 32 consecutive step tokens x 64 value columns
+// value column i (of G * dv, dv even) of one token, turned by the token's position: turns [dv / 2] (cos, sin)
+template <typename T> __device__ __forceinline__ float turned_value(const T* __restrict__ vrow, int i, int dv, const float* __restrict__ turns) {
+    const float v = (float)vrow[i], o = (float)vrow[i ^ 1];
+    const f32x2 cs = *reinterpret_cast<const f32x2*>(turns + ((i % dv) & ~1));
+    return (i & 1) ? v * cs[0] + o * cs[1] : v * cs[0] - o * cs[1];
+}
+
+// Values: blended or turned if asked, then written channel-major.  A workgroup takes 32 consecutive step tokens x 64 value columns
 // through LDS: rows are read as they lie in the projection's output (a token's columns are contiguous), and written with
 // the tokens of a page side by side — a 16-byte store per (column, 8 tokens) wherever 8 neighbours of the step are 8
 // neighbours in a page (prompt portions), single elements otherwise (decoded tokens of different sequences).
 template <typename T>
 __global__ __launch_bounds__(256) void v_write_kernel(const T* __restrict__ qkv, int64_t ld, int64_t v_col0, const int32_t* __restrict__ slots,
                                                       const T* __restrict__ v_first, int64_t ld_vf, const float* __restrict__ lambda_ptr,
-                                                      T* __restrict__ v_pool, int64_t Ttot, int G, int dv) {
+                                                      T* __restrict__ v_pool, int64_t Ttot, int G, int dv, const float* __restrict__ turns) {
     __shared__ float tile[32][65];
     __shared__ int32_t sl[32];
     const int64_t t0 = (int64_t)blockIdx.x * 32;
@@ -180,6 +213,7 @@ __global__ __launch_bounds__(256) void v_write_kernel(const T* __restrict__ qkv,
         if (t0 + tt < Ttot && c0 + cc < C) {
             v = ldf(qkv + (t0 + tt) * ld + v_col0 + c0 + cc);
             if (v_first) v = (1.f - lam) * v + lam * ldf(v_first + (t0 + tt) * ld_vf + c0 + cc);
+            if (turns) v = turned_value(qkv + (t0 + tt) * ld + v_col0, c0 + cc, dv, turns + (t0 + tt) * dv);
         }
         tile[tt][cc] = v;
     }
@@ -289,6 +323,7 @@ __global__ __launch_bounds__(1024) void attn_varlen_kernel(
             const int64_t page = table[j / PAGE];
             s = dot_row<T>(myq, k_pool + ((page * G + g) * PAGE + (j % PAGE)) * dk, dk);
             if (ext.r1) s -= r1h * log1pf(r2h * (float)(pos - j));
+            if (ext.softcap > 0.f) s = capped_score<T>(s, ext.softcap);
         }
         const float mn = fmaxf(m, wave_max(s));  // finite: key `base` is visible
         const float corr = expf(m - mn);         // exp(-inf) = 0 on the first chunk
@@ -356,6 +391,11 @@ __global__ __launch_bounds__(1024) void attn_varlen_kernel(
     const float inv = sink_f / l * head_out_factor<T>(ext, t, g * Rall + r0 + r);
     T* orow = out + (int64_t)t * ld_out + (int64_t)(g * Rall + r0 + r) * dv;
     const T* grow = (ext.gate && !ext.gate_per_head) ? reinterpret_cast<const T*>(ext.gate) + (int64_t)t * ext.ld_gate + (int64_t)(g * Rall + r0 + r) * dv : nullptr;
+    if (ext.turns) {  // dv is even: a channel's partner is in the neighbouring lane and exists when it does
+#pragma unroll
+        for (int c = 0; c < DV_PER_LANE; ++c)
+            if (lane + 64 * c < dv) o[c] = turn_back_lane(ext, t, dv, lane + 64 * c, o[c]);
+    }
 #pragma unroll
     for (int c = 0; c < DV_PER_LANE; ++c)
         if (lane + 64 * c < dv) orow[lane + 64 * c] = (T)(o[c] * inv * (grow ? sigmoid_f32(ldf(grow + lane + 64 * c)) : 1.f));
@@ -455,6 +495,13 @@ __global__ __launch_bounds__(512) void attn_varlen_mfma_kernel(
             for (int i = 0; i < 16; ++i) {
                 const int key = base + (i >> 2) * 8 + (i & 3);
                 S[i] = key_visible(ext, key, pos, lo) ? S[i] * scale - r1h * __logf(1.f + r2h * (float)(pos - key)) : -INFINITY;
+                mx = fmaxf(mx, S[i]);
+            }
+        } else if (ext.softcap > 0.f) {
+#pragma unroll
+            for (int i = 0; i < 16; ++i) {
+                const int key = base + (i >> 2) * 8 + (i & 3);
+                S[i] = key_visible(ext, key, pos, lo) ? capped_score<T>(S[i] * scale, ext.softcap) : -INFINITY;
                 mx = fmaxf(mx, S[i]);
             }
         } else {
@@ -563,6 +610,10 @@ __global__ __launch_bounds__(512) void attn_varlen_mfma_kernel(
 #pragma unroll
                 for (int i = 0; i < 4; ++i) acc[i] += os[((w * DVT + t) * 16 + j * 4 + i) * 64 + lane] * wgt;
             }
+            if (ext.turns) {
+                turn_back(ext, t0 + tq, dv, h * 4 + t * 32 + j * 8, acc[0], acc[1]);
+                turn_back(ext, t0 + tq, dv, h * 4 + t * 32 + j * 8 + 2, acc[2], acc[3]);
+            }
             V4 o4, g4 = {};
             if (grow) g4 = *reinterpret_cast<const V4*>(grow + t * 32 + j * 8);
 #pragma unroll
@@ -581,10 +632,15 @@ __global__ __launch_bounds__(512) void attn_varlen_mfma_kernel(
         if (t < nvt) {
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
+                float acc[4] = {O[t][j * 4], O[t][j * 4 + 1], O[t][j * 4 + 2], O[t][j * 4 + 3]};
+                if (ext.turns) {
+                    turn_back(ext, t0 + tq, dv, h * 4 + t * 32 + j * 8, acc[0], acc[1]);
+                    turn_back(ext, t0 + tq, dv, h * 4 + t * 32 + j * 8 + 2, acc[2], acc[3]);
+                }
                 V4 o4, g4 = {};
                 if (grow) g4 = *reinterpret_cast<const V4*>(grow + t * 32 + j * 8);
 #pragma unroll
-                for (int i = 0; i < 4; ++i) o4[i] = (T)(O[t][j * 4 + i] * inv * (grow ? sigmoid_f32((float)g4[i]) : 1.f));
+                for (int i = 0; i < 4; ++i) o4[i] = (T)(acc[i] * inv * (grow ? sigmoid_f32((float)g4[i]) : 1.f));
                 *reinterpret_cast<V4*>(orow + t * 32 + j * 8) = o4;
             }
         }
@@ -612,6 +668,7 @@ __global__ __launch_bounds__(64) void attn_combine_splits_kernel(const float* __
     for (int c = lane; c < dv; c += 64) {
         float acc = 0.f;
         for (int x = 0; x < X; ++x) acc += p0[x * stride + 2 + c] * wx[x];
+        if (ext.turns) acc = turn_back_lane(ext, t, dv, c, acc);
         out[t * ld_out + (int64_t)head * dv + c] = (T)(acc * (grow ? sigmoid_f32(ldf(grow + c)) : 1.f));
     }
 }
@@ -724,6 +781,13 @@ __global__ __launch_bounds__(256) void attn_varlen_staged_kernel(
                 S[i] = key_visible(ext, key, pos, lo) ? S[i] * scale - r1h * __logf(1.f + r2h * (float)(pos - key)) : -INFINITY;
                 mx = fmaxf(mx, S[i]);
             }
+        } else if (ext.softcap > 0.f) {
+#pragma unroll
+            for (int i = 0; i < 16; ++i) {
+                const int key = base + (i >> 2) * 8 + (i & 3);
+                S[i] = key_visible(ext, key, pos, lo) ? capped_score<T>(S[i] * scale, ext.softcap) : -INFINITY;
+                mx = fmaxf(mx, S[i]);
+            }
         } else {
 #pragma unroll
             for (int i = 0; i < 16; ++i) {
@@ -783,10 +847,15 @@ __global__ __launch_bounds__(256) void attn_varlen_staged_kernel(
         if (t < nvt) {
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
+                float acc[4] = {O[t][j * 4], O[t][j * 4 + 1], O[t][j * 4 + 2], O[t][j * 4 + 3]};
+                if (ext.turns) {
+                    turn_back(ext, t0 + tq, dv, h * 4 + t * 32 + j * 8, acc[0], acc[1]);
+                    turn_back(ext, t0 + tq, dv, h * 4 + t * 32 + j * 8 + 2, acc[2], acc[3]);
+                }
                 V4 o4, g4 = {};
                 if (grow) g4 = *reinterpret_cast<const V4*>(grow + t * 32 + j * 8);
 #pragma unroll
-                for (int i = 0; i < 4; ++i) o4[i] = (T)(O[t][j * 4 + i] * inv * (grow ? sigmoid_f32((float)g4[i]) : 1.f));
+                for (int i = 0; i < 4; ++i) o4[i] = (T)(acc[i] * inv * (grow ? sigmoid_f32((float)g4[i]) : 1.f));
                 *reinterpret_cast<V4*>(orow + t * 32 + j * 8) = o4;
             }
         }
@@ -915,7 +984,8 @@ __global__ __launch_bounds__(256) void rope_rows_kv_write_kernel(T* __restrict__
                                                                  int64_t v_col0, const float* __restrict__ inv_freq,
                                                                  const int32_t* __restrict__ positions, const int32_t* __restrict__ slots,
                                                                  T* __restrict__ k_pool, T* __restrict__ v_pool, int H, int G, int dk,
-                                                                 int dv, int rdims, int v_inline, float unit_eps) {
+                                                                 int dv, int rdims, int v_inline, float unit_eps,
+                                                                 const float* __restrict__ v_turns) {
     const int64_t t = blockIdx.x;
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int slot = slots[t];
@@ -929,7 +999,7 @@ __global__ __launch_bounds__(256) void rope_rows_kv_write_kernel(T* __restrict__
         const int i1 = min(i0 + 1024, G * dv);
         for (int i = i0 + threadIdx.x; i < i1; i += blockDim.x) {
             const int g = i / dv, c = i - g * dv;
-            v_pool[((page * G + g) * dv + c) * PAGE + off] = vrow[i];
+            v_pool[((page * G + g) * dv + c) * PAGE + off] = v_turns ? (T)turned_value(vrow, i, dv, v_turns + t * dv) : vrow[i];
         }
         return;
     }
@@ -986,6 +1056,60 @@ __global__ __launch_bounds__(256) void rope_rows_kv_write_kernel(T* __restrict__
             dst[d + 1] = src[d + 1];
         }
     }
+}
+
+__global__ void pair_turns_kernel(const int32_t* __restrict__ positions, const float* __restrict__ inv_freq, float* __restrict__ turns,
+                                  int64_t total, int n) {
+    const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= total) return;
+    const int64_t t = i / n;
+    float sn, cs;
+    sincosf((float)positions[t] * inv_freq[i - t * n], &sn, &cs);
+    *reinterpret_cast<f32x2*>(turns + 2 * i) = f32x2{cs, sn};
+}
+
+// grid (token): wave 0 the cache latent, wave 1 the query latent (see tgis_latent_norm_write)
+template <typename T>
+__global__ __launch_bounds__(128) void latent_norm_write_kernel(T* __restrict__ down, int64_t ld, int64_t q_col0, int q_rank,
+                                                                const float* __restrict__ q_gain, T* __restrict__ cq, int64_t ld_cq,
+                                                                int64_t c_col0, int rk, const float* __restrict__ c_gain,
+                                                                const int32_t* __restrict__ slots, T* __restrict__ k_pool,
+                                                                T* __restrict__ v_pool, float eps, int v_inline) {
+    const int64_t t = blockIdx.x;
+    const int lane = threadIdx.x & 63;
+    const bool is_q = threadIdx.x >= 64;
+    T* src = down + t * ld + (is_q ? q_col0 : c_col0);
+    const int n = is_q ? q_rank : rk;
+    const float* gain = is_q ? q_gain : c_gain;
+    constexpr int HELD = 16;  // values a lane keeps in registers: rows of up to 1024 are read once
+    float v[HELD], ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < HELD; ++i) {
+        const int c = lane + 64 * i;
+        v[i] = c < n ? ldf(src + c) : 0.f;
+        ss += v[i] * v[i];
+    }
+    for (int c = lane + 64 * HELD; c < n; c += 64) ss += ldf(src + c) * ldf(src + c);
+    ss = wave_sum(ss);
+    const float rinv = 1.0f / sqrtf(ss / (float)n + eps);
+    const int slot = is_q ? 0 : slots[t];
+    const int64_t page = slot / PAGE;
+    const int off = slot % PAGE;
+    T* dst = is_q ? cq + t * ld_cq : k_pool + (page * PAGE + off) * (int64_t)rk;
+    auto put = [&](int c, float x) {
+        const T y = (T)(x * rinv * gain[c]);
+        dst[c] = y;
+        if (!is_q) {
+            if (v_inline)
+                v_pool[(page * rk + c) * PAGE + off] = y;
+            else
+                src[c] = y;
+        }
+    };
+#pragma unroll
+    for (int i = 0; i < HELD; ++i)
+        if (lane + 64 * i < n) put(lane + 64 * i, v[i]);
+    for (int c = lane + 64 * HELD; c < n; c += 64) put(c, ldf(src + c));
 }
 
 template <typename T, int DK16, int DVT>
@@ -1080,7 +1204,7 @@ int launch_prep(void* qkv, int64_t ld, const int32_t* positions, const int32_t* 
                        dv, v_inline);
     if (!v_inline)
         hipLaunchKernelGGL(v_write_kernel<T>, dim3((unsigned)cdiv64(T_, 32), (unsigned)cdiv64((int64_t)G * dv, 64)), dim3(256), 0, st,
-                           (const T*)qkv, ld, (int64_t)(H + G) * dk, slots, (const T*)v_first, ld_vf, lam, (T*)v_pool, T_, G, dv);
+                           (const T*)qkv, ld, (int64_t)(H + G) * dk, slots, (const T*)v_first, ld_vf, lam, (T*)v_pool, T_, G, dv, (const float*)nullptr);
     return 0;
 }
 
@@ -1217,7 +1341,7 @@ extern "C" int tgis_kv_norm_write(void* qkv, int64_t ld, int64_t k_col0, int64_t
     if (!v_inline)
         TGIS_ATTN_BY_DTYPE(dtype, hipLaunchKernelGGL(v_write_kernel<TT>, dim3((unsigned)cdiv64(T, 32), (unsigned)cdiv64((int64_t)G * dv, 64)),
                                                      dim3(256), 0, st, (const TT*)qkv, ld, v_col0, slots, (const TT*)nullptr, (int64_t)0,
-                                                     (const float*)nullptr, (TT*)v_pool, T, G, dv));
+                                                     (const float*)nullptr, (TT*)v_pool, T, G, dv, (const float*)nullptr));
     TGIS_CHECK_LAUNCH();
     return TGIS_OK;
 }
@@ -1245,7 +1369,7 @@ extern "C" int tgis_latent_kv_write(const void* q, int64_t ldq, void* ckv, int64
     if (!v_inline)
         TGIS_ATTN_BY_DTYPE(dtype, hipLaunchKernelGGL(v_write_kernel<TT>, dim3((unsigned)cdiv64(T, 32), (unsigned)cdiv64((int64_t)kv_rank, 64)),
                                                      dim3(256), 0, st, (const TT*)ckv, ld_ckv, (int64_t)0, slots, (const TT*)nullptr, (int64_t)0,
-                                                     (const float*)nullptr, (TT*)v_pool, T, 1, kv_rank));
+                                                     (const float*)nullptr, (TT*)v_pool, T, 1, kv_rank, (const float*)nullptr));
     TGIS_CHECK_LAUNCH();
     return TGIS_OK;
 }
@@ -1255,7 +1379,8 @@ extern "C" int tgis_latent_kv_write(const void* q, int64_t ldq, void* ckv, int64
 // (2i, 2i + 1) of the first rot_dims channels of every head turns by positions[t] * inv_freq[i] (fp32 angle), the rest pass.
 static int rope_rows_impl(void* proj, int64_t ld, int64_t q_col0, int64_t k_col0, int64_t v_col0, const float* inv_freq,
                           const int32_t* positions, const int32_t* slots, void* k_pool, void* v_pool, int64_t T, int H,
-                          int G, int dk, int dv, int rot_dims, float unit_eps, int dtype, void* stream) {
+                          int G, int dk, int dv, int rot_dims, float unit_eps, int dtype, void* stream, const float* v_turns = nullptr) {
+    TGIS_CHECK_ARG(!v_turns || dv % 2 == 0, "tgis_rope_rows_kv_write: values are turned in pairs (width %d)", dv);
     TGIS_CHECK_ARG(proj && positions && slots && k_pool && v_pool && (inv_freq || rot_dims == 0), "tgis_rope_rows_kv_write: null tensor");
     TGIS_CHECK_ARG(H >= 1 && G >= 1 && dk >= 1 && dv >= 1 && rot_dims >= 0 && rot_dims <= dk && rot_dims % 2 == 0 && q_col0 >= 0 &&
                        k_col0 >= 0 && v_col0 >= 0 && ld >= q_col0 + (int64_t)H * dk && ld >= k_col0 + (int64_t)G * dk &&
@@ -1269,11 +1394,11 @@ static int rope_rows_impl(void* proj, int64_t ld, int64_t q_col0, int64_t k_col0
     const int v_blocks = v_inline ? (int)cdiv64((int64_t)G * dv, 1024) : 0;
     TGIS_ATTN_BY_DTYPE(dtype, hipLaunchKernelGGL(rope_rows_kv_write_kernel<TT>, dim3((unsigned)T, (unsigned)((H + G + 3) / 4 + v_blocks)), dim3(256),
                                                  0, st, (TT*)proj, ld, q_col0, k_col0, v_col0, inv_freq, positions, slots, (TT*)k_pool,
-                                                 (TT*)v_pool, H, G, dk, dv, rot_dims, v_inline, unit_eps));
+                                                 (TT*)v_pool, H, G, dk, dv, rot_dims, v_inline, unit_eps, v_turns));
     if (!v_inline)
         TGIS_ATTN_BY_DTYPE(dtype, hipLaunchKernelGGL(v_write_kernel<TT>, dim3((unsigned)cdiv64(T, 32), (unsigned)cdiv64((int64_t)G * dv, 64)),
                                                      dim3(256), 0, st, (const TT*)proj, ld, v_col0, slots, (const TT*)nullptr, (int64_t)0,
-                                                     (const float*)nullptr, (TT*)v_pool, T, G, dv));
+                                                     (const float*)nullptr, (TT*)v_pool, T, G, dv, v_turns));
     TGIS_CHECK_LAUNCH();
     return TGIS_OK;
 }
@@ -1284,12 +1409,81 @@ extern "C" int tgis_rope_rows_kv_write(void* proj, int64_t ld, int64_t q_col0, i
     return rope_rows_impl(proj, ld, q_col0, k_col0, v_col0, inv_freq, positions, slots, k_pool, v_pool, T, H, G, dk, dv, rot_dims, -1.f, dtype, stream);
 }
 
+// The same, and the values are turned by their position on the way into the cache: pair (2m, 2m + 1) of every value head by the
+// angle whose (cos, sin) v_turns [T][dv / 2] holds (tgis_pair_turns).
+extern "C" int tgis_rope_rows_turned_kv_write(void* proj, int64_t ld, int64_t q_col0, int64_t k_col0, int64_t v_col0, const float* inv_freq,
+                                              const int32_t* positions, const int32_t* slots, void* k_pool, void* v_pool, int64_t T, int H,
+                                              int G, int dk, int dv, int rot_dims, const float* v_turns, int dtype, void* stream) {
+    TGIS_CHECK_ARG(v_turns, "tgis_rope_rows_turned_kv_write: null turns");
+    return rope_rows_impl(proj, ld, q_col0, k_col0, v_col0, inv_freq, positions, slots, k_pool, v_pool, T, H, G, dk, dv, rot_dims, -1.f, dtype, stream, v_turns);
+}
+
+// turns[t][i] = (cos, sin) of positions[t] * inv_freq[i] (fp32 angle), i < n
+extern "C" int tgis_pair_turns(const int32_t* positions, const float* inv_freq, float* turns, int64_t T, int n, void* stream) {
+    TGIS_CHECK_ARG(positions && inv_freq && turns && n >= 1, "tgis_pair_turns: bad arguments");
+    if (T == 0) return TGIS_OK;
+    hipStream_t st = (hipStream_t)stream;
+    TgisTimedScope timed(TGIS_OP_ROPE_KV, st);
+    hipLaunchKernelGGL(pair_turns_kernel, dim3((unsigned)cdiv64(T * n, 256)), dim3(256), 0, st, positions, inv_freq, turns, T * n, n);
+    TGIS_CHECK_LAUNCH();
+    return TGIS_OK;
+}
+
+// What a token of a latent-attention layer without positions leaves behind, from ONE down-projection down [T, ld]: the normed query
+// latent (columns q_col0 .. + q_rank, gain q_gain) to cq [T, ld_cq], and the normed cache latent (columns c_col0 .. + kv_rank,
+// gain c_gain) to its page slot, token-major as a key and channel-major as a value (one kv head of width kv_rank; the columns
+// are normed in place when the step is long enough for the transposing writer).  Root mean square norms, eps inside the root.
+extern "C" int tgis_latent_norm_write(void* down, int64_t ld, int64_t q_col0, int64_t q_rank, const float* q_gain, void* cq, int64_t ld_cq,
+                                      int64_t c_col0, int64_t kv_rank, const float* c_gain, const int32_t* slots, void* k_pool, void* v_pool,
+                                      int64_t T, float eps, int dtype, void* stream) {
+    TGIS_CHECK_ARG(down && q_gain && cq && c_gain && slots && k_pool && v_pool, "tgis_latent_norm_write: null tensor");
+    TGIS_CHECK_ARG(q_rank >= 1 && kv_rank >= 1 && q_col0 >= 0 && c_col0 >= 0 && ld >= q_col0 + q_rank && ld >= c_col0 + kv_rank && ld_cq >= q_rank,
+                   "tgis_latent_norm_write: bad geometry (q_rank %ld, kv_rank %ld, ld %ld)", (long)q_rank, (long)kv_rank, (long)ld);
+    TGIS_CHECK_ARG(dtype == TGIS_F16 || dtype == TGIS_BF16 || dtype == TGIS_F32, "tgis_latent_norm_write: bad dtype");
+    if (T == 0) return TGIS_OK;
+    hipStream_t st = (hipStream_t)stream;
+    TgisTimedScope timed(TGIS_OP_ROPE_KV, st);
+    const int v_inline = T < 512 ? 1 : 0;
+    TGIS_ATTN_BY_DTYPE(dtype, hipLaunchKernelGGL(latent_norm_write_kernel<TT>, dim3((unsigned)T), dim3(128), 0, st, (TT*)down, ld, q_col0,
+                                                 (int)q_rank, q_gain, (TT*)cq, ld_cq, c_col0, (int)kv_rank, c_gain, slots, (TT*)k_pool,
+                                                 (TT*)v_pool, eps, v_inline));
+    if (!v_inline)
+        TGIS_ATTN_BY_DTYPE(dtype, hipLaunchKernelGGL(v_write_kernel<TT>, dim3((unsigned)cdiv64(T, 32), (unsigned)cdiv64(kv_rank, 64)), dim3(256), 0,
+                                                     st, (const TT*)down, ld, c_col0, slots, (const TT*)nullptr, (int64_t)0,
+                                                     (const float*)nullptr, (TT*)v_pool, T, 1, (int)kv_rank, (const float*)nullptr));
+    TGIS_CHECK_LAUNCH();
+    return TGIS_OK;
+}
+
 // The same, and every q and k head is divided by its root mean square (sqrt(mean(x^2) + unit_eps), no gain) after the rotation.
 extern "C" int tgis_rope_rows_unit_kv_write(void* proj, int64_t ld, int64_t q_col0, int64_t k_col0, int64_t v_col0, const float* inv_freq,
                                             const int32_t* positions, const int32_t* slots, void* k_pool, void* v_pool, int64_t T, int H,
                                             int G, int dk, int dv, int rot_dims, float unit_eps, int dtype, void* stream) {
     TGIS_CHECK_ARG(unit_eps >= 0.f && dk <= 256, "tgis_rope_rows_unit_kv_write: heads of up to 256 channels, eps >= 0");
     return rope_rows_impl(proj, ld, q_col0, k_col0, v_col0, inv_freq, positions, slots, k_pool, v_pool, T, H, G, dk, dv, rot_dims, unit_eps, dtype, stream);
+}
+
+static int attn_win_impl(const void* q, int64_t ldq, const void* k_pool, const void* v_pool, const int32_t* block_tables, int64_t max_pages,
+                         const int32_t* ctx_lens, const int32_t* cu_seqlens_q, int64_t B, void* out, int64_t ld_out, int64_t total_q,
+                         int64_t max_q_len, int64_t max_ctx, int H, int G, int dk, int dv, float scale, int window, int keep_first,
+                         const float* sink, const void* gate, int64_t ld_gate, int gate_per_head, float out_scale, float softcap,
+                         const float* turns, void* workspace, int64_t workspace_bytes, int impl, int dtype, void* stream) {
+    TGIS_CHECK_ARG(window >= 0 && keep_first >= 0 && (window > 0 || keep_first == 0), "tgis_attn_varlen_win: kept first positions need a window");
+    TGIS_CHECK_ARG(!gate || (gate_per_head ? ld_gate >= H
+                                           : (ld_gate >= (int64_t)H * dv && (dtype == TGIS_F32 || (ld_gate % 4 == 0 && ((uintptr_t)gate & 7) == 0)))),
+                   "tgis_attn_varlen_win: the gate needs a row stride >= H (per head) or >= H dv with 8-byte aligned rows");
+    AttnExt ext{nullptr, nullptr, 0, gate, ld_gate,
+                (int)std::min<int64_t>(64, workspace && ((uintptr_t)workspace & 15) == 0 ? workspace_bytes / std::max<int64_t>(1, total_q * H * (int64_t)(dv + 2) * 4) : 0),
+                (float*)workspace, total_q};
+    ext.window = window;
+    ext.keep_first = keep_first;
+    ext.sink = sink;
+    ext.gate_per_head = gate_per_head ? 1 : 0;
+    ext.out_scale = out_scale;
+    ext.softcap = softcap;
+    ext.turns = turns;
+    return attn_varlen_impl(q, ldq, k_pool, v_pool, block_tables, max_pages, ctx_lens, cu_seqlens_q, B, out, ld_out, total_q, max_q_len,
+                            max_ctx, H, G, dk, dv, scale, impl, dtype, ext, stream);
 }
 
 // tgis_attn_varlen with a sliding window that also keeps the first positions (window > 0: position i sees j <= i only if
@@ -1303,18 +1497,20 @@ extern "C" int tgis_attn_varlen_win(const void* q, int64_t ldq, const void* k_po
                                     float scale, int window, int keep_first, const float* sink, const void* gate, int64_t ld_gate,
                                     int gate_per_head, float out_scale, void* workspace, int64_t workspace_bytes, int impl, int dtype,
                                     void* stream) {
-    TGIS_CHECK_ARG(window >= 0 && keep_first >= 0 && (window > 0 || keep_first == 0), "tgis_attn_varlen_win: kept first positions need a window");
-    TGIS_CHECK_ARG(!gate || (gate_per_head ? ld_gate >= H
-                                           : (ld_gate >= (int64_t)H * dv && (dtype == TGIS_F32 || (ld_gate % 4 == 0 && ((uintptr_t)gate & 7) == 0)))),
-                   "tgis_attn_varlen_win: the gate needs a row stride >= H (per head) or >= H dv with 8-byte aligned rows");
-    AttnExt ext{nullptr, nullptr, 0, gate, ld_gate,
-                (int)std::min<int64_t>(64, workspace && ((uintptr_t)workspace & 15) == 0 ? workspace_bytes / std::max<int64_t>(1, total_q * H * (int64_t)(dv + 2) * 4) : 0),
-                (float*)workspace, total_q};
-    ext.window = window;
-    ext.keep_first = keep_first;
-    ext.sink = sink;
-    ext.gate_per_head = gate_per_head ? 1 : 0;
-    ext.out_scale = out_scale;
-    return attn_varlen_impl(q, ldq, k_pool, v_pool, block_tables, max_pages, ctx_lens, cu_seqlens_q, B, out, ld_out, total_q, max_q_len,
-                            max_ctx, H, G, dk, dv, scale, impl, dtype, ext, stream);
+    return attn_win_impl(q, ldq, k_pool, v_pool, block_tables, max_pages, ctx_lens, cu_seqlens_q, B, out, ld_out, total_q, max_q_len, max_ctx,
+                         H, G, dk, dv, scale, window, keep_first, sink, gate, ld_gate, gate_per_head, out_scale, 0.f, nullptr, workspace,
+                         workspace_bytes, impl, dtype, stream);
+}
+
+// The same with capped scores (softcap > 0: s <- softcap * tanh(s / softcap) after the scale) and / or outputs turned back by the
+// reader's position (turns [total_q][dv / 2] (cos, sin), dv even): the counterpart of values turned by tgis_rope_rows_turned_kv_write.
+extern "C" int tgis_attn_varlen_turned(const void* q, int64_t ldq, const void* k_pool, const void* v_pool, const int32_t* block_tables,
+                                       int64_t max_pages, const int32_t* ctx_lens, const int32_t* cu_seqlens_q, int64_t B, void* out,
+                                       int64_t ld_out, int64_t total_q, int64_t max_q_len, int64_t max_ctx, int H, int G, int dk, int dv,
+                                       float scale, int window, int keep_first, const float* sink, float softcap, const float* turns,
+                                       float out_scale, void* workspace, int64_t workspace_bytes, int impl, int dtype, void* stream) {
+    TGIS_CHECK_ARG(softcap >= 0.f && (!turns || dv % 2 == 0), "tgis_attn_varlen_turned: softcap >= 0; values are turned in pairs (width %d)", dv);
+    return attn_win_impl(q, ldq, k_pool, v_pool, block_tables, max_pages, ctx_lens, cu_seqlens_q, B, out, ld_out, total_q, max_q_len, max_ctx,
+                         H, G, dk, dv, scale, window, keep_first, sink, nullptr, 0, 0, out_scale, softcap, turns, workspace, workspace_bytes,
+                         impl, dtype, stream);
 }

@@ -1,0 +1,198 @@
+// Several fp32 residual streams per token ("hyper-connections"): a sublayer f reads a weighted sum of the s streams and its
+// result is spread over all of them while they are mixed,
+//
+//     u = sum_a c_in[a] X_a;    y = f(u / sqrt(mean u^2 + eps) * g);    X'_b = sum_a M[a][b] X_a + c_out[b] y
+//
+// One launch per sublayer boundary: it applies the update of the sublayer that just ran and makes the normed input of the next
+// one (in front of the first sublayer the streams are s copies of the scaled embedding row, which it looks up itself).  y
+// arrives as the projection left it: a tensor of T, the fp32 split-K slabs of the GEMM, or the unsummed expert rows of a
+// mixture with their weights and a gated shared row.
+//
+// Layout: X [token][stream][W].  A workgroup per token; a column's s values stay in registers between the mix and the next
+// sublayer's sum, whose row waits in LDS for the mean of squares.
+#include "common.h"
+#include "row_io.h"
+
+namespace {
+
+constexpr int MAX_STREAMS = 8;
+
+// What the sublayer left (kind 0: nothing — the streams only feed the next norm).
+struct SublayerResult {
+    int kind;               // 1: T rows, 2: fp32 slabs, 3: mixture
+    const void* p;          // T rows / slabs / expert rows
+    int64_t ld;
+    int slabs;
+    const int32_t* pos;     // mixture: [tokens][k] row of each (token, choice)
+    const float* weight;    // [tokens][k] or null (ones)
+    int k;
+    const void* shared;     // T rows, or slabs if shared_slabs > 0; null: none
+    int64_t ld_shared;
+    int shared_slabs;
+    const float* shared_gate;  // [tokens] or null (ones)
+};
+
+// sum of the split-K slabs [row / 32][S][32][ld] at (row, c), four loads in flight
+template <int V> __device__ __forceinline__ f32x4 slab_sum(const void* p, int64_t ld, int slabs, int64_t row, int64_t c) {
+    const float* sp = reinterpret_cast<const float*>(p) + ((row >> 5) * slabs * 32 + (row & 31)) * ld + c;
+    const int64_t step = 32 * ld;
+    f32x4 v = {};
+    int s = 0;
+    for (; s + 4 <= slabs; s += 4) {
+        f32x4 t[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) t[i] = LdV<float, V>::ld(sp + (int64_t)(s + i) * step);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v += t[i];
+    }
+    for (; s < slabs; ++s) v += LdV<float, V>::ld(sp + (int64_t)s * step);
+    return v;
+}
+
+template <typename T, int V> __device__ __forceinline__ f32x4 result_at(const SublayerResult& r, int64_t row, int64_t c) {
+    if (r.kind == 1) return LdV<T, V>::ld(reinterpret_cast<const T*>(r.p) + row * r.ld + c);
+    if (r.kind == 2) return slab_sum<V>(r.p, r.ld, r.slabs, row, c);
+    const T* rows = reinterpret_cast<const T*>(r.p);
+    f32x4 v = {};
+    int j = 0;
+    for (; j + 2 <= r.k; j += 2) {
+        const int64_t p0 = r.pos[row * r.k + j], p1 = r.pos[row * r.k + j + 1];
+        const f32x4 a = LdV<T, V>::ld(rows + p0 * r.ld + c), b = LdV<T, V>::ld(rows + p1 * r.ld + c);
+        v += a * (r.weight ? r.weight[row * r.k + j] : 1.f);
+        v += b * (r.weight ? r.weight[row * r.k + j + 1] : 1.f);
+    }
+    if (j < r.k) v += LdV<T, V>::ld(rows + (int64_t)r.pos[row * r.k + j] * r.ld + c) * (r.weight ? r.weight[row * r.k + j] : 1.f);
+    if (r.shared) {
+        const f32x4 s = r.shared_slabs > 0 ? slab_sum<V>(r.shared, r.ld_shared, r.shared_slabs, row, c)
+                                           : LdV<T, V>::ld(reinterpret_cast<const T*>(r.shared) + row * r.ld_shared + c);
+        v += s * (r.shared_gate ? r.shared_gate[row] : 1.f);
+    }
+    return v;
+}
+
+// cur: [s * s mix (from, to) | s out] of the sublayer that ran (kind > 0); next: [s in | gain] of the one that comes.
+template <typename T, int S, int V>
+__global__ __launch_bounds__(512) void hyper_update_kernel(const float* x, const int64_t* __restrict__ ids, const T* __restrict__ table,
+                                                           float emb_scale, int64_t vocab, float* x_out, SublayerResult r,
+                                                           const float* __restrict__ cur, const float* __restrict__ next, T* __restrict__ h,
+                                                           int64_t W, float eps) {
+    extern __shared__ float urow[];
+    __shared__ float red[8];
+    const int64_t row = blockIdx.x;
+    const int64_t tok = ids ? min(max(ids[row], (int64_t)0), vocab - 1) : 0;
+    float cin[S], cout[S], mix[S][S];
+#pragma unroll
+    for (int a = 0; a < S; ++a) {
+        cin[a] = next[a];
+        cout[a] = r.kind ? cur[S * S + a] : 0.f;
+#pragma unroll
+        for (int b = 0; b < S; ++b) mix[a][b] = r.kind ? cur[a * S + b] : 0.f;
+    }
+    float ss = 0.f;
+    for (int64_t c = (int64_t)threadIdx.x * V; c < W; c += (int64_t)blockDim.x * V) {
+        f32x4 X[S], N[S];
+        if (ids) {
+            const f32x4 e = LdV<T, V>::ld(table + tok * W + c) * emb_scale;
+#pragma unroll
+            for (int a = 0; a < S; ++a) X[a] = e;
+        } else {
+#pragma unroll
+            for (int a = 0; a < S; ++a) X[a] = LdV<float, V>::ld(x + (row * S + a) * W + c);
+        }
+        if (r.kind) {
+            const f32x4 y = result_at<T, V>(r, row, c);
+#pragma unroll
+            for (int b = 0; b < S; ++b) {
+                N[b] = y * cout[b];
+#pragma unroll
+                for (int a = 0; a < S; ++a) N[b] += X[a] * mix[a][b];
+            }
+        } else {
+#pragma unroll
+            for (int a = 0; a < S; ++a) N[a] = X[a];
+        }
+        f32x4 u = {};
+#pragma unroll
+        for (int a = 0; a < S; ++a) {
+            if (x_out) LdV<float, V>::st(x_out + (row * S + a) * W + c, N[a]);
+            u += N[a] * cin[a];
+        }
+#pragma unroll
+        for (int i = 0; i < V; ++i) {
+            urow[c + i] = u[i];
+            ss += u[i] * u[i];
+        }
+    }
+    ss = block_sum(ss, red);
+    const float f = next[S] / sqrtf(ss / (float)W + eps);
+    // a thread reads back what it wrote itself
+    for (int64_t c = (int64_t)threadIdx.x * V; c < W; c += (int64_t)blockDim.x * V) {
+        f32x4 u = {};
+#pragma unroll
+        for (int i = 0; i < V; ++i) u[i] = urow[c + i] * f;
+        LdV<T, V>::st(h + row * W + c, u);
+    }
+}
+
+template <typename T, int S>
+void launch_s(bool vec, const float* x, const int64_t* ids, const void* table, float emb_scale, int64_t vocab, float* x_out,
+              const SublayerResult& r, const float* cur, const float* next, void* h, int64_t rows, int64_t W, float eps, hipStream_t st) {
+    const int64_t lanes = vec ? W / 4 : W;
+    const int nt = (int)(lanes >= 512 ? 512 : (lanes + 63) / 64 * 64);
+    if (vec)
+        hipLaunchKernelGGL((hyper_update_kernel<T, S, 4>), dim3((unsigned)rows), dim3(nt), (size_t)W * 4, st, x, ids, (const T*)table, emb_scale,
+                           vocab, x_out, r, cur, next, (T*)h, W, eps);
+    else
+        hipLaunchKernelGGL((hyper_update_kernel<T, S, 1>), dim3((unsigned)rows), dim3(nt), (size_t)W * 4, st, x, ids, (const T*)table, emb_scale,
+                           vocab, x_out, r, cur, next, (T*)h, W, eps);
+}
+
+template <typename T>
+void launch_t(int S, bool vec, const float* x, const int64_t* ids, const void* table, float emb_scale, int64_t vocab, float* x_out,
+              const SublayerResult& r, const float* cur, const float* next, void* h, int64_t rows, int64_t W, float eps, hipStream_t st) {
+#define TGIS_HYPER(N) \
+    case N: return launch_s<T, N>(vec, x, ids, table, emb_scale, vocab, x_out, r, cur, next, h, rows, W, eps, st)
+    switch (S) {
+        TGIS_HYPER(1);
+        TGIS_HYPER(2);
+        TGIS_HYPER(3);
+        TGIS_HYPER(4);
+        TGIS_HYPER(5);
+        TGIS_HYPER(6);
+        TGIS_HYPER(7);
+        TGIS_HYPER(8);
+    }
+#undef TGIS_HYPER
+}
+
+}  // namespace
+
+extern "C" int tgis_hyper_update(const float* x, const int64_t* ids, const void* table, int64_t vocab, float emb_scale, float* x_out,
+                                 int kind, const void* y, int64_t ld_y, int slabs, const int32_t* pos, const float* weight, int k,
+                                 const void* shared, int64_t ld_shared, int shared_slabs, const float* shared_gate, const float* cur,
+                                 const float* next, void* h, int64_t rows, int64_t W, int streams, float eps, int dtype, void* stream) {
+    TGIS_CHECK_ARG(dtype == TGIS_F16 || dtype == TGIS_BF16 || dtype == TGIS_F32, "tgis_hyper_update: bad dtype");
+    TGIS_CHECK_ARG((x != nullptr) != (ids != nullptr) && next && h && (!ids || (table && vocab >= 1 && kind == 0)),
+                   "tgis_hyper_update: streams, or token ids and their table (and then no sublayer result)");
+    TGIS_CHECK_ARG(streams >= 1 && streams <= MAX_STREAMS && W >= 1 && W * 4 <= 64 * 1024,
+                   "tgis_hyper_update: 1 .. %d streams of up to 16384 channels (got %d of %ld)", MAX_STREAMS, streams, (long)W);
+    TGIS_CHECK_ARG(kind >= 0 && kind <= 3 && (kind == 0 || (y && cur && ld_y >= W)) && (kind != 2 || slabs >= 1) && (kind != 3 || (pos && k >= 1)) &&
+                       (!shared || (kind == 3 && ld_shared >= W && shared_slabs >= 0)),
+                   "tgis_hyper_update: bad sublayer result (kind %d)", kind);
+    if (rows == 0) return TGIS_OK;
+    hipStream_t st = (hipStream_t)stream;
+    TgisTimedScope timed(TGIS_OP_NORM, st);
+    SublayerResult r{kind, y, ld_y, slabs, pos, weight, k, shared, ld_shared, shared_slabs, shared_gate};
+    auto al = [](const void* p, size_t n) { return ((uintptr_t)p % n) == 0; };
+    const size_t e4 = dtype == TGIS_F32 ? 16 : 8;
+    const bool vec = W % 4 == 0 && al(x, 16) && al(x_out, 16) && al(table, e4) && al(h, e4) && (kind == 0 || ld_y % 4 == 0) &&
+                     al(y, kind == 2 ? 16 : e4) && (!shared || (ld_shared % 4 == 0 && al(shared, shared_slabs > 0 ? 16 : e4)));
+    if (dtype == TGIS_F16)
+        launch_t<f16>(streams, vec, x, ids, table, emb_scale, vocab, x_out, r, cur, next, h, rows, W, eps, st);
+    else if (dtype == TGIS_BF16)
+        launch_t<bf16>(streams, vec, x, ids, table, emb_scale, vocab, x_out, r, cur, next, h, rows, W, eps, st);
+    else
+        launch_t<float>(streams, vec, x, ids, table, emb_scale, vocab, x_out, r, cur, next, h, rows, W, eps, st);
+    TGIS_CHECK_LAUNCH();
+    return TGIS_OK;
+}

@@ -13,6 +13,7 @@
 // The number of tiles is data dependent; the grid is sized for the worst case (T k + E * 31 rows) and tiles past n_tiles
 // leave at once.
 #include "common.h"
+#include "mfma_frag.h"
 
 namespace {
 
@@ -170,55 +171,27 @@ __global__ __launch_bounds__(1024) void moe_align_kernel(const int32_t* __restri
 // Workgroup = 4 waves = one 32-row tile x 128 output columns; a wave owns 32 columns (GLU: 32 gate + the 32 matching up
 // columns).  Operands come straight from global memory / L2 in MFMA fragment order: lane l holds row (l % 32) and 8 (bf16)
 // or 4 (fp32) consecutive k at offset (l / 32) * that — a 16-byte load for A and for B ([out, in] weights are k-contiguous).
-template <typename T> struct Frag;
-template <> struct Frag<bf16> {
-    static constexpr int KSTEP = 16, PER = 8;
-    using V = bf16x8;
-    static __device__ __forceinline__ V zero() { return V{}; }
-    static __device__ __forceinline__ V scaled(V a, float s) {
-        V r;
-#pragma unroll
-        for (int i = 0; i < 8; ++i) r[i] = (bf16)((float)a[i] * s);
-        return r;
-    }
-    static __device__ __forceinline__ void mma(V a, V b, f32x16& c) { c = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, b, c, 0, 0, 0); }
-};
-template <> struct Frag<f16> {
-    static constexpr int KSTEP = 16, PER = 8;
-    using V = f16x8;
-    static __device__ __forceinline__ V zero() { return V{}; }
-    static __device__ __forceinline__ V scaled(V a, float s) {
-        V r;
-#pragma unroll
-        for (int i = 0; i < 8; ++i) r[i] = (f16)((float)a[i] * s);
-        return r;
-    }
-    static __device__ __forceinline__ void mma(V a, V b, f32x16& c) { c = __builtin_amdgcn_mfma_f32_32x32x16_f16(a, b, c, 0, 0, 0); }
-};
-template <> struct Frag<float> {
-    static constexpr int KSTEP = 8, PER = 4;
-    using V = f32x4;
-    static __device__ __forceinline__ V zero() { return V{}; }
-    static __device__ __forceinline__ V scaled(V a, float s) { return a * s; }
-    // four 32x32x2 fp32 products: the k index a lane contributes to product i is (l / 32) * 4 + i, for A and B alike
-    static __device__ __forceinline__ void mma(V a, V b, f32x16& c) {
-#pragma unroll
-        for (int i = 0; i < 4; ++i) c = __builtin_amdgcn_mfma_f32_32x32x2f32(a[i], b[i], c, 0, 0, 0);
-    }
-};
-
 // Two shapes of workgroup (4 waves):
 //   many tiles (prompts): wave w owns row tile 4 y + w and 64 output columns (GLU: 64 gate + the 64 matching up columns).  The
 //     four waves walk the same weight rows at the same time, so an expert's weights come from L2 once per four row tiles
 //     instead of once per tile, and a wave's A fragment feeds two (GLU: four) products;
 //   few tiles (decode, KSPLIT): the four waves split K for ONE 32-row x 32-column block and meet in LDS, so that a launch with a
 //     handful of tiles still has enough waves in flight to stream the expert weights.
-template <typename T, bool GLU, bool KSPLIT>
+//
+// GLU 1: silu(gate) * up.  GLU 2 (clamped unit): g = min(gate, limit), u = clamp(up, +-limit): g sigmoid(alpha g) (u + 1).
+template <int GLU> __device__ __forceinline__ float gated(float g, float u, float alpha, float limit) {
+    if (GLU == 1) return g / (1.f + expf(-g)) * u;
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g / (1.f + expf(-alpha * g)) * (u + 1.f);
+}
+
+template <typename T, int GLU, bool KSPLIT>
 __global__ __launch_bounds__(256) void moe_gemm_kernel(const T* __restrict__ A, int64_t ld_a, const int32_t* __restrict__ sorted,
                                                        int pair_div, const float* __restrict__ pair_scale,
                                                        const int32_t* __restrict__ tile_expert, const int32_t* __restrict__ n_tiles,
                                                        const T* __restrict__ Wt, int64_t expert_stride, int64_t N, int64_t K,
-                                                       T* __restrict__ out, int64_t ld_out) {
+                                                       T* __restrict__ out, int64_t ld_out, float alpha, float limit) {
     using F = Frag<T>;
     using V = typename F::V;
     constexpr int NB = KSPLIT ? 1 : 2;  // 32-column blocks per wave
@@ -290,7 +263,7 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const T* __restrict__ A, 
                 v += part[((w * NA + 0) * 16 + i) * 64 + lane];
                 if (GLU) v2 += part[((w * NA + 1) * 16 + i) * 64 + lane];
             }
-            if (GLU) v = v / (1.f + expf(-v)) * v2;
+            if (GLU) v = gated<GLU>(v, v2, alpha, limit);
             const int m = (i >> 2) * 8 + half * 4 + (i & 3);
             out[((int64_t)tile * TM + m) * ld_out + n0 + row] = (T)v;
         }
@@ -304,7 +277,7 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const T* __restrict__ A, 
             for (int i = 0; i < 16; ++i) {
                 const int m = (i >> 2) * 8 + half * 4 + (i & 3);
                 float v = acc[nb][i];
-                if (GLU) v = v / (1.f + expf(-v)) * acc2[nb][i];
+                if (GLU) v = gated<GLU>(v, acc2[nb][i], alpha, limit);
                 out[((int64_t)tile * TM + m) * ld_out + n] = (T)v;
             }
         }
@@ -331,22 +304,26 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const T* __restrict__ 
 }
 
 template <typename T>
-void launch_gemm(bool glu, const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
+void launch_gemm(int glu, float alpha, float limit, const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
                  const int32_t* tile_expert, const int32_t* n_tiles, const void* Wt, int64_t expert_stride, int64_t N, int64_t K,
                  void* out, int64_t ld_out, int64_t max_tiles, hipStream_t st) {
     const bool ksplit = max_tiles * cdiv64(N, 128) < 1024;
     dim3 grid((unsigned)(ksplit ? cdiv64(N, 32) : cdiv64(N, 64)), (unsigned)(ksplit ? max_tiles : cdiv64(max_tiles, 4)));
 #define TGIS_MOE_LAUNCH(GLU, KS)                                                                                              \
     hipLaunchKernelGGL((moe_gemm_kernel<T, GLU, KS>), grid, dim3(256), 0, st, (const T*)A, ld_a, sorted, pair_div, pair_scale, \
-                       tile_expert, n_tiles, (const T*)Wt, expert_stride, N, K, (T*)out, ld_out)
-    if (glu && ksplit)
-        TGIS_MOE_LAUNCH(true, true);
+                       tile_expert, n_tiles, (const T*)Wt, expert_stride, N, K, (T*)out, ld_out, alpha, limit)
+    if (glu == 2 && ksplit)
+        TGIS_MOE_LAUNCH(2, true);
+    else if (glu == 2)
+        TGIS_MOE_LAUNCH(2, false);
+    else if (glu && ksplit)
+        TGIS_MOE_LAUNCH(1, true);
     else if (glu)
-        TGIS_MOE_LAUNCH(true, false);
+        TGIS_MOE_LAUNCH(1, false);
     else if (ksplit)
-        TGIS_MOE_LAUNCH(false, true);
+        TGIS_MOE_LAUNCH(0, true);
     else
-        TGIS_MOE_LAUNCH(false, false);
+        TGIS_MOE_LAUNCH(0, false);
 #undef TGIS_MOE_LAUNCH
 }
 
@@ -411,9 +388,9 @@ extern "C" int tgis_moe_align(const int32_t* idx, int64_t n_pairs, int E, int32_
     return TGIS_OK;
 }
 
-extern "C" int tgis_moe_gemm(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
+static int moe_gemm_impl(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
                              const int32_t* tile_expert, const int32_t* n_tiles, const void* weights, int64_t expert_stride, int64_t N,
-                             int64_t K, int glu, void* out, int64_t ld_out, int64_t capacity, int dtype, void* stream) {
+                             int64_t K, int glu, void* out, int64_t ld_out, int64_t capacity, int dtype, void* stream, float alpha, float limit) {
     TGIS_CHECK_ARG(A && tile_expert && n_tiles && weights && out, "tgis_moe_gemm: null tensor");
     TGIS_CHECK_ARG(dtype3(dtype), "tgis_moe_gemm: bad dtype");
     const int per = dtype == TGIS_F32 ? 4 : 8;
@@ -429,13 +406,30 @@ extern "C" int tgis_moe_gemm(const void* A, int64_t ld_a, const int32_t* sorted,
     const int64_t tiles = capacity / TM;
     TGIS_CHECK_ARG(tiles <= 65535, "tgis_moe_gemm: %ld tiles exceed one grid", (long)tiles);
     if (dtype == TGIS_F16)
-        launch_gemm<f16>(glu != 0, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, out, ld_out, tiles, st);
+        launch_gemm<f16>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, out, ld_out, tiles, st);
     else if (dtype == TGIS_BF16)
-        launch_gemm<bf16>(glu != 0, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, out, ld_out, tiles, st);
+        launch_gemm<bf16>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, out, ld_out, tiles, st);
     else
-        launch_gemm<float>(glu != 0, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, out, ld_out, tiles, st);
+        launch_gemm<float>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, out, ld_out, tiles, st);
     TGIS_CHECK_LAUNCH();
     return TGIS_OK;
+}
+
+extern "C" int tgis_moe_gemm(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
+                             const int32_t* tile_expert, const int32_t* n_tiles, const void* weights, int64_t expert_stride, int64_t N,
+                             int64_t K, int glu, void* out, int64_t ld_out, int64_t capacity, int dtype, void* stream) {
+    return moe_gemm_impl(A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, glu != 0 ? 1 : 0, out, ld_out,
+                         capacity, dtype, stream, 0.f, 0.f);
+}
+
+// The same over stacked [gate | up] weights with the clamped unit: g = min(gate, limit), u = clamp(up, -limit, limit),
+// g * sigmoid(alpha * g) * (u + 1).
+extern "C" int tgis_moe_gemm_clamped(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
+                                     const int32_t* tile_expert, const int32_t* n_tiles, const void* weights, int64_t expert_stride, int64_t N,
+                                     int64_t K, float alpha, float limit, void* out, int64_t ld_out, int64_t capacity, int dtype,
+                                     void* stream) {
+    return moe_gemm_impl(A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, 2, out, ld_out, capacity,
+                         dtype, stream, alpha, limit);
 }
 
 extern "C" int tgis_moe_combine(const void* rows, int64_t ld_rows, const int32_t* pos_of_pair, const float* pair_weight, int k,

@@ -6,26 +6,9 @@
 // f16 or float; statistics, gains and the residual itself are always float.
 #include <type_traits>
 #include "common.h"
+#include "row_io.h"
 
 namespace {
-
-template <typename T> struct Elem;
-template <> struct Elem<f16> { static __device__ __forceinline__ float ld(const f16* p) { return (float)*p; } };
-template <> struct Elem<bf16> { static __device__ __forceinline__ float ld(const bf16* p) { return (float)*p; } };
-template <> struct Elem<float> { static __device__ __forceinline__ float ld(const float* p) { return *p; } };
-template <typename T> __device__ __forceinline__ T cvt_out(float v) { return (T)v; }
-
-__device__ __forceinline__ float block_sum(float v, float* red) {
-    // every thread of the block calls this; red holds one float per wave (<= 16)
-    v = wave_sum(v);
-    const int wave = threadIdx.x >> 6, nw = (blockDim.x + 63) >> 6;
-    __syncthreads();  // red may still be read from a previous call
-    if ((threadIdx.x & 63) == 0) red[wave] = v;
-    __syncthreads();
-    float s = 0.f;
-    for (int i = 0; i < nw; ++i) s += red[i];
-    return s;
-}
 
 template <typename T>
 __global__ void embedding_scaled_kernel(const int64_t* __restrict__ ids, const T* __restrict__ table, float* __restrict__ out,
@@ -143,33 +126,6 @@ __global__ __launch_bounds__(256) void sandwich_norm_reg_kernel(const float* x, 
 }
 
 
-// The same again for E % 4 == 0 and E <= 512 * 4 * NV: 512 threads, 16-byte loads and stores (a thread owns NV groups of four
-// consecutive elements).  This is the form decode-sized steps run: few rows, so the launch is a chain of round trips and the
-// number of memory instructions in it is what counts.
-template <typename T> struct Vec4;
-template <> struct Vec4<float> {
-    static __device__ __forceinline__ f32x4 ld(const float* p) { return *reinterpret_cast<const f32x4*>(p); }
-    static __device__ __forceinline__ void st(float* p, f32x4 v) { *reinterpret_cast<f32x4*>(p) = v; }
-};
-template <> struct Vec4<bf16> {
-    static __device__ __forceinline__ f32x4 ld(const bf16* p) {
-        bf16x4 v = *reinterpret_cast<const bf16x4*>(p);
-        return f32x4{(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
-    }
-    static __device__ __forceinline__ void st(bf16* p, f32x4 v) {
-        *reinterpret_cast<bf16x4*>(p) = bf16x4{(bf16)v[0], (bf16)v[1], (bf16)v[2], (bf16)v[3]};
-    }
-};
-template <> struct Vec4<f16> {
-    static __device__ __forceinline__ f32x4 ld(const f16* p) {
-        f16x4 v = *reinterpret_cast<const f16x4*>(p);
-        return f32x4{(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
-    }
-    static __device__ __forceinline__ void st(f16* p, f32x4 v) {
-        *reinterpret_cast<f16x4*>(p) = f16x4{(f16)v[0], (f16)v[1], (f16)v[2], (f16)v[3]};
-    }
-};
-
 
 // four elements per thread (I % 4 == 0, rows 8- / 16-byte aligned)
 template <typename T>
@@ -194,6 +150,9 @@ __global__ void glu_vec_kernel(const T* __restrict__ in, int64_t ld_in, T* __res
     }
 }
 
+// The same again for E % 4 == 0 and E <= 512 * 4 * NV: 512 threads, 16-byte loads and stores (a thread owns NV groups of four
+// consecutive elements).  This is the form decode-sized steps run: few rows, so the launch is a chain of round trips and the
+// number of memory instructions in it is what counts.
 // delta may also arrive as the S fp32 split-K slabs of the GEMM that produced it ([row / 32][S][32][slab_ld], TD = float,
 // `delta` then points at the slabs): their sum is taken here instead of by a reduce launch of its own.
 template <typename TD, typename TY, int NV>
@@ -446,16 +405,6 @@ struct GatedDelta {
     const void* gate;
     int64_t ld_gate;
     const void* gate_bias;
-};
-
-template <typename T, int V> struct LdV;
-template <typename T> struct LdV<T, 1> {
-    static __device__ __forceinline__ f32x4 ld(const T* p) { return f32x4{Elem<T>::ld(p), 0.f, 0.f, 0.f}; }
-    static __device__ __forceinline__ void st(T* p, f32x4 v) { *p = cvt_out<T>(v[0]); }
-};
-template <typename T> struct LdV<T, 4> {
-    static __device__ __forceinline__ f32x4 ld(const T* p) { return Vec4<T>::ld(p); }
-    static __device__ __forceinline__ void st(T* p, f32x4 v) { Vec4<T>::st(p, v); }
 };
 
 template <typename TD, int V>

@@ -18,10 +18,11 @@ FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-Xclang", "-tar
 # translation units per family (api.hip: error state / version; elementwise.hip: decode bookkeeping, argmax)
 FAMILY_UNITS = {
     "lenisun": ["api", "elementwise", "gemm_dense", "residual_f32", "attn_varlen", "wkv", "moe", "sampler"],
-    "senadra": ["api", "elementwise", "gemm_dense", "residual_f32", "attn_varlen", "delta_rule", "sampler"],
+    "senadra": ["api", "elementwise", "gemm_dense", "residual_f32", "attn_varlen", "head_product", "delta_rule", "sampler"],
     "mananex": ["api", "elementwise", "gemm_dense", "residual_f32", "attn_varlen", "gated_linear_scan", "moe", "sampler"],
     "tatevik": ["api", "elementwise", "gemm_dense", "residual_f32", "norm_f32", "attn_varlen", "attn_mixed_heads", "gated_linear_scan",
                 "selective_scan", "causal_conv", "moe", "sampler"],
+    "gopetar": ["api", "elementwise", "gemm_dense", "residual_f32", "hyper_streams", "attn_varlen", "head_product", "min_gru", "moe", "sampler"],
 }
 
 

@@ -76,6 +76,7 @@ class KVArgs:
     state: "object" = None             # utils.state_cache.RecurrentStateCache
     state_slots: Optional[torch.Tensor] = None  # [B] int32 (device)
     cu_seqlens_q: Optional[torch.Tensor] = None  # [B + 1] int32, for mixers that get the step description from here
+    turns: Optional[dict] = None       # rotation tables of this step's tokens, made by the first layer that asks (utils/mixers.py)
     residual_trace: Optional[list] = None  # debugging: models that support it append the residual stream after every layer
 
 

@@ -19,7 +19,7 @@ F16, BF16, F32 = 0, 1, 2
 KV_PAGE_TOKENS = 32
 
 OP_GPTQ_GEMM, OP_ATTN, OP_DENSE_GEMM, OP_NORM, OP_ROPE_KV, OP_ACT, OP_SAMPLE = range(7)
-OP_SCAN, OP_MOE_GEMM = 8, 9
+OP_SCAN, OP_MOE_GEMM, OP_HEAD_PRODUCT = 8, 9, 10
 
 _c_i64 = ctypes.c_int64
 _c_int = ctypes.c_int
@@ -159,6 +159,21 @@ SIGNATURES = {
     "tgis_rms_pair_mean": (_c_int, [_vp, _c_i64, _c_int, _vp, _c_f, _vp, _c_i64, _c_int, _vp, _c_f, _vp, _c_i64, _c_i64, _c_f, _c_int, _vp]),
     "tgis_poly_norm": (_c_int, [_vp, _c_i64, _vp, _c_i64, _c_i64, _c_i64, _c_f, _c_f, _c_f, _c_f, _c_f, _c_int, _vp]),
     "tgis_moe_route_grouped": (_c_int, [_vp, _c_i64, _vp, _vp, _c_int, _c_int, _c_f, _vp, _vp, _c_i64, _c_i64, _c_int, _c_int, _c_int, _vp]),
+    "tgis_pair_turns": (_c_int, [_vp, _vp, _vp, _c_i64, _c_int, _vp]),
+    "tgis_rope_rows_turned_kv_write": (_c_int, [_vp, _c_i64, _c_i64, _c_i64, _c_i64, _vp, _vp, _vp, _vp, _vp, _c_i64, _c_int, _c_int,
+                                                _c_int, _c_int, _c_int, _vp, _c_int, _vp]),
+    "tgis_attn_varlen_turned": (_c_int, [_vp, _c_i64, _vp, _vp, _vp, _c_i64, _vp, _vp, _c_i64, _vp, _c_i64, _c_i64, _c_i64, _c_i64,
+                                         _c_int, _c_int, _c_int, _c_int, _c_f, _c_int, _c_int, _vp, _c_f, _vp, _c_f, _vp, _c_i64, _c_int,
+                                         _c_int, _vp]),
+    "tgis_latent_norm_write": (_c_int, [_vp, _c_i64, _c_i64, _c_i64, _vp, _vp, _c_i64, _c_i64, _c_i64, _vp, _vp, _vp, _vp, _c_i64, _c_f,
+                                        _c_int, _vp]),
+    "tgis_head_product": (_c_int, [_vp, _c_i64, _c_i64, _vp, _vp, _c_i64, _c_i64, _c_i64, _c_int, _c_int, _c_int, _c_int, _vp]),
+    "tgis_min_gru_scan": (_c_int, [_vp, _c_i64, _c_i64, _c_i64, _c_i64, _vp, _vp, _vp, _vp, _vp, _c_i64, _c_f, _c_i64, _c_i64, _c_i64,
+                                   _c_i64, _c_int, _vp]),
+    "tgis_moe_gemm_clamped": (_c_int, [_vp, _c_i64, _vp, _c_int, _vp, _vp, _vp, _vp, _c_i64, _c_i64, _c_i64, _c_f, _c_f, _vp, _c_i64,
+                                       _c_i64, _c_int, _vp]),
+    "tgis_hyper_update": (_c_int, [_vp, _vp, _vp, _c_i64, _c_f, _vp, _c_int, _vp, _c_i64, _c_int, _vp, _vp, _c_int, _vp, _c_i64, _c_int,
+                                   _vp, _vp, _vp, _vp, _c_i64, _c_i64, _c_int, _c_f, _c_int, _vp]),
 }
 
 _lib = None
@@ -1020,12 +1035,19 @@ def moe_align(idx: torch.Tensor, E: int):
 
 
 def moe_gemm(A, weights, N: int, tile_expert, n_tiles, capacity: int, sorted_=None, pair_div: int = 1, pair_scale=None,
-             glu_act: bool = False):
-    """weights [E, N (glu: 2 N), K]; returns [capacity, N]."""
+             glu_act: bool = False, clamp=None):
+    """weights [E, N (glu: 2 N), K]; returns [capacity, N].  glu_act: silu(gate) * up, or with clamp = (alpha, limit) the clamped
+    unit."""
     assert A.dim() == 2 and A.stride(1) == 1 and weights.dim() == 3 and weights.is_contiguous() and weights.dtype == A.dtype
     K = weights.shape[2]
     assert weights.shape[1] == (2 * N if glu_act else N) and A.shape[1] == K
     out = torch.empty((capacity, N), dtype=A.dtype, device=A.device)
+    if glu_act and clamp is not None:
+        _check(load_library().tgis_moe_gemm_clamped(
+            _ptr(A), A.stride(0), _i32(sorted_, "sorted"), pair_div, _f32(pair_scale, "pair_scale"), _ptr(tile_expert), _ptr(n_tiles),
+            _ptr(weights), weights.stride(0), N, K, float(clamp[0]), float(clamp[1]), _ptr(out), out.stride(0), capacity,
+            dtype_code3(A.dtype), _stream()), "tgis_moe_gemm_clamped")
+        return out
     _check(load_library().tgis_moe_gemm(
         _ptr(A), A.stride(0), _i32(sorted_, "sorted"), pair_div, _f32(pair_scale, "pair_scale"), _ptr(tile_expert), _ptr(n_tiles),
         _ptr(weights), weights.stride(0), N, K, int(glu_act), _ptr(out), out.stride(0), capacity, dtype_code3(A.dtype), _stream()),
@@ -1468,3 +1490,131 @@ def moe_route_grouped(h, router_w, correction, k: int, n_groups: int = 1, keep_g
                                                  int(n_groups), int(keep_groups), float(renorm_eps), _ptr(idx), _ptr(weight), T, W, E, k,
                                                  dtype_code3(h.dtype), _stream()), "tgis_moe_route_grouped")
     return idx, weight
+
+
+# ---- several residual streams, rotated values, latent attention without positions, minGRU ---------------------------------------
+def pair_turns(positions: torch.Tensor, inv_freq: torch.Tensor) -> torch.Tensor:
+    """[T, n, 2] fp32: (cos, sin) of positions[t] * inv_freq[i]."""
+    T, n = positions.shape[0], inv_freq.shape[0]
+    out = torch.empty((T, n, 2), dtype=torch.float32, device=positions.device)
+    _check(load_library().tgis_pair_turns(_i32(positions, "positions"), _f32(inv_freq, "inv_freq"), _ptr(out), T, n, _stream()),
+           "tgis_pair_turns")
+    return out
+
+
+def rope_rows_turned_kv_write(proj, q_col0: int, k_col0: int, v_col0: int, inv_freq, positions, slots, k_pool, v_pool, H: int, G: int,
+                              dk: int, dv: int, rot_dims: int, v_turns: torch.Tensor):
+    """rope_rows_kv_write, and the values are turned by v_turns [T, dv / 2, 2] on their way into the V pages."""
+    assert proj.dim() == 2 and proj.stride(1) == 1 and k_pool.dtype == proj.dtype and v_pool.dtype == proj.dtype
+    assert positions.shape[0] == proj.shape[0] and slots.shape[0] == proj.shape[0]
+    assert (rot_dims == 0 or inv_freq.shape[0] >= rot_dims // 2) and tuple(v_turns.shape) == (proj.shape[0], dv // 2, 2)
+    _check(load_library().tgis_rope_rows_turned_kv_write(
+        _ptr(proj), proj.stride(0), q_col0, k_col0, v_col0, _f32(inv_freq, "inv_freq") if rot_dims else None, _i32(positions, "positions"),
+        _i32(slots, "slots"), _ptr(k_pool), _ptr(v_pool), proj.shape[0], H, G, dk, dv, rot_dims, _f32(v_turns, "v_turns"),
+        dtype_code3(proj.dtype), _stream()), "tgis_rope_rows_turned_kv_write")
+
+
+def attn_varlen_turned(q, k_pool, v_pool, block_tables, ctx_lens, cu_seqlens_q, H: int, G: int, dk: int, dv: int, scale: float,
+                       window: int = 0, keep_first: int = 0, sink=None, softcap: float = 0.0, turns=None, out_scale: float = 1.0,
+                       out=None, max_q_len: int = 1, max_ctx: int = 1, impl: int = 0, ws: Optional[Workspace] = None):
+    """attn_varlen_win (no gate) with capped scores and / or outputs turned back by turns [T, dv / 2, 2]."""
+    assert q.dim() == 2 and q.stride(1) == 1 and block_tables.dim() == 2
+    T = q.shape[0]
+    assert (sink is None or sink.shape[0] == H) and (turns is None or tuple(turns.shape) == (T, dv // 2, 2))
+    if out is None:
+        out = torch.empty((T, H * dv), dtype=q.dtype, device=q.device)
+    assert out.shape == (T, H * dv) and out.stride(1) == 1 and out.dtype == q.dtype
+    _check(load_library().tgis_attn_varlen_turned(
+        _ptr(q), q.stride(0), _ptr(k_pool), _ptr(v_pool), _i32(block_tables, "block_tables"), block_tables.shape[1],
+        _i32(ctx_lens, "ctx_lens"), _i32(cu_seqlens_q, "cu_seqlens_q"), ctx_lens.shape[0], _ptr(out), out.stride(0), T,
+        max(int(max_q_len), 1), max(int(max_ctx), 1), H, G, dk, dv, float(scale), int(window), int(keep_first), _f32(sink, "sink"),
+        float(softcap), _f32(turns, "turns"), float(out_scale), (ws.ptr + 4096) if ws is not None else None,
+        (ws.nbytes - 4096) if ws is not None else 0, impl, dtype_code3(q.dtype), _stream()), "tgis_attn_varlen_turned")
+    return out
+
+
+def latent_norm_write(down, q_col0: int, q_rank: int, q_gain, c_col0: int, kv_rank: int, c_gain, slots, k_pool, v_pool, eps: float):
+    """The normed query latent [T, q_rank] of the down-projection; the normed cache latent goes to its page slots."""
+    assert down.dim() == 2 and down.stride(1) == 1 and k_pool.dtype == down.dtype and v_pool.dtype == down.dtype
+    assert slots.shape[0] == down.shape[0] and q_gain.shape[0] == q_rank and c_gain.shape[0] == kv_rank
+    cq = torch.empty((down.shape[0], q_rank), dtype=down.dtype, device=down.device)
+    _check(load_library().tgis_latent_norm_write(
+        _ptr(down), down.stride(0), int(q_col0), int(q_rank), _f32(q_gain, "q_gain"), _ptr(cq), cq.stride(0), int(c_col0), int(kv_rank),
+        _f32(c_gain, "c_gain"), _i32(slots, "slots"), _ptr(k_pool), _ptr(v_pool), down.shape[0], float(eps), dtype_code3(down.dtype),
+        _stream()), "tgis_latent_norm_write")
+    return cq
+
+
+def head_product(x: torch.Tensor, head_stride_x: int, w: torch.Tensor, out: torch.Tensor, head_stride_out: int) -> torch.Tensor:
+    """out[t, h * head_stride_out + n] = sum_k x[t, h * head_stride_x + k] w[h, n, k] for w [H, N, K]."""
+    H, N, K = w.shape
+    assert x.dim() == 2 and x.stride(1) == 1 and out.dim() == 2 and out.stride(1) == 1 and out.shape[0] == x.shape[0]
+    assert w.is_contiguous() and w.dtype == x.dtype and out.dtype == x.dtype
+    assert x.shape[1] >= (H - 1) * head_stride_x + K and out.shape[1] >= (H - 1) * head_stride_out + N
+    _check(load_library().tgis_head_product(_ptr(x), x.stride(0), int(head_stride_x), _ptr(w), _ptr(out), out.stride(0), int(head_stride_out),
+                                            x.shape[0], H, N, K, dtype_code3(x.dtype), _stream()), "tgis_head_product")
+    return out
+
+
+def min_gru_scan(proj, z_col0: int, x_col0: int, g_col0: int, state, state_slots, cu_seqlens_q, positions, D: int, out=None,
+                 out_scale: float = 1.0, max_q_len: int = 0) -> torch.Tensor:
+    """S <- (1 - z) S + z cand per channel on columns of proj [T, ld]; S * silu(g) * out_scale -> [T, D] (or the view `out`)."""
+    assert proj.dim() == 2 and proj.stride(1) == 1
+    T = proj.shape[0]
+    if out is None:
+        out = torch.empty((T, D), dtype=proj.dtype, device=proj.device)
+    assert out.shape == (T, D) and out.stride(1) == 1 and out.dtype == proj.dtype
+    assert state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:].numel() == D
+    _check(load_library().tgis_min_gru_scan(
+        _ptr(proj), proj.stride(0), int(z_col0), int(x_col0), int(g_col0), _ptr(state), _i32(state_slots, "state_slots"),
+        _i32(cu_seqlens_q, "cu_seqlens_q"), _i32(positions, "positions"), _ptr(out), out.stride(0), float(out_scale),
+        state_slots.shape[0], T, int(max_q_len) if max_q_len > 0 else max(T, 1), D, dtype_code3(proj.dtype), _stream()),
+        "tgis_min_gru_scan")
+    return out
+
+
+class MixtureRows:
+    """A mixture of experts before its sum: expert rows [cap, W], the row of every (token, choice), the choices' weights, and a
+    gated shared row per token (a tensor or split-K slabs)."""
+
+    def __init__(self, rows, pos, weight, k: int, shared=None, shared_gate=None):
+        self.rows, self.pos, self.weight, self.k, self.shared, self.shared_gate = rows, pos, weight, k, shared, shared_gate
+
+
+def hyper_update(x, y, cur, nxt, eps: float, y_dtype, ids=None, table=None, emb_scale: float = 1.0, x_out=None, streams: int = 0):
+    """x [T, s, W] fp32: x_out (in place unless given) <- mix x + out y, and h = rms_norm(sum_a in[a] x_out[a]) * gain in y_dtype.
+    cur = [s * s | s], nxt = [s | 1] fp32 coefficient rows; y: a tensor of y_dtype, split-K slabs (`Partial`), `MixtureRows`, or None
+    (x stays).  ids + table instead of x: the streams begin as copies of the scaled embedding rows (s = `streams`).  Returns
+    (x_out, h)."""
+    if ids is not None:
+        assert x is None and y is None and ids.dtype == torch.int64 and table.is_contiguous() and table.dtype == y_dtype
+        T, s, W = ids.shape[0], int(streams), table.shape[1]
+        x_out = torch.empty((T, s, W), dtype=torch.float32, device=table.device)
+    else:
+        T, s, W = x.shape
+        assert x.dtype == torch.float32 and x.is_contiguous()
+        x_out = x if x_out is None else x_out
+    assert nxt.shape[0] == s + 1 and (y is None or cur.shape[0] == s * s + s)
+    kind, p, ld, slabs, pos, weight, k, sh, ld_sh, sh_slabs, gate = 0, None, 0, 0, None, None, 0, None, 0, 0, None
+    if isinstance(y, Partial):
+        assert y.shape == (T, W) and y.bias is None
+        kind, p, ld, slabs = 2, _ptr(y.slabs), y.ld, y.S
+    elif isinstance(y, MixtureRows):
+        assert y.rows.dtype == y_dtype and y.rows.shape[1] == W and y.pos.shape[0] == T * y.k
+        kind, p, ld, pos, weight, k = 3, _ptr(y.rows), y.rows.stride(0), _i32(y.pos, "pos"), _f32(y.weight, "weight"), y.k
+        if isinstance(y.shared, Partial):
+            assert y.shared.shape == (T, W) and y.shared.bias is None
+            sh, ld_sh, sh_slabs = _ptr(y.shared.slabs), y.shared.ld, y.shared.S
+        elif y.shared is not None:
+            assert y.shared.shape == (T, W) and y.shared.dtype == y_dtype and y.shared.stride(1) == 1
+            sh, ld_sh = _ptr(y.shared), y.shared.stride(0)
+        gate = _f32(y.shared_gate, "shared_gate")
+    elif y is not None:
+        assert y.shape == (T, W) and y.dtype == y_dtype and y.stride(1) == 1
+        kind, p, ld = 1, _ptr(y), y.stride(0)
+    h = torch.empty((T, W), dtype=y_dtype, device=nxt.device)
+    _check(load_library().tgis_hyper_update(
+        _ptr(x), _ptr(ids), _ptr(table), table.shape[0] if table is not None else 0, float(emb_scale), _ptr(x_out), kind, p, ld, slabs, pos,
+        weight, k, sh, ld_sh, sh_slabs, gate, _f32(cur, "cur") if kind else None, _f32(nxt, "nxt"), _ptr(h), T, W, s, float(eps),
+        dtype_code3(y_dtype), _stream()), "tgis_hyper_update")
+    return x_out, h

@@ -12,13 +12,15 @@ argument, so that a model file only maps its config keys and tensor names onto t
   BlockBiasedAttention  softmax attention without a rotation whose queries see only their own block of positions and whose
                       scores fall with the logarithm of the distance; unit-RMS values; sigmoid output gate; may read the keys
                       and values another layer cached
-  LatentAttention     queries and keys / values through normed low-rank latents, one rotated key part shared by the heads;
-                      the cache holds the latent and the rotated part, the heads' key / value maps are applied to the query
-                      and to the attention output instead of to every cached token
+  LatentAttention     queries and keys / values through normed low-rank latents, optionally one rotated key part shared by the
+                      heads and an output gate; the cache holds the latent and the rotated part, the heads' key / value maps
+                      are applied to the query and to the attention output instead of to every cached token; may read the
+                      latents another layer cached
   DeltaRuleMixer      gated delta rule with a decay per head and key channel, short convolutions in front of q, k and v,
                       low-rank decay and output-gate projections; state in a RecurrentStateCache slot
   WindowSinkAttention rotated (interleaved pairs, partial) GQA softmax attention with a sliding window that keeps the first
-                      positions, a learned sink logit per head in the denominator and a sigmoid gate per head
+                      positions, a learned sink logit per head in the denominator and a sigmoid gate per head; optionally
+                      piecewise scaled frequencies, capped scores, and values rotated by their position and turned back
   GatedLinearRecurrence  HGRN2-style linear attention: S <- diag(f) S + (1 - f) v^T with a forget gate bounded below,
                       o = S^T silu(q), per-head RMS norm; state in a RecurrentStateCache slot
   SideBySideMixers    several mixers reading the same input through ONE stacked projection, their weighted results through
@@ -31,6 +33,9 @@ argument, so that a model file only maps its config keys and tensor names onto t
                       whole-row norm; sigmoid or SiLU output gate
   NormedPairMixers    two mixers on ONE stacked projection whose results are RMS-normed over the width and averaged
   PowerNormMLP        W_down P(W_up h), P a polynomial of the unit-RMS powers z, z^2, z^3
+  MinGRU              S <- (1 - z) S + z c per channel, gate and candidate from the current token only; SiLU output gate
+  HyperStreams        several residual streams: what a sublayer reads is a weighted sum of them, its result is spread over all
+                      of them while they are mixed; scalar-gain RMS norms
   ActivatedMLP        W_down act(W_up h) with the xIELU activation
   TokenSideInput      a slice of a second token embedding, gated by a GELU of a projection of the residual stream itself
 
@@ -177,8 +182,9 @@ class GatedUnit:
 class RoutedExperts:
     def __init__(self, weights, prefix: str, experts: int, top: int, shared: bool, router_bias: bool = False,
                  softmax_top: bool = False, weight_on_input: bool = True, grouped_softmax: bool = False, groups: int = 1,
-                 keep_groups: int = 1, renorm_eps: float = 0.0):
-        """softmax_top: the routing weights are the softmax over the chosen logits (else the sigmoid of each);
+                 keep_groups: int = 1, renorm_eps: float = 0.0, clamp=None, shared_clamp=None):
+        """clamp = (alpha, limit): the experts are clamped gated units (else SiLU); shared_clamp: the same for the shared one.
+        softmax_top: the routing weights are the softmax over the chosen logits (else the sigmoid of each);
         weight_on_input: the weight scales the expert's input (else its output); router_bias: `<prefix>.router.b`.
         grouped_softmax: scores are the softmax over ALL experts; experts are chosen by score + `<prefix>.correction` among the
         `keep_groups` best of `groups` equal groups of neighbours; weights = chosen scores / (their sum + renorm_eps)."""
@@ -202,10 +208,16 @@ class RoutedExperts:
                                                  pad(weights.get_tensor(f"{prefix}.e{e}.up"), self.ff, self.Wp)], 0)
                                       for e in range(experts)]).contiguous()
         self.w_down = torch.stack([pad(weights.get_tensor(f"{prefix}.e{e}.down"), W, self.ff) for e in range(experts)]).contiguous()
-        self.shared = GatedUnit(weights, f"{prefix}.shared") if shared else None
+        self.clamp = clamp
+        self.shared = None
+        if shared and shared_clamp is not None:
+            self.shared = GatedUnit(weights, f"{prefix}.shared", mode="clamped", alpha=shared_clamp[0], limit=shared_clamp[1])
+        elif shared:
+            self.shared = GatedUnit(weights, f"{prefix}.shared")
         self.shared_gate = _f32(weights.get_tensor(f"{prefix}.shared.sg")).reshape(-1) if shared else None
 
-    def forward(self, h: torch.Tensor) -> torch.Tensor:
+    def forward(self, h: torch.Tensor, defer: bool = False):
+        """defer: the sum over a token's rows is left to the consumer (native.MixtureRows)."""
         T, W = h.shape
         if self.grouped_softmax:
             idx, weight = native.moe_route_grouped(h, self.router, self.correction, self.k, self.groups, self.keep_groups, self.renorm_eps)
@@ -216,9 +228,11 @@ class RoutedExperts:
         cap = sorted_.shape[0]
         hp = h if self.Wp == W else torch.nn.functional.pad(h, (0, self.Wp - W))
         act = native.moe_gemm(hp, self.w_gate_up, self.ff, tile_expert, n_tiles, cap, sorted_=sorted_, pair_div=self.k,
-                              pair_scale=weight.view(-1) if self.weight_on_input else None, glu_act=True)
+                              pair_scale=weight.view(-1) if self.weight_on_input else None, glu_act=True, clamp=self.clamp)
         rows = native.moe_gemm(act, self.w_down, W, tile_expert, n_tiles, cap)
-        shared = self.shared(h) if self.shared is not None else None
+        shared = self.shared(h, partial=defer) if self.shared is not None else None
+        if defer:
+            return native.MixtureRows(rows, pos, None if self.weight_on_input else weight.view(-1), self.k, shared, sg)
         return native.moe_combine(rows, pos, self.k, T, pair_weight=None if self.weight_on_input else weight.view(-1),
                                   shared=shared, shared_gate=sg)
 
@@ -286,54 +300,77 @@ def rotary_inverse_frequencies(base: float, dims: int, device) -> torch.Tensor:
     return (float(base) ** (-2.0 * i / dims)).to(torch.float32).to(device)
 
 
+def scaled_inverse_frequencies(base: float, dims: int, scaling: Optional[dict], device) -> torch.Tensor:
+    """rotary_inverse_frequencies with the piecewise scaling by wavelength 2 pi / f: kept below original / high, divided by `factor`
+    above original / low, and in between blended linearly in original / wavelength (float64, rounded once)."""
+    if not scaling:
+        return rotary_inverse_frequencies(base, dims, device)
+    factor, low, high, original = (float(scaling[k]) for k in ("factor", "low", "high", "original"))
+    f = float(base) ** (-2.0 * torch.arange(dims // 2, dtype=torch.float64) / dims)
+    wave = 2.0 * torch.pi / f
+    # the blend is not used where low == high: every wavelength is on one side then
+    s = (original / wave - low) / (high - low) if high != low else torch.zeros_like(f)
+    out = torch.where(wave > original / low, f / factor, (1 - s) * f / factor + s * f)
+    out = torch.where(wave < original / high, f, out)
+    return out.to(torch.float32).to(device)
+
+
 class LatentAttention:
     """c_q = N(W_dq h), q = W_uq c_q = [H][dn | dr];  [c | r] = W_dkv h with c = N(first kv_rank rows);  per head
-    k = [W_uk c | rot(r)], v = W_uv c;  causal softmax;  sigmoid output gate.  Only (c, rot(r)) is cached: a page row is
-    [c | rot(r)] for ONE kv head, so the score of head h is (W_uk,h^T q_n,h) . c + rot(q_r,h) . rot(r) and its output
-    W_uv,h (sum_j p_j c_j) — two batched products per step instead of two per cached token."""
+    k = [W_uk c | rot(r)], v = W_uv c;  causal softmax;  sigmoid output gate (where `<prefix>.g` exists).  Only (c, rot(r)) is
+    cached: a page row is [c | rot(r)] for ONE kv head, so the score of head h is (W_uk,h^T q_n,h) . c + rot(q_r,h) . rot(r) and
+    its output W_uv,h (sum_j p_j c_j) — two products per head and step instead of two per cached token.  rot_dim 0: no
+    positions.  kv_source: the layer whose cached latents this one reads (then it has no down-projection of its own)."""
 
     def __init__(self, weights, prefix: str, layer_id: int, heads: int, dim: int, rot_dim: int, vdim: int, kv_rank: int,
-                 scale: float, eps: float, rot_base: float, rot_dims: int):
-        self.layer_id = layer_id
+                 scale: float, eps: float, rot_base: float = 10000.0, rot_dims: int = 0, kv_source: Optional[int] = None):
+        self.layer_id, self.kv_layer = layer_id, layer_id if kv_source is None else int(kv_source)
+        self.own_kv = kv_source is None
         self.H, self.dn, self.dr, self.dv, self.rk = heads, dim, rot_dim, vdim, kv_rank
         _widths_ok_for_pages(kv_rank + rot_dim, kv_rank)
         self.scale, self.eps, self.rot_dims = float(scale), float(eps), int(rot_dims)
         self.q_rank = weights.get_shape(f"{prefix}.dq")[0]
-        self.down = load_stacked_linear(weights, [f"{prefix}.dq", f"{prefix}.dkv", f"{prefix}.g"])
-        self.c_col = self.q_rank
-        self.g_col = self.q_rank + kv_rank + rot_dim
+        self.has_gate = weights.has(f"{prefix}.g")
+        names = ["dq"] + (["dkv"] if self.own_kv else []) + (["g"] if self.has_gate else [])
+        self.down, cols = load_stacked_blocks(weights, [f"{prefix}.{n}" for n in names], align=8)
+        at = dict(zip(names, cols))
+        self.c_col, self.g_col = at.get("dkv"), at.get("g")
         self.q_gain = _f32(weights.get_tensor(f"{prefix}.dq.norm"))
-        self.c_gain = _f32(weights.get_tensor(f"{prefix}.dkv.norm"))
+        self.c_gain = _f32(weights.get_tensor(f"{prefix}.dkv.norm")) if self.own_kv else None
         self.uq = load_linear(weights, f"{prefix}.uq")
-        # [H, dn, kv_rank]: head h's keys are W_uk,h c, so its query meets the latent as W_uk,h^T q_n
-        self.uk = weights.get_tensor(f"{prefix}.uk").view(heads, dim, kv_rank).contiguous()
-        # [H, kv_rank, dv]: W_uv,h^T, applied to the attention output in latent space
-        self.uv_t = weights.get_tensor(f"{prefix}.uv").view(heads, vdim, kv_rank).transpose(1, 2).contiguous()
-        self.inv_freq = rotary_inverse_frequencies(rot_base, self.rot_dims, self.uk.device) if self.rot_dims else \
-            torch.zeros(1, dtype=torch.float32, device=self.uk.device)
+        # [H, kv_rank, dn]: head h's keys are W_uk,h c, so its query meets the latent as W_uk,h^T q_n
+        self.uk_t = weights.get_tensor(f"{prefix}.uk").view(heads, dim, kv_rank).transpose(1, 2).contiguous()
+        # [H, dv, kv_rank]: W_uv,h, applied to the attention output in latent space
+        self.uv = weights.get_tensor(f"{prefix}.uv").view(heads, vdim, kv_rank).contiguous()
+        self.inv_freq = rotary_inverse_frequencies(rot_base, self.rot_dims, self.uk_t.device) if self.rot_dims else \
+            torch.zeros(1, dtype=torch.float32, device=self.uk_t.device)
         self.o = load_linear(weights, f"{prefix}.o")
         self.defer = can_defer(self.o)
         # cache geometry of this layer: one kv head
-        self.kv_shape = (1, kv_rank + rot_dim, kv_rank)
+        self.kv_shape = (1, kv_rank + rot_dim, kv_rank) if self.own_kv else None
 
     def forward(self, h: torch.Tensor, position_ids, step):
         T = h.shape[0]
         H, dn, dr, rk, dv = self.H, self.dn, self.dr, self.rk, self.dv
         down = self.down(h)
-        cq = native.rms_norm_rows(down[:, :self.q_rank], self.q_gain, self.eps)
-        q = self.uq(cq)
         cache = step.cache
-        k_pool, v_pool = cache.k_pool(self.layer_id), cache.v_pool(self.layer_id)
+        k_pool, v_pool = cache.k_pool(self.kv_layer), cache.v_pool(self.kv_layer)
+        if self.own_kv and not dr:
+            cq = native.latent_norm_write(down, 0, self.q_rank, self.q_gain, self.c_col, rk, self.c_gain, step.slots, k_pool, v_pool, self.eps)
+        else:
+            cq = native.rms_norm_rows(down[:, :self.q_rank], self.q_gain, self.eps)
+        q = self.uq(cq)
         q_abs = torch.empty((T, H * (rk + dr)), dtype=q.dtype, device=q.device)
-        native.latent_kv_write(q, down[:, self.c_col:self.c_col + rk + dr], self.c_gain, self.inv_freq, position_ids, step.slots,
-                               q_abs, k_pool, v_pool, H, dn, dr, rk, self.rot_dims, self.eps)
-        # the unrotated query parts in latent space: [H, T, dn] x [H, dn, rk] (library batched product)
-        qn = q.view(T, H, dn + dr)[:, :, :dn].transpose(0, 1)
-        q_abs.view(T, H, rk + dr)[:, :, :rk].copy_(torch.bmm(qn, self.uk).transpose(0, 1))
+        if dr:
+            native.latent_kv_write(q, down[:, self.c_col:self.c_col + rk + dr], self.c_gain, self.inv_freq, position_ids, step.slots,
+                                   q_abs, k_pool, v_pool, H, dn, dr, rk, self.rot_dims, self.eps)
+        # the unrotated query parts go into latent space, the results come out of it
+        native.head_product(q, dn + dr, self.uk_t, q_abs, rk + dr)
         lat = native.attn_varlen_ext(q_abs, k_pool, v_pool, step.block_tables, step.ctx_lens, step.cu_seqlens_q, H, 1, rk + dr, rk,
                                      self.scale, max_q_len=step.max_q_len, max_ctx=step.max_ctx, ws=workspace(h.device))
-        att = torch.bmm(lat.view(T, H, rk).transpose(0, 1), self.uv_t).transpose(0, 1).reshape(T, H * dv)
-        native.sigmoid_gate_mul(att, down[:, self.g_col:self.g_col + H * dv], out=att)
+        att = native.head_product(lat, rk, self.uv, torch.empty((T, H * dv), dtype=q.dtype, device=q.device), dv)
+        if self.has_gate:
+            native.sigmoid_gate_mul(att, down[:, self.g_col:self.g_col + H * dv], out=att)
         return self.o(att, partial=self.defer)
 
 
@@ -379,9 +416,10 @@ class DeltaRuleMixer:
         return self.o(out, partial=self.defer)
 
 
-def load_stacked_blocks(weights, names, align: int = 8):
+def load_stacked_blocks(weights, names, align: int = 8, biased=()):
     """Several [out_i, in] weights that read the same input as one GEMM whose every block starts on a multiple of `align`
-    output columns (zero rows between them) and whose width is one too: (FastLinear, [first column of each block])."""
+    output columns (zero rows between them) and whose width is one too: (FastLinear, [first column of each block]).  biased: the
+    names whose `<name>.b` (if it exists) the projection adds."""
     parts, cols, at = [], [], 0
     for n in names:
         w = weights.get_tensor(n)
@@ -391,18 +429,34 @@ def load_stacked_blocks(weights, names, align: int = 8):
         if pad:
             parts.append(w.new_zeros((pad, w.shape[1])))
         at += w.shape[0] + pad
-    return FastLinear(torch.cat(parts, dim=0).contiguous(), None), cols
+    return FastLinear(torch.cat(parts, dim=0).contiguous(), stacked_bias(weights, names, cols, at, biased)), cols
+
+
+def stacked_bias(weights, names, cols, width: int, biased) -> Optional[torch.Tensor]:
+    """The biases (`<name>.b`, where they exist) of those `biased` among the weights stacked at output columns `cols`, zeros
+    elsewhere; None without any."""
+    bias = None
+    for n, c in zip(names, cols):
+        if n in biased and weights.has(n + ".b"):
+            b = weights.get_tensor(n + ".b")
+            if bias is None:
+                bias = b.new_zeros(width)
+            bias[c:c + b.shape[0]] = b
+    return bias
 
 
 class WindowSinkAttention:
     """GQA softmax attention: q, k rotated in interleaved pairs (2i, 2i + 1) over their first rot_dims channels by
     position * rot_base^(-2i / rot_dims); position i sees j <= i iff i - j < window or j < keep_first (window 0: plain causal);
     the denominator of head h also holds exp(sink[h]) (`<prefix>.sink`, optional); head h's output is multiplied by
-    sigmoid(W_g h)[h] (`<prefix>.g`, optional).  The mixer reads columns of a projection its owner made (`in_names` are the
-    weights to stack, in this order) and writes its heads into the owner's buffer."""
+    sigmoid(W_g h)[h] (`<prefix>.g`, optional).  rot_scaling: piecewise scaling of the frequencies; softcap: scores become
+    softcap * tanh(score / softcap); turned_values: pair (2m, 2m + 1) of a value turns by position * rot_base^(-2m / vdim) before
+    it is cached and a head's output turns back by the reader's position.  The mixer reads columns of a projection its owner
+    made (`in_names` are the weights to stack, in this order) and writes its heads into the owner's buffer."""
 
     def __init__(self, weights, prefix: str, layer_id: int, heads: int, kv_heads: int, dim: int, vdim: int, scale: float,
-                 window: int = 0, keep_first: int = 0, rot_base: float = 10000.0, rot_dims: int = 0):
+                 window: int = 0, keep_first: int = 0, rot_base: float = 10000.0, rot_dims: int = 0, rot_scaling: Optional[dict] = None,
+                 softcap: float = 0.0, turned_values: bool = False):
         self.layer_id = layer_id
         self.H, self.G, self.dk, self.dv = heads, kv_heads, dim, vdim
         _widths_ok_for_pages(dim, vdim)
@@ -412,10 +466,18 @@ class WindowSinkAttention:
         self.rot_dims = int(rot_dims)
         self.has_gate = weights.has(f"{prefix}.g")
         self.in_names = [f"{prefix}.{n}" for n in (("q", "k", "v", "g") if self.has_gate else ("q", "k", "v"))]
+        self.biased_names = self.in_names[:3]
         self.out_name, self.out_width = f"{prefix}.o", heads * vdim
         self.sink = _f32(weights.get_tensor(f"{prefix}.sink")) if weights.has(f"{prefix}.sink") else None
         dev = weights.device
-        self.inv_freq = rotary_inverse_frequencies(rot_base, self.rot_dims, dev) if self.rot_dims else None
+        self.inv_freq = scaled_inverse_frequencies(rot_base, self.rot_dims, rot_scaling, dev) if self.rot_dims else None
+        self.softcap = float(softcap)
+        self.turn_key = (float(rot_base), vdim) if turned_values else None  # layers with the same key share a step's table
+        self.turn_freq = rotary_inverse_frequencies(rot_base, vdim, dev) if turned_values else None
+        if turned_values and vdim % 2:
+            raise ValueError(f"{prefix}: values of {vdim} channels do not form pairs")
+        if self.has_gate and (self.softcap or turned_values):
+            raise NotImplementedError(f"{prefix}: a per-head gate beside capped scores or turned values")
         self.kv_shape = (kv_heads, dim, vdim)
         self.state_shape = None
 
@@ -423,6 +485,20 @@ class WindowSinkAttention:
         """proj [T, ld] with this mixer's blocks at columns `cols` (one per in_name); out [T, H dv] (a view)."""
         cache = step.cache
         k_pool, v_pool = cache.k_pool(self.layer_id), cache.v_pool(self.layer_id)
+        if self.softcap or self.turn_key:
+            turns = None
+            if self.turn_key:
+                turns = step_turns(step, self.turn_key, self.turn_freq, position_ids)
+                native.rope_rows_turned_kv_write(proj, cols[0], cols[1], cols[2], self.inv_freq, position_ids, step.slots, k_pool, v_pool,
+                                                 self.H, self.G, self.dk, self.dv, self.rot_dims, turns)
+            else:
+                native.rope_rows_kv_write(proj, cols[0], cols[1], cols[2], self.inv_freq, position_ids, step.slots, k_pool, v_pool, self.H,
+                                          self.G, self.dk, self.dv, self.rot_dims)
+            native.attn_varlen_turned(proj[:, cols[0]:cols[0] + self.H * self.dk], k_pool, v_pool, step.block_tables, step.ctx_lens,
+                                      step.cu_seqlens_q, self.H, self.G, self.dk, self.dv, self.scale, window=self.window,
+                                      keep_first=self.keep_first, sink=self.sink, softcap=self.softcap, turns=turns, out_scale=out_scale,
+                                      out=out, max_q_len=step.max_q_len, max_ctx=step.max_ctx, ws=workspace(proj.device))
+            return
         native.rope_rows_kv_write(proj, cols[0], cols[1], cols[2], self.inv_freq, position_ids, step.slots, k_pool, v_pool, self.H,
                                   self.G, self.dk, self.dv, self.rot_dims)
         gate = proj[:, cols[3]:cols[3] + self.H] if self.has_gate else None
@@ -430,6 +506,65 @@ class WindowSinkAttention:
                                step.cu_seqlens_q, self.H, self.G, self.dk, self.dv, self.scale, window=self.window,
                                keep_first=self.keep_first, sink=self.sink, gate=gate, gate_per_head=True, out_scale=out_scale, out=out,
                                max_q_len=step.max_q_len, max_ctx=step.max_ctx, ws=workspace(proj.device))
+
+
+def step_turns(step, key, freq: torch.Tensor, position_ids) -> torch.Tensor:
+    """(cos, sin) of position * freq for a step's tokens: made by the first layer that asks, shared by the others."""
+    if step.turns is None:
+        step.turns = {}
+    if key not in step.turns:
+        step.turns[key] = native.pair_turns(position_ids, freq)
+    return step.turns[key]
+
+
+class MinGRU:
+    """Per channel S <- (1 - z) S + z c with z = sigmoid(W_z h + b_z), u = W_x h + b_x and c = u + 1/2 for u >= 0, sigmoid(u)
+    otherwise; output W_o (S * silu(W_g h)).  Gates, candidates and the state [width] of a slot are fp32.  Reads columns of its
+    owner's projection."""
+
+    def __init__(self, weights, prefix: str, layer_id: int, width: int):
+        self.layer_id, self.D = layer_id, int(width)
+        self.in_names = [f"{prefix}.{n}" for n in ("z", "x", "g")]
+        self.biased_names = self.in_names[:2]
+        self.out_name, self.out_width = f"{prefix}.o", self.D
+        self.kv_shape = None
+        # a slot holds S; nothing else is remembered (a one-float placeholder)
+        self.state_shape = {"matrix": (self.D,), "memory": (1,)}
+
+    def run(self, proj: torch.Tensor, cols, position_ids, step, out: torch.Tensor, out_scale: float = 1.0):
+        native.min_gru_scan(proj, cols[0], cols[1], cols[2], step.state.state[self.layer_id], step.state_slots, step.cu_seqlens_q,
+                            position_ids, self.D, out=out, out_scale=out_scale, max_q_len=step.max_q_len)
+
+
+class HyperStreams:
+    """The residual of a decoder with `streams` fp32 streams X_a per token.  Sublayer f reads u = sum_a in[a] X_a through an RMS norm
+    with one gain for all channels, and X_b <- sum_a mix[a, b] X_a + out[b] f(.).  Sublayers are given in execution order as
+    (connection prefix or None, norm name): `<prefix>.in`, `.out`, `.mix`; prefix None: the plain sum of the streams is read (the
+    end of the stack) or, with one stream and no connection weights, an ordinary pre-norm residual.  One launch per boundary
+    applies a sublayer's result and makes the next one's input."""
+
+    def __init__(self, weights, streams: int, sublayers, eps: float, device):
+        self.s, self.eps = int(streams), float(eps)
+        if not 1 <= self.s <= 8:
+            raise NotImplementedError(f"1 .. 8 residual streams are served (got {streams})")
+        self.cur, self.nxt = [], []
+        for prefix, norm in sublayers:
+            gain = _f32(weights.get_tensor(norm)).reshape(1)
+            if prefix is None:
+                self.nxt.append(torch.cat([torch.ones(self.s, device=device), gain]))
+                self.cur.append(torch.cat([torch.eye(self.s, device=device).reshape(-1), torch.ones(self.s, device=device)]))
+                continue
+            part = lambda n, count: _f32(weights.get_tensor(f"{prefix}.{n}")).reshape(count)
+            self.nxt.append(torch.cat([part("in", self.s), gain]).contiguous())
+            self.cur.append(torch.cat([part("mix", self.s * self.s), part("out", self.s)]).contiguous())
+
+    def begin(self, ids, table, scale: float, dtype):
+        """(streams, normed input of sublayer 0) from the embedding rows."""
+        return native.hyper_update(None, None, None, self.nxt[0], self.eps, dtype, ids=ids, table=table, emb_scale=scale, streams=self.s)
+
+    def step(self, q: int, x, y, dtype):
+        """The result y of sublayer q joins the streams; returns (streams, normed input of sublayer q + 1)."""
+        return native.hyper_update(x, y, self.cur[q], self.nxt[q + 1], self.eps, dtype)
 
 
 class GatedLinearRecurrence:
@@ -466,7 +601,8 @@ class SideBySideMixers:
     def __init__(self, weights, mixers, scales, extra_in=()):
         self.mixers, self.scales = list(mixers), [float(s) for s in scales]
         names = [n for m in self.mixers for n in m.in_names] + list(extra_in)
-        self.proj, cols = load_stacked_blocks(weights, names, align=8)
+        biased = [n for m in self.mixers for n in getattr(m, "biased_names", ())]
+        self.proj, cols = load_stacked_blocks(weights, names, align=8, biased=biased)
         self.cols, at = [], 0
         for m in self.mixers:
             self.cols.append(cols[at:at + len(m.in_names)])
@@ -657,16 +793,9 @@ class StackedInput:
     `extra` more columns behind the blocks for what a mixer computes from them)."""
 
     def __init__(self, weights, names, extra: int = 0):
-        self.proj, self.cols = load_stacked_blocks(weights, names, align=8)
+        self.proj, self.cols = load_stacked_blocks(weights, names, align=8, biased=names)
         self.width = self.proj.out_features
         self.extra_col, self.extra = self.width, int(extra)
-        if any(weights.has(n + ".b") for n in names):
-            bias = torch.zeros(self.width, dtype=self.proj.weight.dtype, device=self.proj.weight.device)
-            for n, c in zip(names, self.cols):
-                if weights.has(n + ".b"):
-                    b = weights.get_tensor(n + ".b")
-                    bias[c:c + b.shape[0]] = b
-            self.proj.bias = bias
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         if not self.extra:
