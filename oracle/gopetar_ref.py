@@ -235,7 +235,7 @@ class GopetarRef:
         return self.advance(self.new_state(), tokens, trace)
 
 
-def clear_cut_tokens(config: dict, tensors, n: int, seed: int, margin: float = 0.05) -> List[int]:
+def clear_cut_tokens(config: dict, tensors, n: int, seed: int, margin: float = 0.15) -> List[int]:
     """n random tokens, each drawn again until no router of the model is within `margin` (in logit) of choosing other experts
     for it: what a reduced-precision run computes for them differs from this restatement by rounding, not by a decision."""
     import copy
@@ -247,7 +247,7 @@ def clear_cut_tokens(config: dict, tensors, n: int, seed: int, margin: float = 0
     try:
         while len(toks) < n:
             best = None
-            for _ in range(30):
+            for _ in range(60):
                 t = int(torch.randint(0, config["vocab"], (1,), generator=g))
                 trial = copy.deepcopy(state)
                 ROUTER_MARGINS = []

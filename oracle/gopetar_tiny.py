@@ -26,7 +26,7 @@ def pair_layer(left: Optional[dict] = None, width=88, left_scale=0.7, right_scal
                                           "right_scale": right_scale}, "mlp": mlp}
 
 
-def latent_layer(heads=3, dim=24, vdim=40, kv_rank=48, q_rank=56, scale=0.35, kv_from: Optional[int] = None, mlp=None) -> dict:
+def latent_layer(heads=3, dim=24, vdim=40, kv_rank=48, q_rank=56, scale=0.2, kv_from: Optional[int] = None, mlp=None) -> dict:
     m = {"heads": heads, "dim": dim, "vdim": vdim, "kv_rank": kv_rank, "q_rank": q_rank, "scale": scale}
     if kv_from is not None:
         m["kv_from"] = kv_from
@@ -72,7 +72,7 @@ def make_tensors(config: dict, seed: int = 0, dtype=torch.bfloat16) -> Dict[str,
             a, q = m["left"], f"{p}.left"
             H, dk = a["heads"], a["dim"]
             G, dv = a.get("kv_heads", H), a.get("vdim", dk)
-            for n_, rows, gain in (("q", H * dk, 2.0), ("k", G * dk, 2.0), ("v", G * dv, 1.0)):
+            for n_, rows, gain in (("q", H * dk, 1.5), ("k", G * dk, 1.5), ("v", G * dv, 1.0)):
                 lin(f"{q}.{n_}", rows, W, gain)
                 vec(f"{q}.{n_}.b", rows, 0.0, 0.3)
             vec(f"{q}.sink", H, 1.0, 1.5)
@@ -118,7 +118,7 @@ def standard_layers() -> List[dict]:
     GQA and MHA, a window and none, full and partial rotation, scaled frequencies and plain ones, no cap, no shared expert."""
     return [latent_layer(mlp=moe_mlp()),
             pair_layer(mlp=moe_mlp(experts=4, top=1, ff=56, shared_ff=None)),
-            latent_layer(heads=4, dim=16, vdim=24, q_rank=40, scale=0.5, kv_from=0, mlp=None),
+            latent_layer(heads=4, dim=16, vdim=24, q_rank=40, scale=0.3, kv_from=0, mlp=None),
             pair_layer(left=attention_part(heads=4, kv_heads=4, dim=16, vdim=16, window=None, rot_dims=16, scaling=None, softcap=None), width=60,
                        mlp=moe_mlp(experts=8, top=3, ff=32, shared_ff=32)),
             latent_layer(heads=2, dim=40, vdim=16, kv_rank=32, q_rank=24, mlp=moe_mlp(experts=3, top=3))]
@@ -144,7 +144,7 @@ def random_config(seed: int) -> dict:
             src = pick(sources) if sources and rnd.random() < 0.5 else None
             rk = src[1] if src else pick([8, 20, 32, 64, 96])
             return latent_layer(heads=pick([1, 2, 3, 5]), dim=pick([8, 12, 32, 40]), vdim=pick([8, 20, 32, 64]), kv_rank=rk, q_rank=pick([6, 16, 40]),
-                                scale=pick([0.2, 0.5]), kv_from=src[0] if src else None, mlp=mlp())
+                                scale=pick([0.1, 0.25]), kv_from=src[0] if src else None, mlp=mlp())
         G = pick([1, 2, 3])
         dk = pick([8, 16, 24, 32, 64])
         left = attention_part(heads=G * pick([1, 2, 3, 4]), kv_heads=G, dim=dk, vdim=pick([8, 16, 32, 48, 64]), scale=pick([0.1, 0.25, dk ** -0.5]),
