@@ -414,13 +414,13 @@ def senadra_layers(variant, width, layers, heads, kv_heads, dim, ff):
     """"senadra_attn": every layer block-masked biased attention (a block longer than any context here, so that the cache bytes
     equal Llama's) + the xIELU feed-forward.  "senadra": delta rule / attention / delta rule / latent attention in turn, the
     second attention layer of every two reading the first one's cache — the design as it is meant.  The delta rule's heads
-    are width / 64 of 64 x 64 (the state bytes of the wkv layers of Lenisun "mixed")."""
+    are width / 64 of 64 x 64 (the state bytes of the wkv layers of Lenisun "mixed").  "senadra_latent": latent layers only."""
     out = []
     attn = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": 8192}}
     first_attn = None
     for i in range(layers):
         mlp = {"kind": "dense", "ff": ff}
-        kind = "attention" if variant == "senadra_attn" else ("channel_delta", "attention", "channel_delta", "latent_attention")[i % 4]
+        kind = {"senadra_attn": "attention", "senadra_latent": "latent_attention"}.get(variant) or ("channel_delta", "attention", "channel_delta", "latent_attention")[i % 4]
         if kind == "attention":
             m = dict(attn)
             if variant == "senadra" and first_attn is not None and (i // 4) % 2 == 1:
@@ -439,16 +439,16 @@ def senadra_layers(variant, width, layers, heads, kv_heads, dim, ff):
 
 
 def mananex_layers(variant, width, layers, heads, kv_heads, dim, ff):
-    """"mananex_dense": every layer the two mixers side by side (attention with a window longer than any context here, so that
+    """"mananex_moe": "mananex" with the mixture in every layer.  "mananex_dense": every layer the two mixers side by side (attention with a window longer than any context here, so that
     the cache bytes equal Llama's, and a recurrence of width / 256 heads of 64 x 128) + the gated unit with biases.
     "mananex": a window of 512 positions that keeps the first 4, and every second feed-forward a mixture of 8 experts of
     ff / 4, top 2 — the design as it is meant."""
     out = []
     for i in range(layers):
         mlp = {"kind": "dense", "ff": ff}
-        if variant == "mananex" and i % 2 == 1:
+        if variant == "mananex_moe" or (variant == "mananex" and i % 2 == 1):
             mlp = {"kind": "moe", "expert": {"ff": ff // 4}, "router": {"experts": 8, "top": 2}}
-        window = 512 if variant == "mananex" else 8192
+        window = 8192 if variant == "mananex_dense" else 512
         out.append({"type": "parallel", "mlp": mlp,
                     "mixer": {"left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5,
                                        "mask": {"size": window, "keep_first": 4}, "rot": {"base": 10000.0, "dims": dim}},
@@ -488,6 +488,28 @@ def tatevik_layers(variant, width, layers, heads, kv_heads, dim, ff):
     return out, {"start": 1, "stop": 1 + span, "times": 2}, 4
 
 
+def gopetar_layers(variant, width, layers, heads, kv_heads, dim, ff):
+    """"gopetar_pair": every layer attention with rotated values, capped scores, a sink and a window of 512 beside a minGRU of `width`
+    channels — like for like with Mananex "mananex_moe".  "gopetar_latent": every layer latent attention (rank 192, the cached width
+    of the latent layers of Senadra's variants without their rotated part) — beside "senadra_latent".  "gopetar": latent / pair /
+    pair / latent in turn, the second latent layer of every four reading the first one's latents — the design as it is meant.
+    Every feed-forward is a mixture of 8 clamped units of ff / 4, top 2, and a shared one; four residual streams."""
+    out = []
+    for i in range(layers):
+        mlp = {"kind": "moe", "expert": {"ff": ff // 4, "limit": 7.0}, "router": {"experts": 8, "top": 2}, "shared": {"ff": ff // 4, "limit": 7.0}}
+        kind = {"gopetar_pair": "pair", "gopetar_latent": "latent"}.get(variant) or ("latent", "pair", "pair", "reader")[i % 4]
+        if kind == "pair":
+            left = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "softcap": 30.0, "mask": {"size": 512},
+                    "rot": {"base": 500000.0, "dims": dim // 2, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+            out.append({"type": "parallel", "mlp": mlp, "mixer": {"left": left, "left_scale": 0.7, "right": {"width": width}, "right_scale": 0.7}})
+        else:
+            m = {"heads": heads, "dim": dim, "vdim": dim, "kv_rank": 192, "q_rank": 768, "scale": dim ** -0.5}
+            if kind == "reader":
+                m["kv_from"] = i - 3
+            out.append({"type": "latent_attention", "mlp": mlp, "mixer": m})
+    return out
+
+
 def bench_hybrid(args):
     """Prefill and decode throughput + per-kernel-class device time (HIP events, eager pass) of Lenisun variants and of
     Llama at the same size, through the same entry points (from_pb -> generate_token).  One JSON line."""
@@ -512,7 +534,7 @@ def bench_hybrid(args):
     Bp, Lp = args.prefill_batch, args.prefill_len
     tok = SyntheticTokenizer(vocab)
     ops = {"attention": native.OP_ATTN, "dense_gemm": native.OP_DENSE_GEMM, "norm": native.OP_NORM, "qk_prep": native.OP_ROPE_KV,
-           "act": native.OP_ACT, "scan": native.OP_SCAN, "moe_gemm": native.OP_MOE_GEMM}
+           "act": native.OP_ACT, "scan": native.OP_SCAN, "moe_gemm": native.OP_MOE_GEMM, "head_product": native.OP_HEAD_PRODUCT}
     results = []
     for name in [v for v in args.hybrid_models.split(",") if v]:
         if name == "llama":
@@ -536,6 +558,14 @@ def bench_hybrid(args):
             tensors = tatevik_tensors(cfg, seed=1234, device=device, dtype=dtype)
             n_attn = sum(cfg.layers[i]["type"] == "parallel" for i, _ in cfg.runs)
             n_scan = len(cfg.runs)  # every run has one: selective scan, fixed-decay or channel-decay linear attention
+        elif name.startswith("gopetar"):
+            from tgis_amd.inference_engine.synthetic import gopetar_tensors
+            from tgis_amd.models.custom_modeling.flash_gopetar_modeling import GopetarConfig
+
+            cfg = GopetarConfig(width=width, vocab=vocab, norm={"eps": 1e-5}, streams=4, embedding={"scale": 1.0},
+                                layers=gopetar_layers(name, width, layers, heads, kv_heads, dim, ff))
+            tensors = gopetar_tensors(cfg, seed=1234, device=device, dtype=dtype)
+            n_attn, n_scan = layers, sum(l["type"] == "parallel" for l in cfg.layers)
         elif name.startswith("senadra"):
             cfg = SenadraConfig(width=width, vocab=vocab, norm={"eps": 1e-5}, residual_mult=0.25, token_side={"dim": 64},
                                 logit_softcap=25.0, layers=senadra_layers(name, width, layers, heads, kv_heads, dim, ff))
@@ -605,8 +635,10 @@ def bench_hybrid(args):
             ctx_now = L_in + W + K + 2
             if "attention" in kern:
                 # bytes one attention launch has to read: every cached key and value of the batch once
-                keys = min(ctx_now, 512 + 4 + 32) if name in ("mananex", "tatevik") else ctx_now  # a window, its kept positions, a page's slack
+                keys = min(ctx_now, 512 + 4 + 32) if name in ("mananex", "mananex_moe", "tatevik", "gopetar_pair") else ctx_now  # a window, its kept positions, a page's slack
                 by = B * keys * kv_heads * 2 * dim * 2
+                if name.endswith("_latent"):  # a token's latent, as a key row and as value columns (and Senadra's rotated part)
+                    by = B * ctx_now * (2 * 192 + (dim // 2 if name.startswith("senadra") else 0)) * 2
                 kern["attention"]["algorithmic_bytes"] = by
                 kern["attention"]["frac_of_hbm_peak"] = round(by / (kern["attention"]["us_per_launch"] * 1e-6) / 1e9 / HBM_PEAK_GBS, 4)
             rec["decode"] = {"batch": B, "ctx": ctx_now, "ms_per_step": round(dt * 1e3, 4), "tokens_per_s": round(B / dt, 1),
@@ -642,7 +674,8 @@ def main():
     ap.add_argument("--hybrid", choices=sorted(HYBRID_SIZES), default=None,
                     help="instead of the default workload: Lenisun / Senadra variants beside Llama at this size (prefill + decode)")
     ap.add_argument("--hybrid-models", default="llama,attn,mixed",
-                    help="comma list of llama, attn, mixed (Lenisun), senadra_attn, senadra, mananex_dense, mananex, tatevik_pair, tatevik")
+                    help="comma list of llama, attn, mixed (Lenisun), senadra_attn, senadra_latent, senadra, mananex_dense, mananex_moe, mananex, "
+                         "tatevik_pair, tatevik, gopetar_pair, gopetar_latent, gopetar")
     ap.add_argument("--prefill-batch", type=int, default=4)
     ap.add_argument("--prefill-len", type=int, default=1024)
     ap.add_argument("--prefill-reps", type=int, default=3)

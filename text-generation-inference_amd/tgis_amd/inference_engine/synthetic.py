@@ -412,3 +412,69 @@ def tatevik_tensors(config, seed: int, device="cpu", dtype=torch.bfloat16, decay
     vec("final.norm", W, 1.0)
     lin("head", config.vocab, W)
     return t
+
+
+def gopetar_tensors(config, seed: int, device="cpu", dtype=torch.bfloat16) -> Dict[str, torch.Tensor]:
+    """Seeded full Gopetar checkpoint in the family's tensor naming for a `GopetarConfig`: N(0, 1 / fan_in) projections, gains around
+    one, stream mixes near the identity."""
+    g = torch.Generator(device=device).manual_seed(seed)
+    W, s = config.width, config.streams
+    t: Dict[str, torch.Tensor] = {}
+
+    def lin(name, n, k, gain=1.0):
+        t[name] = (torch.randn(n, k, generator=g, device=device) * gain * k ** -0.5).to(dtype)
+
+    def vec(name, n, mean=0.0, std=0.05):
+        t[name] = (mean + torch.randn(n, generator=g, device=device) * std).to(dtype)
+
+    def sublayer(i, q):
+        t[f"l{i}.norm{q}"] = torch.ones((), device=device).to(dtype)
+        vec(f"l{i}.hc{q}.in", s, 1.0 / s, 0.1)
+        vec(f"l{i}.hc{q}.out", s, 0.5, 0.1)
+        t[f"l{i}.hc{q}.mix"] = (torch.eye(s, device=device) * 0.9 + torch.randn(s, s, generator=g, device=device) * 0.05).to(dtype)
+
+    t["embed"] = torch.randn(config.vocab, W, generator=g, device=device).to(dtype)
+    for i, lay in enumerate(config.layers):
+        m, p = lay["mixer"], f"l{i}.mix"
+        sublayer(i, 1)
+        if lay["type"] == "parallel":
+            a, q = m["left"], f"{p}.left"
+            H, dk = a["heads"], a["dim"]
+            G, dv = a.get("kv_heads", H), a.get("vdim", dk)
+            for n_, rows in (("q", H * dk), ("k", G * dk), ("v", G * dv)):
+                lin(f"{q}.{n_}", rows, W)
+                vec(f"{q}.{n_}.b", rows, 0.0, 0.1)
+            vec(f"{q}.sink", H, 0.0, 1.0)
+            lin(f"{q}.o", W, H * dv)
+            D, q = m["right"]["width"], f"{p}.right"
+            for n_ in ("z", "x", "g"):
+                lin(f"{q}.{n_}", D, W)
+            vec(f"{q}.z.b", D, -2.0, 1.0)
+            vec(f"{q}.x.b", D, 0.0, 0.1)
+            lin(f"{q}.o", W, D)
+        else:
+            H, dk, dv, rk, rq = m["heads"], m["dim"], m["vdim"], m["kv_rank"], m["q_rank"]
+            lin(f"{p}.dq", rq, W)
+            vec(f"{p}.dq.norm", rq, 1.0)
+            lin(f"{p}.uq", H * dk, rq)
+            if m.get("kv_from") is None:
+                lin(f"{p}.dkv", rk, W)
+                vec(f"{p}.dkv.norm", rk, 1.0)
+            lin(f"{p}.uk", H * dk, rk)
+            lin(f"{p}.uv", H * dv, rk)
+            lin(f"{p}.o", W, H * dv)
+        f = lay.get("mlp")
+        if f:
+            sublayer(i, 2)
+            q, E = f"l{i}.mlp", f["router"]["experts"]
+            units = [(f"{q}.e{e}", f["expert"]["ff"]) for e in range(E)] + ([(f"{q}.shared", f["shared"]["ff"])] if f.get("shared") else [])
+            for name, n_ in units:
+                lin(f"{name}.gate", n_, W)
+                lin(f"{name}.up", n_, W)
+                lin(f"{name}.down", W, n_)
+            lin(f"{q}.router", E, W)
+            if f.get("shared"):
+                lin(f"{q}.shared.sg", 1, W)
+    t["final.norm"] = torch.ones((), device=device).to(dtype)
+    lin("head", config.vocab, W)
+    return t
