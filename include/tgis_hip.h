@@ -646,6 +646,18 @@ int tgis_min_gru_scan(const void* proj, int64_t ld, int64_t z_col0, int64_t x_co
 int tgis_moe_gemm_clamped(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
                           const int32_t* tile_expert, const int32_t* n_tiles, const void* weights, int64_t expert_stride, int64_t N,
                           int64_t K, float alpha, float limit, void* out, int64_t ld_out, int64_t capacity, int dtype, void* stream);
+/* Tiles of 128 rows for long steps: tgis_moe_tile_rows names the alignment (32 or 128) a mixture of n_pairs pairs over E experts of
+ * W -> ff -> W should use; tgis_moe_tiled_capacity, tgis_moe_align_tiled and tgis_moe_gemm_tiled are tgis_moe_row_capacity,
+ * tgis_moe_align and tgis_moe_gemm for that alignment (glu 0: plain, 1: silu(gate) * up, 2: the clamped unit with alpha, limit).
+ * 128-row tiles: f16 / bf16, K a multiple of 32. */
+int tgis_moe_tile_rows(int64_t n_pairs, int64_t E, int64_t W, int64_t ff, int dtype);
+int64_t tgis_moe_tiled_capacity(int64_t n_pairs, int64_t E, int tile_rows);
+int tgis_moe_align_tiled(const int32_t* idx, int64_t n_pairs, int E, int32_t* sorted, int64_t capacity, int32_t* tile_expert,
+                         int32_t* pos_of_pair, int32_t* n_tiles, int tile_rows, void* stream);
+int tgis_moe_gemm_tiled(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
+                        const int32_t* tile_expert, const int32_t* n_tiles, const void* weights, int64_t expert_stride, int64_t N,
+                        int64_t K, int glu, float alpha, float limit, void* out, int64_t ld_out, int64_t capacity, int tile_rows,
+                        int dtype, void* stream);
 /* s residual streams per token, X [T][s][W] fp32 (s <= 8): the update of the sublayer that ran and the input of the next one,
  *   X'_b = sum_a cur.mix[a][b] X_a + cur.out[b] y   (kind 0: X' = X);   u = sum_a next.in[a] X'_a;
  *   h = u / sqrt(mean u^2 + eps) * next.gain   (h [T, W] of `dtype`)

@@ -594,7 +594,7 @@ def test_latent_attention_finds_a_far_token(gpu_device, dtype):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("T", [5, 37, 600])
-@pytest.mark.parametrize("E,k,W,ff,shared", [(6, 2, 72, 40, 56), (12, 4, 64, 96, None), (3, 3, 37, 21, 13), (1, 1, 40, 16, 40)])
+@pytest.mark.parametrize("E,k,W,ff,shared", [(6, 2, 72, 40, 56), (12, 4, 64, 96, None), (3, 3, 37, 21, 13), (1, 1, 40, 16, 40), (4, 2, 96, 160, 32)])
 def test_mixture_of_clamped_units(gpu_device, dtype, T, E, k, W, ff, shared):
     """Routed and shared clamped units (gates and ups on both sides of their limits), summed by the combine launch and left to the
     consumer."""
@@ -632,6 +632,52 @@ def test_mixture_of_clamped_units(gpu_device, dtype, T, E, k, W, ff, shared):
     nxt = torch.tensor([1.0, 1.0], device=gpu_device)
     X, _ = native.hyper_update(torch.randn(T, 1, W, device=gpu_device), rows, one, nxt, 1e-5, dtype)
     assert float((X[:, 0].double().cpu() - want)[sure].abs().max()) <= tol * float(want.abs().max())
+
+
+@pytest.mark.parametrize("dtype", [torch.float16, torch.bfloat16])
+@pytest.mark.parametrize("N,K", [(64, 32), (200, 96), (320, 512), (1024, 160)])
+@pytest.mark.parametrize("glu", [0, 1, 2])
+def test_grouped_products_in_tiles_of_128_rows(gpu_device, dtype, N, K, glu):
+    """Pairs spread unevenly over seven experts, one without any: gathered rows with a weight on the input and rows in place, every
+    activation, against plain products; the 32-row tiles must agree."""
+    from tgis_amd import native
+
+    g = torch.Generator().manual_seed(N + K + glu)
+    dev, T, k, E = gpu_device, 450, 2, 7
+    share = torch.tensor([0.4, 0.02, 0.2, 0.0, 0.1, 0.18, 0.1])
+    idx = torch.stack([torch.multinomial(share, k, generator=g) for _ in range(T)]).to(torch.int32)
+    h = torch.randn(T, K, generator=g).to(dtype)
+    w = (torch.randn(E, 2 * N if glu else N, K, generator=g) * K ** -0.5).to(dtype)
+    scale = torch.rand(T * k, generator=g) + 0.5
+    clamp = (1.702, 0.6) if glu == 2 else None
+
+    def act(z):
+        if not glu:
+            return z
+        a, b = z[..., :N], z[..., N:]
+        if glu == 1:
+            return ref.silu(a) * b
+        a, b = a.clamp(max=0.6), b.clamp(-0.6, 0.6)
+        return a * torch.sigmoid(1.702 * a) * (b + 1)
+
+    rows = h.double().repeat_interleave(k, 0)
+    flat = idx.view(-1).long()
+    prod = lambda x: act(torch.stack([x[i] @ w[flat[i]].double().T for i in range(T * k)]))
+    want, want_scaled = prod(rows), prod((rows * scale.double()[:, None]).to(dtype).double())
+    assert native.moe_tile_rows(T * k, E, 32, 32, dtype) == 128 and native.moe_tile_rows(T * k, E, 32, 40, dtype) == 32
+    tol = 0.02 if dtype == torch.bfloat16 else 0.003
+    for tile in (128, 32):
+        srt, te, pos, nt = native.moe_align(idx.to(dev), E, tile)
+        cap = srt.shape[0]
+        kw = dict(glu_act=bool(glu), clamp=clamp, tile_rows=tile)
+        got = native.moe_gemm(h.to(dev), w.to(dev), N, te, nt, cap, sorted_=srt, pair_div=k, **kw)
+        got_s = native.moe_gemm(h.to(dev), w.to(dev), N, te, nt, cap, sorted_=srt, pair_div=k, pair_scale=scale.to(dev), **kw)
+        placed = torch.zeros(cap, K, dtype=dtype, device=dev)
+        placed[pos.long()] = h.to(dev).repeat_interleave(k, 0)
+        got_p = native.moe_gemm(placed, w.to(dev), N, te, nt, cap, **kw)
+        for out, ref_out in ((got, want), (got_s, want_scaled), (got_p, want)):
+            o = out[pos.long()].double().cpu()
+            assert float((o - ref_out).abs().max()) <= tol * float(ref_out.abs().max()), tile
 
 
 # ---- generation through the serving entry points ---------------------------------------------------------------------------

@@ -410,8 +410,10 @@ __global__ __launch_bounds__(1024) void attn_varlen_kernel(
 // the V^T fragment that matches k-slot order is two 8-byte loads of the channel-major V page.
 //   mode 0 (a step with long runs):   the NW waves of a workgroup own NW neighbouring column tiles and all their keys;
 //   mode 1 (runs * R <= 32, decode):  the NW waves split the pages of ONE tile and meet in LDS.
+// Wide values (DVT 8) need more than the 256 registers a lane of an eight-wave workgroup can have, and their merge area in LDS never
+// holds eight waves' sums anyway: their workgroups are of four waves.
 template <typename T, int DK16, int DVT>
-__global__ __launch_bounds__(512) void attn_varlen_mfma_kernel(
+__global__ __launch_bounds__(DVT >= 8 ? 256 : 512) void attn_varlen_mfma_kernel(
     const T* __restrict__ q, int64_t ldq, const T* __restrict__ k_pool, const T* __restrict__ v_pool,
     const int32_t* __restrict__ bt, int64_t bt_ld, const int32_t* __restrict__ ctx_lens, const int32_t* __restrict__ cu_q,
     T* __restrict__ out, int64_t ld_out, int H, int G, int dk, int dv, float scale, int split, AttnExt ext) {
@@ -1068,36 +1070,41 @@ __global__ void pair_turns_kernel(const int32_t* __restrict__ positions, const f
     *reinterpret_cast<f32x2*>(turns + 2 * i) = f32x2{cs, sn};
 }
 
-// grid (token): wave 0 the cache latent, wave 1 the query latent (see tgis_latent_norm_write)
+// grid (token, 2): block row 0 the cache latent, 1 the query latent (see tgis_latent_norm_write)
 template <typename T>
-__global__ __launch_bounds__(128) void latent_norm_write_kernel(T* __restrict__ down, int64_t ld, int64_t q_col0, int q_rank,
+__global__ __launch_bounds__(256) void latent_norm_write_kernel(T* __restrict__ down, int64_t ld, int64_t q_col0, int q_rank,
                                                                 const float* __restrict__ q_gain, T* __restrict__ cq, int64_t ld_cq,
                                                                 int64_t c_col0, int rk, const float* __restrict__ c_gain,
                                                                 const int32_t* __restrict__ slots, T* __restrict__ k_pool,
                                                                 T* __restrict__ v_pool, float eps, int v_inline) {
+    __shared__ float part[4];
     const int64_t t = blockIdx.x;
-    const int lane = threadIdx.x & 63;
-    const bool is_q = threadIdx.x >= 64;
+    const int tid = threadIdx.x;
+    const bool is_q = blockIdx.y != 0;
     T* src = down + t * ld + (is_q ? q_col0 : c_col0);
     const int n = is_q ? q_rank : rk;
     const float* gain = is_q ? q_gain : c_gain;
-    constexpr int HELD = 16;  // values a lane keeps in registers: rows of up to 1024 are read once
-    float v[HELD], ss = 0.f;
+    constexpr int HELD = 4;  // values a thread keeps in registers: rows of up to 1024 are read once
+    float v[HELD], w[HELD], ss = 0.f;
 #pragma unroll
     for (int i = 0; i < HELD; ++i) {
-        const int c = lane + 64 * i;
+        const int c = tid + 256 * i;
         v[i] = c < n ? ldf(src + c) : 0.f;
+        w[i] = c < n ? gain[c] : 0.f;
         ss += v[i] * v[i];
     }
-    for (int c = lane + 64 * HELD; c < n; c += 64) ss += ldf(src + c) * ldf(src + c);
+    for (int c = tid + 256 * HELD; c < n; c += 256) ss += ldf(src + c) * ldf(src + c);
     ss = wave_sum(ss);
-    const float rinv = 1.0f / sqrtf(ss / (float)n + eps);
+    if ((tid & 63) == 0) part[tid >> 6] = ss;
     const int slot = is_q ? 0 : slots[t];
+    __syncthreads();
+    ss = part[0] + part[1] + part[2] + part[3];
+    const float rinv = 1.0f / sqrtf(ss / (float)n + eps);
     const int64_t page = slot / PAGE;
     const int off = slot % PAGE;
     T* dst = is_q ? cq + t * ld_cq : k_pool + (page * PAGE + off) * (int64_t)rk;
     auto put = [&](int c, float x) {
-        const T y = (T)(x * rinv * gain[c]);
+        const T y = (T)x;
         dst[c] = y;
         if (!is_q) {
             if (v_inline)
@@ -1108,8 +1115,8 @@ __global__ __launch_bounds__(128) void latent_norm_write_kernel(T* __restrict__ 
     };
 #pragma unroll
     for (int i = 0; i < HELD; ++i)
-        if (lane + 64 * i < n) put(lane + 64 * i, v[i]);
-    for (int c = lane + 64 * HELD; c < n; c += 64) put(c, ldf(src + c));
+        if (tid + 256 * i < n) put(tid + 256 * i, v[i] * rinv * w[i]);
+    for (int c = tid + 256 * HELD; c < n; c += 256) put(c, ldf(src + c) * rinv * gain[c]);
 }
 
 template <typename T, int DK16, int DVT>
@@ -1139,7 +1146,7 @@ void launch_mfma_one(const void* q, int64_t ldq, const void* k_pool, const void*
         gx = (unsigned)key_splits;
         const size_t per_wave = (128 + (size_t)DVT * 16 * 64) * sizeof(float);
         // eight waves share a tile's pages when the contexts are long or the grid alone would leave most of the chip idle
-        nw = (key_splits == 1 && (max_ctx > 2048 || (int64_t)B * G < 512) && max_ctx > 4 * PAGE && 8 * per_wave <= 150 * 1024) ? 8 : 4;
+        nw = (DVT < 8 && key_splits == 1 && (max_ctx > 2048 || (int64_t)B * G < 512) && max_ctx > 4 * PAGE && 8 * per_wave <= 150 * 1024) ? 8 : 4;
         lds = nw * per_wave;
         if (lds > 48 * 1024)
             (void)hipFuncSetAttribute((const void*)attn_varlen_mfma_kernel<T, DK16, DVT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
@@ -1149,7 +1156,10 @@ void launch_mfma_one(const void* q, int64_t ldq, const void* k_pool, const void*
         // and loses for wide ones (dk 128 / dv 128, MHA: 10.4 against 8.4 ms for 32 layers: two barriers per page and one LDS
         // buffer cost more than the second trip to L1 saves), so wide heads keep taking their fragments straight from L2 / L1.
         static const bool direct = getenv("TGIS_ATTN_VARLEN_DIRECT") != nullptr;  // A/B switch
-        if (!direct && DK16 <= 4 && DVT <= 2) {
+        // Many query heads on one cached head (a latent cache): a workgroup's 128 columns are a few neighbouring tokens, all of its
+        // waves need the same pages, and wide rows are worth staging.
+        const bool shared_wide = DK16 == 16 && DVT == 8 && R >= 8;
+        if (!direct && ((DK16 <= 4 && DVT <= 2) || shared_wide)) {
             hipLaunchKernelGGL((attn_varlen_staged_kernel<T, DK16, DVT>), dim3(gx, (unsigned)G, (unsigned)B), dim3(256), 0, st,
                                (const T*)q, ldq, (const T*)k_pool, (const T*)v_pool, bt, bt_ld, ctx_lens, cu_q, (T*)out, ld_out, H, G,
                                dk, dv, scale, ext);
@@ -1444,7 +1454,7 @@ extern "C" int tgis_latent_norm_write(void* down, int64_t ld, int64_t q_col0, in
     hipStream_t st = (hipStream_t)stream;
     TgisTimedScope timed(TGIS_OP_ROPE_KV, st);
     const int v_inline = T < 512 ? 1 : 0;
-    TGIS_ATTN_BY_DTYPE(dtype, hipLaunchKernelGGL(latent_norm_write_kernel<TT>, dim3((unsigned)T), dim3(128), 0, st, (TT*)down, ld, q_col0,
+    TGIS_ATTN_BY_DTYPE(dtype, hipLaunchKernelGGL(latent_norm_write_kernel<TT>, dim3((unsigned)T, 2), dim3(256), 0, st, (TT*)down, ld, q_col0,
                                                  (int)q_rank, q_gain, (TT*)cq, ld_cq, c_col0, (int)kv_rank, c_gain, slots, (TT*)k_pool,
                                                  (TT*)v_pool, eps, v_inline));
     if (!v_inline)

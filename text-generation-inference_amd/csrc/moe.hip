@@ -3,21 +3,22 @@
 // the combine that sums a token's rows (plus an optional gated shared expert).
 //
 //   route    logits = W_r h (fp32);  score = sigmoid(logit);  the k largest -> idx[T][k], weight[T][k]
-//   align    pairs p = t * k + j sorted by expert; every expert's run padded to a multiple of 32 rows:
-//            sorted[pos] = p or -1, tile_expert[pos / 32], pos_of_pair[p] = pos, n_tiles
+//   align    pairs p = t * k + j sorted by expert; every expert's run padded to a multiple of the tile rows (32, long steps 128):
+//            sorted[pos] = p or -1, tile_expert[pos / tile rows], pos_of_pair[p] = pos, n_tiles
 //   gemm     out[pos][n] = sum_c A[row(pos)][c] * s(pos) * W[expert(pos)][n][c]        (s = 1 or the routing weight, applied
 //            to the INPUT row and rounded to T like any other GEMM operand), optionally silu(gate) * up over a stacked
 //            [gate | up] weight
 //   combine  y[t] = sum_j rows[pos_of_pair[t k + j]] * (w[t][j] or 1) + g[t] * shared[t]
 //
-// The number of tiles is data dependent; the grid is sized for the worst case (T k + E * 31 rows) and tiles past n_tiles
-// leave at once.
+// The number of tiles is data dependent; the grid is sized for the worst case (T k + E * (tile rows - 1) rows) and tiles past
+// n_tiles leave at once.
 #include "common.h"
 #include "mfma_frag.h"
 
 namespace {
 
-constexpr int TM = 32;  // rows per tile = one 32x32 MFMA block
+constexpr int TM = 32;        // rows per tile = one 32x32 MFMA block
+constexpr int TM_LONG = 128;  // rows per tile of long steps (moe_gemm_tiled_kernel)
 
 template <typename T> __device__ __forceinline__ float ldf(const T* p) { return (float)*p; }
 
@@ -136,7 +137,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
 // ---- align: one workgroup ---------------------------------------------------------------------------------------------
 __global__ __launch_bounds__(1024) void moe_align_kernel(const int32_t* __restrict__ idx, int64_t n_pairs, int E,
                                                          int32_t* __restrict__ sorted, int64_t cap, int32_t* __restrict__ tile_expert,
-                                                         int32_t* __restrict__ pos_of_pair, int32_t* __restrict__ n_tiles) {
+                                                         int32_t* __restrict__ pos_of_pair, int32_t* __restrict__ n_tiles, int tm) {
     extern __shared__ int32_t si[];
     int32_t* count = si;            // [E]
     int32_t* start = si + E;        // [E + 1]
@@ -150,14 +151,14 @@ __global__ __launch_bounds__(1024) void moe_align_kernel(const int32_t* __restri
         int32_t at = 0;
         for (int e = 0; e < E; ++e) {
             start[e] = at;
-            at += (count[e] + TM - 1) / TM * TM;
+            at += (count[e] + tm - 1) / tm * tm;
         }
         start[E] = at;
-        *n_tiles = at / TM;
+        *n_tiles = at / tm;
     }
     __syncthreads();
     for (int e = threadIdx.x; e < E; e += blockDim.x)
-        for (int32_t tl = start[e] / TM; tl < start[e + 1] / TM; ++tl) tile_expert[tl] = e;
+        for (int32_t tl = start[e] / tm; tl < start[e + 1] / tm; ++tl) tile_expert[tl] = e;
     // arrival order within an expert: the rows of a tile are independent of each other, so the order changes no result
     for (int64_t p = threadIdx.x; p < n_pairs; p += blockDim.x) {
         const int e = idx[p];
@@ -228,7 +229,7 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const T* __restrict__ A, 
     // this wave's k range, in whole steps
     const int64_t steps = (K + F::KSTEP - 1) / F::KSTEP;
     const int64_t s0 = KSPLIT ? steps * wave / 4 : 0, s1 = KSPLIT ? steps * (wave + 1) / 4 : steps;
-#pragma unroll 2
+#pragma unroll(KSPLIT ? 4 : 2)
     for (int64_t kk = s0 * F::KSTEP; kk < s1 * F::KSTEP; kk += F::KSTEP) {
         const bool in = kk + half * F::PER + F::PER <= K;  // K is a multiple of PER: a fragment is whole or absent
         V a = in ? *reinterpret_cast<const V*>(ap + kk) : F::zero();
@@ -284,6 +285,154 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const T* __restrict__ A, 
     }
 }
 
+// ---- grouped GEMM of long steps -----------------------------------------------------------------------------------------
+// Workgroup = 4 waves (2 x 2) = one 128-row tile x BN weight rows (GLU: BN / 2 gate rows and the matching up rows); a wave owns
+// 64 rows x BN / 2 weight rows: 2 x BN / 64 accumulators of 32x32.  Both operands go through LDS in slices of 32 k, two slices
+// deep: the next slice is on its way to registers while the matrix cores work on the current one, one barrier per slice.  A slice
+// row is four 16-byte pieces, stored at piece ^ swz(row) so that the fragment reads of neighbouring rows fall on different banks.
+// Workgroups are dealt so that an XCD (one in eight workgroup ids) works on eight row tiles x a run of column blocks at a time:
+// what they read again is in its own L2.
+template <typename T, int GLU, int BN>
+__global__ __launch_bounds__(256, 2) void moe_gemm_tiled_kernel(const T* __restrict__ A, int64_t ld_a, const int32_t* __restrict__ sorted,
+                                                                int pair_div, const float* __restrict__ pair_scale,
+                                                                const int32_t* __restrict__ tile_expert, const int32_t* __restrict__ n_tiles,
+                                                                const T* __restrict__ Wt, int64_t expert_stride, int64_t N, int64_t K,
+                                                                T* __restrict__ out, int64_t ld_out, float alpha, float limit, int ncb) {
+    using V = typename Frag<T>::V;
+    constexpr int BK = 32, AL = TM_LONG * 4 / 256, BL = BN * 4 / 256, NJ = BN / 64;
+    constexpr int HALF = BN / 2;                      // weight rows of a wave
+    constexpr int OUTC = GLU ? BN / 2 : BN;           // output columns of the workgroup
+    __shared__ __attribute__((aligned(16))) T as[2][TM_LONG * BK];
+    __shared__ __attribute__((aligned(16))) T bs[2][BN * BK];
+    const int total = *n_tiles * ncb;
+    const int chunk = (total + 7) >> 3;
+    const int lin = (int)(blockIdx.x & 7) * chunk + (int)(blockIdx.x >> 3);
+    if ((int)(blockIdx.x >> 3) >= chunk || lin >= total) return;  // the whole workgroup
+    // groups of eight row tiles; inside a group the row tile moves fastest
+    const int group = lin / (8 * ncb), in_group = lin - group * 8 * ncb;
+    const int rows_here = min(8, *n_tiles - group * 8);
+    const int tile = group * 8 + in_group % rows_here, cb = in_group / rows_here;
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+    const int wr = wave >> 1, wc = wave & 1, r = lane & 31, half = lane >> 5;
+    const T* W = Wt + (int64_t)tile_expert[tile] * expert_stride;
+    const int64_t n0 = (int64_t)cb * OUTC;
+    auto swz = [](int row) { return ((row >> 1) ^ (row >> 3)) & 3; };
+    const T* ap[AL];
+    float asc[AL];
+    int aoff[AL];
+#pragma unroll
+    for (int i = 0; i < AL; ++i) {
+        const int e = tid + i * 256, row = e >> 2, piece = e & 3;
+        const int64_t pos = (int64_t)tile * TM_LONG + row;
+        int64_t arow = pos;
+        asc[i] = 1.f;
+        if (sorted) {
+            const int32_t p = sorted[pos];
+            arow = p >= 0 ? p / pair_div : 0;
+            if (pair_scale) asc[i] = p >= 0 ? pair_scale[p] : 0.f;
+        }
+        ap[i] = A + arow * ld_a + piece * 8;
+        aoff[i] = row * BK + ((piece ^ swz(row)) * 8);
+    }
+    const T* bp[BL];
+    int boff[BL];
+#pragma unroll
+    for (int i = 0; i < BL; ++i) {
+        const int e = tid + i * 256, row = e >> 2, piece = e & 3;
+        int64_t n;
+        if (GLU) {  // a wave's rows: HALF / 2 gate rows, then the matching up rows
+            const int w = row / HALF, x = row % HALF;
+            n = n0 + w * (HALF / 2) + x % (HALF / 2);
+            n = (n < N ? n : N - 1) + (x >= HALF / 2 ? N : 0);
+        } else {
+            n = n0 + row;
+            n = n < N ? n : N - 1;  // clamped: columns past N are computed and dropped
+        }
+        bp[i] = W + n * K + piece * 8;
+        boff[i] = row * BK + ((piece ^ swz(row)) * 8);
+    }
+    f32x16 acc[2][NJ];
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int j = 0; j < NJ; ++j) acc[i][j] = f32x16{};
+    V ar[AL], br[BL];
+    auto fetch = [&](int64_t k) {
+#pragma unroll
+        for (int i = 0; i < AL; ++i) ar[i] = *reinterpret_cast<const V*>(ap[i] + k);
+#pragma unroll
+        for (int i = 0; i < BL; ++i) br[i] = *reinterpret_cast<const V*>(bp[i] + k);
+    };
+    auto store = [&](int buf) {
+#pragma unroll
+        for (int i = 0; i < AL; ++i) *reinterpret_cast<V*>(&as[buf][aoff[i]]) = pair_scale ? Frag<T>::scaled(ar[i], asc[i]) : ar[i];
+#pragma unroll
+        for (int i = 0; i < BL; ++i) *reinterpret_cast<V*>(&bs[buf][boff[i]]) = br[i];
+    };
+    fetch(0);
+    store(0);
+    __syncthreads();
+    int buf = 0;
+    for (int64_t k = 0; k < K; k += BK, buf ^= 1) {
+        const bool more = k + BK < K;
+        if (more) fetch(k + BK);
+#pragma unroll
+        for (int s = 0; s < 2; ++s) {
+            V a[2], b[NJ];
+#pragma unroll
+            for (int i = 0; i < 2; ++i) {
+                const int row = wr * 64 + i * 32 + r;
+                a[i] = *reinterpret_cast<const V*>(&as[buf][row * BK + (((s * 2 + half) ^ swz(row)) * 8)]);
+            }
+#pragma unroll
+            for (int j = 0; j < NJ; ++j) {
+                const int row = wc * HALF + j * 32 + r;
+                b[j] = *reinterpret_cast<const V*>(&bs[buf][row * BK + (((s * 2 + half) ^ swz(row)) * 8)]);
+            }
+#pragma unroll
+            for (int i = 0; i < 2; ++i)
+#pragma unroll
+                for (int j = 0; j < NJ; ++j) Frag<T>::mma(a[i], b[j], acc[i][j]);
+        }
+        if (more) store(buf ^ 1);  // its last readers passed the barrier at the end of the slice before
+        __syncthreads();
+    }
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int j = 0; j < (GLU ? NJ / 2 : NJ); ++j) {
+            const int64_t n = n0 + (GLU ? wc * (HALF / 2) : wc * HALF) + j * 32 + r;
+            if (n >= N) continue;
+#pragma unroll
+            for (int q = 0; q < 16; ++q) {
+                const int64_t row = (int64_t)tile * TM_LONG + wr * 64 + i * 32 + (q >> 2) * 8 + half * 4 + (q & 3);
+                float v = acc[i][j][q];
+                if (GLU) v = gated<GLU ? GLU : 1>(v, acc[i][GLU ? j + NJ / 2 : j][q], alpha, limit);
+                out[row * ld_out + n] = (T)v;
+            }
+        }
+}
+
+template <typename T>
+void launch_gemm_tiled(int glu, float alpha, float limit, const void* A, int64_t ld_a, const int32_t* sorted, int pair_div,
+                       const float* pair_scale, const int32_t* tile_expert, const int32_t* n_tiles, const void* Wt, int64_t expert_stride,
+                       int64_t N, int64_t K, void* out, int64_t ld_out, int64_t max_tiles, hipStream_t st) {
+#define TGIS_MOE_TILED(GLU, BN)                                                                                                        \
+    do {                                                                                                                               \
+        const int ncb = (int)cdiv64(N, GLU ? BN / 2 : BN);                                                                             \
+        hipLaunchKernelGGL((moe_gemm_tiled_kernel<T, GLU, BN>), dim3((unsigned)((max_tiles * ncb + 7) / 8 * 8)), dim3(256), 0, st,     \
+                           (const T*)A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, (const T*)Wt, expert_stride, N, K,   \
+                           (T*)out, ld_out, alpha, limit, ncb);                                                                        \
+    } while (0)
+    if (glu == 2)
+        TGIS_MOE_TILED(2, 256);
+    else if (glu)
+        TGIS_MOE_TILED(1, 256);
+    else
+        TGIS_MOE_TILED(0, 256);
+#undef TGIS_MOE_TILED
+}
+
 // ---- combine: one workgroup per token -----------------------------------------------------------------------------------
 template <typename T>
 __global__ __launch_bounds__(256) void moe_combine_kernel(const T* __restrict__ rows, int64_t ld_rows, const int32_t* __restrict__ pos_of_pair,
@@ -331,7 +480,15 @@ void launch_gemm(int glu, float alpha, float limit, const void* A, int64_t ld_a,
 
 static bool dtype3(int d) { return d == TGIS_F16 || d == TGIS_BF16 || d == TGIS_F32; }
 
-extern "C" int64_t tgis_moe_row_capacity(int64_t n_pairs, int64_t E) { return (n_pairs + E * (TM - 1) + TM - 1) / TM * TM; }
+static int64_t row_capacity(int64_t n_pairs, int64_t E, int64_t tm) { return (n_pairs + E * (tm - 1) + tm - 1) / tm * tm; }
+extern "C" int64_t tgis_moe_row_capacity(int64_t n_pairs, int64_t E) { return row_capacity(n_pairs, E, TM); }
+
+// Rows per tile a mixture of n_pairs (token, choice) pairs over E experts should be aligned to: 128 where the experts' runs are long
+// enough to fill such tiles and both products' inner widths fit the LDS-staged kernel (two-byte dtypes, multiples of 32), else 32.
+extern "C" int tgis_moe_tile_rows(int64_t n_pairs, int64_t E, int64_t W, int64_t ff, int dtype) {
+    return dtype != TGIS_F32 && n_pairs >= 96 * E && W % 32 == 0 && ff % 32 == 0 ? TM_LONG : TM;
+}
+extern "C" int64_t tgis_moe_tiled_capacity(int64_t n_pairs, int64_t E, int tile_rows) { return row_capacity(n_pairs, E, tile_rows); }
 
 static int moe_route_impl(const void* h, int64_t ld_h, const float* router_w, const float* shared_gate_w, int32_t* idx,
                           float* weight, float* shared_gate, int64_t T, int64_t W, int E, int k, int dtype, void* stream,
@@ -377,20 +534,31 @@ extern "C" int tgis_moe_route_grouped(const void* h, int64_t ld_h, const float* 
                           keep_groups, renorm_eps);
 }
 
-extern "C" int tgis_moe_align(const int32_t* idx, int64_t n_pairs, int E, int32_t* sorted, int64_t capacity, int32_t* tile_expert,
-                              int32_t* pos_of_pair, int32_t* n_tiles, void* stream) {
+static int moe_align_impl(const int32_t* idx, int64_t n_pairs, int E, int32_t* sorted, int64_t capacity, int32_t* tile_expert,
+                          int32_t* pos_of_pair, int32_t* n_tiles, int tile_rows, void* stream) {
     TGIS_CHECK_ARG(idx && sorted && tile_expert && pos_of_pair && n_tiles, "tgis_moe_align: null tensor");
-    TGIS_CHECK_ARG(E >= 1 && E <= 4096 && n_pairs >= 0 && capacity >= tgis_moe_row_capacity(n_pairs, E),
-                   "tgis_moe_align: capacity %ld below tgis_moe_row_capacity", (long)capacity);
+    TGIS_CHECK_ARG(tile_rows == TM || tile_rows == TM_LONG, "tgis_moe_align: tiles of %d or %d rows", TM, TM_LONG);
+    TGIS_CHECK_ARG(E >= 1 && E <= 4096 && n_pairs >= 0 && capacity >= row_capacity(n_pairs, E, tile_rows) && capacity % tile_rows == 0,
+                   "tgis_moe_align: capacity %ld below the rows of %ld pairs", (long)capacity, (long)n_pairs);
     hipLaunchKernelGGL(moe_align_kernel, dim3(1), dim3(1024), (size_t)(3 * E + 1) * sizeof(int32_t), (hipStream_t)stream, idx, n_pairs,
-                       E, sorted, capacity, tile_expert, pos_of_pair, n_tiles);
+                       E, sorted, capacity, tile_expert, pos_of_pair, n_tiles, tile_rows);
     TGIS_CHECK_LAUNCH();
     return TGIS_OK;
 }
 
+extern "C" int tgis_moe_align(const int32_t* idx, int64_t n_pairs, int E, int32_t* sorted, int64_t capacity, int32_t* tile_expert,
+                              int32_t* pos_of_pair, int32_t* n_tiles, void* stream) {
+    return moe_align_impl(idx, n_pairs, E, sorted, capacity, tile_expert, pos_of_pair, n_tiles, TM, stream);
+}
+
+extern "C" int tgis_moe_align_tiled(const int32_t* idx, int64_t n_pairs, int E, int32_t* sorted, int64_t capacity, int32_t* tile_expert,
+                                    int32_t* pos_of_pair, int32_t* n_tiles, int tile_rows, void* stream) {
+    return moe_align_impl(idx, n_pairs, E, sorted, capacity, tile_expert, pos_of_pair, n_tiles, tile_rows, stream);
+}
+
 static int moe_gemm_impl(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
                              const int32_t* tile_expert, const int32_t* n_tiles, const void* weights, int64_t expert_stride, int64_t N,
-                             int64_t K, int glu, void* out, int64_t ld_out, int64_t capacity, int dtype, void* stream, float alpha, float limit) {
+                             int64_t K, int glu, void* out, int64_t ld_out, int64_t capacity, int dtype, void* stream, float alpha, float limit, int tile_rows = TM) {
     TGIS_CHECK_ARG(A && tile_expert && n_tiles && weights && out, "tgis_moe_gemm: null tensor");
     TGIS_CHECK_ARG(dtype3(dtype), "tgis_moe_gemm: bad dtype");
     const int per = dtype == TGIS_F32 ? 4 : 8;
@@ -403,6 +571,17 @@ static int moe_gemm_impl(const void* A, int64_t ld_a, const int32_t* sorted, int
     if (capacity == 0) return TGIS_OK;
     hipStream_t st = (hipStream_t)stream;
     TgisTimedScope timed(TGIS_OP_MOE_GEMM, st);
+    if (tile_rows == TM_LONG) {
+        TGIS_CHECK_ARG(dtype != TGIS_F32 && K % 32 == 0 && capacity % TM_LONG == 0 && capacity / TM_LONG * cdiv64(N, 128) < (1ll << 30),
+                       "tgis_moe_gemm: 128-row tiles take two-byte dtypes and K a multiple of 32 (got %ld)", (long)K);
+        if (dtype == TGIS_F16)
+            launch_gemm_tiled<f16>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, out, ld_out, capacity / TM_LONG, st);
+        else
+            launch_gemm_tiled<bf16>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, out, ld_out, capacity / TM_LONG, st);
+        TGIS_CHECK_LAUNCH();
+        return TGIS_OK;
+    }
+    TGIS_CHECK_ARG(tile_rows == TM, "tgis_moe_gemm: tiles of %d or %d rows", TM, TM_LONG);
     const int64_t tiles = capacity / TM;
     TGIS_CHECK_ARG(tiles <= 65535, "tgis_moe_gemm: %ld tiles exceed one grid", (long)tiles);
     if (dtype == TGIS_F16)
@@ -430,6 +609,16 @@ extern "C" int tgis_moe_gemm_clamped(const void* A, int64_t ld_a, const int32_t*
                                      void* stream) {
     return moe_gemm_impl(A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, 2, out, ld_out, capacity,
                          dtype, stream, alpha, limit);
+}
+
+// Any of the three (glu 0: plain, 1: silu(gate) * up, 2: the clamped unit) over pairs aligned to tiles of tile_rows rows.
+extern "C" int tgis_moe_gemm_tiled(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
+                                   const int32_t* tile_expert, const int32_t* n_tiles, const void* weights, int64_t expert_stride, int64_t N,
+                                   int64_t K, int glu, float alpha, float limit, void* out, int64_t ld_out, int64_t capacity, int tile_rows,
+                                   int dtype, void* stream) {
+    TGIS_CHECK_ARG(glu >= 0 && glu <= 2, "tgis_moe_gemm_tiled: glu 0, 1 or 2");
+    return moe_gemm_impl(A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, glu, out, ld_out, capacity,
+                         dtype, stream, alpha, limit, tile_rows);
 }
 
 extern "C" int tgis_moe_combine(const void* rows, int64_t ld_rows, const int32_t* pos_of_pair, const float* pair_weight, int k,

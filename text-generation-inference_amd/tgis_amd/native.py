@@ -172,6 +172,11 @@ SIGNATURES = {
                                    _c_i64, _c_int, _vp]),
     "tgis_moe_gemm_clamped": (_c_int, [_vp, _c_i64, _vp, _c_int, _vp, _vp, _vp, _vp, _c_i64, _c_i64, _c_i64, _c_f, _c_f, _vp, _c_i64,
                                        _c_i64, _c_int, _vp]),
+    "tgis_moe_tile_rows": (_c_int, [_c_i64, _c_i64, _c_i64, _c_i64, _c_int]),
+    "tgis_moe_tiled_capacity": (_c_i64, [_c_i64, _c_i64, _c_int]),
+    "tgis_moe_align_tiled": (_c_int, [_vp, _c_i64, _c_int, _vp, _c_i64, _vp, _vp, _vp, _c_int, _vp]),
+    "tgis_moe_gemm_tiled": (_c_int, [_vp, _c_i64, _vp, _c_int, _vp, _vp, _vp, _vp, _c_i64, _c_i64, _c_i64, _c_int, _c_f, _c_f, _vp, _c_i64,
+                                     _c_i64, _c_int, _c_int, _vp]),
     "tgis_hyper_update": (_c_int, [_vp, _vp, _vp, _c_i64, _c_f, _vp, _c_int, _vp, _c_i64, _c_int, _vp, _vp, _c_int, _vp, _c_i64, _c_int,
                                    _vp, _vp, _vp, _vp, _c_i64, _c_i64, _c_int, _c_f, _c_int, _vp]),
 }
@@ -1020,38 +1025,40 @@ def moe_route(h, router_w, shared_gate_w, k: int, router_b=None, softmax_top: bo
     return idx, weight, sg
 
 
-def moe_align(idx: torch.Tensor, E: int):
-    """(sorted [cap], tile_expert [cap / 32], pos_of_pair [pairs], n_tiles [1]) for idx [T, k]."""
+def moe_tile_rows(n_pairs: int, E: int, W: int, ff: int, dtype: torch.dtype) -> int:
+    return load_library().tgis_moe_tile_rows(n_pairs, E, W, ff, dtype_code3(dtype))
+
+
+def moe_align(idx: torch.Tensor, E: int, tile_rows: int = 32):
+    """(sorted [cap], tile_expert [cap / tile_rows], pos_of_pair [pairs], n_tiles [1]) for idx [T, k]."""
     n = idx.numel()
-    cap = moe_row_capacity(n, E)
+    lib = load_library()
+    cap = lib.tgis_moe_tiled_capacity(n, E, tile_rows)
     dev = idx.device
     sorted_ = torch.empty((cap,), dtype=torch.int32, device=dev)
-    tile_expert = torch.empty((cap // 32,), dtype=torch.int32, device=dev)
+    tile_expert = torch.empty((cap // tile_rows,), dtype=torch.int32, device=dev)
     pos = torch.empty((n,), dtype=torch.int32, device=dev)
     n_tiles = torch.empty((1,), dtype=torch.int32, device=dev)
-    _check(load_library().tgis_moe_align(_i32(idx, "idx"), n, E, _ptr(sorted_), cap, _ptr(tile_expert), _ptr(pos), _ptr(n_tiles),
-                                         _stream()), "tgis_moe_align")
+    _check(lib.tgis_moe_align_tiled(_i32(idx, "idx"), n, E, _ptr(sorted_), cap, _ptr(tile_expert), _ptr(pos), _ptr(n_tiles), tile_rows,
+                                    _stream()), "tgis_moe_align_tiled")
     return sorted_, tile_expert, pos, n_tiles
 
 
 def moe_gemm(A, weights, N: int, tile_expert, n_tiles, capacity: int, sorted_=None, pair_div: int = 1, pair_scale=None,
-             glu_act: bool = False, clamp=None):
+             glu_act: bool = False, clamp=None, tile_rows: int = 32):
     """weights [E, N (glu: 2 N), K]; returns [capacity, N].  glu_act: silu(gate) * up, or with clamp = (alpha, limit) the clamped
-    unit."""
+    unit.  tile_rows: the alignment moe_align was asked for."""
     assert A.dim() == 2 and A.stride(1) == 1 and weights.dim() == 3 and weights.is_contiguous() and weights.dtype == A.dtype
     K = weights.shape[2]
     assert weights.shape[1] == (2 * N if glu_act else N) and A.shape[1] == K
+    assert capacity % tile_rows == 0 and tile_expert.shape[0] * tile_rows == capacity and (sorted_ is not None or A.shape[0] >= capacity)
     out = torch.empty((capacity, N), dtype=A.dtype, device=A.device)
-    if glu_act and clamp is not None:
-        _check(load_library().tgis_moe_gemm_clamped(
-            _ptr(A), A.stride(0), _i32(sorted_, "sorted"), pair_div, _f32(pair_scale, "pair_scale"), _ptr(tile_expert), _ptr(n_tiles),
-            _ptr(weights), weights.stride(0), N, K, float(clamp[0]), float(clamp[1]), _ptr(out), out.stride(0), capacity,
-            dtype_code3(A.dtype), _stream()), "tgis_moe_gemm_clamped")
-        return out
-    _check(load_library().tgis_moe_gemm(
+    glu = (2 if clamp is not None else 1) if glu_act else 0
+    alpha, limit = clamp if clamp is not None else (0.0, 0.0)
+    _check(load_library().tgis_moe_gemm_tiled(
         _ptr(A), A.stride(0), _i32(sorted_, "sorted"), pair_div, _f32(pair_scale, "pair_scale"), _ptr(tile_expert), _ptr(n_tiles),
-        _ptr(weights), weights.stride(0), N, K, int(glu_act), _ptr(out), out.stride(0), capacity, dtype_code3(A.dtype), _stream()),
-        "tgis_moe_gemm")
+        _ptr(weights), weights.stride(0), N, K, glu, float(alpha), float(limit), _ptr(out), out.stride(0), capacity, tile_rows,
+        dtype_code3(A.dtype), _stream()), "tgis_moe_gemm_tiled")
     return out
 
 

@@ -224,12 +224,13 @@ class RoutedExperts:
             sg = None
         else:
             idx, weight, sg = native.moe_route(h, self.router, self.shared_gate, self.k, self.router_b, self.softmax_top)
-        sorted_, tile_expert, pos, n_tiles = native.moe_align(idx, self.E)
+        tm = native.moe_tile_rows(idx.numel(), self.E, self.Wp, self.ff, h.dtype)
+        sorted_, tile_expert, pos, n_tiles = native.moe_align(idx, self.E, tm)
         cap = sorted_.shape[0]
         hp = h if self.Wp == W else torch.nn.functional.pad(h, (0, self.Wp - W))
         act = native.moe_gemm(hp, self.w_gate_up, self.ff, tile_expert, n_tiles, cap, sorted_=sorted_, pair_div=self.k,
-                              pair_scale=weight.view(-1) if self.weight_on_input else None, glu_act=True, clamp=self.clamp)
-        rows = native.moe_gemm(act, self.w_down, W, tile_expert, n_tiles, cap)
+                              pair_scale=weight.view(-1) if self.weight_on_input else None, glu_act=True, clamp=self.clamp, tile_rows=tm)
+        rows = native.moe_gemm(act, self.w_down, W, tile_expert, n_tiles, cap, tile_rows=tm)
         shared = self.shared(h, partial=defer) if self.shared is not None else None
         if defer:
             return native.MixtureRows(rows, pos, None if self.weight_on_input else weight.view(-1), self.k, shared, sg)
