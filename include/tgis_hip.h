@@ -389,22 +389,27 @@ int tgis_wkv_scan(const void* r, const void* k, const void* v, const void* gate,
                   const int32_t* state_slots, const int32_t* cu_seqlens_q, const int32_t* positions, void* out,
                   int64_t ld_out, int64_t B, int H, int d, float eps, int dtype, void* stream);
 
-/* Mixture of experts, no host round trip.  Pairs p = t * k + j.  Rows of the grouped GEMMs live in 32-row tiles, one
- * expert per tile; tgis_moe_row_capacity(n_pairs, E) rows always suffice. */
-int64_t tgis_moe_row_capacity(int64_t n_pairs, int64_t E);
+/* Mixture of experts, no host round trip.  Pairs p = t * k + j.  Rows of the grouped GEMMs live in tiles of tile_rows (32 or 128)
+ * rows, one expert per tile; tgis_moe_row_capacity rows always suffice.  tgis_moe_tile_rows names the tile_rows a mixture of n_pairs
+ * pairs over E experts of W -> ff -> W should use (128: long steps, f16 / bf16, inner widths that are multiples of 32). */
+int64_t tgis_moe_row_capacity(int64_t n_pairs, int64_t E, int tile_rows);
+int tgis_moe_tile_rows(int64_t n_pairs, int64_t E, int64_t W, int64_t ff, int dtype);
 /* idx / weight [T][k]: the k experts with the largest router_w[e] . h[t] (fp32) and sigmoid of that logit;
  * shared_gate[t] = sigmoid(shared_gate_w . h[t]) when shared_gate_w != NULL. */
 int tgis_moe_route(const void* h, int64_t ld_h, const float* router_w, const float* shared_gate_w, int32_t* idx,
                    float* weight, float* shared_gate, int64_t T, int64_t W, int E, int k, int dtype, void* stream);
-/* sorted [capacity] = pair per row (-1: padding), tile_expert [capacity / 32], pos_of_pair [n_pairs], n_tiles [1]. */
+/* sorted [capacity] = pair per row (-1: padding), tile_expert [capacity / tile_rows], pos_of_pair [n_pairs], n_tiles [1]. */
 int tgis_moe_align(const int32_t* idx, int64_t n_pairs, int E, int32_t* sorted, int64_t capacity, int32_t* tile_expert,
-                   int32_t* pos_of_pair, int32_t* n_tiles, void* stream);
-/* out[row][n] = sum_c a(row)[c] * W[tile_expert[row / 32]][n][c], weights [E][N (glu: 2 N)][K] k-contiguous.
+                   int32_t* pos_of_pair, int32_t* n_tiles, int tile_rows, void* stream);
+/* out[row][n] = sum_c a(row)[c] * W[tile_expert[row / tile_rows]][n][c].
  * a(row) = A[sorted[row] / pair_div] * pair_scale[sorted[row]] (rounded to T) when sorted != NULL, else A[row].
- * glu: out = silu(gate) * up with gate rows [0, N) and up rows [N, 2 N) of each expert. */
+ * glu 1: out = silu(gate) * up;  2: g = min(gate, limit), u = clamp(up, -limit, limit), out = g sigmoid(alpha g) (u + 1).
+ * image: the experts' weights in fragment order, per expert [ceil(N / 32) blocks of weight rows (glu: the gate rows' blocks, then
+ * the up rows')][ceil(K / 16) steps (fp32: K / 8)][64 lanes][8 (fp32: 4) elements]: lane l of a step holds row l % 32 of the block
+ * and the elements k = step * 16 (8) + l / 32 * 8 (4) and on; rows and k padded with zeros. */
 int tgis_moe_gemm(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
-                  const int32_t* tile_expert, const int32_t* n_tiles, const void* weights, int64_t expert_stride, int64_t N,
-                  int64_t K, int glu, void* out, int64_t ld_out, int64_t capacity, int dtype, void* stream);
+                  const int32_t* tile_expert, const int32_t* n_tiles, const void* image, int64_t N, int64_t K, int glu,
+                  float alpha, float limit, void* out, int64_t ld_out, int64_t capacity, int tile_rows, int dtype, void* stream);
 /* out[t] = sum_j rows[pos_of_pair[t k + j]] * (pair_weight[t k + j] or 1) + (shared_gate[t] or 1) * shared[t]. */
 int tgis_moe_combine(const void* rows, int64_t ld_rows, const int32_t* pos_of_pair, const float* pair_weight, int k,
                      const void* shared, int64_t ld_shared, const float* shared_gate, void* out, int64_t ld_out, int64_t T,
@@ -641,23 +646,6 @@ int tgis_head_product(const void* x, int64_t ld_x, int64_t head_stride_x, const 
 int tgis_min_gru_scan(const void* proj, int64_t ld, int64_t z_col0, int64_t x_col0, int64_t g_col0, float* state,
                       const int32_t* state_slots, const int32_t* cu_seqlens_q, const int32_t* positions, void* out,
                       int64_t ld_out, float out_scale, int64_t B, int64_t T, int64_t max_q_len, int64_t D, int dtype, void* stream);
-/* tgis_moe_gemm over stacked [gate | up] weights with the clamped unit g = min(gate, limit), u = clamp(up, -limit, limit):
- * g sigmoid(alpha g) (u + 1). */
-int tgis_moe_gemm_clamped(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
-                          const int32_t* tile_expert, const int32_t* n_tiles, const void* weights, int64_t expert_stride, int64_t N,
-                          int64_t K, float alpha, float limit, void* out, int64_t ld_out, int64_t capacity, int dtype, void* stream);
-/* Tiles of 128 rows for long steps: tgis_moe_tile_rows names the alignment (32 or 128) a mixture of n_pairs pairs over E experts of
- * W -> ff -> W should use; tgis_moe_tiled_capacity, tgis_moe_align_tiled and tgis_moe_gemm_tiled are tgis_moe_row_capacity,
- * tgis_moe_align and tgis_moe_gemm for that alignment (glu 0: plain, 1: silu(gate) * up, 2: the clamped unit with alpha, limit).
- * 128-row tiles: f16 / bf16, K a multiple of 32. */
-int tgis_moe_tile_rows(int64_t n_pairs, int64_t E, int64_t W, int64_t ff, int dtype);
-int64_t tgis_moe_tiled_capacity(int64_t n_pairs, int64_t E, int tile_rows);
-int tgis_moe_align_tiled(const int32_t* idx, int64_t n_pairs, int E, int32_t* sorted, int64_t capacity, int32_t* tile_expert,
-                         int32_t* pos_of_pair, int32_t* n_tiles, int tile_rows, void* stream);
-int tgis_moe_gemm_tiled(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
-                        const int32_t* tile_expert, const int32_t* n_tiles, const void* weights, int64_t expert_stride, int64_t N,
-                        int64_t K, int glu, float alpha, float limit, void* out, int64_t ld_out, int64_t capacity, int tile_rows,
-                        int dtype, void* stream);
 /* s residual streams per token, X [T][s][W] fp32 (s <= 8): the update of the sublayer that ran and the input of the next one,
  *   X'_b = sum_a cur.mix[a][b] X_a + cur.out[b] y   (kind 0: X' = X);   u = sum_a next.in[a] X'_a;
  *   h = u / sqrt(mean u^2 + eps) * next.gain   (h [T, W] of `dtype`)

@@ -669,12 +669,13 @@ def test_grouped_products_in_tiles_of_128_rows(gpu_device, dtype, N, K, glu):
     for tile in (128, 32):
         srt, te, pos, nt = native.moe_align(idx.to(dev), E, tile)
         cap = srt.shape[0]
-        kw = dict(glu_act=bool(glu), clamp=clamp, tile_rows=tile)
-        got = native.moe_gemm(h.to(dev), w.to(dev), N, te, nt, cap, sorted_=srt, pair_div=k, **kw)
-        got_s = native.moe_gemm(h.to(dev), w.to(dev), N, te, nt, cap, sorted_=srt, pair_div=k, pair_scale=scale.to(dev), **kw)
+        kw = dict(clamp=clamp, tile_rows=tile)
+        wi = native.MoeWeight(w.to(dev), glu=bool(glu))
+        got = native.moe_gemm(h.to(dev), wi, te, nt, cap, sorted_=srt, pair_div=k, **kw)
+        got_s = native.moe_gemm(h.to(dev), wi, te, nt, cap, sorted_=srt, pair_div=k, pair_scale=scale.to(dev), **kw)
         placed = torch.zeros(cap, K, dtype=dtype, device=dev)
         placed[pos.long()] = h.to(dev).repeat_interleave(k, 0)
-        got_p = native.moe_gemm(placed, w.to(dev), N, te, nt, cap, **kw)
+        got_p = native.moe_gemm(placed, wi, te, nt, cap, **kw)
         for out, ref_out in ((got, want), (got_s, want_scaled), (got_p, want)):
             o = out[pos.long()].double().cpu()
             assert float((o - ref_out).abs().max()) <= tol * float(ref_out.abs().max()), tile

@@ -171,12 +171,17 @@ __global__ __launch_bounds__(1024) void moe_align_kernel(const int32_t* __restri
 // ---- grouped GEMM -----------------------------------------------------------------------------------------------------
 // Workgroup = 4 waves = one 32-row tile x 128 output columns; a wave owns 32 columns (GLU: 32 gate + the 32 matching up
 // columns).  Operands come straight from global memory / L2 in MFMA fragment order: lane l holds row (l % 32) and 8 (bf16)
-// or 4 (fp32) consecutive k at offset (l / 32) * that — a 16-byte load for A and for B ([out, in] weights are k-contiguous).
-// Two shapes of workgroup (4 waves):
+// or 4 (fp32) consecutive k at offset (l / 32) * that — a 16-byte load for A and for B.
+//
+// Weights come as an IMAGE in that order: per expert [block of 32 weight rows][step of 16 (fp32: 8) k][lane][8 (4) elements], rows
+// and k padded with zeros, GLU: the gate rows' blocks, then the up rows' — a step of a block is 1 KiB in one piece, so a decode
+// step streams an expert's weights in whole lines.
+//
+// Two shapes of workgroup:
 //   many tiles (prompts): wave w owns row tile 4 y + w and 64 output columns (GLU: 64 gate + the 64 matching up columns).  The
 //     four waves walk the same weight rows at the same time, so an expert's weights come from L2 once per four row tiles
 //     instead of once per tile, and a wave's A fragment feeds two (GLU: four) products;
-//   few tiles (decode, KSPLIT): the four waves split K for ONE 32-row x 32-column block and meet in LDS, so that a launch with a
+//   few tiles (decode, KW > 1): KW waves split K for ONE 32-row x 32-column block and meet in LDS, so that a launch with a
 //     handful of tiles still has enough waves in flight to stream the expert weights.
 //
 // GLU 1: silu(gate) * up.  GLU 2 (clamped unit): g = min(gate, limit), u = clamp(up, +-limit): g sigmoid(alpha g) (u + 1).
@@ -187,23 +192,29 @@ template <int GLU> __device__ __forceinline__ float gated(float g, float u, floa
     return g / (1.f + expf(-alpha * g)) * (u + 1.f);
 }
 
-template <typename T, int GLU, bool KSPLIT>
-__global__ __launch_bounds__(256) void moe_gemm_kernel(const T* __restrict__ A, int64_t ld_a, const int32_t* __restrict__ sorted,
+template <typename T> __device__ __forceinline__ int64_t image_block(int64_t K) {  // elements of a block of 32 weight rows
+    return (K + Frag<T>::KSTEP - 1) / Frag<T>::KSTEP * (64 * Frag<T>::PER);
+}
+
+template <typename T, int GLU, int KW>
+__global__ __launch_bounds__(KW > 4 ? 512 : 256) void moe_gemm_kernel(const T* __restrict__ A, int64_t ld_a, const int32_t* __restrict__ sorted,
                                                        int pair_div, const float* __restrict__ pair_scale,
                                                        const int32_t* __restrict__ tile_expert, const int32_t* __restrict__ n_tiles,
-                                                       const T* __restrict__ Wt, int64_t expert_stride, int64_t N, int64_t K,
+                                                       const T* __restrict__ Wt, int64_t N, int64_t K,
                                                        T* __restrict__ out, int64_t ld_out, float alpha, float limit) {
+    constexpr bool KSPLIT = KW > 1;
     using F = Frag<T>;
     using V = typename F::V;
     constexpr int NB = KSPLIT ? 1 : 2;  // 32-column blocks per wave
-    __shared__ float part[KSPLIT ? 4 * (GLU ? 2 : 1) * 16 * 64 : 1];
+    __shared__ float part[KSPLIT ? KW * (GLU ? 2 : 1) * 16 * 64 : 1];
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int tile = KSPLIT ? blockIdx.y : blockIdx.y * 4 + wave;
     if (tile >= *n_tiles) return;  // KSPLIT: the whole workgroup
     const int row = lane & 31, half = lane >> 5;
     const int64_t n0 = (int64_t)blockIdx.x * 32 * NB;
     const int64_t pos = (int64_t)tile * TM + row;
-    const T* W = Wt + (int64_t)tile_expert[tile] * expert_stride;
+    const int64_t block = image_block<T>(K), nblocks = (N + 31) >> 5;
+    const T* W = Wt + (int64_t)tile_expert[tile] * nblocks * (GLU ? 2 : 1) * block;
     // A row of this lane
     int64_t arow = pos;
     float scale = 1.f;
@@ -218,28 +229,28 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const T* __restrict__ A, 
     const T* bp2[NB];
 #pragma unroll
     for (int nb = 0; nb < NB; ++nb) {
-        const int64_t n = n0 + nb * 32 + row;
-        const int64_t ncol = n < N ? n : N - 1;  // clamped: columns past N are computed and dropped
-        bp[nb] = W + ncol * K + half * F::PER;
-        bp2[nb] = GLU ? W + (N + ncol) * K + half * F::PER : nullptr;
+        const int64_t nblk = min((n0 >> 5) + nb, nblocks - 1);  // clamped: a block past the last is computed and dropped
+        bp[nb] = W + nblk * block + lane * F::PER;
+        bp2[nb] = GLU ? W + (nblocks + nblk) * block + lane * F::PER : nullptr;
     }
     f32x16 acc[NB], acc2[NB];
 #pragma unroll
     for (int nb = 0; nb < NB; ++nb) acc[nb] = acc2[nb] = f32x16{};
     // this wave's k range, in whole steps
     const int64_t steps = (K + F::KSTEP - 1) / F::KSTEP;
-    const int64_t s0 = KSPLIT ? steps * wave / 4 : 0, s1 = KSPLIT ? steps * (wave + 1) / 4 : steps;
+    const int64_t s0 = KSPLIT ? steps * wave / KW : 0, s1 = KSPLIT ? steps * (wave + 1) / KW : steps;
 #pragma unroll(KSPLIT ? 4 : 2)
-    for (int64_t kk = s0 * F::KSTEP; kk < s1 * F::KSTEP; kk += F::KSTEP) {
+    for (int64_t st = s0; st < s1; ++st) {
+        const int64_t kk = st * F::KSTEP;
         const bool in = kk + half * F::PER + F::PER <= K;  // K is a multiple of PER: a fragment is whole or absent
         V a = in ? *reinterpret_cast<const V*>(ap + kk) : F::zero();
         if (pair_scale) a = F::scaled(a, scale);
 #pragma unroll
         for (int nb = 0; nb < NB; ++nb) {
-            V b = in ? *reinterpret_cast<const V*>(bp[nb] + kk) : F::zero();
+            const V b = *reinterpret_cast<const V*>(bp[nb] + st * (64 * F::PER));
             F::mma(a, b, acc[nb]);
             if (GLU) {
-                V b2 = in ? *reinterpret_cast<const V*>(bp2[nb] + kk) : F::zero();
+                const V b2 = *reinterpret_cast<const V*>(bp2[nb] + st * (64 * F::PER));
                 F::mma(a, b2, acc2[nb]);
             }
         }
@@ -254,13 +265,13 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const T* __restrict__ A, 
         }
         __syncthreads();
         if (n0 + row >= N) return;
-        // wave w finishes accumulators 4 w .. 4 w + 3
+        // wave w finishes accumulators 16 / KW * w and on
 #pragma unroll
-        for (int q = 0; q < 4; ++q) {
-            const int i = wave * 4 + q;
+        for (int q = 0; q < 16 / KW; ++q) {
+            const int i = wave * (16 / KW) + q;
             float v = 0.f, v2 = 0.f;
 #pragma unroll
-            for (int w = 0; w < 4; ++w) {
+            for (int w = 0; w < KW; ++w) {
                 v += part[((w * NA + 0) * 16 + i) * 64 + lane];
                 if (GLU) v2 += part[((w * NA + 1) * 16 + i) * 64 + lane];
             }
@@ -296,7 +307,7 @@ template <typename T, int GLU, int BN>
 __global__ __launch_bounds__(256, 2) void moe_gemm_tiled_kernel(const T* __restrict__ A, int64_t ld_a, const int32_t* __restrict__ sorted,
                                                                 int pair_div, const float* __restrict__ pair_scale,
                                                                 const int32_t* __restrict__ tile_expert, const int32_t* __restrict__ n_tiles,
-                                                                const T* __restrict__ Wt, int64_t expert_stride, int64_t N, int64_t K,
+                                                                const T* __restrict__ Wt, int64_t N, int64_t K,
                                                                 T* __restrict__ out, int64_t ld_out, float alpha, float limit, int ncb) {
     using V = typename Frag<T>::V;
     constexpr int BK = 32, AL = TM_LONG * 4 / 256, BL = BN * 4 / 256, NJ = BN / 64;
@@ -314,7 +325,8 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_tiled_kernel(const T* __restr
     const int tile = group * 8 + in_group % rows_here, cb = in_group / rows_here;
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
     const int wr = wave >> 1, wc = wave & 1, r = lane & 31, half = lane >> 5;
-    const T* W = Wt + (int64_t)tile_expert[tile] * expert_stride;
+    const int64_t block = image_block<T>(K), nblocks = (N + 31) >> 5;
+    const T* W = Wt + (int64_t)tile_expert[tile] * nblocks * (GLU ? 2 : 1) * block;
     const int64_t n0 = (int64_t)cb * OUTC;
     auto swz = [](int row) { return ((row >> 1) ^ (row >> 3)) & 3; };
     const T* ap[AL];
@@ -338,17 +350,18 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_tiled_kernel(const T* __restr
     int boff[BL];
 #pragma unroll
     for (int i = 0; i < BL; ++i) {
-        const int e = tid + i * 256, row = e >> 2, piece = e & 3;
-        int64_t n;
-        if (GLU) {  // a wave's rows: HALF / 2 gate rows, then the matching up rows
-            const int w = row / HALF, x = row % HALF;
-            n = n0 + w * (HALF / 2) + x % (HALF / 2);
-            n = (n < N ? n : N - 1) + (x >= HALF / 2 ? N : 0);
+        // the image's order: 32 rows of one piece lie side by side
+        const int e = tid + i * 256, rb = e >> 7, piece = (e >> 5) & 3, row = rb * 32 + (e & 31);
+        int64_t nblk;
+        if (GLU) {  // a wave's blocks: HALF / 64 of gate rows, then the matching up rows'
+            constexpr int PB = HALF / 32;
+            const int w = rb / PB, x = rb % PB;
+            nblk = (n0 >> 5) + w * (PB / 2) + x % (PB / 2);
+            nblk = min(nblk, nblocks - 1) + (x >= PB / 2 ? nblocks : 0);
         } else {
-            n = n0 + row;
-            n = n < N ? n : N - 1;  // clamped: columns past N are computed and dropped
+            nblk = min((n0 >> 5) + rb, nblocks - 1);  // clamped: a block past the last is computed and dropped
         }
-        bp[i] = W + n * K + piece * 8;
+        bp[i] = W + nblk * block + ((piece >> 1) * 64 + (piece & 1) * 32 + (e & 31)) * 8;
         boff[i] = row * BK + ((piece ^ swz(row)) * 8);
     }
     f32x16 acc[2][NJ];
@@ -361,7 +374,7 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_tiled_kernel(const T* __restr
 #pragma unroll
         for (int i = 0; i < AL; ++i) ar[i] = *reinterpret_cast<const V*>(ap[i] + k);
 #pragma unroll
-        for (int i = 0; i < BL; ++i) br[i] = *reinterpret_cast<const V*>(bp[i] + k);
+        for (int i = 0; i < BL; ++i) br[i] = *reinterpret_cast<const V*>(bp[i] + k * 32);  // two steps of 512 elements per slice
     };
     auto store = [&](int buf) {
 #pragma unroll
@@ -415,13 +428,13 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_tiled_kernel(const T* __restr
 
 template <typename T>
 void launch_gemm_tiled(int glu, float alpha, float limit, const void* A, int64_t ld_a, const int32_t* sorted, int pair_div,
-                       const float* pair_scale, const int32_t* tile_expert, const int32_t* n_tiles, const void* Wt, int64_t expert_stride,
+                       const float* pair_scale, const int32_t* tile_expert, const int32_t* n_tiles, const void* Wt,
                        int64_t N, int64_t K, void* out, int64_t ld_out, int64_t max_tiles, hipStream_t st) {
 #define TGIS_MOE_TILED(GLU, BN)                                                                                                        \
     do {                                                                                                                               \
         const int ncb = (int)cdiv64(N, GLU ? BN / 2 : BN);                                                                             \
         hipLaunchKernelGGL((moe_gemm_tiled_kernel<T, GLU, BN>), dim3((unsigned)((max_tiles * ncb + 7) / 8 * 8)), dim3(256), 0, st,     \
-                           (const T*)A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, (const T*)Wt, expert_stride, N, K,   \
+                           (const T*)A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, (const T*)Wt, N, K,   \
                            (T*)out, ld_out, alpha, limit, ncb);                                                                        \
     } while (0)
     if (glu == 2)
@@ -454,25 +467,31 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const T* __restrict__ 
 
 template <typename T>
 void launch_gemm(int glu, float alpha, float limit, const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
-                 const int32_t* tile_expert, const int32_t* n_tiles, const void* Wt, int64_t expert_stride, int64_t N, int64_t K,
+                 const int32_t* tile_expert, const int32_t* n_tiles, const void* Wt, int64_t N, int64_t K,
                  void* out, int64_t ld_out, int64_t max_tiles, hipStream_t st) {
     const bool ksplit = max_tiles * cdiv64(N, 128) < 1024;
+    // few blocks (narrow experts): eight waves per block, or the launch is over before the memory system is busy
+    const bool deep = ksplit && max_tiles * cdiv64(N, 32) < 1024 && K >= 1024;
     dim3 grid((unsigned)(ksplit ? cdiv64(N, 32) : cdiv64(N, 64)), (unsigned)(ksplit ? max_tiles : cdiv64(max_tiles, 4)));
-#define TGIS_MOE_LAUNCH(GLU, KS)                                                                                              \
-    hipLaunchKernelGGL((moe_gemm_kernel<T, GLU, KS>), grid, dim3(256), 0, st, (const T*)A, ld_a, sorted, pair_div, pair_scale, \
-                       tile_expert, n_tiles, (const T*)Wt, expert_stride, N, K, (T*)out, ld_out, alpha, limit)
-    if (glu == 2 && ksplit)
-        TGIS_MOE_LAUNCH(2, true);
-    else if (glu == 2)
-        TGIS_MOE_LAUNCH(2, false);
-    else if (glu && ksplit)
-        TGIS_MOE_LAUNCH(1, true);
-    else if (glu)
-        TGIS_MOE_LAUNCH(1, false);
+#define TGIS_MOE_LAUNCH(GLU, KW)                                                                                                       \
+    hipLaunchKernelGGL((moe_gemm_kernel<T, GLU, KW>), grid, dim3(KW > 4 ? 512 : 256), 0, st, (const T*)A, ld_a, sorted, pair_div, pair_scale, \
+                       tile_expert, n_tiles, (const T*)Wt, N, K, (T*)out, ld_out, alpha, limit)
+#define TGIS_MOE_GLU(KW)                     \
+    do {                                     \
+        if (glu == 2)                        \
+            TGIS_MOE_LAUNCH(2, KW);          \
+        else if (glu)                        \
+            TGIS_MOE_LAUNCH(1, KW);          \
+        else                                 \
+            TGIS_MOE_LAUNCH(0, KW);          \
+    } while (0)
+    if (deep)
+        TGIS_MOE_GLU(8);
     else if (ksplit)
-        TGIS_MOE_LAUNCH(0, true);
+        TGIS_MOE_GLU(4);
     else
-        TGIS_MOE_LAUNCH(0, false);
+        TGIS_MOE_GLU(1);
+#undef TGIS_MOE_GLU
 #undef TGIS_MOE_LAUNCH
 }
 
@@ -481,14 +500,13 @@ void launch_gemm(int glu, float alpha, float limit, const void* A, int64_t ld_a,
 static bool dtype3(int d) { return d == TGIS_F16 || d == TGIS_BF16 || d == TGIS_F32; }
 
 static int64_t row_capacity(int64_t n_pairs, int64_t E, int64_t tm) { return (n_pairs + E * (tm - 1) + tm - 1) / tm * tm; }
-extern "C" int64_t tgis_moe_row_capacity(int64_t n_pairs, int64_t E) { return row_capacity(n_pairs, E, TM); }
+extern "C" int64_t tgis_moe_row_capacity(int64_t n_pairs, int64_t E, int tile_rows) { return row_capacity(n_pairs, E, tile_rows); }
 
 // Rows per tile a mixture of n_pairs (token, choice) pairs over E experts should be aligned to: 128 where the experts' runs are long
 // enough to fill such tiles and both products' inner widths fit the LDS-staged kernel (two-byte dtypes, multiples of 32), else 32.
 extern "C" int tgis_moe_tile_rows(int64_t n_pairs, int64_t E, int64_t W, int64_t ff, int dtype) {
     return dtype != TGIS_F32 && n_pairs >= 96 * E && W % 32 == 0 && ff % 32 == 0 ? TM_LONG : TM;
 }
-extern "C" int64_t tgis_moe_tiled_capacity(int64_t n_pairs, int64_t E, int tile_rows) { return row_capacity(n_pairs, E, tile_rows); }
 
 static int moe_route_impl(const void* h, int64_t ld_h, const float* router_w, const float* shared_gate_w, int32_t* idx,
                           float* weight, float* shared_gate, int64_t T, int64_t W, int E, int k, int dtype, void* stream,
@@ -534,91 +552,54 @@ extern "C" int tgis_moe_route_grouped(const void* h, int64_t ld_h, const float* 
                           keep_groups, renorm_eps);
 }
 
-static int moe_align_impl(const int32_t* idx, int64_t n_pairs, int E, int32_t* sorted, int64_t capacity, int32_t* tile_expert,
-                          int32_t* pos_of_pair, int32_t* n_tiles, int tile_rows, void* stream) {
+extern "C" int tgis_moe_align(const int32_t* idx, int64_t n_pairs, int E, int32_t* sorted, int64_t capacity, int32_t* tile_expert,
+                              int32_t* pos_of_pair, int32_t* n_tiles, int tile_rows, void* stream) {
     TGIS_CHECK_ARG(idx && sorted && tile_expert && pos_of_pair && n_tiles, "tgis_moe_align: null tensor");
     TGIS_CHECK_ARG(tile_rows == TM || tile_rows == TM_LONG, "tgis_moe_align: tiles of %d or %d rows", TM, TM_LONG);
     TGIS_CHECK_ARG(E >= 1 && E <= 4096 && n_pairs >= 0 && capacity >= row_capacity(n_pairs, E, tile_rows) && capacity % tile_rows == 0,
-                   "tgis_moe_align: capacity %ld below the rows of %ld pairs", (long)capacity, (long)n_pairs);
-    hipLaunchKernelGGL(moe_align_kernel, dim3(1), dim3(1024), (size_t)(3 * E + 1) * sizeof(int32_t), (hipStream_t)stream, idx, n_pairs,
+                   "tgis_moe_align: capacity %ld below tgis_moe_row_capacity", (long)capacity);
+    const int threads = n_pairs <= 1024 && capacity <= 4096 ? 256 : 1024;  // decode: barriers of four waves instead of sixteen
+    hipLaunchKernelGGL(moe_align_kernel, dim3(1), dim3(threads), (size_t)(3 * E + 1) * sizeof(int32_t), (hipStream_t)stream, idx, n_pairs,
                        E, sorted, capacity, tile_expert, pos_of_pair, n_tiles, tile_rows);
     TGIS_CHECK_LAUNCH();
     return TGIS_OK;
 }
 
-extern "C" int tgis_moe_align(const int32_t* idx, int64_t n_pairs, int E, int32_t* sorted, int64_t capacity, int32_t* tile_expert,
-                              int32_t* pos_of_pair, int32_t* n_tiles, void* stream) {
-    return moe_align_impl(idx, n_pairs, E, sorted, capacity, tile_expert, pos_of_pair, n_tiles, TM, stream);
-}
-
-extern "C" int tgis_moe_align_tiled(const int32_t* idx, int64_t n_pairs, int E, int32_t* sorted, int64_t capacity, int32_t* tile_expert,
-                                    int32_t* pos_of_pair, int32_t* n_tiles, int tile_rows, void* stream) {
-    return moe_align_impl(idx, n_pairs, E, sorted, capacity, tile_expert, pos_of_pair, n_tiles, tile_rows, stream);
-}
-
-static int moe_gemm_impl(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
-                             const int32_t* tile_expert, const int32_t* n_tiles, const void* weights, int64_t expert_stride, int64_t N,
-                             int64_t K, int glu, void* out, int64_t ld_out, int64_t capacity, int dtype, void* stream, float alpha, float limit, int tile_rows = TM) {
-    TGIS_CHECK_ARG(A && tile_expert && n_tiles && weights && out, "tgis_moe_gemm: null tensor");
-    TGIS_CHECK_ARG(dtype3(dtype), "tgis_moe_gemm: bad dtype");
+extern "C" int tgis_moe_gemm(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
+                             const int32_t* tile_expert, const int32_t* n_tiles, const void* image, int64_t N, int64_t K, int glu,
+                             float alpha, float limit, void* out, int64_t ld_out, int64_t capacity, int tile_rows, int dtype, void* stream) {
+    TGIS_CHECK_ARG(A && tile_expert && n_tiles && image && out, "tgis_moe_gemm: null tensor");
+    TGIS_CHECK_ARG(dtype3(dtype) && glu >= 0 && glu <= 2, "tgis_moe_gemm: bad dtype or glu");
     const int per = dtype == TGIS_F32 ? 4 : 8;
-    TGIS_CHECK_ARG(N >= 1 && K >= per && K % per == 0 && ld_a % per == 0 && ld_a >= K && ld_out >= N && capacity % TM == 0,
+    TGIS_CHECK_ARG(N >= 1 && K >= per && K % per == 0 && ld_a % per == 0 && ld_a >= K && ld_out >= N,
                    "tgis_moe_gemm: K (%ld) and the A row stride (%ld) must be multiples of %d", (long)K, (long)ld_a, per);
-    TGIS_CHECK_ARG((((uintptr_t)A) & 15) == 0 && (((uintptr_t)weights) & 15) == 0 && (expert_stride * (dtype == TGIS_F32 ? 4 : 2)) % 16 == 0,
-                   "tgis_moe_gemm: operands must be 16-byte aligned");
+    TGIS_CHECK_ARG((((uintptr_t)A) & 15) == 0 && (((uintptr_t)image) & 15) == 0, "tgis_moe_gemm: operands must be 16-byte aligned");
     TGIS_CHECK_ARG(!sorted || pair_div >= 1, "tgis_moe_gemm: gathered rows need pair_div >= 1");
     TGIS_CHECK_ARG(!pair_scale || sorted, "tgis_moe_gemm: a per-pair scale needs the sorted pair list");
+    TGIS_CHECK_ARG((tile_rows == TM || tile_rows == TM_LONG) && capacity % tile_rows == 0, "tgis_moe_gemm: tiles of %d or %d rows", TM, TM_LONG);
     if (capacity == 0) return TGIS_OK;
     hipStream_t st = (hipStream_t)stream;
     TgisTimedScope timed(TGIS_OP_MOE_GEMM, st);
+    const int64_t tiles = capacity / tile_rows;
     if (tile_rows == TM_LONG) {
-        TGIS_CHECK_ARG(dtype != TGIS_F32 && K % 32 == 0 && capacity % TM_LONG == 0 && capacity / TM_LONG * cdiv64(N, 128) < (1ll << 30),
+        TGIS_CHECK_ARG(dtype != TGIS_F32 && K % 32 == 0 && tiles * cdiv64(N, 128) < (1ll << 30),
                        "tgis_moe_gemm: 128-row tiles take two-byte dtypes and K a multiple of 32 (got %ld)", (long)K);
         if (dtype == TGIS_F16)
-            launch_gemm_tiled<f16>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, out, ld_out, capacity / TM_LONG, st);
+            launch_gemm_tiled<f16>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, image, N, K, out, ld_out, tiles, st);
         else
-            launch_gemm_tiled<bf16>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, out, ld_out, capacity / TM_LONG, st);
+            launch_gemm_tiled<bf16>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, image, N, K, out, ld_out, tiles, st);
         TGIS_CHECK_LAUNCH();
         return TGIS_OK;
     }
-    TGIS_CHECK_ARG(tile_rows == TM, "tgis_moe_gemm: tiles of %d or %d rows", TM, TM_LONG);
-    const int64_t tiles = capacity / TM;
     TGIS_CHECK_ARG(tiles <= 65535, "tgis_moe_gemm: %ld tiles exceed one grid", (long)tiles);
     if (dtype == TGIS_F16)
-        launch_gemm<f16>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, out, ld_out, tiles, st);
+        launch_gemm<f16>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, image, N, K, out, ld_out, tiles, st);
     else if (dtype == TGIS_BF16)
-        launch_gemm<bf16>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, out, ld_out, tiles, st);
+        launch_gemm<bf16>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, image, N, K, out, ld_out, tiles, st);
     else
-        launch_gemm<float>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, out, ld_out, tiles, st);
+        launch_gemm<float>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, image, N, K, out, ld_out, tiles, st);
     TGIS_CHECK_LAUNCH();
     return TGIS_OK;
-}
-
-extern "C" int tgis_moe_gemm(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
-                             const int32_t* tile_expert, const int32_t* n_tiles, const void* weights, int64_t expert_stride, int64_t N,
-                             int64_t K, int glu, void* out, int64_t ld_out, int64_t capacity, int dtype, void* stream) {
-    return moe_gemm_impl(A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, glu != 0 ? 1 : 0, out, ld_out,
-                         capacity, dtype, stream, 0.f, 0.f);
-}
-
-// The same over stacked [gate | up] weights with the clamped unit: g = min(gate, limit), u = clamp(up, -limit, limit),
-// g * sigmoid(alpha * g) * (u + 1).
-extern "C" int tgis_moe_gemm_clamped(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
-                                     const int32_t* tile_expert, const int32_t* n_tiles, const void* weights, int64_t expert_stride, int64_t N,
-                                     int64_t K, float alpha, float limit, void* out, int64_t ld_out, int64_t capacity, int dtype,
-                                     void* stream) {
-    return moe_gemm_impl(A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, 2, out, ld_out, capacity,
-                         dtype, stream, alpha, limit);
-}
-
-// Any of the three (glu 0: plain, 1: silu(gate) * up, 2: the clamped unit) over pairs aligned to tiles of tile_rows rows.
-extern "C" int tgis_moe_gemm_tiled(const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
-                                   const int32_t* tile_expert, const int32_t* n_tiles, const void* weights, int64_t expert_stride, int64_t N,
-                                   int64_t K, int glu, float alpha, float limit, void* out, int64_t ld_out, int64_t capacity, int tile_rows,
-                                   int dtype, void* stream) {
-    TGIS_CHECK_ARG(glu >= 0 && glu <= 2, "tgis_moe_gemm_tiled: glu 0, 1 or 2");
-    return moe_gemm_impl(A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, weights, expert_stride, N, K, glu, out, ld_out, capacity,
-                         dtype, stream, alpha, limit, tile_rows);
 }
 
 extern "C" int tgis_moe_combine(const void* rows, int64_t ld_rows, const int32_t* pos_of_pair, const float* pair_weight, int k,

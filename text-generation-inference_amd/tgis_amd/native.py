@@ -104,11 +104,11 @@ SIGNATURES = {
     "tgis_wkv_decay": (_c_int, [_vp, _c_i64, _vp, _vp, _vp, _c_i64, _c_int, _c_i64, _c_int, _vp]),
     "tgis_wkv_scan": (_c_int, [_vp, _vp, _vp, _vp, _c_i64, _vp, _vp, _vp, _vp, _vp, _vp, _c_i64, _vp, _vp, _vp, _vp, _c_i64,
                                _c_i64, _c_int, _c_int, _c_f, _c_int, _vp]),
-    "tgis_moe_row_capacity": (_c_i64, [_c_i64, _c_i64]),
+    "tgis_moe_row_capacity": (_c_i64, [_c_i64, _c_i64, _c_int]),
     "tgis_moe_route": (_c_int, [_vp, _c_i64, _vp, _vp, _vp, _vp, _vp, _c_i64, _c_i64, _c_int, _c_int, _c_int, _vp]),
-    "tgis_moe_align": (_c_int, [_vp, _c_i64, _c_int, _vp, _c_i64, _vp, _vp, _vp, _vp]),
-    "tgis_moe_gemm": (_c_int, [_vp, _c_i64, _vp, _c_int, _vp, _vp, _vp, _vp, _c_i64, _c_i64, _c_i64, _c_int, _vp, _c_i64, _c_i64,
-                               _c_int, _vp]),
+    "tgis_moe_align": (_c_int, [_vp, _c_i64, _c_int, _vp, _c_i64, _vp, _vp, _vp, _c_int, _vp]),
+    "tgis_moe_gemm": (_c_int, [_vp, _c_i64, _vp, _c_int, _vp, _vp, _vp, _vp, _c_i64, _c_i64, _c_int, _c_f, _c_f, _vp, _c_i64, _c_i64,
+                               _c_int, _c_int, _vp]),
     "tgis_moe_combine": (_c_int, [_vp, _c_i64, _vp, _vp, _c_int, _vp, _c_i64, _vp, _vp, _c_i64, _c_i64, _c_i64, _c_int, _vp]),
     "tgis_residual_update_f32": (_c_int, [_vp, _vp, _c_i64, _c_int, _vp, _c_f, _c_f, _vp, _vp, _c_f, _vp, _c_int, _c_i64, _c_i64,
                                           _c_f, _vp]),
@@ -170,13 +170,7 @@ SIGNATURES = {
     "tgis_head_product": (_c_int, [_vp, _c_i64, _c_i64, _vp, _vp, _c_i64, _c_i64, _c_i64, _c_int, _c_int, _c_int, _c_int, _vp]),
     "tgis_min_gru_scan": (_c_int, [_vp, _c_i64, _c_i64, _c_i64, _c_i64, _vp, _vp, _vp, _vp, _vp, _c_i64, _c_f, _c_i64, _c_i64, _c_i64,
                                    _c_i64, _c_int, _vp]),
-    "tgis_moe_gemm_clamped": (_c_int, [_vp, _c_i64, _vp, _c_int, _vp, _vp, _vp, _vp, _c_i64, _c_i64, _c_i64, _c_f, _c_f, _vp, _c_i64,
-                                       _c_i64, _c_int, _vp]),
     "tgis_moe_tile_rows": (_c_int, [_c_i64, _c_i64, _c_i64, _c_i64, _c_int]),
-    "tgis_moe_tiled_capacity": (_c_i64, [_c_i64, _c_i64, _c_int]),
-    "tgis_moe_align_tiled": (_c_int, [_vp, _c_i64, _c_int, _vp, _c_i64, _vp, _vp, _vp, _c_int, _vp]),
-    "tgis_moe_gemm_tiled": (_c_int, [_vp, _c_i64, _vp, _c_int, _vp, _vp, _vp, _vp, _c_i64, _c_i64, _c_i64, _c_int, _c_f, _c_f, _vp, _c_i64,
-                                     _c_i64, _c_int, _c_int, _vp]),
     "tgis_hyper_update": (_c_int, [_vp, _vp, _vp, _c_i64, _c_f, _vp, _c_int, _vp, _c_i64, _c_int, _vp, _vp, _c_int, _vp, _c_i64, _c_int,
                                    _vp, _vp, _vp, _vp, _c_i64, _c_i64, _c_int, _c_f, _c_int, _vp]),
 }
@@ -1002,8 +996,8 @@ def wkv_scan(r, k, v, gate, logw, u, gain, state, shift_state, h, state_slots, c
     return out
 
 
-def moe_row_capacity(n_pairs: int, E: int) -> int:
-    return load_library().tgis_moe_row_capacity(n_pairs, E)
+def moe_row_capacity(n_pairs: int, E: int, tile_rows: int = 32) -> int:
+    return load_library().tgis_moe_row_capacity(n_pairs, E, tile_rows)
 
 
 def moe_route(h, router_w, shared_gate_w, k: int, router_b=None, softmax_top: bool = False):
@@ -1032,33 +1026,46 @@ def moe_tile_rows(n_pairs: int, E: int, W: int, ff: int, dtype: torch.dtype) -> 
 def moe_align(idx: torch.Tensor, E: int, tile_rows: int = 32):
     """(sorted [cap], tile_expert [cap / tile_rows], pos_of_pair [pairs], n_tiles [1]) for idx [T, k]."""
     n = idx.numel()
-    lib = load_library()
-    cap = lib.tgis_moe_tiled_capacity(n, E, tile_rows)
+    cap = moe_row_capacity(n, E, tile_rows)
     dev = idx.device
     sorted_ = torch.empty((cap,), dtype=torch.int32, device=dev)
     tile_expert = torch.empty((cap // tile_rows,), dtype=torch.int32, device=dev)
     pos = torch.empty((n,), dtype=torch.int32, device=dev)
     n_tiles = torch.empty((1,), dtype=torch.int32, device=dev)
-    _check(lib.tgis_moe_align_tiled(_i32(idx, "idx"), n, E, _ptr(sorted_), cap, _ptr(tile_expert), _ptr(pos), _ptr(n_tiles), tile_rows,
-                                    _stream()), "tgis_moe_align_tiled")
+    _check(load_library().tgis_moe_align(_i32(idx, "idx"), n, E, _ptr(sorted_), cap, _ptr(tile_expert), _ptr(pos), _ptr(n_tiles), tile_rows,
+                                         _stream()), "tgis_moe_align")
     return sorted_, tile_expert, pos, n_tiles
 
 
-def moe_gemm(A, weights, N: int, tile_expert, n_tiles, capacity: int, sorted_=None, pair_div: int = 1, pair_scale=None,
-             glu_act: bool = False, clamp=None, tile_rows: int = 32):
-    """weights [E, N (glu: 2 N), K]; returns [capacity, N].  glu_act: silu(gate) * up, or with clamp = (alpha, limit) the clamped
-    unit.  tile_rows: the alignment moe_align was asked for."""
-    assert A.dim() == 2 and A.stride(1) == 1 and weights.dim() == 3 and weights.is_contiguous() and weights.dtype == A.dtype
-    K = weights.shape[2]
-    assert weights.shape[1] == (2 * N if glu_act else N) and A.shape[1] == K
+class MoeWeight:
+    """The experts' weights [E, N (glu: 2 N, gate rows then up rows), K] as the image tgis_moe_gemm streams: per expert, blocks of 32
+    rows x steps of 16 (fp32: 8) k in fragment order, padded with zeros."""
+
+    def __init__(self, weights: torch.Tensor, glu: bool):
+        E, R, K = weights.shape
+        self.E, self.glu, self.N, self.K, self.dtype = E, bool(glu), R // 2 if glu else R, K, weights.dtype
+        step, per = (8, 4) if weights.dtype == torch.float32 else (16, 8)
+        parts = 2 if glu else 1
+        w = weights.reshape(E, parts, self.N, K)
+        w = torch.nn.functional.pad(w, (0, -K % step, 0, -self.N % 32))
+        nb, ks = w.shape[2] // 32, w.shape[3] // step
+        # [E, parts, block, row, step, half, per] -> [E, parts, block, step, half, row, per]
+        self.image = w.reshape(E, parts, nb, 32, ks, 2, per).permute(0, 1, 2, 4, 5, 3, 6).contiguous()
+
+
+def moe_gemm(A, w: MoeWeight, tile_expert, n_tiles, capacity: int, sorted_=None, pair_div: int = 1, pair_scale=None, clamp=None,
+             tile_rows: int = 32):
+    """Returns [capacity, w.N].  A gate | up weight is activated: silu(gate) * up, or with clamp = (alpha, limit) the clamped unit.
+    tile_rows: the alignment moe_align was asked for."""
+    assert A.dim() == 2 and A.stride(1) == 1 and w.dtype == A.dtype and A.shape[1] == w.K
     assert capacity % tile_rows == 0 and tile_expert.shape[0] * tile_rows == capacity and (sorted_ is not None or A.shape[0] >= capacity)
-    out = torch.empty((capacity, N), dtype=A.dtype, device=A.device)
-    glu = (2 if clamp is not None else 1) if glu_act else 0
+    out = torch.empty((capacity, w.N), dtype=A.dtype, device=A.device)
+    glu = (2 if clamp is not None else 1) if w.glu else 0
     alpha, limit = clamp if clamp is not None else (0.0, 0.0)
-    _check(load_library().tgis_moe_gemm_tiled(
+    _check(load_library().tgis_moe_gemm(
         _ptr(A), A.stride(0), _i32(sorted_, "sorted"), pair_div, _f32(pair_scale, "pair_scale"), _ptr(tile_expert), _ptr(n_tiles),
-        _ptr(weights), weights.stride(0), N, K, glu, float(alpha), float(limit), _ptr(out), out.stride(0), capacity, tile_rows,
-        dtype_code3(A.dtype), _stream()), "tgis_moe_gemm_tiled")
+        _ptr(w.image), w.N, w.K, glu, float(alpha), float(limit), _ptr(out), out.stride(0), capacity, tile_rows, dtype_code3(A.dtype),
+        _stream()), "tgis_moe_gemm")
     return out
 
 

@@ -203,11 +203,11 @@ class RoutedExperts:
         # with zero rows / columns once, here (silu(0) * 0 = 0 keeps a padded hidden channel out of the result)
         self.W, self.Wp, self.ff = W, pad8(W), pad8(ff)
         pad = lambda t, rows, cols: torch.nn.functional.pad(t, (0, cols - t.shape[1], 0, rows - t.shape[0]))
-        # [E, 2 ff, W] (gate rows, then up rows) and [E, W, ff]
-        self.w_gate_up = torch.stack([torch.cat([pad(gate[e], self.ff, self.Wp),
-                                                 pad(weights.get_tensor(f"{prefix}.e{e}.up"), self.ff, self.Wp)], 0)
-                                      for e in range(experts)]).contiguous()
-        self.w_down = torch.stack([pad(weights.get_tensor(f"{prefix}.e{e}.down"), W, self.ff) for e in range(experts)]).contiguous()
+        # [E, 2 ff, W] (gate rows, then up rows) and [E, W, ff], each as the image the grouped GEMM streams
+        self.w_gate_up = native.MoeWeight(torch.stack([torch.cat([pad(gate[e], self.ff, self.Wp),
+                                                                  pad(weights.get_tensor(f"{prefix}.e{e}.up"), self.ff, self.Wp)], 0)
+                                                       for e in range(experts)]), glu=True)
+        self.w_down = native.MoeWeight(torch.stack([pad(weights.get_tensor(f"{prefix}.e{e}.down"), W, self.ff) for e in range(experts)]), glu=False)
         self.clamp = clamp
         self.shared = None
         if shared and shared_clamp is not None:
@@ -228,9 +228,9 @@ class RoutedExperts:
         sorted_, tile_expert, pos, n_tiles = native.moe_align(idx, self.E, tm)
         cap = sorted_.shape[0]
         hp = h if self.Wp == W else torch.nn.functional.pad(h, (0, self.Wp - W))
-        act = native.moe_gemm(hp, self.w_gate_up, self.ff, tile_expert, n_tiles, cap, sorted_=sorted_, pair_div=self.k,
-                              pair_scale=weight.view(-1) if self.weight_on_input else None, glu_act=True, clamp=self.clamp, tile_rows=tm)
-        rows = native.moe_gemm(act, self.w_down, W, tile_expert, n_tiles, cap, tile_rows=tm)
+        act = native.moe_gemm(hp, self.w_gate_up, tile_expert, n_tiles, cap, sorted_=sorted_, pair_div=self.k,
+                              pair_scale=weight.view(-1) if self.weight_on_input else None, clamp=self.clamp, tile_rows=tm)
+        rows = native.moe_gemm(act, self.w_down, tile_expert, n_tiles, cap, tile_rows=tm)
         shared = self.shared(h, partial=defer) if self.shared is not None else None
         if defer:
             return native.MixtureRows(rows, pos, None if self.weight_on_input else weight.view(-1), self.k, shared, sg)
