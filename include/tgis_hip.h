@@ -402,7 +402,8 @@ int tgis_moe_route(const void* h, int64_t ld_h, const float* router_w, const flo
 int tgis_moe_align(const int32_t* idx, int64_t n_pairs, int E, int32_t* sorted, int64_t capacity, int32_t* tile_expert,
                    int32_t* pos_of_pair, int32_t* n_tiles, int tile_rows, void* stream);
 /* out[row][n] = sum_c a(row)[c] * W[tile_expert[row / tile_rows]][n][c].
- * a(row) = A[sorted[row] / pair_div] * pair_scale[sorted[row]] (rounded to T) when sorted != NULL, else A[row].
+ * a(row) = A[sorted[row] / pair_div] * pair_scale[sorted[row]] (rounded to T) when sorted != NULL, else A[row]; with sorted and
+ * pair_div 0 the rows are in place and the list only tells which of them are padding.
  * glu 1: out = silu(gate) * up;  2: g = min(gate, limit), u = clamp(up, -limit, limit), out = g sigmoid(alpha g) (u + 1).
  * image: the experts' weights in fragment order, per expert [ceil(N / 32) blocks of weight rows (glu: the gate rows' blocks, then
  * the up rows')][ceil(K / 16) steps (fp32: K / 8)][64 lanes][8 (fp32: 4) elements]: lane l of a step holds row l % 32 of the block
@@ -652,11 +653,15 @@ int tgis_min_gru_scan(const void* proj, int64_t ld, int64_t z_col0, int64_t x_co
  * cur = [s * s mix (from, to) | s out], next = [s in | gain], fp32.  y by kind: 1 a [T, ld_y] tensor of `dtype`; 2 the fp32 split-K
  * slabs of tgis_dense_gemm_partial (ld_y their row stride); 3 a mixture: sum_j weight[t][j] y[pos[t][j]] over k expert rows, plus
  * shared_gate[t] * shared[t] (shared: rows of `dtype`, or slabs if shared_slabs > 0; weight, shared, shared_gate may be NULL).
+ * router_w [E][W] fp32 (or NULL): the next sublayer is a mixture — idx / route_weight [T][top] and route_gate [T] (with router_sg [W])
+ * receive what tgis_moe_route_ext makes of the (unrounded) row h; top <= 64.
  * ids instead of x (kind 0): every stream is table[ids[t]] * emb_scale.  x_out (may alias x, may be NULL) receives X'. */
 int tgis_hyper_update(const float* x, const int64_t* ids, const void* table, int64_t vocab, float emb_scale, float* x_out,
                       int kind, const void* y, int64_t ld_y, int slabs, const int32_t* pos, const float* weight, int k,
                       const void* shared, int64_t ld_shared, int shared_slabs, const float* shared_gate, const float* cur,
-                      const float* next, void* h, int64_t rows, int64_t W, int streams, float eps, int dtype, void* stream);
+                      const float* next, void* h, int64_t rows, int64_t W, int streams, float eps, const float* router_w,
+                      const float* router_sg, int E, int top, int softmax_top, int32_t* idx, float* route_weight,
+                      float* route_gate, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

@@ -310,6 +310,39 @@ def test_stream_mix_and_norm(gpu_device, dtype, streams, W, T):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("W,E,k,softmax_top,gate", [(72, 6, 2, True, True), (37, 3, 3, True, False), (256, 130, 8, False, True), (64, 1, 1, True, True)])
+def test_routing_inside_the_stream_update(gpu_device, dtype, W, E, k, softmax_top, gate):
+    """The update's own routing against the router launch on the same row, and against its definition."""
+    from tgis_amd import native
+
+    g = torch.Generator().manual_seed(W + E)
+    dev, T, s = gpu_device, 33, 2
+    X, y = torch.randn(T, s, W, generator=g), torch.randn(T, W, generator=g).to(dtype)
+    cur, nxt = torch.randn(s * s + s, generator=g), torch.cat([torch.randn(s, generator=g), torch.tensor([1.1])])
+    rw, sg = torch.randn(E, W, generator=g) * W ** -0.5, torch.randn(W, generator=g) * W ** -0.5
+    sg = sg if gate else None
+    new = torch.einsum("ab,taw->tbw", cur[:s * s].view(s, s).double(), X.double()) + cur[s * s:].double()[None, :, None] * y.double()[:, None]
+    h = ref.rms_unit(torch.einsum("a,taw->tw", nxt[:s].double(), new), 1e-5) * nxt[s].double()
+    logits = h @ rw.double().T
+    _, _, (idx, wt, gt) = native.hyper_update(X.to(dev), y.to(dev), cur.to(dev), nxt.to(dev), 1e-5, dtype,
+                                              router=(rw.to(dev), sg.to(dev) if gate else None, k, softmax_top))
+    ri, rwt, rg = native.moe_route(h.float().to(dev), rw.to(dev), sg.to(dev) if gate else None, k, softmax_top=softmax_top)
+    val, want = logits.topk(k, dim=-1)
+    ww = torch.softmax(val, -1) if softmax_top else torch.sigmoid(val)
+    for i, w in ((idx, wt), (ri, rwt)):
+        sure = torch.ones(T, dtype=torch.bool)
+        if k < E:
+            b = logits.sort(-1, descending=True).values[:, :k + 1]
+            sure = (b[:, :-1] - b[:, 1:]).min(-1).values > 1e-4
+        assert torch.equal(i.cpu().long()[sure], want[sure]) and float((w.double().cpu() - ww)[sure].abs().max()) < 1e-4
+    if gate:
+        for x in (gt, rg):
+            assert float((x.double().cpu() - torch.sigmoid(h @ sg.double())).abs().max()) < 1e-5
+    else:
+        assert gt is None
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
 def test_streams_begin_as_copies_of_the_embedding(gpu_device, dtype):
     from tgis_amd import native
 
@@ -676,7 +709,8 @@ def test_grouped_products_in_tiles_of_128_rows(gpu_device, dtype, N, K, glu):
         placed = torch.zeros(cap, K, dtype=dtype, device=dev)
         placed[pos.long()] = h.to(dev).repeat_interleave(k, 0)
         got_p = native.moe_gemm(placed, wi, te, nt, cap, **kw)
-        for out, ref_out in ((got, want), (got_s, want_scaled), (got_p, want)):
+        got_m = native.moe_gemm(placed, wi, te, nt, cap, sorted_=srt, pair_div=0, **kw)
+        for out, ref_out in ((got, want), (got_s, want_scaled), (got_p, want), (got_m, want)):
             o = out[pos.long()].double().cpu()
             assert float((o - ref_out).abs().max()) <= tol * float(ref_out.abs().max()), tile
 

@@ -14,6 +14,7 @@
 // n_tiles leave at once.
 #include "common.h"
 #include "mfma_frag.h"
+#include "route_top.h"
 
 namespace {
 
@@ -56,6 +57,12 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
         if (lane == 0) logit[e] = s + ((router_b && e < E) ? router_b[e] : 0.f);
     }
     __syncthreads();
+    if (softmax_top != 2 && k <= 64) {
+        if (wave != 0) return;
+        if (lane == 0 && wg) shared_gate[t] = 1.f / (1.f + expf(-logit[E]));
+        route_top_wave(logit, E, k, softmax_top, idx + t * k, weight + t * k);
+        return;
+    }
     if (threadIdx.x == 0) {
         if (wg) shared_gate[t] = 1.f / (1.f + expf(-logit[E]));
         if (softmax_top == 2) {
@@ -218,10 +225,11 @@ __global__ __launch_bounds__(KW > 4 ? 512 : 256) void moe_gemm_kernel(const T* _
     // A row of this lane
     int64_t arow = pos;
     float scale = 1.f;
+    bool live = true;
     if (sorted) {
         const int32_t p = sorted[pos];
-        const bool live = p >= 0;
-        arow = live ? p / pair_div : 0;
+        live = p >= 0;
+        if (pair_div > 0) arow = live ? p / pair_div : 0;
         if (pair_scale) scale = live ? pair_scale[p] : 0.f;
     }
     const T* ap = A + arow * ld_a + half * F::PER;
@@ -242,7 +250,9 @@ __global__ __launch_bounds__(KW > 4 ? 512 : 256) void moe_gemm_kernel(const T* _
 #pragma unroll(KSPLIT ? 4 : 2)
     for (int64_t st = s0; st < s1; ++st) {
         const int64_t kk = st * F::KSTEP;
-        const bool in = kk + half * F::PER + F::PER <= K;  // K is a multiple of PER: a fragment is whole or absent
+        // K is a multiple of PER: a fragment is whole or absent.  Padding rows are not fetched: a decode step has a few live rows
+        // per tile, and their lines are as many as the weights' otherwise
+        const bool in = live && kk + half * F::PER + F::PER <= K;
         V a = in ? *reinterpret_cast<const V*>(ap + kk) : F::zero();
         if (pair_scale) a = F::scaled(a, scale);
 #pragma unroll
@@ -340,7 +350,7 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_tiled_kernel(const T* __restr
         asc[i] = 1.f;
         if (sorted) {
             const int32_t p = sorted[pos];
-            arow = p >= 0 ? p / pair_div : 0;
+            if (pair_div > 0) arow = p >= 0 ? p / pair_div : 0;
             if (pair_scale) asc[i] = p >= 0 ? pair_scale[p] : 0.f;
         }
         ap[i] = A + arow * ld_a + piece * 8;
@@ -574,7 +584,7 @@ extern "C" int tgis_moe_gemm(const void* A, int64_t ld_a, const int32_t* sorted,
     TGIS_CHECK_ARG(N >= 1 && K >= per && K % per == 0 && ld_a % per == 0 && ld_a >= K && ld_out >= N,
                    "tgis_moe_gemm: K (%ld) and the A row stride (%ld) must be multiples of %d", (long)K, (long)ld_a, per);
     TGIS_CHECK_ARG((((uintptr_t)A) & 15) == 0 && (((uintptr_t)image) & 15) == 0, "tgis_moe_gemm: operands must be 16-byte aligned");
-    TGIS_CHECK_ARG(!sorted || pair_div >= 1, "tgis_moe_gemm: gathered rows need pair_div >= 1");
+    TGIS_CHECK_ARG(!sorted || pair_div >= 0, "tgis_moe_gemm: gathered rows need pair_div >= 1, rows in place pair_div 0");
     TGIS_CHECK_ARG(!pair_scale || sorted, "tgis_moe_gemm: a per-pair scale needs the sorted pair list");
     TGIS_CHECK_ARG((tile_rows == TM || tile_rows == TM_LONG) && capacity % tile_rows == 0, "tgis_moe_gemm: tiles of %d or %d rows", TM, TM_LONG);
     if (capacity == 0) return TGIS_OK;

@@ -135,10 +135,12 @@ class FlashGopetarModel:
         X, h = residual.begin(input_ids, self.embed, self.config.embedding_scale, dt)
         q = 0
         for layer in self.layers:
-            X, h = residual.step(q, X, layer.mix(h, position_ids, kv), dt)
+            # the mixture's router rides in the update in front of it, its sum in the update behind it
+            router = layer.ff.plain_router if layer.ff is not None else None
+            X, h, routed = residual.step(q, X, layer.mix(h, position_ids, kv), dt, router)
             q += 1
             if layer.ff is not None:
-                X, h = residual.step(q, X, layer.ff(h, defer=True), dt)
+                X, h, _ = residual.step(q, X, layer.ff(h, defer=True, routed=routed), dt)
                 q += 1
             if kv.residual_trace is not None:
                 kv.residual_trace.append(X.sum(1))

@@ -172,7 +172,8 @@ SIGNATURES = {
                                    _c_i64, _c_int, _vp]),
     "tgis_moe_tile_rows": (_c_int, [_c_i64, _c_i64, _c_i64, _c_i64, _c_int]),
     "tgis_hyper_update": (_c_int, [_vp, _vp, _vp, _c_i64, _c_f, _vp, _c_int, _vp, _c_i64, _c_int, _vp, _vp, _c_int, _vp, _c_i64, _c_int,
-                                   _vp, _vp, _vp, _vp, _c_i64, _c_i64, _c_int, _c_f, _c_int, _vp]),
+                                   _vp, _vp, _vp, _vp, _c_i64, _c_i64, _c_int, _c_f, _vp, _vp, _c_int, _c_int, _c_int, _vp, _vp, _vp,
+                                   _c_int, _vp]),
 }
 
 _lib = None
@@ -1055,10 +1056,10 @@ class MoeWeight:
 
 def moe_gemm(A, w: MoeWeight, tile_expert, n_tiles, capacity: int, sorted_=None, pair_div: int = 1, pair_scale=None, clamp=None,
              tile_rows: int = 32):
-    """Returns [capacity, w.N].  A gate | up weight is activated: silu(gate) * up, or with clamp = (alpha, limit) the clamped unit.
+    """Returns [capacity, w.N].  sorted_ with pair_div 0: rows in place, the list marks padding.  A gate | up weight is activated: silu(gate) * up, or with clamp = (alpha, limit) the clamped unit.
     tile_rows: the alignment moe_align was asked for."""
     assert A.dim() == 2 and A.stride(1) == 1 and w.dtype == A.dtype and A.shape[1] == w.K
-    assert capacity % tile_rows == 0 and tile_expert.shape[0] * tile_rows == capacity and (sorted_ is not None or A.shape[0] >= capacity)
+    assert capacity % tile_rows == 0 and tile_expert.shape[0] * tile_rows == capacity and ((sorted_ is not None and pair_div > 0) or A.shape[0] >= capacity)
     out = torch.empty((capacity, w.N), dtype=A.dtype, device=A.device)
     glu = (2 if clamp is not None else 1) if w.glu else 0
     alpha, limit = clamp if clamp is not None else (0.0, 0.0)
@@ -1595,11 +1596,12 @@ class MixtureRows:
         self.rows, self.pos, self.weight, self.k, self.shared, self.shared_gate = rows, pos, weight, k, shared, shared_gate
 
 
-def hyper_update(x, y, cur, nxt, eps: float, y_dtype, ids=None, table=None, emb_scale: float = 1.0, x_out=None, streams: int = 0):
+def hyper_update(x, y, cur, nxt, eps: float, y_dtype, ids=None, table=None, emb_scale: float = 1.0, x_out=None, streams: int = 0, router=None):
     """x [T, s, W] fp32: x_out (in place unless given) <- mix x + out y, and h = rms_norm(sum_a in[a] x_out[a]) * gain in y_dtype.
     cur = [s * s | s], nxt = [s | 1] fp32 coefficient rows; y: a tensor of y_dtype, split-K slabs (`Partial`), `MixtureRows`, or None
-    (x stays).  ids + table instead of x: the streams begin as copies of the scaled embedding rows (s = `streams`).  Returns
-    (x_out, h)."""
+    (x stays).  ids + table instead of x: the streams begin as copies of the scaled embedding rows (s = `streams`).  router =
+    (weight [E, W] fp32, shared gate [W] fp32 or None, top, softmax_top): the next sublayer's routing is made on the way.  Returns
+    (x_out, h), with a router (x_out, h, (idx, weight, gate) as moe_route does)."""
     if ids is not None:
         assert x is None and y is None and ids.dtype == torch.int64 and table.is_contiguous() and table.dtype == y_dtype
         T, s, W = ids.shape[0], int(streams), table.shape[1]
@@ -1627,8 +1629,15 @@ def hyper_update(x, y, cur, nxt, eps: float, y_dtype, ids=None, table=None, emb_
         assert y.shape == (T, W) and y.dtype == y_dtype and y.stride(1) == 1
         kind, p, ld = 1, _ptr(y), y.stride(0)
     h = torch.empty((T, W), dtype=y_dtype, device=nxt.device)
+    routed, r_args = None, (None, None, 0, 0, 0, None, None, None)
+    if router is not None:
+        rw, rsg, top, softmax_top = router
+        assert rw.shape[1] == W and (rsg is None or rsg.shape[0] == W)
+        routed = (torch.empty((T, top), dtype=torch.int32, device=h.device), torch.empty((T, top), dtype=torch.float32, device=h.device),
+                  torch.empty((T,), dtype=torch.float32, device=h.device) if rsg is not None else None)
+        r_args = (_f32(rw, "router_w"), _f32(rsg, "router_sg"), rw.shape[0], top, int(softmax_top), _ptr(routed[0]), _ptr(routed[1]), _ptr(routed[2]))
     _check(load_library().tgis_hyper_update(
         _ptr(x), _ptr(ids), _ptr(table), table.shape[0] if table is not None else 0, float(emb_scale), _ptr(x_out), kind, p, ld, slabs, pos,
         weight, k, sh, ld_sh, sh_slabs, gate, _f32(cur, "cur") if kind else None, _f32(nxt, "nxt"), _ptr(h), T, W, s, float(eps),
-        dtype_code3(y_dtype), _stream()), "tgis_hyper_update")
-    return x_out, h
+        *r_args, dtype_code3(y_dtype), _stream()), "tgis_hyper_update")
+    return (x_out, h) if routed is None else (x_out, h, routed)

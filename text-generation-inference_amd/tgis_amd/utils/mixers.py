@@ -216,10 +216,20 @@ class RoutedExperts:
             self.shared = GatedUnit(weights, f"{prefix}.shared")
         self.shared_gate = _f32(weights.get_tensor(f"{prefix}.shared.sg")).reshape(-1) if shared else None
 
-    def forward(self, h: torch.Tensor, defer: bool = False):
-        """defer: the sum over a token's rows is left to the consumer (native.MixtureRows)."""
+    @property
+    def plain_router(self):
+        """What a residual update needs to route for this mixture on the way (native.hyper_update), or None."""
+        if self.grouped_softmax or self.router_b is not None or self.k > 64:
+            return None
+        return self.router, self.shared_gate, self.k, self.softmax_top
+
+    def forward(self, h: torch.Tensor, defer: bool = False, routed=None):
+        """defer: the sum over a token's rows is left to the consumer (native.MixtureRows).  routed: (idx, weight, shared gate), if
+        the routing is made already."""
         T, W = h.shape
-        if self.grouped_softmax:
+        if routed is not None:
+            idx, weight, sg = routed
+        elif self.grouped_softmax:
             idx, weight = native.moe_route_grouped(h, self.router, self.correction, self.k, self.groups, self.keep_groups, self.renorm_eps)
             sg = None
         else:
@@ -230,7 +240,7 @@ class RoutedExperts:
         hp = h if self.Wp == W else torch.nn.functional.pad(h, (0, self.Wp - W))
         act = native.moe_gemm(hp, self.w_gate_up, tile_expert, n_tiles, cap, sorted_=sorted_, pair_div=self.k,
                               pair_scale=weight.view(-1) if self.weight_on_input else None, clamp=self.clamp, tile_rows=tm)
-        rows = native.moe_gemm(act, self.w_down, tile_expert, n_tiles, cap, tile_rows=tm)
+        rows = native.moe_gemm(act, self.w_down, tile_expert, n_tiles, cap, sorted_=sorted_, pair_div=0, tile_rows=tm)
         shared = self.shared(h, partial=defer) if self.shared is not None else None
         if defer:
             return native.MixtureRows(rows, pos, None if self.weight_on_input else weight.view(-1), self.k, shared, sg)
@@ -563,9 +573,10 @@ class HyperStreams:
         """(streams, normed input of sublayer 0) from the embedding rows."""
         return native.hyper_update(None, None, None, self.nxt[0], self.eps, dtype, ids=ids, table=table, emb_scale=scale, streams=self.s)
 
-    def step(self, q: int, x, y, dtype):
-        """The result y of sublayer q joins the streams; returns (streams, normed input of sublayer q + 1)."""
-        return native.hyper_update(x, y, self.cur[q], self.nxt[q + 1], self.eps, dtype)
+    def step(self, q: int, x, y, dtype, router=None):
+        """The result y of sublayer q joins the streams; returns (streams, normed input of sublayer q + 1, its routing or None)."""
+        out = native.hyper_update(x, y, self.cur[q], self.nxt[q + 1], self.eps, dtype, router=router)
+        return out if router is not None else (*out, None)
 
 
 class GatedLinearRecurrence:
