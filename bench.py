@@ -637,8 +637,12 @@ def bench_hybrid(args):
                 # bytes one attention launch has to read: every cached key and value of the batch once
                 keys = min(ctx_now, 512 + 4 + 32) if name in ("mananex", "mananex_moe", "tatevik", "gopetar_pair") else ctx_now  # a window, its kept positions, a page's slack
                 by = B * keys * kv_heads * 2 * dim * 2
+                latent = B * ctx_now * (2 * 192 + (dim // 2 if name.startswith("senadra") else 0)) * 2
                 if name.endswith("_latent"):  # a token's latent, as a key row and as value columns (and Senadra's rotated part)
-                    by = B * ctx_now * (2 * 192 + (dim // 2 if name.startswith("senadra") else 0)) * 2
+                    by = latent
+                elif name == "gopetar":  # the mean over its layers
+                    pairs = sum(l["type"] == "parallel" for l in cfg.layers)
+                    by = (pairs * B * min(ctx_now, 512 + 4 + 32) * kv_heads * 2 * dim * 2 + (layers - pairs) * latent) // layers
                 kern["attention"]["algorithmic_bytes"] = by
                 kern["attention"]["frac_of_hbm_peak"] = round(by / (kern["attention"]["us_per_launch"] * 1e-6) / 1e9 / HBM_PEAK_GBS, 4)
             rec["decode"] = {"batch": B, "ctx": ctx_now, "ms_per_step": round(dt * 1e3, 4), "tokens_per_s": round(B / dt, 1),
