@@ -404,7 +404,8 @@ int tgis_moe_align(const int32_t* idx, int64_t n_pairs, int E, int32_t* sorted, 
 /* out[row][n] = sum_c a(row)[c] * W[tile_expert[row / tile_rows]][n][c].
  * a(row) = A[sorted[row] / pair_div] * pair_scale[sorted[row]] (rounded to T) when sorted != NULL, else A[row]; with sorted and
  * pair_div 0 the rows are in place and the list only tells which of them are padding.
- * glu 1: out = silu(gate) * up;  2: g = min(gate, limit), u = clamp(up, -limit, limit), out = g sigmoid(alpha g) (u + 1).
+ * glu 1: out = silu(gate) * up;  2: g = min(gate, limit), u = clamp(up, -limit, limit), out = g sigmoid(alpha g) (u + 1);
+ * 3: a plain weight, out = max(product, 0)^2.
  * image: the experts' weights in fragment order, per expert [ceil(N / 32) blocks of weight rows (glu: the gate rows' blocks, then
  * the up rows')][ceil(K / 16) steps (fp32: K / 8)][64 lanes][8 (fp32: 4) elements]: lane l of a step holds row l % 32 of the block
  * and the elements k = step * 16 (8) + l / 32 * 8 (4) and on; rows and k padded with zeros. */
@@ -662,6 +663,58 @@ int tgis_hyper_update(const float* x, const int64_t* ids, const void* table, int
                       const float* next, void* h, int64_t rows, int64_t W, int streams, float eps, const float* router_w,
                       const float* router_sg, int E, int top, int softmax_top, int32_t* idx, float* route_weight,
                       float* route_gate, int dtype, void* stream);
+
+/* ---- norm after the sum, matrix memory with exponential gates, block-masked attention with normed half-rotated q and k ---- */
+/* Residual update of designs that norm after the sum, x <- N(alpha x + y) * w with N(z) = z / sqrt(mean z^2 + eps):
+ * x [rows, W] fp32, or ids instead (x = table[ids[t]] * emb_scale, vocab rows of `dtype`); y by kind as in tgis_hyper_update
+ * (0 none: no sum; 1 tensor, 2 split-K slabs, 3 rows of a mixture with pair_weight or ones); w NULL: no norm.  x_out (may alias x,
+ * may be NULL) receives the new stream; h [rows, W] of `dtype` its rounding, or with w2 N(x) * w2.
+ * dot_w [R][W] fp32 (or NULL): fp32 products of the rounded row h with R rows — to dot_out [rows][R], or (idx not NULL) as router
+ * logits: idx / route_weight [rows][top] receive what tgis_moe_choose makes of them. */
+int tgis_post_norm_update(const float* x, const int64_t* ids, const void* table, int64_t vocab, float emb_scale, float alpha,
+                          float* x_out, int kind, const void* y, int64_t ld_y, int slabs, const int32_t* pos,
+                          const float* pair_weight, int pairs, const float* w, const float* w2, void* h, int64_t rows, int64_t W,
+                          float eps, const float* dot_w, int R, float* dot_out, int32_t* idx, float* route_weight, int top,
+                          int groups, int keep, float route_scale, int dtype, void* stream);
+/* out[t][n] = sum_c h[t][c] w[n][c], fp32 [rows][R], for few outputs and many rows: h [rows, ld_h] and w [R][W] of a two-byte
+ * `dtype`, W and ld_h multiples of 8, 16-byte aligned. */
+int tgis_narrow_product(const void* h, int64_t ld_h, const void* w, float* out, int64_t rows, int R, int64_t W, int dtype,
+                        void* stream);
+/* The choice of a router from its logits [T][E] fp32: scores are their sigmoids; the k experts with the largest scores among the
+ * `keep` best of `groups` equal groups of neighbours (a group counts by the sum of its two largest scores; keep == groups: all);
+ * weight = chosen score * scale.  k <= 64, E <= 2048, keep * E / groups >= k. */
+int tgis_moe_choose(const float* logits, int64_t T, int E, int k, int groups, int keep, float scale, int32_t* idx, float* weight,
+                    void* stream);
+/* out = max(in, 0)^2, and the same where a decode-sized projection finishes its output. */
+int tgis_relu2(const void* in, int64_t ld_in, void* out, int64_t ld_out, int64_t rows, int64_t C, int dtype, void* stream);
+int tgis_dense_gemm_relu2(const void* x, int64_t ldx, const void* prepared, void* out, int64_t ldo, int64_t M, int64_t K,
+                          int64_t N, int dtype, void* workspace, int64_t workspace_bytes, void* stream);
+/* Matrix memory with exponential gates per (sequence, head), tokens in order (the running maximum m starts at 0):
+ *   i = cap tanh((z_i + i_bias) / cap);  f = ln sigmoid(cap tanh((z_f + f_bias) / cap));  m' = max(f + m, i);
+ *   S <- e^(f + m - m') S + e^(i - m') k v^T;  n likewise with k;  o = c S^T q / (max(|c n . q|, e^-m') + read_eps), c = q_scale;
+ *   out = o / sqrt(mean o^2 + eps) * gain[h dv ..] * sigmoid(g)      (the mean over the head; g_col0 < 0: no gate)
+ * q, k, v, g: columns of proj [T, ld] (head h at col0 + h dk / dv); gates [T, ld_gates] fp32: z_i of head h at h, z_f at H + h.
+ * state [slots][H][dk][dv] and memory [slots][H][dk + 1] (n, then m) fp32, read unless the step starts at position 0, written back.
+ * dk, dv <= 256.  impl 0: by size; 1: token by token; 2: chunks on the matrix cores (two-byte dtypes, dk, dv <= 128). */
+int tgis_matrix_memory(const void* proj, int64_t ld, int64_t q_col0, int64_t k_col0, int64_t v_col0, int64_t g_col0,
+                       const float* gates, int64_t ld_gates, const float* i_bias, const float* f_bias, float cap,
+                       const float* gain, float* state, float* memory, const int32_t* state_slots,
+                       const int32_t* cu_seqlens_q, const int32_t* positions, void* out, int64_t ld_out, int64_t B, int64_t T,
+                       int64_t max_q_len, int H, int dk, int dv, float q_scale, float eps, float read_eps, int impl, int dtype,
+                       void* stream);
+/* Every q and k head divided by its root mean square (eps inside) times q_gain / k_gain [dk]; channels (i, i + rot_dims / 2),
+ * i < rot_dims / 2, turned by the token's angle i — (cos, sin) in turns [T][rot_dims / 2][2] (tgis_pair_turns) — and multiplied by
+ * amp; q in place, k and v to their page slots as in tgis_rope_rows_kv_write.  dk <= 256. */
+int tgis_norm_rope_rows_kv_write(void* proj, int64_t ld, int64_t q_col0, int64_t k_col0, int64_t v_col0, const float* q_gain,
+                                 const float* k_gain, float eps, const float* turns, float amp, const int32_t* slots, void* k_pool,
+                                 void* v_pool, int64_t T, int H, int G, int dk, int dv, int rot_dims, int dtype, void* stream);
+/* tgis_attn_varlen with a block mask (chunk > 0: position i sees j <= i only if floor(i / chunk) == floor(j / chunk)) and a sink
+ * logit per query head in the softmax denominator (sink [H] fp32 or NULL); out may be a column range of a wider buffer. */
+int tgis_attn_varlen_blocks(const void* q, int64_t ldq, const void* k_pool, const void* v_pool, const int32_t* block_tables,
+                            int64_t max_pages, const int32_t* ctx_lens, const int32_t* cu_seqlens_q, int64_t B, void* out,
+                            int64_t ld_out, int64_t total_q, int64_t max_q_len, int64_t max_ctx, int H, int G, int dk, int dv,
+                            float scale, int chunk, const float* sink, void* workspace, int64_t workspace_bytes, int impl,
+                            int dtype, void* stream);
 
 #ifdef __cplusplus
 }

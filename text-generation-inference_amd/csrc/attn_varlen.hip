@@ -1060,6 +1060,76 @@ __global__ __launch_bounds__(256) void rope_rows_kv_write_kernel(T* __restrict__
     }
 }
 
+// Gained norm, half-split rotation and cache write: every q and k head is divided by its root mean square, times gain[dk] (one for
+// all q heads, one for all k heads); then channels (i, i + rdims / 2), i < rdims / 2, turn by the token's angle i, whose (cos, sin)
+// turns [T][rdims / 2][2] holds, and grow by `amp`.  q stays in place, k goes to its page slot, v as in rope_rows_kv_write_kernel.
+// grid (token, ceil((H + G) / 4) [+ value blocks]): a wave per q / k head, whose channels wait in registers and LDS.
+template <typename T>
+__global__ __launch_bounds__(256) void norm_rope_rows_kv_write_kernel(T* __restrict__ qkv, int64_t ld, int64_t q_col0, int64_t k_col0,
+                                                                      int64_t v_col0, const float* __restrict__ q_gain,
+                                                                      const float* __restrict__ k_gain, float eps, const float* __restrict__ turns,
+                                                                      float amp, const int32_t* __restrict__ slots, T* __restrict__ k_pool,
+                                                                      T* __restrict__ v_pool, int H, int G, int dk, int dv, int rdims, int v_inline) {
+    __shared__ float normed[4][256];
+    const int64_t t = blockIdx.x;
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    const int slot = slots[t];
+    const int64_t page = slot / PAGE;
+    const int off = slot % PAGE;
+    T* row = qkv + t * ld;
+    const int head_blocks = (H + G + 3) / 4;
+    if ((int)blockIdx.y >= head_blocks) {
+        const T* vrow = row + v_col0;
+        const int i0 = ((int)blockIdx.y - head_blocks) * 1024;
+        const int i1 = min(i0 + 1024, G * dv);
+        for (int i = i0 + threadIdx.x; i < i1; i += blockDim.x) {
+            const int g = i / dv, c = i - g * dv;
+            v_pool[((page * G + g) * dv + c) * PAGE + off] = vrow[i];
+        }
+        return;
+    }
+    const int h = blockIdx.y * 4 + wave;
+    if (h >= H + G) return;  // the whole wave; no workgroup barrier follows
+    const bool is_q = h < H;
+    T* src = is_q ? row + q_col0 + (int64_t)h * dk : row + k_col0 + (int64_t)(h - H) * dk;
+    T* dst = is_q ? src : k_pool + ((page * G + (h - H)) * PAGE + off) * dk;
+    const float* gain = is_q ? q_gain : k_gain;
+    float x[4], ss = 0.f;  // dk <= 256
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int c = lane + 64 * i;
+        x[i] = c < dk ? ldf(src + c) : 0.f;
+        ss += x[i] * x[i];
+    }
+    ss = wave_sum(ss);
+    const float rinv = 1.f / sqrtf(ss / (float)dk + eps);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int c = lane + 64 * i;
+        if (c < dk) {
+            x[i] *= rinv * gain[c];
+            normed[wave][c] = x[i];
+        }
+    }
+    __threadfence_block();
+    __builtin_amdgcn_wave_barrier();
+    const int half = rdims >> 1;
+    const f32x2* cs = reinterpret_cast<const f32x2*>(turns + t * rdims);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int c = lane + 64 * i;
+        if (c >= dk) continue;
+        float y = x[i];
+        if (c < rdims) {
+            const bool second = c >= half;
+            const f32x2 a = cs[second ? c - half : c];
+            const float other = normed[wave][second ? c - half : c + half];
+            y = (second ? y * a[0] + other * a[1] : y * a[0] - other * a[1]) * amp;
+        }
+        dst[c] = (T)y;
+    }
+}
+
 __global__ void pair_turns_kernel(const int32_t* __restrict__ positions, const float* __restrict__ inv_freq, float* __restrict__ turns,
                                   int64_t total, int n) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
@@ -1127,6 +1197,8 @@ void launch_mfma_one(const void* q, int64_t ldq, const void* k_pool, const void*
     const bool split = max_q_len * R <= 32;
     // a windowed query walks its window's pages and the kept first ones, whatever the context
     if (ext.window > 0) max_ctx = std::min<int64_t>(max_ctx, (int64_t)ext.window + ext.keep_first + 2 * PAGE);
+    // ... a query of a block at most that block's
+    if (ext.chunk > 0) max_ctx = std::min<int64_t>(max_ctx, (int64_t)ext.chunk + 2 * PAGE);
     int nw = 4;
     size_t lds = 0;
     unsigned gx = 1;
@@ -1523,4 +1595,46 @@ extern "C" int tgis_attn_varlen_turned(const void* q, int64_t ldq, const void* k
     return attn_win_impl(q, ldq, k_pool, v_pool, block_tables, max_pages, ctx_lens, cu_seqlens_q, B, out, ld_out, total_q, max_q_len, max_ctx,
                          H, G, dk, dv, scale, window, keep_first, sink, nullptr, 0, 0, out_scale, softcap, turns, workspace, workspace_bytes,
                          impl, dtype, stream);
+}
+
+// tgis_attn_varlen with a block mask (chunk > 0) AND a sink logit per query head in the softmax denominator (sink [H] fp32 or NULL).
+// out may be a column range of a wider buffer (ld_out).  workspace: as for tgis_attn_varlen_ext.
+extern "C" int tgis_attn_varlen_blocks(const void* q, int64_t ldq, const void* k_pool, const void* v_pool, const int32_t* block_tables,
+                                       int64_t max_pages, const int32_t* ctx_lens, const int32_t* cu_seqlens_q, int64_t B, void* out,
+                                       int64_t ld_out, int64_t total_q, int64_t max_q_len, int64_t max_ctx, int H, int G, int dk, int dv,
+                                       float scale, int chunk, const float* sink, void* workspace, int64_t workspace_bytes, int impl, int dtype,
+                                       void* stream) {
+    TGIS_CHECK_ARG(chunk >= 0, "tgis_attn_varlen_blocks: chunk >= 0");
+    AttnExt ext{nullptr, nullptr, chunk, nullptr, 0,
+                (int)std::min<int64_t>(64, workspace && ((uintptr_t)workspace & 15) == 0 ? workspace_bytes / std::max<int64_t>(1, total_q * H * (int64_t)(dv + 2) * 4) : 0),
+                (float*)workspace, total_q};
+    ext.sink = sink;
+    return attn_varlen_impl(q, ldq, k_pool, v_pool, block_tables, max_pages, ctx_lens, cu_seqlens_q, B, out, ld_out, total_q, max_q_len,
+                            max_ctx, H, G, dk, dv, scale, impl, dtype, ext, stream);
+}
+
+// Per-head norm of q and k with gains, half-split rotation by a step's table of turns, and the cache write (see
+// norm_rope_rows_kv_write_kernel).  proj [T, ld] as in tgis_rope_rows_kv_write; turns [T][rot_dims / 2][2] from tgis_pair_turns.
+extern "C" int tgis_norm_rope_rows_kv_write(void* proj, int64_t ld, int64_t q_col0, int64_t k_col0, int64_t v_col0, const float* q_gain,
+                                            const float* k_gain, float eps, const float* turns, float amp, const int32_t* slots, void* k_pool,
+                                            void* v_pool, int64_t T, int H, int G, int dk, int dv, int rot_dims, int dtype, void* stream) {
+    TGIS_CHECK_ARG(proj && q_gain && k_gain && slots && k_pool && v_pool && (turns || rot_dims == 0), "tgis_norm_rope_rows_kv_write: null tensor");
+    TGIS_CHECK_ARG(H >= 1 && G >= 1 && dk >= 1 && dk <= 256 && dv >= 1 && rot_dims >= 0 && rot_dims <= dk && rot_dims % 2 == 0 && q_col0 >= 0 &&
+                       k_col0 >= 0 && v_col0 >= 0 && ld >= q_col0 + (int64_t)H * dk && ld >= k_col0 + (int64_t)G * dk && ld >= v_col0 + (int64_t)G * dv,
+                   "tgis_norm_rope_rows_kv_write: bad geometry (H %d, G %d, dk %d, dv %d, rot_dims %d, ld %ld)", H, G, dk, dv, rot_dims, (long)ld);
+    TGIS_CHECK_ARG(dtype == TGIS_F16 || dtype == TGIS_BF16 || dtype == TGIS_F32, "tgis_norm_rope_rows_kv_write: bad dtype");
+    if (T == 0) return TGIS_OK;
+    hipStream_t st = (hipStream_t)stream;
+    TgisTimedScope timed(TGIS_OP_ROPE_KV, st);
+    const int v_inline = T < 512 ? 1 : 0;
+    const int v_blocks = v_inline ? (int)cdiv64((int64_t)G * dv, 1024) : 0;
+    TGIS_ATTN_BY_DTYPE(dtype, hipLaunchKernelGGL(norm_rope_rows_kv_write_kernel<TT>, dim3((unsigned)T, (unsigned)((H + G + 3) / 4 + v_blocks)),
+                                                 dim3(256), 0, st, (TT*)proj, ld, q_col0, k_col0, v_col0, q_gain, k_gain, eps, turns, amp, slots,
+                                                 (TT*)k_pool, (TT*)v_pool, H, G, dk, dv, rot_dims, v_inline));
+    if (!v_inline)
+        TGIS_ATTN_BY_DTYPE(dtype, hipLaunchKernelGGL(v_write_kernel<TT>, dim3((unsigned)cdiv64(T, 32), (unsigned)cdiv64((int64_t)G * dv, 64)),
+                                                     dim3(256), 0, st, (const TT*)proj, ld, v_col0, slots, (const TT*)nullptr, (int64_t)0,
+                                                     (const float*)nullptr, (TT*)v_pool, T, G, dv, (const float*)nullptr));
+    TGIS_CHECK_LAUNCH();
+    return TGIS_OK;
 }

@@ -22,8 +22,8 @@ struct DenseArgs {
     int out_f32;
     float* slabs;  // [Mslabs][S][32][NT*32] f32 partial sums (S > 1 or partial mode)
     int partial;   // 1: always leave fp32 slabs (deferred reduce), never write `out`
-    int gelu;      // model-dtype output only: 0 none, 1 GELU (erf), 2 GELU (tanh), 3 xIELU (coefficients act_p0 / act_p1)
-                   // applied to the rounded sum + bias
+    int gelu;      // model-dtype output only: 0 none, 1 GELU (erf), 2 GELU (tanh), 3 xIELU (coefficients act_p0 / act_p1),
+                   // 5 the square of relu; applied to the rounded sum + bias
     // ACT == 3 (rope image, tgis_dense_prepare flags bit 1): the epilogue rotates q / k heads and writes k / v into their
     // cache pages; `out` is the q tensor (see tgis_dense_gemm_rope)
     const int32_t* positions;  // [M]
@@ -66,6 +66,9 @@ __device__ __forceinline__ T finish_out(float v, int gelu, float p0 = 0.f, float
     if (gelu == 3) {
         const float z = to_f32(t);
         t = from_f32<T>(z > 0.f ? p0 * z * z + 0.5f * z : p1 * (expm1f(z) - z) + 0.5f * z);
+    } else if (gelu == 5) {
+        const float z = fmaxf(to_f32(t), 0.f);
+        t = from_f32<T>(z * z);
     } else if (gelu) {
         t = from_f32<T>(gelu_f32(to_f32(t), gelu == 2));
     }

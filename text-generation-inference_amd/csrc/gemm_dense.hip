@@ -304,6 +304,25 @@ extern "C" int tgis_dense_gemm_xielu(const void* x, int64_t ldx, const void* pre
     return dtype == TGIS_F16 ? launch_dense<f16>(a, pl, 0, cdiv64(M, 32), st) : launch_dense<bf16>(a, pl, 0, cdiv64(M, 32), st);
 }
 
+// A plain projection with the square of relu applied where the output is finished (epilogue, or the split-K reduce): the same bits as
+// tgis_dense_gemm followed by tgis_relu2.
+extern "C" int tgis_dense_gemm_relu2(const void* x, int64_t ldx, const void* prepared, void* out, int64_t ldo, int64_t M, int64_t K,
+                                     int64_t N, int dtype, void* workspace, int64_t workspace_bytes, void* stream) {
+    int rc = dense_check(x, ldx, prepared, M, K, N, dtype, 0);
+    if (rc != TGIS_OK) return rc;
+    TGIS_CHECK_ARG(out, "tgis_dense_gemm_relu2: null out");
+    if (M == 0) return TGIS_OK;
+    hipStream_t st = (hipStream_t)stream;
+    DensePlan pl = plan_dense(K, N, M, 0);
+    const int64_t need = tgis_dense_gemm_workspace_bytes(M, K, N);
+    TGIS_CHECK_ARG(workspace && workspace_bytes >= need, "tgis_dense_gemm_relu2: workspace too small (%ld < %ld)", (long)workspace_bytes, (long)need);
+    TgisTimedScope timed(TGIS_OP_DENSE_GEMM, st);
+    DenseArgs a;
+    dense_fill(a, x, ldx, prepared, nullptr, out, ldo, M, K, N, 0, (float*)((uint8_t*)workspace + 4096), 0, pl);
+    a.gelu = 5;
+    return dtype == TGIS_F16 ? launch_dense<f16>(a, pl, 0, cdiv64(M, 32), st) : launch_dense<bf16>(a, pl, 0, cdiv64(M, 32), st);
+}
+
 // out[m][n] = gelu_tanh(x[m] . W[n]) * table[ids[m]][col0 + n]: a plain projection whose activated output gates a slice of
 // an embedding row of the row's token, finished in the epilogue (or the split-K reduce): the same bits as tgis_dense_gemm
 // followed by tgis_gelu_gated_lookup.

@@ -1,0 +1,317 @@
+// Matrix memory with exponential gates (mLSTM), per sequence and head, S [dk, dv], n [dk] and m in fp32:
+//
+//     m_t = max(f_t + m_(t-1), i_t)          i = soft(z_i + b_i),  f = ln sigmoid(soft(z_f + b_f)),  soft(z) = cap tanh(z / cap)
+//     S_t = e^(f_t + m_(t-1) - m_t) S_(t-1) + e^(i_t - m_t) k_t v_t^T;      n_t likewise with k_t alone
+//     o_t = c S_t^T q_t / (max(|c n_t . q_t|, e^(-m_t)) + read_eps)
+//     out_t = o_t / sqrt(mean(o_t^2) + eps) * gain[h] * sigmoid(g_t)       (norm per head over dv, gains of all heads side by side)
+//
+// Every sequence starts from S = 0, n = 0, m = 0.  q, k, v and the output gate's logits g are columns of one projection (activation
+// dtype T); z_i, z_f are fp32 [T][2 H].  A slot of the state cache holds S [H][dk][dv] and (n, m) [H][dk + 1]; a step that starts at
+// position 0 starts from zeros whatever the slot holds.
+//
+// matrix_memory_scan_kernel: token by token, any dtype and size up to 256 x 256 (decode, short runs, fp32 serving).  Workgroup =
+// (sequence, head) = LPC dv_pad / CPL threads: LPC neighbouring lanes share column j of S (with CPL = 2 also j + dv_pad / 2), each
+// keeps RPL rows of it in registers.  Tokens go through LDS in stages of `ts`, two buffers deep, the next stage on its way to
+// registers while the current one is worked on; the stage's decays and write weights (one pair per token and head) are made by one
+// wave, which carries m from stage to stage token by token; rows of n belong to the first dk threads.
+#include <algorithm>
+#include "common.h"
+
+namespace {
+
+constexpr int SEG_PAD = 4;  // floats between the row groups' segments
+constexpr int PFQ = 4;      // (q, k) pairs and
+constexpr int PFV = 4;      // values of the next stage that a thread holds in registers: ts dk <= PFQ threads, ts dv_pad <= PFV threads
+constexpr int MAX_TS = 32;  // a stage's gates are made by one wave, half of it idle
+
+struct MemoryArgs {
+    const void* proj;
+    int64_t ld, q_col0, k_col0, v_col0, g_col0;  // g_col0 < 0: no output gate
+    const float* gates;                          // [T][ld_gates]: z_i of head h at h, z_f at H + h
+    int64_t ld_gates;
+    const float* i_bias;
+    const float* f_bias;
+    float cap;
+    const float* gain;  // [H dv]
+    float* state;
+    float* memory;
+    const int32_t* state_slots;
+    const int32_t* cu_q;
+    const int32_t* positions;
+    void* out;
+    int64_t ld_out;
+    int H, dk, dv;
+    float q_scale, eps, read_eps;
+    int dv_pad, ts;
+};
+
+__device__ __forceinline__ float soft_capped(float z, float cap) { return cap * tanhf(z / cap); }
+// ln(sigmoid(z)) without cancellation at either end
+__device__ __forceinline__ float log_sigmoid(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
+__device__ __forceinline__ float lane_value(float v, int lane) {
+    return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), lane));
+}
+// (i, f) of head h at token t
+__device__ __forceinline__ void log_gates(const MemoryArgs& a, int64_t t, int h, float& li, float& lf) {
+    const float* z = a.gates + t * a.ld_gates;
+    li = soft_capped(z[h] + (a.i_bias ? a.i_bias[h] : 0.f), a.cap);
+    lf = log_sigmoid(soft_capped(z[a.H + h] + (a.f_bias ? a.f_bias[h] : 0.f), a.cap));
+}
+template <typename T> __device__ __forceinline__ float output_gate(const MemoryArgs& a, int64_t t, int col) {
+    if (a.g_col0 < 0) return 1.f;
+    const float g = (float)reinterpret_cast<const T*>(a.proj)[t * a.ld + a.g_col0 + col];
+    return 1.f / (1.f + expf(-g));
+}
+
+template <typename T, int RPL, int CPL, int LPC, int MAXT>
+__global__ __launch_bounds__(MAXT) void matrix_memory_scan_kernel(MemoryArgs a) {
+    extern __shared__ __attribute__((aligned(16))) float smem[];
+    constexpr int SEG = RPL + SEG_PAD, ROW = LPC * SEG;
+    const int ts = a.ts, dk = a.dk, dv = a.dv, dv_pad = a.dv_pad;
+    float* qs = smem;                    // [2][ts][ROW]
+    float* ks = qs + 2 * ts * ROW;       // [2][ts][ROW]
+    float* vs = ks + 2 * ts * ROW;       // [2][ts][dv_pad]
+    float* os = vs + 2 * ts * dv_pad;    // [ts][dv_pad]
+    float* nq = os + ts * dv_pad;        // [ts][dk]: products of n and q
+    f32x2* gs = reinterpret_cast<f32x2*>(nq + ((ts * dk + 1) & ~1));  // [2][ts]: (decay, write weight)
+    float* fl = reinterpret_cast<float*>(gs + 2 * ts);                 // [2][ts]: e^-m
+    const int b = blockIdx.x, h = blockIdx.y;
+    const int tid = threadIdx.x, j = tid / LPC, qd = tid % LPC;
+    const int t0 = a.cu_q[b], qlen = a.cu_q[b + 1] - t0;
+    if (qlen <= 0) return;
+    const int nthreads = blockDim.x;
+    const int wave = tid >> 6, lane = tid & 63, nw = nthreads >> 6;
+    const bool fresh = a.positions[t0] == 0;
+    const T* proj = reinterpret_cast<const T*>(a.proj);
+    const int64_t slot = a.state_slots[b];
+    float* S = a.state + (slot * a.H + h) * (int64_t)dk * dv;
+    float* N = a.memory + (slot * a.H + h) * (int64_t)(dk + 1);
+    const int jstep = dv_pad / CPL;
+    float s[CPL][RPL];
+#pragma unroll
+    for (int c = 0; c < CPL; ++c)
+#pragma unroll
+        for (int r = 0; r < RPL; ++r) {
+            const int i = qd * RPL + r, jc = j + c * jstep;
+            s[c][r] = (!fresh && i < dk && jc < dv) ? S[(int64_t)i * dv + jc] : 0.f;
+        }
+    float nrow[4];  // rows tid, tid + nthreads, ... of n: dk <= 256, at least 64 threads
+#pragma unroll
+    for (int u = 0; u < 4; ++u) nrow[u] = (!fresh && tid + u * nthreads < dk) ? N[tid + u * nthreads] : 0.f;
+    float m_run = fresh ? 0.f : N[dk];  // carried by wave 0
+    // rows past dk and columns past dv of both buffers stay zero
+    for (int e = tid; e < 2 * ts * ROW; e += nthreads) {
+        qs[e] = 0.f;
+        ks[e] = 0.f;
+    }
+    for (int e = tid; e < 2 * ts * dv_pad; e += nthreads) vs[e] = 0.f;
+    // a thread's share of a stage is the same in every stage: where it comes from and goes to is worked out once
+    T qr[PFQ], kr[PFQ], vr[PFV];
+    int q_tt[PFQ], q_src[PFQ], q_dst[PFQ], v_tt[PFV], v_src[PFV];
+#pragma unroll
+    for (int u = 0; u < PFQ; ++u) {
+        const int e = tid + u * nthreads;
+        const int tt = e / dk, i = e - tt * dk;
+        q_tt[u] = tt;
+        q_src[u] = tt * (int)a.ld + h * dk + i;
+        q_dst[u] = tt * ROW + (i / RPL) * SEG + (i % RPL);
+    }
+#pragma unroll
+    for (int u = 0; u < PFV; ++u) {
+        const int e = tid + u * nthreads;
+        const int tt = e / dv_pad, c = e - tt * dv_pad;
+        v_tt[u] = c < dv ? tt : 1 << 30;  // a column past the head's width is never fetched
+        v_src[u] = tt * (int)a.ld + h * dv + c;
+    }
+    auto fetch = [&](int first, int n) {
+        const T* base = proj + (int64_t)(t0 + first) * a.ld;
+#pragma unroll
+        for (int u = 0; u < PFQ; ++u)
+            if (q_tt[u] < n) {
+                qr[u] = base[a.q_col0 + q_src[u]];
+                kr[u] = base[a.k_col0 + q_src[u]];
+            }
+#pragma unroll
+        for (int u = 0; u < PFV; ++u)
+            if (v_tt[u] < n) vr[u] = base[a.v_col0 + v_src[u]];
+    };
+    // ... into stage buffer `buf`, and the gates of those tokens by wave 0
+    auto commit = [&](int first, int n, int buf) {
+#pragma unroll
+        for (int u = 0; u < PFQ; ++u)
+            if (q_tt[u] < n) {
+                qs[buf * ts * ROW + q_dst[u]] = (float)qr[u] * a.q_scale;
+                ks[buf * ts * ROW + q_dst[u]] = (float)kr[u];
+            }
+#pragma unroll
+        for (int u = 0; u < PFV; ++u)
+            if (v_tt[u] < n) vs[buf * ts * dv_pad + tid + u * nthreads] = (float)vr[u];
+        if (wave != 0) return;
+        float li = 0.f, lf = 0.f, before = 0.f, after = 0.f;
+        if (lane < n) log_gates(a, t0 + first + lane, h, li, lf);
+        for (int tt = 0; tt < n; ++tt) {
+            const float top = fmaxf(lane_value(lf, tt) + m_run, lane_value(li, tt));
+            if (lane == tt) {
+                before = m_run;
+                after = top;
+            }
+            m_run = top;
+        }
+        if (lane < n) {
+            gs[buf * ts + lane] = f32x2{expf(lf + before - after), expf(li - after)};
+            fl[buf * ts + lane] = expf(-after);
+        }
+    };
+    fetch(0, min(ts, qlen));
+    __syncthreads();  // the buffers are cleared
+    commit(0, min(ts, qlen), 0);
+    __syncthreads();
+    T* out = reinterpret_cast<T*>(a.out);
+    int buf = 0;
+    for (int base = 0; base < qlen; base += ts, buf ^= 1) {
+        const int n = min(ts, qlen - base);
+        const int n_next = min(ts, qlen - base - ts);
+        if (n_next > 0) fetch(base + ts, n_next);
+        const float* qb = qs + buf * ts * ROW + qd * SEG;
+        const float* kb = ks + buf * ts * ROW + qd * SEG;
+        const float* vb = vs + buf * ts * dv_pad + j;
+        const f32x2* gb = gs + buf * ts;
+#pragma unroll 1
+        for (int tt = 0; tt < n; ++tt) {
+            const f32x2 g = gb[tt];
+            float vj[CPL], acc[CPL];
+#pragma unroll
+            for (int c = 0; c < CPL; ++c) {
+                vj[c] = vb[tt * dv_pad + c * jstep] * g[1];
+                acc[c] = 0.f;
+            }
+#pragma unroll
+            for (int r4 = 0; r4 < RPL; r4 += 4) {
+                const f32x4 q4 = *reinterpret_cast<const f32x4*>(qb + tt * ROW + r4);
+                const f32x4 k4 = *reinterpret_cast<const f32x4*>(kb + tt * ROW + r4);
+#pragma unroll
+                for (int u = 0; u < 4; ++u)
+#pragma unroll
+                    for (int c = 0; c < CPL; ++c) {
+                        s[c][r4 + u] = fmaf(g[0], s[c][r4 + u], k4[u] * vj[c]);
+                        acc[c] = fmaf(s[c][r4 + u], q4[u], acc[c]);
+                    }
+            }
+#pragma unroll
+            for (int c = 0; c < CPL; ++c) {
+                float t = acc[c];
+                t += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, t), 0xB1, 0xF, 0xF, true));  // lane ^ 1
+                t += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, t), 0x4E, 0xF, 0xF, true));  // lane ^ 2
+                if (LPC == 8)  // the other quad of the eight: lane 7 - i of the half row holds its total
+                    t += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, t), 0x141, 0xF, 0xF, true));
+                if (qd == 0) os[tt * dv_pad + j + c * jstep] = t;
+            }
+        }
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+            const int i = tid + u * nthreads;
+            if (i < dk) {
+                const int at = buf * ts * ROW + (i / RPL) * SEG + (i % RPL);
+                for (int tt = 0; tt < n; ++tt) {
+                    const f32x2 g = gb[tt];
+                    nrow[u] = fmaf(g[0], nrow[u], g[1] * ks[at + tt * ROW]);
+                    nq[tt * dk + i] = nrow[u] * qs[at + tt * ROW];
+                }
+            }
+        }
+        __syncthreads();
+        for (int tt = wave; tt < n; tt += nw) {
+            float d = 0.f, ss = 0.f;
+            for (int i = lane; i < dk; i += 64) d += nq[tt * dk + i];
+            for (int c = lane; c < dv; c += 64) ss += os[tt * dv_pad + c] * os[tt * dv_pad + c];
+            d = wave_sum(d);
+            ss = wave_sum(ss);
+            const float den = fmaxf(fabsf(d), fl[buf * ts + tt]) + a.read_eps;
+            // o / den normed: mean((o / den)^2) + eps under the root
+            const float rinv = 1.f / (den * sqrtf(ss / ((float)dv * den * den) + a.eps));
+            const int64_t t = t0 + base + tt;
+            T* orow = out + t * a.ld_out + (int64_t)h * dv;
+            for (int c = lane; c < dv; c += 64)
+                orow[c] = (T)(os[tt * dv_pad + c] * rinv * a.gain[h * dv + c] * output_gate<T>(a, t, h * dv + c));
+        }
+        if (n_next > 0) commit(base + ts, n_next, buf ^ 1);
+        __syncthreads();  // the outputs are out, the next stage is in
+    }
+#pragma unroll
+    for (int c = 0; c < CPL; ++c)
+#pragma unroll
+        for (int r = 0; r < RPL; ++r) {
+            const int i = qd * RPL + r, jc = j + c * jstep;
+            if (i < dk && jc < dv) S[(int64_t)i * dv + jc] = s[c][r];
+        }
+#pragma unroll
+    for (int u = 0; u < 4; ++u)
+        if (tid + u * nthreads < dk) N[tid + u * nthreads] = nrow[u];
+    if (tid == 0) N[dk] = m_run;
+}
+
+template <typename T, int RPL, int CPL, int LPC, int MAXT>
+void launch_memory_as(MemoryArgs a, int64_t B, int64_t max_q_len, int cols, hipStream_t st) {
+    a.dv_pad = cols;
+    const int threads = LPC * cols / CPL;
+    auto bytes = [&](int ts) {
+        return ((size_t)4 * ts * LPC * (RPL + SEG_PAD) + (size_t)3 * ts * cols + ((size_t)ts * a.dk + 1) / 2 * 2 + (size_t)6 * ts) * sizeof(float);
+    };
+    int ts = MAX_TS;
+    while (ts > 1 && (bytes(ts) > 140 * 1024 || ts >= 2 * max_q_len || ts * a.dk > PFQ * threads || ts * cols > PFV * threads)) ts >>= 1;
+    a.ts = ts;
+    const size_t lds = bytes(ts);
+    if (lds > 48 * 1024)
+        (void)hipFuncSetAttribute((const void*)matrix_memory_scan_kernel<T, RPL, CPL, LPC, MAXT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    hipLaunchKernelGGL((matrix_memory_scan_kernel<T, RPL, CPL, LPC, MAXT>), dim3((unsigned)B, (unsigned)a.H), dim3(threads), lds, st, a);
+}
+
+// R4: rows per lane with four lanes per column.  Steps of one or two tokens are mostly the state's trip from and to memory: two
+// columns per lane from 64 value channels on; longer runs spread a column over eight lanes where 1024 threads allow it.
+template <typename T, int R4>
+void launch_memory(const MemoryArgs& a, int64_t B, int64_t max_q_len, hipStream_t st) {
+    const int pad16 = (a.dv + 15) / 16 * 16;
+    if constexpr (R4 <= 32) {
+        if (a.dv >= 64 && max_q_len <= 2) return launch_memory_as<T, R4, 2, 4, 512>(a, B, max_q_len, (a.dv + 31) / 32 * 32, st);
+    }
+    if constexpr (R4 >= 8) {
+        if (max_q_len > 2 && 8 * pad16 <= 1024) return launch_memory_as<T, R4 / 2, 1, 8, 1024>(a, B, max_q_len, pad16, st);
+    }
+    launch_memory_as<T, R4, 1, 4, 1024>(a, B, max_q_len, pad16, st);
+}
+
+template <typename T>
+void launch_memory_rows(const MemoryArgs& a, int64_t B, int64_t max_q_len, hipStream_t st) {
+    if (a.dk <= 16) launch_memory<T, 4>(a, B, max_q_len, st);
+    else if (a.dk <= 32) launch_memory<T, 8>(a, B, max_q_len, st);
+    else if (a.dk <= 64) launch_memory<T, 16>(a, B, max_q_len, st);
+    else if (a.dk <= 128) launch_memory<T, 32>(a, B, max_q_len, st);
+    else launch_memory<T, 64>(a, B, max_q_len, st);
+}
+
+}  // namespace
+
+extern "C" int tgis_matrix_memory(const void* proj, int64_t ld, int64_t q_col0, int64_t k_col0, int64_t v_col0, int64_t g_col0,
+                                  const float* gates, int64_t ld_gates, const float* i_bias, const float* f_bias, float cap, const float* gain,
+                                  float* state, float* memory, const int32_t* state_slots, const int32_t* cu_seqlens_q,
+                                  const int32_t* positions, void* out, int64_t ld_out, int64_t B, int64_t T, int64_t max_q_len, int H, int dk,
+                                  int dv, float q_scale, float eps, float read_eps, int impl, int dtype, void* stream) {
+    TGIS_CHECK_ARG(proj && gates && gain && state && memory && state_slots && cu_seqlens_q && positions && out, "tgis_matrix_memory: null tensor");
+    TGIS_CHECK_ARG(H >= 1 && H <= 65535 && dk >= 1 && dk <= 256 && dv >= 1 && dv <= 256, "tgis_matrix_memory: heads of up to 256 x 256 (got %d x %d)", dk, dv);
+    TGIS_CHECK_ARG(q_col0 >= 0 && k_col0 >= 0 && v_col0 >= 0 && ld >= q_col0 + (int64_t)H * dk && ld >= k_col0 + (int64_t)H * dk &&
+                       ld >= v_col0 + (int64_t)H * dv && (g_col0 < 0 || ld >= g_col0 + (int64_t)H * dv) && ld_gates >= 2 * (int64_t)H &&
+                       ld_out >= (int64_t)H * dv && max_q_len >= 1 && T >= 0 && ld <= (1 << 24),
+                   "tgis_matrix_memory: bad strides");
+    TGIS_CHECK_ARG(cap > 0.f && impl >= 0 && impl <= 2, "tgis_matrix_memory: cap > 0; impl 0 (auto), 1 (token by token), 2 (chunks)");
+    TGIS_CHECK_ARG(dtype == TGIS_F16 || dtype == TGIS_BF16 || dtype == TGIS_F32, "tgis_matrix_memory: bad dtype");
+    if (B == 0 || T == 0) return TGIS_OK;
+    hipStream_t st = (hipStream_t)stream;
+    TgisTimedScope timed(TGIS_OP_SCAN, st);
+    const MemoryArgs a{proj, ld, q_col0, k_col0, v_col0, g_col0, gates, ld_gates, i_bias, f_bias, cap, gain, state, memory, state_slots,
+                       cu_seqlens_q, positions, out, ld_out, H, dk, dv, q_scale, eps, read_eps, 0, 0};
+    if (dtype == TGIS_F16) launch_memory_rows<f16>(a, B, max_q_len, st);
+    else if (dtype == TGIS_BF16) launch_memory_rows<bf16>(a, B, max_q_len, st);
+    else launch_memory_rows<float>(a, B, max_q_len, st);
+    TGIS_CHECK_LAUNCH();
+    return TGIS_OK;
+}

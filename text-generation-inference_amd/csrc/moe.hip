@@ -7,7 +7,7 @@
 //            sorted[pos] = p or -1, tile_expert[pos / tile rows], pos_of_pair[p] = pos, n_tiles
 //   gemm     out[pos][n] = sum_c A[row(pos)][c] * s(pos) * W[expert(pos)][n][c]        (s = 1 or the routing weight, applied
 //            to the INPUT row and rounded to T like any other GEMM operand), optionally silu(gate) * up over a stacked
-//            [gate | up] weight
+//            [gate | up] weight or the square of relu of a plain one
 //   combine  y[t] = sum_j rows[pos_of_pair[t k + j]] * (w[t][j] or 1) + g[t] * shared[t]
 //
 // The number of tiles is data dependent; the grid is sized for the worst case (T k + E * (tile rows - 1) rows) and tiles past
@@ -141,6 +141,18 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
     }
 }
 
+// Choice among logits that are there already (tgis_narrow_product): a wave per token, four tokens per workgroup.
+__global__ __launch_bounds__(256) void moe_choose_kernel(const float* __restrict__ logits, int64_t rows, int E, int k, int groups, int keep,
+                                                         float scale, int32_t* __restrict__ idx, float* __restrict__ weight) {
+    extern __shared__ float sm[];  // [4][E + groups]
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    const int64_t t = (int64_t)blockIdx.x * 4 + wave;
+    if (t >= rows) return;  // the whole wave; no workgroup barrier follows
+    float* mine = sm + wave * (E + groups);
+    for (int e = lane; e < E; e += 64) mine[e] = logits[t * E + e];
+    route_grouped_sigmoid_wave(mine, mine + E, E, k, groups, keep, scale, idx + t * k, weight + t * k);
+}
+
 // ---- align: one workgroup ---------------------------------------------------------------------------------------------
 __global__ __launch_bounds__(1024) void moe_align_kernel(const int32_t* __restrict__ idx, int64_t n_pairs, int E,
                                                          int32_t* __restrict__ sorted, int64_t cap, int32_t* __restrict__ tile_expert,
@@ -199,6 +211,12 @@ template <int GLU> __device__ __forceinline__ float gated(float g, float u, floa
     return g / (1.f + expf(-alpha * g)) * (u + 1.f);
 }
 
+// what a plain product (GLU 0) becomes where it is written: act 1 the square of relu
+__device__ __forceinline__ float plain_out(float v, int act) {
+    const float p = fmaxf(v, 0.f);
+    return act ? p * p : v;
+}
+
 template <typename T> __device__ __forceinline__ int64_t image_block(int64_t K) {  // elements of a block of 32 weight rows
     return (K + Frag<T>::KSTEP - 1) / Frag<T>::KSTEP * (64 * Frag<T>::PER);
 }
@@ -208,7 +226,7 @@ __global__ __launch_bounds__(KW > 4 ? 512 : 256) void moe_gemm_kernel(const T* _
                                                        int pair_div, const float* __restrict__ pair_scale,
                                                        const int32_t* __restrict__ tile_expert, const int32_t* __restrict__ n_tiles,
                                                        const T* __restrict__ Wt, int64_t N, int64_t K,
-                                                       T* __restrict__ out, int64_t ld_out, float alpha, float limit) {
+                                                       T* __restrict__ out, int64_t ld_out, float alpha, float limit, int act) {
     constexpr bool KSPLIT = KW > 1;
     using F = Frag<T>;
     using V = typename F::V;
@@ -285,7 +303,7 @@ __global__ __launch_bounds__(KW > 4 ? 512 : 256) void moe_gemm_kernel(const T* _
                 v += part[((w * NA + 0) * 16 + i) * 64 + lane];
                 if (GLU) v2 += part[((w * NA + 1) * 16 + i) * 64 + lane];
             }
-            if (GLU) v = gated<GLU>(v, v2, alpha, limit);
+            v = GLU ? gated<GLU>(v, v2, alpha, limit) : plain_out(v, act);
             const int m = (i >> 2) * 8 + half * 4 + (i & 3);
             out[((int64_t)tile * TM + m) * ld_out + n0 + row] = (T)v;
         }
@@ -299,7 +317,7 @@ __global__ __launch_bounds__(KW > 4 ? 512 : 256) void moe_gemm_kernel(const T* _
             for (int i = 0; i < 16; ++i) {
                 const int m = (i >> 2) * 8 + half * 4 + (i & 3);
                 float v = acc[nb][i];
-                if (GLU) v = gated<GLU>(v, acc2[nb][i], alpha, limit);
+                v = GLU ? gated<GLU>(v, acc2[nb][i], alpha, limit) : plain_out(v, act);
                 out[((int64_t)tile * TM + m) * ld_out + n] = (T)v;
             }
         }
@@ -318,7 +336,7 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_tiled_kernel(const T* __restr
                                                                 int pair_div, const float* __restrict__ pair_scale,
                                                                 const int32_t* __restrict__ tile_expert, const int32_t* __restrict__ n_tiles,
                                                                 const T* __restrict__ Wt, int64_t N, int64_t K,
-                                                                T* __restrict__ out, int64_t ld_out, float alpha, float limit, int ncb) {
+                                                                T* __restrict__ out, int64_t ld_out, float alpha, float limit, int ncb, int act) {
     using V = typename Frag<T>::V;
     constexpr int BK = 32, AL = TM_LONG * 4 / 256, BL = BN * 4 / 256, NJ = BN / 64;
     constexpr int HALF = BN / 2;                      // weight rows of a wave
@@ -430,14 +448,14 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_tiled_kernel(const T* __restr
             for (int q = 0; q < 16; ++q) {
                 const int64_t row = (int64_t)tile * TM_LONG + wr * 64 + i * 32 + (q >> 2) * 8 + half * 4 + (q & 3);
                 float v = acc[i][j][q];
-                if (GLU) v = gated<GLU ? GLU : 1>(v, acc[i][GLU ? j + NJ / 2 : j][q], alpha, limit);
+                v = GLU ? gated<GLU ? GLU : 1>(v, acc[i][GLU ? j + NJ / 2 : j][q], alpha, limit) : plain_out(v, act);
                 out[row * ld_out + n] = (T)v;
             }
         }
 }
 
 template <typename T>
-void launch_gemm_tiled(int glu, float alpha, float limit, const void* A, int64_t ld_a, const int32_t* sorted, int pair_div,
+void launch_gemm_tiled(int glu, int act, float alpha, float limit, const void* A, int64_t ld_a, const int32_t* sorted, int pair_div,
                        const float* pair_scale, const int32_t* tile_expert, const int32_t* n_tiles, const void* Wt,
                        int64_t N, int64_t K, void* out, int64_t ld_out, int64_t max_tiles, hipStream_t st) {
 #define TGIS_MOE_TILED(GLU, BN)                                                                                                        \
@@ -445,7 +463,7 @@ void launch_gemm_tiled(int glu, float alpha, float limit, const void* A, int64_t
         const int ncb = (int)cdiv64(N, GLU ? BN / 2 : BN);                                                                             \
         hipLaunchKernelGGL((moe_gemm_tiled_kernel<T, GLU, BN>), dim3((unsigned)((max_tiles * ncb + 7) / 8 * 8)), dim3(256), 0, st,     \
                            (const T*)A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, (const T*)Wt, N, K,   \
-                           (T*)out, ld_out, alpha, limit, ncb);                                                                        \
+                           (T*)out, ld_out, alpha, limit, ncb, act);                                                                   \
     } while (0)
     if (glu == 2)
         TGIS_MOE_TILED(2, 256);
@@ -476,7 +494,7 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const T* __restrict__ 
 }
 
 template <typename T>
-void launch_gemm(int glu, float alpha, float limit, const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
+void launch_gemm(int glu, int act, float alpha, float limit, const void* A, int64_t ld_a, const int32_t* sorted, int pair_div, const float* pair_scale,
                  const int32_t* tile_expert, const int32_t* n_tiles, const void* Wt, int64_t N, int64_t K,
                  void* out, int64_t ld_out, int64_t max_tiles, hipStream_t st) {
     const bool ksplit = max_tiles * cdiv64(N, 128) < 1024;
@@ -485,7 +503,7 @@ void launch_gemm(int glu, float alpha, float limit, const void* A, int64_t ld_a,
     dim3 grid((unsigned)(ksplit ? cdiv64(N, 32) : cdiv64(N, 64)), (unsigned)(ksplit ? max_tiles : cdiv64(max_tiles, 4)));
 #define TGIS_MOE_LAUNCH(GLU, KW)                                                                                                       \
     hipLaunchKernelGGL((moe_gemm_kernel<T, GLU, KW>), grid, dim3(KW > 4 ? 512 : 256), 0, st, (const T*)A, ld_a, sorted, pair_div, pair_scale, \
-                       tile_expert, n_tiles, (const T*)Wt, N, K, (T*)out, ld_out, alpha, limit)
+                       tile_expert, n_tiles, (const T*)Wt, N, K, (T*)out, ld_out, alpha, limit, act)
 #define TGIS_MOE_GLU(KW)                     \
     do {                                     \
         if (glu == 2)                        \
@@ -562,6 +580,20 @@ extern "C" int tgis_moe_route_grouped(const void* h, int64_t ld_h, const float* 
                           keep_groups, renorm_eps);
 }
 
+// The choice alone, from logits [T][E] fp32: scores are their sigmoids; experts come from the `keep` best of `groups` equal groups of
+// neighbours (a group counts by the sum of its two largest scores); weights = chosen scores * scale.
+extern "C" int tgis_moe_choose(const float* logits, int64_t T, int E, int k, int groups, int keep, float scale, int32_t* idx, float* weight,
+                               void* stream) {
+    TGIS_CHECK_ARG(logits && idx && weight && E >= 1 && E <= 2048 && k >= 1 && k <= 64 && groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups &&
+                       (int64_t)keep * (E / groups) >= k,
+                   "tgis_moe_choose: cannot choose %d of %d experts in the best %d of %d groups", k, E, keep, groups);
+    if (T == 0) return TGIS_OK;
+    hipLaunchKernelGGL(moe_choose_kernel, dim3((unsigned)cdiv64(T, 4)), dim3(256), (size_t)4 * (E + groups) * sizeof(float), (hipStream_t)stream, logits,
+                       T, E, k, groups, keep, scale, idx, weight);
+    TGIS_CHECK_LAUNCH();
+    return TGIS_OK;
+}
+
 extern "C" int tgis_moe_align(const int32_t* idx, int64_t n_pairs, int E, int32_t* sorted, int64_t capacity, int32_t* tile_expert,
                               int32_t* pos_of_pair, int32_t* n_tiles, int tile_rows, void* stream) {
     TGIS_CHECK_ARG(idx && sorted && tile_expert && pos_of_pair && n_tiles, "tgis_moe_align: null tensor");
@@ -579,7 +611,9 @@ extern "C" int tgis_moe_gemm(const void* A, int64_t ld_a, const int32_t* sorted,
                              const int32_t* tile_expert, const int32_t* n_tiles, const void* image, int64_t N, int64_t K, int glu,
                              float alpha, float limit, void* out, int64_t ld_out, int64_t capacity, int tile_rows, int dtype, void* stream) {
     TGIS_CHECK_ARG(A && tile_expert && n_tiles && image && out, "tgis_moe_gemm: null tensor");
-    TGIS_CHECK_ARG(dtype3(dtype) && glu >= 0 && glu <= 2, "tgis_moe_gemm: bad dtype or glu");
+    TGIS_CHECK_ARG(dtype3(dtype) && glu >= 0 && glu <= 3, "tgis_moe_gemm: bad dtype or glu");
+    const int act = glu == 3 ? 1 : 0;  // a plain weight whose product is squared where it is positive
+    if (act) glu = 0;
     const int per = dtype == TGIS_F32 ? 4 : 8;
     TGIS_CHECK_ARG(N >= 1 && K >= per && K % per == 0 && ld_a % per == 0 && ld_a >= K && ld_out >= N,
                    "tgis_moe_gemm: K (%ld) and the A row stride (%ld) must be multiples of %d", (long)K, (long)ld_a, per);
@@ -595,19 +629,19 @@ extern "C" int tgis_moe_gemm(const void* A, int64_t ld_a, const int32_t* sorted,
         TGIS_CHECK_ARG(dtype != TGIS_F32 && K % 32 == 0 && tiles * cdiv64(N, 128) < (1ll << 30),
                        "tgis_moe_gemm: 128-row tiles take two-byte dtypes and K a multiple of 32 (got %ld)", (long)K);
         if (dtype == TGIS_F16)
-            launch_gemm_tiled<f16>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, image, N, K, out, ld_out, tiles, st);
+            launch_gemm_tiled<f16>(glu, act, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, image, N, K, out, ld_out, tiles, st);
         else
-            launch_gemm_tiled<bf16>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, image, N, K, out, ld_out, tiles, st);
+            launch_gemm_tiled<bf16>(glu, act, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, image, N, K, out, ld_out, tiles, st);
         TGIS_CHECK_LAUNCH();
         return TGIS_OK;
     }
     TGIS_CHECK_ARG(tiles <= 65535, "tgis_moe_gemm: %ld tiles exceed one grid", (long)tiles);
     if (dtype == TGIS_F16)
-        launch_gemm<f16>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, image, N, K, out, ld_out, tiles, st);
+        launch_gemm<f16>(glu, act, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, image, N, K, out, ld_out, tiles, st);
     else if (dtype == TGIS_BF16)
-        launch_gemm<bf16>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, image, N, K, out, ld_out, tiles, st);
+        launch_gemm<bf16>(glu, act, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, image, N, K, out, ld_out, tiles, st);
     else
-        launch_gemm<float>(glu, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, image, N, K, out, ld_out, tiles, st);
+        launch_gemm<float>(glu, act, alpha, limit, A, ld_a, sorted, pair_div, pair_scale, tile_expert, n_tiles, image, N, K, out, ld_out, tiles, st);
     TGIS_CHECK_LAUNCH();
     return TGIS_OK;
 }

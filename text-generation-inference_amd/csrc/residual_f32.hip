@@ -295,7 +295,7 @@ __device__ __forceinline__ float xielu_f32(float z, float ap, float an) {
     return z > 0.f ? ap * z * z + 0.5f * z : an * (expm1f(z) - z) + 0.5f * z;
 }
 
-// act 0: xIELU(in)   act 1: in * sigmoid(other)   act 2: cap * tanh(in / cap) (p0 = cap)
+// act 0: xIELU(in)   act 1: in * sigmoid(other)   act 2: cap * tanh(in / cap) (p0 = cap)   act 3: max(in, 0)^2
 template <typename T, typename TO>
 __global__ void unary_rows_kernel(const T* __restrict__ in, int64_t ld_in, const T* __restrict__ other, int64_t ld_other,
                                   TO* __restrict__ out, int64_t ld_out, int64_t rows, int64_t C, int act, float p0, float p1) {
@@ -308,8 +308,10 @@ __global__ void unary_rows_kernel(const T* __restrict__ in, int64_t ld_in, const
             r = xielu_f32(z, p0, p1);
         } else if (act == 1) {
             r = z / (1.f + expf(-Elem<T>::ld(other + t * ld_other + c)));
-        } else {
+        } else if (act == 2) {
             r = p0 * tanhf(z / p0);
+        } else {
+            r = fmaxf(z, 0.f) * fmaxf(z, 0.f);
         }
         out[t * ld_out + c] = cvt_out<TO>(r);
     }
@@ -331,9 +333,12 @@ __global__ void unary_rows_vec_kernel(const T* __restrict__ in, int64_t ld_in, c
             const f32x4 g = Vec4<T>::ld(other + t * ld_other + c);
 #pragma unroll
             for (int e = 0; e < 4; ++e) r[e] = z[e] / (1.f + expf(-g[e]));
-        } else {
+        } else if (act == 2) {
 #pragma unroll
             for (int e = 0; e < 4; ++e) r[e] = p0 * tanhf(z[e] / p0);
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) r[e] = fmaxf(z[e], 0.f) * fmaxf(z[e], 0.f);
         }
         Vec4<T>::st(out + t * ld_out + c, r);
     }
@@ -700,6 +705,17 @@ extern "C" int tgis_xielu(const void* in, int64_t ld_in, void* out, int64_t ld_o
     hipStream_t st = (hipStream_t)stream;
     TgisTimedScope timed(TGIS_OP_ACT, st);
     TGIS_BY_DTYPE(dtype, launch_unary<TT, TT>(in, ld_in, nullptr, 0, out, ld_out, rows, C, 0, ap, an, st));
+    TGIS_CHECK_LAUNCH();
+    return TGIS_OK;
+}
+
+// out = max(in, 0)^2 (out may alias in)
+extern "C" int tgis_relu2(const void* in, int64_t ld_in, void* out, int64_t ld_out, int64_t rows, int64_t C, int dtype, void* stream) {
+    TGIS_CHECK_ARG(in && out && C > 0 && ld_in >= C && ld_out >= C && dtype3(dtype), "tgis_relu2: bad arguments");
+    if (rows == 0) return TGIS_OK;
+    hipStream_t st = (hipStream_t)stream;
+    TgisTimedScope timed(TGIS_OP_ACT, st);
+    TGIS_BY_DTYPE(dtype, launch_unary<TT, TT>(in, ld_in, nullptr, 0, out, ld_out, rows, C, 3, 0.f, 0.f, st));
     TGIS_CHECK_LAUNCH();
     return TGIS_OK;
 }

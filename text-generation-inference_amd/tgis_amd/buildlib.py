@@ -23,6 +23,7 @@ FAMILY_UNITS = {
     "tatevik": ["api", "elementwise", "gemm_dense", "residual_f32", "norm_f32", "attn_varlen", "attn_mixed_heads", "gated_linear_scan",
                 "selective_scan", "causal_conv", "moe", "sampler"],
     "gopetar": ["api", "elementwise", "gemm_dense", "residual_f32", "hyper_streams", "attn_varlen", "head_product", "min_gru", "moe", "sampler"],
+    "fidatar": ["api", "elementwise", "gemm_dense", "residual_f32", "post_norm", "attn_varlen", "matrix_memory", "moe", "sampler"],
 }
 
 

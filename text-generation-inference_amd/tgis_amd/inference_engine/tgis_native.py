@@ -12,7 +12,7 @@ from tgis_amd.utils.dist import initialize_torch_distributed
 from tgis_amd.utils.hub import local_weight_files
 from tgis_amd.utils.weights import Weights
 
-FLASH_TYPES = ["llama", "gpt_bigcode", "lenisun", "senadra", "mananex", "tatevik", "gopetar"]
+FLASH_TYPES = ["llama", "gpt_bigcode", "lenisun", "senadra", "mananex", "tatevik", "gopetar", "fidatar"]
 
 
 def _barrier(group):
@@ -58,6 +58,10 @@ def model_class_for(config):
         from tgis_amd.models.custom_modeling.flash_gopetar_modeling import FlashGopetarForCausalLM
 
         return FlashGopetarForCausalLM, None
+    if model_type == "fidatar":
+        from tgis_amd.models.custom_modeling.flash_fidatar_modeling import FlashFidatarForCausalLM
+
+        return FlashFidatarForCausalLM, None
     raise NotImplementedError(f"Flash attention currently only supported by the following model types: {FLASH_TYPES}")
 
 

@@ -174,6 +174,18 @@ SIGNATURES = {
     "tgis_hyper_update": (_c_int, [_vp, _vp, _vp, _c_i64, _c_f, _vp, _c_int, _vp, _c_i64, _c_int, _vp, _vp, _c_int, _vp, _c_i64, _c_int,
                                    _vp, _vp, _vp, _vp, _c_i64, _c_i64, _c_int, _c_f, _vp, _vp, _c_int, _c_int, _c_int, _vp, _vp, _vp,
                                    _c_int, _vp]),
+    "tgis_post_norm_update": (_c_int, [_vp, _vp, _vp, _c_i64, _c_f, _c_f, _vp, _c_int, _vp, _c_i64, _c_int, _vp, _vp, _c_int, _vp, _vp,
+                                       _vp, _c_i64, _c_i64, _c_f, _vp, _c_int, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_f, _c_int, _vp]),
+    "tgis_narrow_product": (_c_int, [_vp, _c_i64, _vp, _vp, _c_i64, _c_int, _c_i64, _c_int, _vp]),
+    "tgis_moe_choose": (_c_int, [_vp, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_f, _vp, _vp, _vp]),
+    "tgis_relu2": (_c_int, [_vp, _c_i64, _vp, _c_i64, _c_i64, _c_i64, _c_int, _vp]),
+    "tgis_dense_gemm_relu2": (_c_int, [_vp, _c_i64, _vp, _vp, _c_i64, _c_i64, _c_i64, _c_i64, _c_int, _vp, _c_i64, _vp]),
+    "tgis_matrix_memory": (_c_int, [_vp, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _vp, _c_i64, _vp, _vp, _c_f, _vp, _vp, _vp, _vp, _vp, _vp,
+                                    _vp, _c_i64, _c_i64, _c_i64, _c_i64, _c_int, _c_int, _c_int, _c_f, _c_f, _c_f, _c_int, _c_int, _vp]),
+    "tgis_norm_rope_rows_kv_write": (_c_int, [_vp, _c_i64, _c_i64, _c_i64, _c_i64, _vp, _vp, _c_f, _vp, _c_f, _vp, _vp, _vp, _c_i64, _c_int,
+                                              _c_int, _c_int, _c_int, _c_int, _c_int, _vp]),
+    "tgis_attn_varlen_blocks": (_c_int, [_vp, _c_i64, _vp, _vp, _vp, _c_i64, _vp, _vp, _c_i64, _vp, _c_i64, _c_i64, _c_i64, _c_i64,
+                                         _c_int, _c_int, _c_int, _c_int, _c_f, _c_int, _vp, _vp, _c_i64, _c_int, _c_int, _vp]),
 }
 
 _lib = None
@@ -1055,13 +1067,15 @@ class MoeWeight:
 
 
 def moe_gemm(A, w: MoeWeight, tile_expert, n_tiles, capacity: int, sorted_=None, pair_div: int = 1, pair_scale=None, clamp=None,
-             tile_rows: int = 32):
+             tile_rows: int = 32, relu2: bool = False):
     """Returns [capacity, w.N].  sorted_ with pair_div 0: rows in place, the list marks padding.  A gate | up weight is activated: silu(gate) * up, or with clamp = (alpha, limit) the clamped unit.
-    tile_rows: the alignment moe_align was asked for."""
+    relu2: the product of a plain weight is squared where it is positive, zero elsewhere.  tile_rows: the alignment moe_align was asked
+    for."""
+    assert not (relu2 and w.glu)
     assert A.dim() == 2 and A.stride(1) == 1 and w.dtype == A.dtype and A.shape[1] == w.K
     assert capacity % tile_rows == 0 and tile_expert.shape[0] * tile_rows == capacity and ((sorted_ is not None and pair_div > 0) or A.shape[0] >= capacity)
     out = torch.empty((capacity, w.N), dtype=A.dtype, device=A.device)
-    glu = (2 if clamp is not None else 1) if w.glu else 0
+    glu = (2 if clamp is not None else 1) if w.glu else (3 if relu2 else 0)
     alpha, limit = clamp if clamp is not None else (0.0, 0.0)
     _check(load_library().tgis_moe_gemm(
         _ptr(A), A.stride(0), _i32(sorted_, "sorted"), pair_div, _f32(pair_scale, "pair_scale"), _ptr(tile_expert), _ptr(n_tiles),
@@ -1641,3 +1655,137 @@ def hyper_update(x, y, cur, nxt, eps: float, y_dtype, ids=None, table=None, emb_
         weight, k, sh, ld_sh, sh_slabs, gate, _f32(cur, "cur") if kind else None, _f32(nxt, "nxt"), _ptr(h), T, W, s, float(eps),
         *r_args, dtype_code3(y_dtype), _stream()), "tgis_hyper_update")
     return (x_out, h) if routed is None else (x_out, h, routed)
+
+
+# ---- norm after the sum, matrix memory with exponential gates, normed half-rotated q and k ---------------------------------------
+def post_norm_update(x, y, alpha: float, w, eps: float, y_dtype, ids=None, table=None, emb_scale: float = 1.0, w2=None, keep_x: bool = True,
+                     dots=None, router=None):
+    """x [T, W] fp32 (in place): x <- rms_norm(alpha x + y) * w, h = x rounded to y_dtype (or rms_norm(x) * w2).  y: a tensor of
+    y_dtype, split-K slabs (`Partial`), `MixtureRows` without a shared row, or None; ids + table instead of x: the scaled embedding
+    rows begin the stream.  dots [R, W] fp32: products of the row h; router = (top, groups, keep, scale): they are logits to choose
+    from.  Returns (x or None, h, products [T, R] / (idx, weight) / None)."""
+    if ids is not None:
+        assert x is None and y is None and ids.dtype == torch.int64 and table.is_contiguous() and table.dtype == y_dtype
+        T, W, dev = ids.shape[0], table.shape[1], table.device
+        x_out = torch.empty((T, W), dtype=torch.float32, device=dev) if keep_x else None
+    else:
+        T, W = x.shape
+        assert x.dtype == torch.float32 and x.is_contiguous()
+        x_out, dev = (x if keep_x else None), x.device
+    kind, p, ld, slabs, pos, weight, k = 0, None, 0, 0, None, None, 0
+    if isinstance(y, Partial):
+        assert y.shape == (T, W) and y.bias is None
+        kind, p, ld, slabs = 2, _ptr(y.slabs), y.ld, y.S
+    elif isinstance(y, MixtureRows):
+        assert y.rows.dtype == y_dtype and y.rows.shape[1] == W and y.pos.shape[0] == T * y.k and y.shared is None
+        kind, p, ld, pos, weight, k = 3, _ptr(y.rows), y.rows.stride(0), _i32(y.pos, "pos"), _f32(y.weight, "weight"), y.k
+    elif y is not None:
+        assert y.shape == (T, W) and y.dtype == y_dtype and y.stride(1) == 1
+        kind, p, ld = 1, _ptr(y), y.stride(0)
+    for g in (w, w2):
+        assert g is None or g.shape[0] == W
+    h = torch.empty((T, W), dtype=y_dtype, device=dev)
+    R, extra, out, idx, wt, (top, groups, keep, scale) = 0, None, None, None, None, (0, 1, 1, 1.0)
+    if dots is not None:
+        R = dots.shape[0]
+        assert dots.shape[1] == W
+        if router is not None:
+            top, groups, keep, scale = router
+            extra = idx, wt = (torch.empty((T, top), dtype=torch.int32, device=dev), torch.empty((T, top), dtype=torch.float32, device=dev))
+        else:
+            extra = out = torch.empty((T, R), dtype=torch.float32, device=dev)
+    _check(load_library().tgis_post_norm_update(
+        _ptr(x), _ptr(ids), _ptr(table), table.shape[0] if table is not None else 0, float(emb_scale), float(alpha), _ptr(x_out), kind, p, ld,
+        slabs, pos, weight, k, _f32(w, "w"), _f32(w2, "w2"), _ptr(h), T, W, float(eps), _f32(dots, "dots"), R, _ptr(out), _ptr(idx), _ptr(wt),
+        int(top), int(groups), int(keep), float(scale), dtype_code3(y_dtype), _stream()), "tgis_post_norm_update")
+    return x_out, h, extra
+
+
+def narrow_product(h: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """h [T, W] @ w [R, W]^T in fp32 (two-byte operands, few outputs, many rows)."""
+    assert h.dim() == 2 and h.stride(1) == 1 and w.is_contiguous() and h.dtype == w.dtype and h.shape[1] == w.shape[1]
+    out = torch.empty((h.shape[0], w.shape[0]), dtype=torch.float32, device=h.device)
+    _check(load_library().tgis_narrow_product(_ptr(h), h.stride(0), _ptr(w), _ptr(out), h.shape[0], w.shape[0], h.shape[1],
+                                              dtype_code(h.dtype), _stream()), "tgis_narrow_product")
+    return out
+
+
+def moe_choose(logits: torch.Tensor, k: int, groups: int, keep: int, scale: float):
+    """(idx [T, k] int32, weight [T, k] fp32) from router logits [T, E]: sigmoid scores, the best groups by their two best scores."""
+    assert logits.is_contiguous()
+    T, E = logits.shape
+    idx = torch.empty((T, k), dtype=torch.int32, device=logits.device)
+    weight = torch.empty((T, k), dtype=torch.float32, device=logits.device)
+    _check(load_library().tgis_moe_choose(_f32(logits, "logits"), T, E, int(k), int(groups), int(keep), float(scale), _ptr(idx), _ptr(weight),
+                                          _stream()), "tgis_moe_choose")
+    return idx, weight
+
+
+def relu2(x: torch.Tensor) -> torch.Tensor:
+    assert x.dim() == 2 and x.stride(1) == 1
+    out = torch.empty((x.shape[0], x.shape[1]), dtype=x.dtype, device=x.device)
+    _check(load_library().tgis_relu2(_ptr(x), x.stride(0), _ptr(out), out.stride(0), x.shape[0], x.shape[1], dtype_code3(x.dtype), _stream()),
+           "tgis_relu2")
+    return out
+
+
+def dense_gemm_relu2(x: torch.Tensor, w: DenseWeight, ws: Workspace) -> torch.Tensor:
+    """relu2(x @ W^T) in one launch (decode-sized M, plain image)."""
+    assert x.dim() == 2 and x.stride(1) == 1 and x.dtype == w.dtype and x.shape[1] == w.K and not w.flags
+    M = x.shape[0]
+    out = torch.empty((M, w.N), dtype=w.dtype, device=x.device)
+    ws.ensure(w.workspace_bytes(M))
+    _check(load_library().tgis_dense_gemm_relu2(_ptr(x), x.stride(0), _ptr(w.image), _ptr(out), out.stride(0), M, w.K, w.N,
+                                                dtype_code(w.dtype), ws.ptr, ws.nbytes, _stream()), "tgis_dense_gemm_relu2")
+    return out
+
+
+def matrix_memory(proj, q_col0: int, k_col0: int, v_col0: int, g_col0: int, gates, i_bias, f_bias, cap: float, gain, state, memory,
+                  state_slots, cu_seqlens_q, positions, H: int, dk: int, dv: int, q_scale: float, eps: float, read_eps: float,
+                  max_q_len: int = 0, impl: int = 0) -> torch.Tensor:
+    """Matrix memory with exponential gates on columns of proj [T, ld]; see tgis_matrix_memory.  -> [T, H dv]."""
+    assert proj.dim() == 2 and proj.stride(1) == 1
+    T = proj.shape[0]
+    out = torch.empty((T, H * dv), dtype=proj.dtype, device=proj.device)
+    assert gates.shape == (T, 2 * H) and gates.is_contiguous() and gain.shape[0] == H * dv
+    assert state.dtype == torch.float32 and state.is_contiguous() and tuple(state.shape[1:]) == (H, dk, dv)
+    assert memory.dtype == torch.float32 and memory.is_contiguous() and tuple(memory.shape[1:]) == (H, dk + 1)
+    assert (i_bias is None or i_bias.shape[0] == H) and (f_bias is None or f_bias.shape[0] == H)
+    _check(load_library().tgis_matrix_memory(
+        _ptr(proj), proj.stride(0), int(q_col0), int(k_col0), int(v_col0), int(g_col0), _f32(gates, "gates"), gates.stride(0),
+        _f32(i_bias, "i_bias"), _f32(f_bias, "f_bias"), float(cap), _f32(gain, "gain"), _ptr(state), _ptr(memory),
+        _i32(state_slots, "state_slots"), _i32(cu_seqlens_q, "cu_seqlens_q"), _i32(positions, "positions"), _ptr(out), out.stride(0),
+        state_slots.shape[0], T, int(max_q_len) if max_q_len > 0 else max(T, 1), H, dk, dv, float(q_scale), float(eps), float(read_eps),
+        int(impl), dtype_code3(proj.dtype), _stream()), "tgis_matrix_memory")
+    return out
+
+
+def norm_rope_rows_kv_write(proj, q_col0: int, k_col0: int, v_col0: int, q_gain, k_gain, eps: float, turns, amp: float, slots, k_pool, v_pool,
+                            H: int, G: int, dk: int, dv: int, rot_dims: int):
+    """Normed, gained and half-split rotated q (in place) and k, and v, of a step: the latter two into their page slots."""
+    assert proj.dim() == 2 and proj.stride(1) == 1 and k_pool.dtype == proj.dtype and v_pool.dtype == proj.dtype
+    assert slots.shape[0] == proj.shape[0] and q_gain.shape[0] == dk and k_gain.shape[0] == dk
+    assert rot_dims == 0 or tuple(turns.shape) == (proj.shape[0], rot_dims // 2, 2)
+    _check(load_library().tgis_norm_rope_rows_kv_write(
+        _ptr(proj), proj.stride(0), q_col0, k_col0, v_col0, _f32(q_gain, "q_gain"), _f32(k_gain, "k_gain"), float(eps),
+        _f32(turns, "turns") if rot_dims else None, float(amp), _i32(slots, "slots"), _ptr(k_pool), _ptr(v_pool), proj.shape[0], H, G, dk, dv,
+        rot_dims, dtype_code3(proj.dtype), _stream()), "tgis_norm_rope_rows_kv_write")
+
+
+def attn_varlen_blocks(q, k_pool, v_pool, block_tables, ctx_lens, cu_seqlens_q, H: int, G: int, dk: int, dv: int, scale: float,
+                       chunk: int = 0, sink=None, out=None, max_q_len: int = 1, max_ctx: int = 1, impl: int = 0,
+                       ws: Optional[Workspace] = None):
+    """attn_varlen with a block mask and a sink logit per query head in the denominator."""
+    assert q.dim() == 2 and q.stride(1) == 1 and block_tables.dim() == 2
+    T = q.shape[0]
+    assert sink is None or sink.shape[0] == H
+    if out is None:
+        out = torch.empty((T, H * dv), dtype=q.dtype, device=q.device)
+    assert out.shape == (T, H * dv) and out.stride(1) == 1 and out.dtype == q.dtype
+    _check(load_library().tgis_attn_varlen_blocks(
+        _ptr(q), q.stride(0), _ptr(k_pool), _ptr(v_pool), _i32(block_tables, "block_tables"), block_tables.shape[1],
+        _i32(ctx_lens, "ctx_lens"), _i32(cu_seqlens_q, "cu_seqlens_q"), ctx_lens.shape[0], _ptr(out), out.stride(0), T,
+        max(int(max_q_len), 1), max(int(max_ctx), 1), H, G, dk, dv, float(scale), int(chunk), _f32(sink, "sink"),
+        (ws.ptr + 4096) if ws is not None else None, (ws.nbytes - 4096) if ws is not None else 0, impl, dtype_code3(q.dtype), _stream()),
+        "tgis_attn_varlen_blocks")
+    return out

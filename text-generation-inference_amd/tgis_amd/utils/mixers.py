@@ -36,13 +36,20 @@ argument, so that a model file only maps its config keys and tensor names onto t
   MinGRU              S <- (1 - z) S + z c per channel, gate and candidate from the current token only; SiLU output gate
   HyperStreams        several residual streams: what a sublayer reads is a weighted sum of them, its result is spread over all
                       of them while they are mixed; scalar-gain RMS norms
-  ActivatedMLP        W_down act(W_up h) with the xIELU activation
+  ActivatedMLP        W_down act(W_up h) with the xIELU activation or the square of relu
+  PostNormResidual    one fp32 stream, x <- N(c x + sublayer(x)) w: the norm comes after the sum and the sublayers read x itself
+  RowProducts         a few fp32 products of the stream that a sublayer needs (router logits, gates of a recurrence)
+  HalfRotatedBlockAttention  GQA softmax attention with biases, gained per-head norms of q and k, half-split rotation with YaRN
+                      frequencies, queries that see their own block of positions only, and a 1 in the softmax denominator
+  MatrixMemory        mLSTM: a matrix state with exponential input and forget gates kept in range by a running maximum, a normaliser
+                      beside it; per-head RMS norm, sigmoid output gate
   TokenSideInput      a slice of a second token embedding, gated by a GELU of a projection of the residual stream itself
 
 Activations between kernels are in the serving dtype (bfloat16 or float32); what has to be 32-bit (norm statistics, scores,
 softmax weights, router logits, decays, recurrent state) is 32-bit inside the kernels whatever the serving dtype.
 All of them run ragged steps: a step's tokens are concatenated by sequence and described by a `StepArgs`-like object with
 `cu_seqlens_q`, `ctx_lens`, `slots`, `block_tables`, `state_slots`, `cache`, `state` (models.custom_modeling KVArgs)."""
+import math
 from typing import Optional
 
 import torch
@@ -182,31 +189,43 @@ class GatedUnit:
 class RoutedExperts:
     def __init__(self, weights, prefix: str, experts: int, top: int, shared: bool, router_bias: bool = False,
                  softmax_top: bool = False, weight_on_input: bool = True, grouped_softmax: bool = False, groups: int = 1,
-                 keep_groups: int = 1, renorm_eps: float = 0.0, clamp=None, shared_clamp=None):
+                 keep_groups: int = 1, renorm_eps: float = 0.0, clamp=None, shared_clamp=None, unit: str = "gated",
+                 grouped_sigmoid: Optional[float] = None):
         """clamp = (alpha, limit): the experts are clamped gated units (else SiLU); shared_clamp: the same for the shared one.
         softmax_top: the routing weights are the softmax over the chosen logits (else the sigmoid of each);
         weight_on_input: the weight scales the expert's input (else its output); router_bias: `<prefix>.router.b`.
         grouped_softmax: scores are the softmax over ALL experts; experts are chosen by score + `<prefix>.correction` among the
-        `keep_groups` best of `groups` equal groups of neighbours; weights = chosen scores / (their sum + renorm_eps)."""
+        `keep_groups` best of `groups` equal groups of neighbours; weights = chosen scores / (their sum + renorm_eps).
+        grouped_sigmoid: scores are sigmoids, a group of neighbours counts by the sum of its two largest, weights = chosen scores times
+        this number (the routing then comes from `products`).  unit "relu2": the experts are W_down relu(W_up h)^2."""
         self.E, self.k = experts, top
+        self.relu2 = {"gated": False, "relu2": True}[unit]
+        self.products = None
         self.grouped_softmax, self.groups, self.keep_groups, self.renorm_eps = bool(grouped_softmax), int(groups), int(keep_groups), float(renorm_eps)
-        if grouped_softmax and (experts % self.groups or not 1 <= self.keep_groups <= self.groups):
+        if (grouped_softmax or grouped_sigmoid is not None) and (experts % self.groups or not 1 <= self.keep_groups <= self.groups):
             raise ValueError(f"{prefix}: {experts} experts in {groups} groups, {keep_groups} kept")
         self.correction = _f32(weights.get_tensor(f"{prefix}.correction")) if grouped_softmax and weights.has(f"{prefix}.correction") else None
         self.softmax_top, self.weight_on_input = bool(softmax_top), bool(weight_on_input)
-        self.router = _f32(weights.get_tensor(f"{prefix}.router"))
+        if grouped_sigmoid is not None:
+            if top > 64 or top > self.keep_groups * (experts // self.groups):
+                raise ValueError(f"{prefix}: {top} of {experts} experts in the best {self.keep_groups} of {self.groups} groups")
+            self.products = RowProducts(weights.get_tensor(f"{prefix}.router"), router=(top, self.groups, self.keep_groups, float(grouped_sigmoid)))
+        self.router = _f32(weights.get_tensor(f"{prefix}.router")) if self.products is None else self.products.w32
         self.router_b = _f32(weights.get_tensor(f"{prefix}.router.b")) if router_bias else None
         pad8 = lambda n: (n + 7) // 8 * 8
-        gate = [weights.get_tensor(f"{prefix}.e{e}.gate") for e in range(experts)]
-        ff, W = gate[0].shape
+        gate = [weights.get_tensor(f"{prefix}.e{e}.gate") for e in range(experts)] if not self.relu2 else None
+        up = [weights.get_tensor(f"{prefix}.e{e}.up") for e in range(experts)]
+        ff, W = up[0].shape
         # the grouped GEMM reads 16-byte fragments along its inner dimension: widths that are not multiples of 8 are padded
-        # with zero rows / columns once, here (silu(0) * 0 = 0 keeps a padded hidden channel out of the result)
+        # with zero rows / columns once, here (silu(0) * 0 = relu(0)^2 = 0 keeps a padded hidden channel out of the result)
         self.W, self.Wp, self.ff = W, pad8(W), pad8(ff)
         pad = lambda t, rows, cols: torch.nn.functional.pad(t, (0, cols - t.shape[1], 0, rows - t.shape[0]))
-        # [E, 2 ff, W] (gate rows, then up rows) and [E, W, ff], each as the image the grouped GEMM streams
-        self.w_gate_up = native.MoeWeight(torch.stack([torch.cat([pad(gate[e], self.ff, self.Wp),
-                                                                  pad(weights.get_tensor(f"{prefix}.e{e}.up"), self.ff, self.Wp)], 0)
-                                                       for e in range(experts)]), glu=True)
+        # [E, 2 ff, W] (gate rows, then up rows; plain units: [E, ff, W]) and [E, W, ff], each as the image the grouped GEMM streams
+        if self.relu2:
+            self.w_in = native.MoeWeight(torch.stack([pad(u, self.ff, self.Wp) for u in up]), glu=False)
+        else:
+            self.w_in = native.MoeWeight(torch.stack([torch.cat([pad(g, self.ff, self.Wp), pad(u, self.ff, self.Wp)], 0) for g, u in zip(gate, up)]),
+                                         glu=True)
         self.w_down = native.MoeWeight(torch.stack([pad(weights.get_tensor(f"{prefix}.e{e}.down"), W, self.ff) for e in range(experts)]), glu=False)
         self.clamp = clamp
         self.shared = None
@@ -219,7 +238,7 @@ class RoutedExperts:
     @property
     def plain_router(self):
         """What a residual update needs to route for this mixture on the way (native.hyper_update), or None."""
-        if self.grouped_softmax or self.router_b is not None or self.k > 64:
+        if self.grouped_softmax or self.products is not None or self.router_b is not None or self.k > 64:
             return None
         return self.router, self.shared_gate, self.k, self.softmax_top
 
@@ -229,6 +248,8 @@ class RoutedExperts:
         T, W = h.shape
         if routed is not None:
             idx, weight, sg = routed
+        elif self.products is not None:
+            (idx, weight), sg = self.products.of(h), None
         elif self.grouped_softmax:
             idx, weight = native.moe_route_grouped(h, self.router, self.correction, self.k, self.groups, self.keep_groups, self.renorm_eps)
             sg = None
@@ -238,8 +259,8 @@ class RoutedExperts:
         sorted_, tile_expert, pos, n_tiles = native.moe_align(idx, self.E, tm)
         cap = sorted_.shape[0]
         hp = h if self.Wp == W else torch.nn.functional.pad(h, (0, self.Wp - W))
-        act = native.moe_gemm(hp, self.w_gate_up, tile_expert, n_tiles, cap, sorted_=sorted_, pair_div=self.k,
-                              pair_scale=weight.view(-1) if self.weight_on_input else None, clamp=self.clamp, tile_rows=tm)
+        act = native.moe_gemm(hp, self.w_in, tile_expert, n_tiles, cap, sorted_=sorted_, pair_div=self.k,
+                              pair_scale=weight.view(-1) if self.weight_on_input else None, clamp=self.clamp, tile_rows=tm, relu2=self.relu2)
         rows = native.moe_gemm(act, self.w_down, tile_expert, n_tiles, cap, sorted_=sorted_, pair_div=0, tile_rows=tm)
         shared = self.shared(h, partial=defer) if self.shared is not None else None
         if defer:
@@ -324,6 +345,21 @@ def scaled_inverse_frequencies(base: float, dims: int, scaling: Optional[dict], 
     out = torch.where(wave > original / low, f / factor, (1 - s) * f / factor + s * f)
     out = torch.where(wave < original / high, f, out)
     return out.to(torch.float32).to(device)
+
+
+def yarn_inverse_frequencies(base: float, dims: int, scaling: Optional[dict], device):
+    """(frequencies, factor on cos and sin) with YaRN scaling: pairs that turn more than `fast` times over `original` positions keep
+    base^(-2i / dims), those that turn less than `slow` times are divided by `factor`, with a linear ramp over the pair's index in
+    between; the factor is 0.1 ln(factor) + 1 (float64, rounded once)."""
+    if not scaling:
+        return rotary_inverse_frequencies(base, dims, device), 1.0
+    factor, original, fast, slow = (float(scaling[k]) for k in ("factor", "original", "fast", "slow"))
+    pair_of = lambda turns: dims * math.log(original / (2 * math.pi * turns)) / (2 * math.log(float(base)))
+    lo, hi = max(math.floor(pair_of(fast)), 0), min(math.ceil(pair_of(slow)), dims - 1)
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    f = float(base) ** (-2.0 * i / dims)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0, 1)
+    return (f / factor * ramp + f * (1 - ramp)).to(torch.float32).to(device), 0.1 * math.log(factor) + 1.0
 
 
 class LatentAttention:
@@ -878,31 +914,163 @@ class PowerNormMLP:
 
 
 def _softplus(z: float) -> float:
-    import math
-
     return z if z > 30 else math.log1p(math.exp(z))
 
 
 class ActivatedMLP:
-    """W_down xielu(W_up h);  xielu(z) = ap z^2 + z / 2 for z > 0, an (exp(z) - 1 - z) + z / 2 otherwise, with
-    ap = softplus(p), an = 1/2 + softplus(q) from the layer's two learned numbers."""
+    """W_down act(W_up h).  act "xielu": ap z^2 + z / 2 for z > 0, an (exp(z) - 1 - z) + z / 2 otherwise, with ap = softplus(p),
+    an = 1/2 + softplus(q) from the layer's two learned numbers (`<prefix>.act`);  "relu2": max(z, 0)^2."""
 
-    def __init__(self, weights, prefix: str):
+    def __init__(self, weights, prefix: str, act: str = "xielu"):
         self.up = load_linear(weights, f"{prefix}.up")
         self.down = load_linear(weights, f"{prefix}.down")
-        p, q = weights.get_tensor(f"{prefix}.act").float().tolist()
-        self.ap, self.an = _softplus(p), 0.5 + _softplus(q)
+        if act not in ("xielu", "relu2"):
+            raise ValueError(f"{prefix}: unknown activation {act!r}")
+        self.relu2 = act == "relu2"
+        if not self.relu2:
+            p, q = weights.get_tensor(f"{prefix}.act").float().tolist()
+            self.ap, self.an = _softplus(p), 0.5 + _softplus(q)
 
     def forward(self, h: torch.Tensor, partial: bool = False):
         partial = partial and can_defer(self.down)
         if self.up.streams and h.shape[0] <= SKINNY_MAX_M:
             # decode-sized steps: the activation where the weight-streaming GEMM finishes its output
-            act = native.dense_gemm_xielu(h, self.up.prepared, workspace(h.device), self.ap, self.an)
+            if self.relu2:
+                act = native.dense_gemm_relu2(h, self.up.prepared, workspace(h.device))
+            else:
+                act = native.dense_gemm_xielu(h, self.up.prepared, workspace(h.device), self.ap, self.an)
         else:
-            act = native.xielu(self.up(h), self.ap, self.an)
+            act = native.relu2(self.up(h)) if self.relu2 else native.xielu(self.up(h), self.ap, self.an)
         return self.down(act, partial=partial)
 
     __call__ = forward
+
+
+# rows up to which a sublayer's fp32 products of the stream ride in the residual update in front of it
+ROW_PRODUCTS_FUSED_MAX_ROWS = 64
+
+
+class RowProducts:
+    """fp32 products of the stream's row with the few rows of `weight` [R, W] that a sublayer needs: the logits of a router
+    (router = (top, groups, kept groups, scale): experts are chosen from them) or the gates of a recurrence."""
+
+    def __init__(self, weight: torch.Tensor, router=None):
+        self.w32 = _f32(weight)
+        self.w = weight.contiguous()
+        self.router = router
+
+    def rides(self, rows: int) -> bool:
+        """In the residual update (steps of few tokens; fp32 serving, odd widths), or by launches of their own on the matrix cores?"""
+        return rows <= ROW_PRODUCTS_FUSED_MAX_ROWS or self.w.dtype == torch.float32 or self.w.shape[1] % 8 != 0
+
+    def of(self, h: torch.Tensor):
+        z = native.narrow_product(h, self.w) if h.dtype != torch.float32 and h.shape[1] % 8 == 0 else torch.nn.functional.linear(h.float(), self.w32)
+        return native.moe_choose(z, *self.router) if self.router is not None else z
+
+
+class PostNormResidual:
+    """The residual of a decoder that norms after the sum: x <- N(alpha x + y) * w, N(z) = z / sqrt(mean z^2 + eps), x fp32.  Norms are
+    given in execution order, then the one behind the whole stack.  One launch per boundary applies a sublayer's result, leaves the
+    next one's input (x rounded to the serving dtype) and, on steps of few tokens, its RowProducts."""
+
+    def __init__(self, weights, norms, final_norm: str, alpha: float, eps: float):
+        self.norms = [_f32(weights.get_tensor(n)) for n in norms]
+        self.final = _f32(weights.get_tensor(final_norm))
+        self.alpha, self.eps = float(alpha), float(eps)
+
+    def _update(self, rows: int, products: Optional[RowProducts], **kw):
+        ride = products is not None and products.rides(rows)
+        x, h, extra = native.post_norm_update(alpha=self.alpha, eps=self.eps, dots=products.w32 if ride else None,
+                                              router=products.router if ride else None, **kw)
+        if products is not None and not ride:
+            extra = products.of(h)
+        return x, h, extra
+
+    def begin(self, ids, table, scale: float, dtype, products: Optional[RowProducts] = None):
+        """(stream, first sublayer's input, its products) from the embedding rows."""
+        return self._update(ids.shape[0], products, x=None, y=None, w=None, y_dtype=dtype, ids=ids, table=table, emb_scale=scale)
+
+    def step(self, q: int, x, y, dtype, products: Optional[RowProducts] = None, last: bool = False, keep_x: bool = True):
+        """The result y of sublayer q joins the stream; (stream, next input, its products).  last: the final norm follows."""
+        return self._update(x.shape[0], products, x=x, y=y, w=self.norms[q], y_dtype=dtype, w2=self.final if last else None,
+                            keep_x=keep_x)
+
+
+class HalfRotatedBlockAttention:
+    """GQA softmax attention: q, k and v with biases (`<prefix>.q.b`, ...); every q and k head divided by its root mean square times
+    `<prefix>.q.norm` / `.k.norm` [dim]; channels (i, i + rot_dims / 2) of the first rot_dims turned by position * frequency (YaRN, see
+    yarn_inverse_frequencies); position i sees j <= i of its own block of `chunk` positions (0: plain causal); unit_sink: the softmax
+    denominator is 1 + sum exp(score)."""
+
+    def __init__(self, weights, prefix: str, layer_id: int, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, eps: float,
+                 chunk: int = 0, rot_base: float = 10000.0, rot_dims: int = 0, rot_scaling: Optional[dict] = None, unit_sink: bool = True):
+        self.layer_id = layer_id
+        self.H, self.G, self.dk, self.dv = heads, kv_heads, dim, vdim
+        _widths_ok_for_pages(dim, vdim)
+        if heads % kv_heads or rot_dims % 2 or rot_dims > dim:
+            raise ValueError(f"{prefix}: {heads} heads on {kv_heads} kv heads, {rot_dims} rotated of {dim} channels")
+        self.scale, self.eps, self.chunk, self.rot_dims = float(scale), float(eps), int(chunk), int(rot_dims)
+        names = [f"{prefix}.{n}" for n in ("q", "k", "v")]
+        self.proj, self.cols = load_stacked_blocks(weights, names, align=8, biased=names)
+        self.q_gain = _f32(weights.get_tensor(f"{prefix}.q.norm"))
+        self.k_gain = _f32(weights.get_tensor(f"{prefix}.k.norm"))
+        dev = weights.device
+        self.inv_freq, self.amp = yarn_inverse_frequencies(rot_base, self.rot_dims, rot_scaling, dev) if self.rot_dims else (None, 1.0)
+        # layers with the same key share a step's table of turns
+        self.turn_key = ("half", self.rot_dims, float(rot_base), tuple(sorted((rot_scaling or {}).items())))
+        self.sink = torch.zeros(heads, dtype=torch.float32, device=dev) if unit_sink else None
+        self.o = load_linear(weights, f"{prefix}.o")
+        self.defer = can_defer(self.o)
+        self.kv_shape, self.state_shape, self.products = (kv_heads, dim, vdim), None, None
+
+    def forward(self, h: torch.Tensor, products, position_ids, step):
+        proj = self.proj(h)
+        cache = step.cache
+        k_pool, v_pool = cache.k_pool(self.layer_id), cache.v_pool(self.layer_id)
+        turns = step_turns(step, self.turn_key, self.inv_freq, position_ids) if self.rot_dims else None
+        q, k, v = self.cols
+        native.norm_rope_rows_kv_write(proj, q, k, v, self.q_gain, self.k_gain, self.eps, turns, self.amp, step.slots, k_pool, v_pool, self.H,
+                                       self.G, self.dk, self.dv, self.rot_dims)
+        att = native.attn_varlen_blocks(proj[:, q:q + self.H * self.dk], k_pool, v_pool, step.block_tables, step.ctx_lens, step.cu_seqlens_q,
+                                        self.H, self.G, self.dk, self.dv, self.scale, chunk=self.chunk, sink=self.sink,
+                                        max_q_len=step.max_q_len, max_ctx=step.max_ctx, ws=workspace(h.device))
+        return self.o(att, partial=self.defer)
+
+
+class MatrixMemory:
+    """mLSTM per head, S [dim, vdim], n [dim] and a running maximum m that starts at 0, all fp32 in a state slot:
+    m' = max(f + m, i);  S <- e^(f + m - m') S + e^(i - m') k v^T, n likewise with k;  o = S^T q / (max(|n . q|, e^-m') + read_eps)
+    with q = dim^-1/2 W_q h and soft-capped gates i = soft(W_i h + b_i), f = ln sigmoid(soft(W_f h + b_f)), soft(z) = cap tanh(z / cap);
+    then o / rms(o) per head, times `<prefix>.norm` (all heads' width), times sigmoid(W_g h).  The gates' products with the stream are
+    fp32 (`products`, made by the owner)."""
+
+    def __init__(self, weights, prefix: str, layer_id: int, heads: int, dim: int, vdim: int, gate_cap: float, eps: float,
+                 read_eps: float = 1e-6):
+        self.layer_id = layer_id
+        self.H, self.dk, self.dv = heads, dim, vdim
+        if dim > 256 or vdim > 256:
+            raise NotImplementedError(f"{prefix}: matrix memories of up to 256 x 256 per head are served (got {dim} x {vdim})")
+        self.cap, self.eps, self.read_eps, self.q_scale = float(gate_cap), float(eps), float(read_eps), dim ** -0.5
+        self.proj, self.cols = load_stacked_blocks(weights, [f"{prefix}.{n}" for n in ("q", "k", "v", "g")], align=8)
+        self.products = RowProducts(torch.cat([weights.get_tensor(f"{prefix}.i"), weights.get_tensor(f"{prefix}.f")], 0))
+        bias = lambda n: _f32(weights.get_tensor(f"{prefix}.{n}.b")) if weights.has(f"{prefix}.{n}.b") else None
+        self.i_bias, self.f_bias = bias("i"), bias("f")
+        self.gain = _f32(weights.get_tensor(f"{prefix}.norm"))
+        if self.gain.shape[0] != heads * vdim:
+            raise ValueError(f"{prefix}.norm: {self.gain.shape[0]} gains for {heads} heads of {vdim}")
+        self.o = load_linear(weights, f"{prefix}.o")
+        self.defer = can_defer(self.o)
+        self.kv_shape = None
+        self.state_shape = {"matrix": (heads, dim, vdim), "memory": (heads, dim + 1)}
+
+    def forward(self, h: torch.Tensor, products, position_ids, step):
+        """products: the gates' [T, 2 heads] fp32 (input gates, then forget gates)."""
+        proj = self.proj(h)
+        q, k, v, g = self.cols
+        out = native.matrix_memory(proj, q, k, v, g, products, self.i_bias, self.f_bias, self.cap, self.gain, step.state.state[self.layer_id],
+                                   step.state.shift[self.layer_id], step.state_slots, step.cu_seqlens_q, position_ids, self.H, self.dk, self.dv,
+                                   self.q_scale, self.eps, self.read_eps, max_q_len=step.max_q_len)
+        return self.o(out, partial=self.defer)
 
 
 class TokenSideInput:
