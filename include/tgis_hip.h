@@ -695,7 +695,8 @@ int tgis_dense_gemm_relu2(const void* x, int64_t ldx, const void* prepared, void
  *   out = o / sqrt(mean o^2 + eps) * gain[h dv ..] * sigmoid(g)      (the mean over the head; g_col0 < 0: no gate)
  * q, k, v, g: columns of proj [T, ld] (head h at col0 + h dk / dv); gates [T, ld_gates] fp32: z_i of head h at h, z_f at H + h.
  * state [slots][H][dk][dv] and memory [slots][H][dk + 1] (n, then m) fp32, read unless the step starts at position 0, written back.
- * dk, dv <= 256.  impl 0: by size; 1: token by token; 2: chunks on the matrix cores (two-byte dtypes, dk, dv <= 128). */
+ * dk, dv <= 256.  impl 0: by size; 1: token by token; 2: chunks of 64 on the matrix cores (bf16, dk and
+ * dv multiples of 8 up to 128, q, k, v columns and rows 16-byte aligned). */
 int tgis_matrix_memory(const void* proj, int64_t ld, int64_t q_col0, int64_t k_col0, int64_t v_col0, int64_t g_col0,
                        const float* gates, int64_t ld_gates, const float* i_bias, const float* f_bias, float cap,
                        const float* gain, float* state, float* memory, const int32_t* state_slots,

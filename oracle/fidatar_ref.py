@@ -24,6 +24,9 @@ DT = torch.float64
 READ_EPS = 1e-6
 # filled by `route` while not None: how far (in score) a token's choice of groups and of experts is from another choice
 ROUTER_MARGINS: Optional[list] = None
+# filled by `mlstm` while not None: |S^T q| sqrt(dk) / (|S| |q|) per token and head, about one for a q of no particular direction.  The
+# read-out is normed, so a q all but orthogonal to what S holds (the first tokens' S has rank one!) turns rounding into direction.
+READ_MARGINS: Optional[list] = None
 
 
 # ---- small pieces ---------------------------------------------------------------------------------------------------------
@@ -121,6 +124,9 @@ def mlstm(h, p, m: dict, eps: float, st: dict):
     for t in range(T):
         S, n, mx, o = matrix_memory_step(S, n, mx, q[t], k[t], v[t], i[t], f[t])
         rows.append(o)
+        if READ_MARGINS is not None:
+            size = (S * S).sum((1, 2)).sqrt() * (q[t] * q[t]).sum(-1).sqrt()
+            READ_MARGINS.extend(((S * q[t][:, :, None]).sum(1).norm(dim=-1) * dk ** 0.5 / size.clamp_min(1e-30)).tolist())
     st["S"], st["n"], st["m"] = S, n, mx
     o = rms_unit(torch.stack(rows), eps).reshape(T, H * dv) * p["norm"]
     return (o * torch.sigmoid(h @ p["g"].T)) @ p["o"].T
@@ -219,10 +225,11 @@ class FidatarRef:
         return self.advance(self.new_state(), tokens, trace)
 
 
-def clear_cut_tokens(config: dict, tensors, n: int, seed: int, margin: float = 0.03) -> List[int]:
-    """n random tokens, each drawn again until no router of the model is within `margin` (in score) of choosing other experts
-    for it: what a reduced-precision run computes for them differs from this restatement by rounding, not by a decision."""
-    global ROUTER_MARGINS
+def clear_cut_tokens(config: dict, tensors, n: int, seed: int, margin: float = 0.03, read_margin: float = 0.3) -> List[int]:
+    """n random tokens, each drawn again until no router of the model is within `margin` (in score) of choosing other experts for it
+    and no memory's read-out is below `read_margin` of its usual size: what a reduced-precision run computes for them differs from
+    this restatement by rounding, not by a decision."""
+    global ROUTER_MARGINS, READ_MARGINS
     g = torch.Generator().manual_seed(seed)
     ref = FidatarRef(config, tensors)
     state, toks = ref.new_state(), []
@@ -232,15 +239,15 @@ def clear_cut_tokens(config: dict, tensors, n: int, seed: int, margin: float = 0
             for _ in range(60):
                 t = int(torch.randint(0, config["vocab"], (1,), generator=g))
                 trial = copy.deepcopy(state)
-                ROUTER_MARGINS = []
+                ROUTER_MARGINS, READ_MARGINS = [], []
                 ref.advance(trial, [t])
-                closest = min(ROUTER_MARGINS, default=margin)
+                closest = min(min(ROUTER_MARGINS, default=margin) / margin, min(READ_MARGINS, default=read_margin) / read_margin)
                 if best is None or closest > best[0]:
                     best = (closest, t, trial)
-                if closest >= margin:
+                if closest >= 1.0:
                     break
             state = best[2]
             toks.append(best[1])
     finally:
-        ROUTER_MARGINS = None
+        ROUTER_MARGINS = READ_MARGINS = None
     return toks

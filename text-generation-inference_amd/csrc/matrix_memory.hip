@@ -14,6 +14,16 @@
 // keeps RPL rows of it in registers.  Tokens go through LDS in stages of `ts`, two buffers deep, the next stage on its way to
 // registers while the current one is worked on; the stage's decays and write weights (one pair per token and head) are made by one
 // wave, which carries m from stage to stage token by token; rows of n belong to the first dk threads.
+//
+// matrix_memory_chunk_kernel: long runs of bf16 models, heads of up to 128 x 128, 64 tokens at a time on the matrix cores.  With
+// F_t = sum_(s <= t) f_s counted from the chunk's start and a_s = i_s - F_s, the maximum is m_t = F_t + M_t with M_t = max(m_0, max_(s <= t) a_s)
+// and the recurrence becomes
+//     S_t^T q_t = e^(m_0 - M_t) S_0^T q_t + sum_(s <= t) e^(a_s - M_t) (q_t . k_s) v_s        n_t . q_t the same with 1 for v_s
+//     S_C = e^(m_0 - M_C) S_0 + sum_s e^(a_s - M_C) k_s v_s^T                                  (every exponent <= 0)
+// q, k and v are bf16 already, so the products q . k are exact in fp32; the weighted scores, the state as an operand and the weighted
+// values are fp32 numbers, each taken as the sum of two bf16 (16 bits of mantissa) with fp32 accumulation; the state itself stays in
+// fp32 accumulators from the first chunk to the last.  Workgroup = (sequence, head) = four waves; wave w owns value columns 32 w ..
+// with all their rows of S; the score tiles are shared through LDS.
 #include <algorithm>
 #include "common.h"
 
@@ -289,6 +299,343 @@ void launch_memory_rows(const MemoryArgs& a, int64_t B, int64_t max_q_len, hipSt
     else launch_memory<T, 64>(a, B, max_q_len, st);
 }
 
+// ---- chunks on the matrix cores -----------------------------------------------------------------------------------------
+constexpr int CT = 64;        // tokens per chunk
+constexpr int TROW = CT + 8;  // LDS row of a channel-major operand: the chunk's tokens + 16 bytes
+
+template <int KT, int VT> struct ChunkLds {
+    static constexpr int DKP = KT * 32, DVP = VT * 32;
+    static constexpr int QROW = DKP + 8;
+    static constexpr int OROW = DVP + 16;
+    bf16 qs[CT * QROW];      // [token][channel]
+    bf16 ks[CT * QROW];
+    bf16 kt[DKP * TROW];     // [channel][token]
+    bf16 vt[DVP * TROW];
+    bf16 ph[CT * TROW];      // weighted scores [t][s], high and low parts
+    bf16 pl[CT * TROW];
+    float o[CT * OROW];      // read-outs [t][value channel]
+    float n[DKP];
+    float a[CT];             // a_s
+    float top[CT];           // M_t
+    float d0[CT];            // e^(m_0 - M_t)
+    float fl[CT];            // e^(-m_t)
+    float w[CT];             // e^(a_s - M_C)
+    float part[2][CT];       // sums of the weighted scores over the chunk's first and second 32 tokens
+    float nq[CT];            // n_0 . q_t
+    float keep;              // e^(m_0 - M_C)
+};
+
+__device__ __forceinline__ void split_bf16(float x, bf16& hi, bf16& lo) {
+    hi = (bf16)x;
+    lo = (bf16)(x - (float)hi);
+}
+
+template <int KT, int VT>
+__global__ __launch_bounds__(256) void matrix_memory_chunk_kernel(MemoryArgs a) {
+    extern __shared__ __attribute__((aligned(16))) unsigned char raw[];
+    using L = ChunkLds<KT, VT>;
+    L& sm = *reinterpret_cast<L*>(raw);
+    constexpr int QROW = L::QROW, OROW = L::OROW;
+    const int b = blockIdx.x, h = blockIdx.y;
+    const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, c = lane & 31, half = lane >> 5;
+    const int t0 = a.cu_q[b], qlen = a.cu_q[b + 1] - t0;
+    if (qlen <= 0) return;
+    const int dk = a.dk, dv = a.dv;
+    const bool fresh = a.positions[t0] == 0;
+    const bf16* proj = reinterpret_cast<const bf16*>(a.proj);
+    const int64_t slot = a.state_slots[b];
+    float* Sg = a.state + (slot * a.H + h) * (int64_t)dk * dv;
+    float* Ng = a.memory + (slot * a.H + h) * (int64_t)(dk + 1);
+    const bool owner = wave < VT;  // has value columns
+    const int col = wave * 32 + c;
+    f32x16 S[KT];  // accumulator i of lane (c, half): row 8 (i / 4) + 4 half + i % 4 of the 32-row tile, column c
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt)
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            const int r = kt * 32 + (i >> 2) * 8 + half * 4 + (i & 3);
+            S[kt][i] = (owner && !fresh && r < dk && col < dv) ? Sg[(int64_t)r * dv + col] : 0.f;
+        }
+    if (tid < L::DKP) sm.n[tid] = (!fresh && tid < dk) ? Ng[tid] : 0.f;
+    float m_run = fresh ? 0.f : Ng[dk];  // wave 0
+    // a thread's share of a chunk: token tid % 64, pieces of 8 channels; and the output gates of token tid / 4
+    bf16x8 qr[KT], kr[KT], vr[VT];
+    bf16x4 gr[VT * 2];
+    float zi = 0.f, zf = 0.f;
+    const int st = tid & 63, piece = tid >> 6;
+    const int ot = tid >> 2, oq = tid & 3;
+    auto fetch = [&](int base, int n) {
+        const bf16* row = proj + (int64_t)(t0 + base + st) * a.ld;
+        const bool in = st < n;
+#pragma unroll
+        for (int u = 0; u < KT; ++u) {
+            const int ch = (piece + u * 4) * 8;
+            qr[u] = in && ch < dk ? *reinterpret_cast<const bf16x8*>(row + a.q_col0 + h * dk + ch) : bf16x8{};
+            kr[u] = in && ch < dk ? *reinterpret_cast<const bf16x8*>(row + a.k_col0 + h * dk + ch) : bf16x8{};
+        }
+#pragma unroll
+        for (int u = 0; u < VT; ++u) {
+            const int ch = (piece + u * 4) * 8;
+            vr[u] = in && ch < dv ? *reinterpret_cast<const bf16x8*>(row + a.v_col0 + h * dv + ch) : bf16x8{};
+        }
+        if (wave == 0 && in) {
+            const float* z = a.gates + (int64_t)(t0 + base + st) * a.ld_gates;
+            zi = z[h];
+            zf = z[a.H + h];
+        }
+    };
+    fetch(0, min(CT, qlen));
+    for (int base = 0; base < qlen; base += CT) {
+        const int n = min(CT, qlen - base);
+        // ---- the chunk into LDS; its gates
+        if (wave == 0) {
+            float li = -INFINITY, F = 0.f;  // tokens past the end keep everything and write nothing
+            if (lane < n) {
+                li = soft_capped(zi + (a.i_bias ? a.i_bias[h] : 0.f), a.cap);
+                F = log_sigmoid(soft_capped(zf + (a.f_bias ? a.f_bias[h] : 0.f), a.cap));
+            }
+#pragma unroll
+            for (int o = 1; o < 64; o <<= 1) {
+                const float up = __shfl_up(F, o, 64);
+                if (lane >= o) F += up;
+            }
+            const float as = li - F;
+            float top = as;
+#pragma unroll
+            for (int o = 1; o < 64; o <<= 1) {
+                const float up = __shfl_up(top, o, 64);
+                if (lane >= o) top = fmaxf(top, up);
+            }
+            top = fmaxf(top, m_run);
+            const float end = lane_value(top, 63);
+            sm.a[lane] = as;
+            sm.top[lane] = top;
+            sm.d0[lane] = expf(m_run - top);
+            sm.fl[lane] = expf(-(F + top));
+            sm.w[lane] = expf(as - end);
+            if (lane == 0) sm.keep = expf(m_run - end);
+            m_run = lane_value(F, 63) + end;
+        }
+#pragma unroll
+        for (int u = 0; u < KT; ++u) {
+            const int ch = (piece + u * 4) * 8;
+            *reinterpret_cast<bf16x8*>(sm.qs + st * QROW + ch) = qr[u];
+            *reinterpret_cast<bf16x8*>(sm.ks + st * QROW + ch) = kr[u];
+#pragma unroll
+            for (int j = 0; j < 8; ++j) sm.kt[(ch + j) * TROW + st] = kr[u][j];
+        }
+#pragma unroll
+        for (int u = 0; u < VT; ++u) {
+            const int ch = (piece + u * 4) * 8;
+#pragma unroll
+            for (int j = 0; j < 8; ++j) sm.vt[(ch + j) * TROW + st] = vr[u][j];
+        }
+        __syncthreads();
+        if (base + CT < qlen) fetch(base + CT, min(CT, qlen - base - CT));
+        if (a.g_col0 >= 0 && ot < n) {
+            const bf16* g = proj + (int64_t)(t0 + base + ot) * a.ld + a.g_col0 + h * dv;
+#pragma unroll
+            for (int j = 0; j < VT * 2; ++j) gr[j] = j * 16 + oq * 4 < dv ? *reinterpret_cast<const bf16x4*>(g + j * 16 + oq * 4) : bf16x4{};
+        }
+        // ---- weighted scores: waves 0, 1, 2 take the (s, t) tiles (0, 0), (0, 1), (1, 1), transposed (a lane has one t)
+        if (wave < 3) {
+            const int ts = wave >> 1, tt = (wave + 1) >> 1;
+            f32x16 P = {};
+#pragma unroll
+            for (int s = 0; s < KT * 2; ++s) {
+                const bf16x8 x = *reinterpret_cast<const bf16x8*>(sm.ks + (ts * 32 + c) * QROW + s * 16 + half * 8);
+                const bf16x8 y = *reinterpret_cast<const bf16x8*>(sm.qs + (tt * 32 + c) * QROW + s * 16 + half * 8);
+                P = mfma32(x, y, P);
+            }
+            const int t = tt * 32 + c;
+            const float top = sm.top[t];
+            float sum = 0.f;
+#pragma unroll
+            for (int g = 0; g < 4; ++g) {
+                const int s0 = ts * 32 + g * 8 + half * 4;
+                const f32x4 as = *reinterpret_cast<const f32x4*>(sm.a + s0);
+                bf16x4 hi, lo;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const float p = s0 + i <= t ? P[g * 4 + i] * __expf(as[i] - top) : 0.f;
+                    sum += p;
+                    bf16 x, y;
+                    split_bf16(p, x, y);
+                    hi[i] = x;
+                    lo[i] = y;
+                }
+                *reinterpret_cast<bf16x4*>(sm.ph + t * TROW + s0) = hi;
+                *reinterpret_cast<bf16x4*>(sm.pl + t * TROW + s0) = lo;
+            }
+            sum += __shfl_xor(sum, 32, 64);
+            if (half == 0) {
+                sm.part[ts][t] = sum;
+                if (wave == 0) sm.part[1][t] = 0.f;  // no later keys for the first 32 tokens
+            }
+        }
+        // ---- what the state of the chunk's start gives: S_0^T q and n_0 . q
+        f32x16 O[2] = {};
+        if (owner) {
+#pragma unroll
+            for (int kt = 0; kt < KT; ++kt)
+#pragma unroll
+                for (int x = 0; x < 2; ++x) {
+                    bf16x8 hi, lo;  // rows 16 x + 8 (j / 4) + 4 half + j % 4 of the tile: the A operand follows that order
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) {
+                        bf16 u, v;
+                        split_bf16(S[kt][x * 8 + j], u, v);
+                        hi[j] = u;
+                        lo[j] = v;
+                    }
+#pragma unroll
+                    for (int tt = 0; tt < 2; ++tt) {
+                        const bf16* q = sm.qs + (tt * 32 + c) * QROW + kt * 32 + x * 16 + half * 4;
+                        const bf16x4 q0 = *reinterpret_cast<const bf16x4*>(q), q1 = *reinterpret_cast<const bf16x4*>(q + 8);
+                        const bf16x8 qa = __builtin_shufflevector(q0, q1, 0, 1, 2, 3, 4, 5, 6, 7);
+                        O[tt] = mfma32(qa, hi, O[tt]);
+                        O[tt] = mfma32(qa, lo, O[tt]);
+                    }
+                }
+#pragma unroll
+            for (int tt = 0; tt < 2; ++tt)
+#pragma unroll
+                for (int g = 0; g < 4; ++g) {
+                    const f32x4 d = *reinterpret_cast<const f32x4*>(sm.d0 + tt * 32 + g * 8 + half * 4);
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) O[tt][g * 4 + i] *= d[i];
+                }
+        }
+        {
+            float d = 0.f;
+#pragma unroll
+            for (int u = 0; u < KT; ++u) {
+                const bf16x8 q = *reinterpret_cast<const bf16x8*>(sm.qs + ot * QROW + (u * 4 + oq) * 8);
+                const f32x4 n0 = *reinterpret_cast<const f32x4*>(sm.n + (u * 4 + oq) * 8), n1 = *reinterpret_cast<const f32x4*>(sm.n + (u * 4 + oq) * 8 + 4);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) d += (float)q[i] * n0[i] + (float)q[4 + i] * n1[i];
+            }
+            d += __shfl_xor(d, 1, 64);
+            d += __shfl_xor(d, 2, 64);
+            if (oq == 0) sm.nq[ot] = d;
+        }
+        __syncthreads();
+        // ---- the chunk's own keys and values; the state of its end
+        const float keep = sm.keep;
+        if (owner) {
+            const bf16* vrow = sm.vt + col * TROW + half * 8;
+#pragma unroll
+            for (int kk = 0; kk < 4; ++kk) {
+                const bf16x8 v = *reinterpret_cast<const bf16x8*>(vrow + kk * 16);
+                // read-outs: tokens of the first half see keys of the first half only
+#pragma unroll
+                for (int tt = 0; tt < 2; ++tt) {
+                    if (tt == 0 && kk >= 2) continue;
+                    const int at = (tt * 32 + c) * TROW + kk * 16 + half * 8;
+                    O[tt] = mfma32(*reinterpret_cast<const bf16x8*>(sm.ph + at), v, O[tt]);
+                    O[tt] = mfma32(*reinterpret_cast<const bf16x8*>(sm.pl + at), v, O[tt]);
+                }
+                // values times their write weights
+                const f32x4 w0 = *reinterpret_cast<const f32x4*>(sm.w + kk * 16 + half * 8), w1 = *reinterpret_cast<const f32x4*>(sm.w + kk * 16 + half * 8 + 4);
+                bf16x8 hi, lo;
+#pragma unroll
+                for (int j = 0; j < 8; ++j) {
+                    bf16 x, y;
+                    split_bf16((float)v[j] * (j < 4 ? w0[j & 3] : w1[j & 3]), x, y);
+                    hi[j] = x;
+                    lo[j] = y;
+                }
+#pragma unroll
+                for (int kt = 0; kt < KT; ++kt) {
+                    if (kk == 0) S[kt] *= keep;
+                    const bf16x8 k = *reinterpret_cast<const bf16x8*>(sm.kt + (kt * 32 + c) * TROW + kk * 16 + half * 8);
+                    S[kt] = mfma32(k, hi, S[kt]);
+                    S[kt] = mfma32(k, lo, S[kt]);
+                }
+            }
+#pragma unroll
+            for (int tt = 0; tt < 2; ++tt)
+#pragma unroll
+                for (int i = 0; i < 16; ++i) sm.o[(tt * 32 + (i >> 2) * 8 + half * 4 + (i & 3)) * OROW + col] = O[tt][i];
+        }
+        if (tid >= 256 - L::DKP) {  // the last waves have least else to do
+            const int i = tid - (256 - L::DKP);
+            float s = sm.n[i] * keep;
+#pragma unroll
+            for (int p = 0; p < CT / 8; ++p) {
+                const bf16x8 k = *reinterpret_cast<const bf16x8*>(sm.kt + i * TROW + p * 8);
+                const f32x4 w0 = *reinterpret_cast<const f32x4*>(sm.w + p * 8), w1 = *reinterpret_cast<const f32x4*>(sm.w + p * 8 + 4);
+#pragma unroll
+                for (int j = 0; j < 4; ++j) s += (float)k[j] * w0[j] + (float)k[4 + j] * w1[j];
+            }
+            sm.n[i] = s;
+        }
+        __syncthreads();
+        // ---- normaliser, norm and gate: four neighbouring lanes per token
+        {
+            const float nq = (sm.nq[ot] * sm.d0[ot] + sm.part[0][ot] + sm.part[1][ot]) * a.q_scale;
+            const float den = fmaxf(fabsf(nq), sm.fl[ot]) + a.read_eps;
+            f32x4 v[VT * 2];
+            float ss = 0.f;
+#pragma unroll
+            for (int j = 0; j < VT * 2; ++j) {
+                v[j] = *reinterpret_cast<const f32x4*>(sm.o + ot * OROW + j * 16 + oq * 4) * a.q_scale;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) ss += v[j][i] * v[j][i];  // columns past dv are zero
+            }
+            ss += __shfl_xor(ss, 1, 64);
+            ss += __shfl_xor(ss, 2, 64);
+            const float rinv = 1.f / (den * sqrtf(ss / ((float)dv * den * den) + a.eps));
+            if (ot < n) {
+                bf16* orow = reinterpret_cast<bf16*>(a.out) + (int64_t)(t0 + base + ot) * a.ld_out + (int64_t)h * dv;
+#pragma unroll
+                for (int j = 0; j < VT * 2; ++j) {
+                    const int at = j * 16 + oq * 4;
+                    if (at >= dv) continue;
+                    const f32x4 gain = *reinterpret_cast<const f32x4*>(a.gain + h * dv + at);
+                    bf16x4 y;
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) {
+                        const float g = a.g_col0 >= 0 ? __builtin_amdgcn_rcpf(1.f + __expf(-(float)gr[j][i])) : 1.f;
+                        y[i] = (bf16)(v[j][i] * rinv * gain[i] * g);
+                    }
+                    *reinterpret_cast<bf16x4*>(orow + at) = y;
+                }
+            }
+        }
+        // the next chunk's buffers: everything the last part reads (o, nq, part, fl, d0) is written behind the next barriers, except
+        // d0 and fl, which wave 0 writes in front of the first of them
+        __syncthreads();
+    }
+    if (owner) {
+#pragma unroll
+        for (int kt = 0; kt < KT; ++kt)
+#pragma unroll
+            for (int i = 0; i < 16; ++i) {
+                const int r = kt * 32 + (i >> 2) * 8 + half * 4 + (i & 3);
+                if (r < dk && col < dv) Sg[(int64_t)r * dv + col] = S[kt][i];
+            }
+    }
+    if (tid < dk) Ng[tid] = sm.n[tid];
+    if (tid == 0) Ng[dk] = m_run;
+}
+
+template <int KT, int VT> void launch_chunks(const MemoryArgs& a, int64_t B, hipStream_t st) {
+    constexpr size_t lds = sizeof(ChunkLds<KT, VT>);
+    static_assert(lds <= 160 * 1024, "a chunk's operands fit the LDS of a compute unit");
+    (void)hipFuncSetAttribute((const void*)matrix_memory_chunk_kernel<KT, VT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    hipLaunchKernelGGL((matrix_memory_chunk_kernel<KT, VT>), dim3((unsigned)B, (unsigned)a.H), dim3(256), lds, st, a);
+}
+
+// runs from this length on are worth a chunk of 64 (a single token costs a whole one)
+constexpr int64_t CHUNKS_FROM = 12;
+
+bool chunks_ok(const MemoryArgs& a, int dtype) {
+    auto al = [](const void* p, size_t n) { return ((uintptr_t)p % n) == 0; };
+    return dtype == TGIS_BF16 && a.dk <= 128 && a.dv <= 128 && a.dk % 8 == 0 && a.dv % 8 == 0 && a.ld % 8 == 0 && a.q_col0 % 8 == 0 && a.k_col0 % 8 == 0 &&
+           a.v_col0 % 8 == 0 && (a.g_col0 < 0 || a.g_col0 % 4 == 0) && a.ld_out % 4 == 0 && al(a.proj, 16) && al(a.out, 8) && al(a.gain, 16);
+}
+
 }  // namespace
 
 extern "C" int tgis_matrix_memory(const void* proj, int64_t ld, int64_t q_col0, int64_t k_col0, int64_t v_col0, int64_t g_col0,
@@ -309,6 +656,16 @@ extern "C" int tgis_matrix_memory(const void* proj, int64_t ld, int64_t q_col0, 
     TgisTimedScope timed(TGIS_OP_SCAN, st);
     const MemoryArgs a{proj, ld, q_col0, k_col0, v_col0, g_col0, gates, ld_gates, i_bias, f_bias, cap, gain, state, memory, state_slots,
                        cu_seqlens_q, positions, out, ld_out, H, dk, dv, q_scale, eps, read_eps, 0, 0};
+    const bool can = chunks_ok(a, dtype);
+    TGIS_CHECK_ARG(impl != 2 || can, "tgis_matrix_memory: chunks take bf16, dk and dv multiples of 8 up to 128, aligned operands");
+    if (impl == 2 || (impl == 0 && can && max_q_len >= CHUNKS_FROM)) {
+        if (dk <= 64 && dv <= 64) launch_chunks<2, 2>(a, B, st);
+        else if (dk <= 64) launch_chunks<2, 4>(a, B, st);
+        else if (dv <= 64) launch_chunks<4, 2>(a, B, st);
+        else launch_chunks<4, 4>(a, B, st);
+        TGIS_CHECK_LAUNCH();
+        return TGIS_OK;
+    }
     if (dtype == TGIS_F16) launch_memory_rows<f16>(a, B, max_q_len, st);
     else if (dtype == TGIS_BF16) launch_memory_rows<bf16>(a, B, max_q_len, st);
     else launch_memory_rows<float>(a, B, max_q_len, st);
