@@ -510,6 +510,27 @@ def gopetar_layers(variant, width, layers, heads, kv_heads, dim, ff):
     return out
 
 
+def fidatar_layers(variant, width, layers, heads, kv_heads, dim, ff):
+    """"fidatar_attn": every layer block-masked attention (a block longer than any context here, so that the cache bytes equal Llama's)
+    + the dense squared-relu unit — like for like with Senadra "senadra_attn".  "fidatar_mlstm": every layer a matrix memory of
+    width / 256 heads of 64 x 128 (the state of Mananex's recurrence) + a mixture of 8 plain units of ff / 4, top 2, among the best
+    2 of 4 groups — its scan and its products beside those of "mananex_moe".  "fidatar": attention in blocks of 512 and matrix
+    memories of width / 256 heads of 128 x 128 in turn, every second feed-forward the mixture — the design as it is meant."""
+    out = []
+    for i in range(layers):
+        mlp = {"kind": "dense", "ff": ff}
+        if variant == "fidatar_mlstm" or (variant == "fidatar" and i % 2 == 1):
+            mlp = {"kind": "moe", "expert": {"ff": ff // 4}, "router": {"experts": 8, "top": 2, "scale": 1.0, "groups": {"count": 4, "keep": 2}}}
+        if variant == "fidatar_mlstm" or (variant == "fidatar" and i % 2 == 1):
+            m = {"heads": max(1, width // 256), "dim": 64 if variant == "fidatar_mlstm" else 128, "vdim": 128, "gate_cap": 15.0}
+            out.append({"type": "mlstm", "mixer": m, "mlp": mlp})
+        else:
+            m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": 8192 if variant == "fidatar_attn" else 512},
+                 "rot": {"base": 500000.0, "dims": dim // 2, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+            out.append({"type": "attention", "mixer": m, "mlp": mlp})
+    return out
+
+
 def bench_hybrid(args):
     """Prefill and decode throughput + per-kernel-class device time (HIP events, eager pass) of Lenisun variants and of
     Llama at the same size, through the same entry points (from_pb -> generate_token).  One JSON line."""
@@ -566,6 +587,15 @@ def bench_hybrid(args):
                                 layers=gopetar_layers(name, width, layers, heads, kv_heads, dim, ff))
             tensors = gopetar_tensors(cfg, seed=1234, device=device, dtype=dtype)
             n_attn, n_scan = layers, sum(l["type"] == "parallel" for l in cfg.layers)
+        elif name.startswith("fidatar"):
+            from tgis_amd.inference_engine.synthetic import fidatar_tensors
+            from tgis_amd.models.custom_modeling.flash_fidatar_modeling import FidatarConfig
+
+            cfg = FidatarConfig(width=width, vocab=vocab, norm={"eps": 1e-5}, embedding={"scale": 1.0}, postln_alpha=2.0, logit_softcap=30.0,
+                                layers=fidatar_layers(name, width, layers, heads, kv_heads, dim, ff))
+            tensors = fidatar_tensors(cfg, seed=1234, device=device, dtype=dtype)
+            n_attn = sum(l["type"] == "attention" for l in cfg.layers)
+            n_scan = layers - n_attn
         elif name.startswith("senadra"):
             cfg = SenadraConfig(width=width, vocab=vocab, norm={"eps": 1e-5}, residual_mult=0.25, token_side={"dim": 64},
                                 logit_softcap=25.0, layers=senadra_layers(name, width, layers, heads, kv_heads, dim, ff))
@@ -637,6 +667,8 @@ def bench_hybrid(args):
                 # bytes one attention launch has to read: every cached key and value of the batch once
                 keys = min(ctx_now, 512 + 4 + 32) if name in ("mananex", "mananex_moe", "tatevik", "gopetar_pair") else ctx_now  # a window, its kept positions, a page's slack
                 by = B * keys * kv_heads * 2 * dim * 2
+                if name == "fidatar":  # what a token's own block of 512 holds
+                    by = B * (ctx_now % 512 + 1) * kv_heads * 2 * dim * 2
                 latent = B * ctx_now * (2 * 192 + (dim // 2 if name.startswith("senadra") else 0)) * 2
                 if name.endswith("_latent"):  # a token's latent, as a key row and as value columns (and Senadra's rotated part)
                     by = latent
@@ -679,7 +711,7 @@ def main():
                     help="instead of the default workload: Lenisun / Senadra variants beside Llama at this size (prefill + decode)")
     ap.add_argument("--hybrid-models", default="llama,attn,mixed",
                     help="comma list of llama, attn, mixed (Lenisun), senadra_attn, senadra_latent, senadra, mananex_dense, mananex_moe, mananex, "
-                         "tatevik_pair, tatevik, gopetar_pair, gopetar_latent, gopetar")
+                         "tatevik_pair, tatevik, gopetar_pair, gopetar_latent, gopetar, fidatar_attn, fidatar_mlstm, fidatar")
     ap.add_argument("--prefill-batch", type=int, default=4)
     ap.add_argument("--prefill-len", type=int, default=1024)
     ap.add_argument("--prefill-reps", type=int, default=3)

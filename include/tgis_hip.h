@@ -669,12 +669,12 @@ int tgis_hyper_update(const float* x, const int64_t* ids, const void* table, int
  * x [rows, W] fp32, or ids instead (x = table[ids[t]] * emb_scale, vocab rows of `dtype`); y by kind as in tgis_hyper_update
  * (0 none: no sum; 1 tensor, 2 split-K slabs, 3 rows of a mixture with pair_weight or ones); w NULL: no norm.  x_out (may alias x,
  * may be NULL) receives the new stream; h [rows, W] of `dtype` its rounding, or with w2 N(x) * w2.
- * dot_w [R][W] fp32 (or NULL): fp32 products of the rounded row h with R rows — to dot_out [rows][R], or (idx not NULL) as router
+ * dot_w [R][W] of `dtype` (or NULL): fp32 products of the rounded row h with R rows — to dot_out [rows][R], or (idx not NULL) as router
  * logits: idx / route_weight [rows][top] receive what tgis_moe_choose makes of them. */
 int tgis_post_norm_update(const float* x, const int64_t* ids, const void* table, int64_t vocab, float emb_scale, float alpha,
                           float* x_out, int kind, const void* y, int64_t ld_y, int slabs, const int32_t* pos,
                           const float* pair_weight, int pairs, const float* w, const float* w2, void* h, int64_t rows, int64_t W,
-                          float eps, const float* dot_w, int R, float* dot_out, int32_t* idx, float* route_weight, int top,
+                          float eps, const void* dot_w, int R, float* dot_out, int32_t* idx, float* route_weight, int top,
                           int groups, int keep, float route_scale, int dtype, void* stream);
 /* out[t][n] = sum_c h[t][c] w[n][c], fp32 [rows][R], for few outputs and many rows: h [rows, ld_h] and w [R][W] of a two-byte
  * `dtype`, W and ld_h multiples of 8, 16-byte aligned. */

@@ -276,7 +276,7 @@ def test_norm_after_the_sum(gpu_device, dtype, W, T):
     g = torch.Generator().manual_seed(W + T)
     dev, alpha, eps = gpu_device, 1.9, 1e-5
     rnd = lambda *sh: torch.randn(*sh, generator=g)
-    X, w, w2, dots = rnd(T, W), 1 + 0.3 * rnd(W), 1 + 0.3 * rnd(W), rnd(11, W)
+    X, w, w2, dots = rnd(T, W), 1 + 0.3 * rnd(W), 1 + 0.3 * rnd(W), rnd(21, W).to(dtype)
     tol = 2e-5 if dtype == torch.float32 else 0.012
 
     def check(y_dev, y):
@@ -311,7 +311,7 @@ def test_the_stream_begins_with_the_scaled_embedding(gpu_device, dtype):
     from tgis_amd import native
 
     g = torch.Generator().manual_seed(0)
-    table, ids, dots = torch.randn(50, 24, generator=g).to(dtype), torch.tensor([3, 49, 0, 7]), torch.randn(6, 24, generator=g)
+    table, ids, dots = torch.randn(50, 24, generator=g).to(dtype), torch.tensor([3, 49, 0, 7]), torch.randn(6, 24, generator=g).to(dtype)
     x, h, z = native.post_norm_update(None, None, 2.0, None, 1e-5, dtype, ids=ids.to(gpu_device), table=table.to(gpu_device), emb_scale=3.0,
                                       dots=dots.to(gpu_device))
     want = table.double()[ids] * 3.0

@@ -14,6 +14,7 @@
 #include <algorithm>
 #include <type_traits>
 #include "common.h"
+#include "wave_dpp.h"
 
 namespace {
 
@@ -1130,6 +1131,70 @@ __global__ __launch_bounds__(256) void norm_rope_rows_kv_write_kernel(T* __restr
     }
 }
 
+// The same for two-byte dtypes whose head is a power of two of 8-channel pieces (LPH of them) and whose rotated half is whole pieces: a
+// lane owns one piece, 64 / LPH heads share a wave, and a piece's rotation partner is read again (it is in L1) instead of exchanged.
+template <typename T, int LPH>
+__global__ __launch_bounds__(256) void norm_rope_rows_kv_write_vec_kernel(T* __restrict__ qkv, int64_t ld, int64_t q_col0, int64_t k_col0,
+                                                                          int64_t v_col0, const float* __restrict__ q_gain,
+                                                                          const float* __restrict__ k_gain, float eps, const float* __restrict__ turns,
+                                                                          float amp, const int32_t* __restrict__ slots, T* __restrict__ k_pool,
+                                                                          T* __restrict__ v_pool, int H, int G, int dk, int dv, int rdims, int v_inline) {
+    using V8 = typename VecT<T>::x8;
+    constexpr int PER_WG = 256 / LPH;  // heads
+    const int64_t t = blockIdx.x;
+    const int slot = slots[t];
+    const int64_t page = slot / PAGE;
+    const int off = slot % PAGE;
+    T* row = qkv + t * ld;
+    const int head_blocks = (H + G + PER_WG - 1) / PER_WG;
+    if ((int)blockIdx.y >= head_blocks) {
+        const T* vrow = row + v_col0;
+        const int i0 = ((int)blockIdx.y - head_blocks) * 1024;
+        const int i1 = min(i0 + 1024, G * dv);
+        for (int i = i0 + threadIdx.x; i < i1; i += blockDim.x) {
+            const int g = i / dv, c = i - g * dv;
+            v_pool[((page * G + g) * dv + c) * PAGE + off] = vrow[i];
+        }
+        return;
+    }
+    const int h = blockIdx.y * PER_WG + threadIdx.x / LPH, c = threadIdx.x % LPH * 8;
+    const bool in = h < H + G;
+    const bool is_q = h < H;
+    T* src = is_q ? row + q_col0 + (int64_t)h * dk : row + k_col0 + (int64_t)(h - H) * dk;
+    const float* gain = is_q ? q_gain : k_gain;
+    const int half = rdims >> 1;
+    const bool turned = c < rdims, second = c >= half;
+    const int pc = second ? c - half : c + half;  // the partner's piece
+    V8 x = {}, p = {};
+    float ss = 0.f;
+    if (in) {
+        x = *reinterpret_cast<const V8*>(src + c);
+        if (turned) p = *reinterpret_cast<const V8*>(src + pc);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) ss += (float)x[i] * (float)x[i];
+    }
+    ss = sum_neighbours<LPH < 16 ? LPH : 16>(ss);
+    if (LPH == 32) ss += __shfl_xor(ss, 16, 64);
+    const float rinv = 1.f / sqrtf(ss / (float)dk + eps);
+    if (!in) return;
+    V8 y;
+    if (turned) {
+        const f32x4* cs = reinterpret_cast<const f32x4*>(turns + t * rdims + 2 * (second ? c - half : c));  // (cos, sin) pairs
+        const float sign = second ? 1.f : -1.f;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            const f32x4 a = cs[i >> 1];
+            y[i] = (T)(rinv * amp * ((float)x[i] * gain[c + i] * a[(i & 1) * 2] + sign * (float)p[i] * gain[pc + i] * a[(i & 1) * 2 + 1]));
+        }
+    } else {
+#pragma unroll
+        for (int i = 0; i < 8; ++i) y[i] = (T)((float)x[i] * rinv * gain[c + i]);
+    }
+    // a head's pieces are lanes of one wave: all of them have read before one of them writes
+    T* dst = is_q ? src : k_pool + ((page * G + (h - H)) * PAGE + off) * dk;
+    *reinterpret_cast<V8*>(dst + c) = y;
+}
+
 __global__ void pair_turns_kernel(const int32_t* __restrict__ positions, const float* __restrict__ inv_freq, float* __restrict__ turns,
                                   int64_t total, int n) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
@@ -1628,6 +1693,30 @@ extern "C" int tgis_norm_rope_rows_kv_write(void* proj, int64_t ld, int64_t q_co
     TgisTimedScope timed(TGIS_OP_ROPE_KV, st);
     const int v_inline = T < 512 ? 1 : 0;
     const int v_blocks = v_inline ? (int)cdiv64((int64_t)G * dv, 1024) : 0;
+    const int lph = dk / 8;
+    const bool vec = dtype != TGIS_F32 && dk % 8 == 0 && (lph & (lph - 1)) == 0 && rot_dims % 16 == 0 && ld % 8 == 0 && q_col0 % 8 == 0 && k_col0 % 8 == 0 &&
+                     (((uintptr_t)proj | (uintptr_t)k_pool | (uintptr_t)turns) & 15) == 0;
+    if (vec) {
+#define TGIS_NORM_ROPE_VEC(TT, LPH)                                                                                                          \
+    hipLaunchKernelGGL((norm_rope_rows_kv_write_vec_kernel<TT, LPH>), dim3((unsigned)T, (unsigned)((H + G + 256 / LPH - 1) / (256 / LPH) + v_blocks)), \
+                       dim3(256), 0, st, (TT*)proj, ld, q_col0, k_col0, v_col0, q_gain, k_gain, eps, turns, amp, slots, (TT*)k_pool, (TT*)v_pool, H,  \
+                       G, dk, dv, rot_dims, v_inline)
+#define TGIS_NORM_ROPE_LPH(LPH)                            \
+    case LPH:                                              \
+        if (dtype == TGIS_F16) TGIS_NORM_ROPE_VEC(f16, LPH); \
+        else TGIS_NORM_ROPE_VEC(bf16, LPH);                \
+        break
+        switch (lph) {
+            TGIS_NORM_ROPE_LPH(1);
+            TGIS_NORM_ROPE_LPH(2);
+            TGIS_NORM_ROPE_LPH(4);
+            TGIS_NORM_ROPE_LPH(8);
+            TGIS_NORM_ROPE_LPH(16);
+            TGIS_NORM_ROPE_LPH(32);
+        }
+#undef TGIS_NORM_ROPE_LPH
+#undef TGIS_NORM_ROPE_VEC
+    } else
     TGIS_ATTN_BY_DTYPE(dtype, hipLaunchKernelGGL(norm_rope_rows_kv_write_kernel<TT>, dim3((unsigned)T, (unsigned)((H + G + 3) / 4 + v_blocks)),
                                                  dim3(256), 0, st, (TT*)proj, ld, q_col0, k_col0, v_col0, q_gain, k_gain, eps, turns, amp, slots,
                                                  (TT*)k_pool, (TT*)v_pool, H, G, dk, dv, rot_dims, v_inline));

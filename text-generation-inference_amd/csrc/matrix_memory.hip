@@ -22,10 +22,12 @@
 //     S_C = e^(m_0 - M_C) S_0 + sum_s e^(a_s - M_C) k_s v_s^T                                  (every exponent <= 0)
 // q, k and v are bf16 already, so the products q . k are exact in fp32; the weighted scores, the state as an operand and the weighted
 // values are fp32 numbers, each taken as the sum of two bf16 (16 bits of mantissa) with fp32 accumulation; the state itself stays in
-// fp32 accumulators from the first chunk to the last.  Workgroup = (sequence, head) = four waves; wave w owns value columns 32 w ..
-// with all their rows of S; the score tiles are shared through LDS.
+// fp32 accumulators from the first chunk to the last.  Workgroup = (sequence, head) = eight waves; wave w owns value columns
+// 32 (w % 4) .. with half of their rows of S, and leaves its share of the read-outs in LDS, where the two halves meet; the score tiles
+// are shared through LDS too.
 #include <algorithm>
 #include "common.h"
+#include "wave_dpp.h"
 
 namespace {
 
@@ -58,9 +60,6 @@ struct MemoryArgs {
 __device__ __forceinline__ float soft_capped(float z, float cap) { return cap * tanhf(z / cap); }
 // ln(sigmoid(z)) without cancellation at either end
 __device__ __forceinline__ float log_sigmoid(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
-__device__ __forceinline__ float lane_value(float v, int lane) {
-    return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), lane));
-}
 // (i, f) of head h at token t
 __device__ __forceinline__ void log_gates(const MemoryArgs& a, int64_t t, int h, float& li, float& lf) {
     const float* z = a.gates + t * a.ld_gates;
@@ -209,11 +208,7 @@ __global__ __launch_bounds__(MAXT) void matrix_memory_scan_kernel(MemoryArgs a) 
             }
 #pragma unroll
             for (int c = 0; c < CPL; ++c) {
-                float t = acc[c];
-                t += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, t), 0xB1, 0xF, 0xF, true));  // lane ^ 1
-                t += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, t), 0x4E, 0xF, 0xF, true));  // lane ^ 2
-                if (LPC == 8)  // the other quad of the eight: lane 7 - i of the half row holds its total
-                    t += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, t), 0x141, 0xF, 0xF, true));
+                const float t = sum_neighbours<LPC>(acc[c]);
                 if (qd == 0) os[tt * dv_pad + j + c * jstep] = t;
             }
         }
@@ -234,11 +229,10 @@ __global__ __launch_bounds__(MAXT) void matrix_memory_scan_kernel(MemoryArgs a) 
             float d = 0.f, ss = 0.f;
             for (int i = lane; i < dk; i += 64) d += nq[tt * dk + i];
             for (int c = lane; c < dv; c += 64) ss += os[tt * dv_pad + c] * os[tt * dv_pad + c];
-            d = wave_sum(d);
-            ss = wave_sum(ss);
+            d = wave_total(d);
+            ss = wave_total(ss);
             const float den = fmaxf(fabsf(d), fl[buf * ts + tt]) + a.read_eps;
-            // o / den normed: mean((o / den)^2) + eps under the root
-            const float rinv = 1.f / (den * sqrtf(ss / ((float)dv * den * den) + a.eps));
+            const float rinv = 1.f / sqrtf(ss / (float)dv + a.eps * den * den);  // o / den, normed
             const int64_t t = t0 + base + tt;
             T* orow = out + t * a.ld_out + (int64_t)h * dv;
             for (int c = lane; c < dv; c += 64)
@@ -306,24 +300,32 @@ constexpr int TROW = CT + 8;  // LDS row of a channel-major operand: the chunk's
 template <int KT, int VT> struct ChunkLds {
     static constexpr int DKP = KT * 32, DVP = VT * 32;
     static constexpr int QROW = DKP + 8;
-    static constexpr int OROW = DVP + 16;
+    static constexpr int OROW = DVP + 4;
     bf16 qs[CT * QROW];      // [token][channel]
     bf16 ks[CT * QROW];
-    bf16 kt[DKP * TROW];     // [channel][token]
+    bf16 kt[DKP * TROW];     // [channel][token], groups of 8 tokens swizzled (token_group)
     bf16 vt[DVP * TROW];
     bf16 ph[CT * TROW];      // weighted scores [t][s], high and low parts
     bf16 pl[CT * TROW];
-    float o[CT * OROW];      // read-outs [t][value channel]
+    float o[2][CT * OROW];   // read-outs [t][value channel], a part from either half of the waves
+    float gain[DVP];
     float n[DKP];
-    float a[CT];             // a_s
-    float top[CT];           // M_t
-    float d0[CT];            // e^(m_0 - M_t)
-    float fl[CT];            // e^(-m_t)
-    float w[CT];             // e^(a_s - M_C)
+    struct Gates {
+        float a[CT];         // a_s
+        float top[CT];       // M_t
+        float d0[CT];        // e^(m_0 - M_t)
+        float fl[CT];        // e^(-m_t)
+        float w[CT];         // e^(a_s - M_C)
+        float keep;          // e^(m_0 - M_C)
+        float pad[3];
+    } gates[2];
     float part[2][CT];       // sums of the weighted scores over the chunk's first and second 32 tokens
     float nq[CT];            // n_0 . q_t
-    float keep;              // e^(m_0 - M_C)
 };
+
+// where group g of 8 tokens of a channel lies in its row: the transposing stores of 8 neighbouring channel pieces then hit
+// different banks, and so do the 16-byte reads of 8 neighbouring channels
+__device__ __forceinline__ int token_group(int channel, int g) { return (g ^ (channel >> 3 & 7)) * 8; }
 
 __device__ __forceinline__ void split_bf16(float x, bf16& hi, bf16& lo) {
     hi = (bf16)x;
@@ -331,7 +333,7 @@ __device__ __forceinline__ void split_bf16(float x, bf16& hi, bf16& lo) {
 }
 
 template <int KT, int VT>
-__global__ __launch_bounds__(256) void matrix_memory_chunk_kernel(MemoryArgs a) {
+__global__ __launch_bounds__(512) void matrix_memory_chunk_kernel(MemoryArgs a) {
     extern __shared__ __attribute__((aligned(16))) unsigned char raw[];
     using L = ChunkLds<KT, VT>;
     L& sm = *reinterpret_cast<L*>(raw);
@@ -346,100 +348,108 @@ __global__ __launch_bounds__(256) void matrix_memory_chunk_kernel(MemoryArgs a) 
     const int64_t slot = a.state_slots[b];
     float* Sg = a.state + (slot * a.H + h) * (int64_t)dk * dv;
     float* Ng = a.memory + (slot * a.H + h) * (int64_t)(dk + 1);
-    const bool owner = wave < VT;  // has value columns
-    const int col = wave * 32 + c;
-    f32x16 S[KT];  // accumulator i of lane (c, half): row 8 (i / 4) + 4 half + i % 4 of the 32-row tile, column c
+    constexpr int KH = KT / 2, VH = VT / 2;  // KT, VT: 2 or 4
+    const bool owner = (wave & 3) < VT;      // has value columns
+    const int col = (wave & 3) * 32 + c, hw = wave >> 2;
+    f32x16 S[KH];  // this wave's tiles of S, rows 32 KH hw and on; accumulator i of lane (c, half): row 8 (i / 4) + 4 half + i % 4 of the 32-row tile, column c
 #pragma unroll
-    for (int kt = 0; kt < KT; ++kt)
+    for (int kt = 0; kt < KH; ++kt)
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
-            const int r = kt * 32 + (i >> 2) * 8 + half * 4 + (i & 3);
+            const int r = (hw * KH + kt) * 32 + (i >> 2) * 8 + half * 4 + (i & 3);
             S[kt][i] = (owner && !fresh && r < dk && col < dv) ? Sg[(int64_t)r * dv + col] : 0.f;
         }
     if (tid < L::DKP) sm.n[tid] = (!fresh && tid < dk) ? Ng[tid] : 0.f;
-    float m_run = fresh ? 0.f : Ng[dk];  // wave 0
-    // a thread's share of a chunk: token tid % 64, pieces of 8 channels; and the output gates of token tid / 4
-    bf16x8 qr[KT], kr[KT], vr[VT];
-    bf16x4 gr[VT * 2];
-    float zi = 0.f, zf = 0.f;
-    const int st = tid & 63, piece = tid >> 6;
-    const int ot = tid >> 2, oq = tid & 3;
+    // tokens of the first half never see keys of the second: that corner of the weighted scores stays zero
+    if (tid < 256) {
+        const int at = (tid >> 3) * TROW + 32 + (tid & 7) * 4;
+        *reinterpret_cast<bf16x4*>(sm.ph + at) = bf16x4{};
+        *reinterpret_cast<bf16x4*>(sm.pl + at) = bf16x4{};
+    }
+    if (tid < L::DVP) sm.gain[tid] = tid < dv ? a.gain[h * dv + tid] : 0.f;
+    // A thread's share of a chunk: 8 of every 64 channels of one token, eight neighbouring lanes fetch a line
+    bf16x8 qr[KH], kr[KH], vr[VH], gr[VH];
+    const int st_t = tid >> 3, st_p = tid & 7;
     auto fetch = [&](int base, int n) {
-        const bf16* row = proj + (int64_t)(t0 + base + st) * a.ld;
-        const bool in = st < n;
+        const bf16* row = proj + (int64_t)(t0 + base + st_t) * a.ld + st_p * 8;
 #pragma unroll
-        for (int u = 0; u < KT; ++u) {
-            const int ch = (piece + u * 4) * 8;
-            qr[u] = in && ch < dk ? *reinterpret_cast<const bf16x8*>(row + a.q_col0 + h * dk + ch) : bf16x8{};
-            kr[u] = in && ch < dk ? *reinterpret_cast<const bf16x8*>(row + a.k_col0 + h * dk + ch) : bf16x8{};
+        for (int u = 0; u < KH; ++u) {
+            const bool in = st_t < n && u * 64 + st_p * 8 < dk;
+            qr[u] = in ? *reinterpret_cast<const bf16x8*>(row + a.q_col0 + h * dk + u * 64) : bf16x8{};
+            kr[u] = in ? *reinterpret_cast<const bf16x8*>(row + a.k_col0 + h * dk + u * 64) : bf16x8{};
         }
 #pragma unroll
-        for (int u = 0; u < VT; ++u) {
-            const int ch = (piece + u * 4) * 8;
-            vr[u] = in && ch < dv ? *reinterpret_cast<const bf16x8*>(row + a.v_col0 + h * dv + ch) : bf16x8{};
+        for (int u = 0; u < VH; ++u) {
+            const bool in = st_t < n && u * 64 + st_p * 8 < dv;
+            vr[u] = in ? *reinterpret_cast<const bf16x8*>(row + a.v_col0 + h * dv + u * 64) : bf16x8{};
         }
-        if (wave == 0 && in) {
-            const float* z = a.gates + (int64_t)(t0 + base + st) * a.ld_gates;
+    };
+    // one wave without score tiles makes the gates, one chunk ahead, and carries m
+    float zi = 0.f, zf = 0.f, m_run = fresh ? 0.f : Ng[dk];
+    auto fetch_gates = [&](int base, int n) {
+        if (lane < n) {
+            const float* z = a.gates + (int64_t)(t0 + base + lane) * a.ld_gates;
             zi = z[h];
             zf = z[a.H + h];
         }
     };
+    const float inv_dv = 1.f / (float)dv;
+    const float ib = a.i_bias ? a.i_bias[h] : 0.f, fb = a.f_bias ? a.f_bias[h] : 0.f;
+    auto make_gates = [&](int n, typename L::Gates& g) {
+        float li = -INFINITY, F = 0.f;  // tokens past the end keep everything and write nothing
+        if (lane < n) {
+            li = soft_capped(zi + ib, a.cap);
+            F = log_sigmoid(soft_capped(zf + fb, a.cap));
+        }
+        F = scan_sum(F);
+        const float as = li - F;
+        const float top = fmaxf(scan_max(as), m_run);
+        const float end = lane_value(top, 63);
+        g.a[lane] = as;
+        g.top[lane] = top;
+        g.d0[lane] = expf(m_run - top);
+        g.fl[lane] = expf(-(F + top));
+        g.w[lane] = expf(as - end);
+        if (lane == 0) g.keep = expf(m_run - end);
+        m_run = lane_value(F, 63) + end;
+    };
     fetch(0, min(CT, qlen));
-    for (int base = 0; base < qlen; base += CT) {
-        const int n = min(CT, qlen - base);
-        // ---- the chunk into LDS; its gates
-        if (wave == 0) {
-            float li = -INFINITY, F = 0.f;  // tokens past the end keep everything and write nothing
-            if (lane < n) {
-                li = soft_capped(zi + (a.i_bias ? a.i_bias[h] : 0.f), a.cap);
-                F = log_sigmoid(soft_capped(zf + (a.f_bias ? a.f_bias[h] : 0.f), a.cap));
-            }
+    if (wave == 3) {
+        fetch_gates(0, min(CT, qlen));
+        make_gates(min(CT, qlen), sm.gates[0]);
+    }
+    int buf = 0;
+    for (int base = 0; base < qlen; base += CT, buf ^= 1) {
+        const int n = min(CT, qlen - base), n_next = min(CT, qlen - base - CT);
+        const typename L::Gates& G = sm.gates[buf];
+        // ---- the chunk into LDS
 #pragma unroll
-            for (int o = 1; o < 64; o <<= 1) {
-                const float up = __shfl_up(F, o, 64);
-                if (lane >= o) F += up;
-            }
-            const float as = li - F;
-            float top = as;
+        for (int u = 0; u < KH; ++u) {
+            const int ch = u * 64 + st_p * 8;
+            *reinterpret_cast<bf16x8*>(sm.qs + st_t * QROW + ch) = qr[u];
+            *reinterpret_cast<bf16x8*>(sm.ks + st_t * QROW + ch) = kr[u];
+            bf16* dst = sm.kt + ch * TROW + token_group(ch, st_t >> 3) + (st_t & 7);
 #pragma unroll
-            for (int o = 1; o < 64; o <<= 1) {
-                const float up = __shfl_up(top, o, 64);
-                if (lane >= o) top = fmaxf(top, up);
-            }
-            top = fmaxf(top, m_run);
-            const float end = lane_value(top, 63);
-            sm.a[lane] = as;
-            sm.top[lane] = top;
-            sm.d0[lane] = expf(m_run - top);
-            sm.fl[lane] = expf(-(F + top));
-            sm.w[lane] = expf(as - end);
-            if (lane == 0) sm.keep = expf(m_run - end);
-            m_run = lane_value(F, 63) + end;
+            for (int j = 0; j < 8; ++j) dst[j * TROW] = kr[u][j];
         }
 #pragma unroll
-        for (int u = 0; u < KT; ++u) {
-            const int ch = (piece + u * 4) * 8;
-            *reinterpret_cast<bf16x8*>(sm.qs + st * QROW + ch) = qr[u];
-            *reinterpret_cast<bf16x8*>(sm.ks + st * QROW + ch) = kr[u];
+        for (int u = 0; u < VH; ++u) {
+            const int ch = u * 64 + st_p * 8;
+            bf16* dst = sm.vt + ch * TROW + token_group(ch, st_t >> 3) + (st_t & 7);
 #pragma unroll
-            for (int j = 0; j < 8; ++j) sm.kt[(ch + j) * TROW + st] = kr[u][j];
+            for (int j = 0; j < 8; ++j) dst[j * TROW] = vr[u][j];
         }
-#pragma unroll
-        for (int u = 0; u < VT; ++u) {
-            const int ch = (piece + u * 4) * 8;
-#pragma unroll
-            for (int j = 0; j < 8; ++j) sm.vt[(ch + j) * TROW + st] = vr[u][j];
-        }
+        if (wave == 3 && n_next > 0) fetch_gates(base + CT, n_next);
         __syncthreads();
-        if (base + CT < qlen) fetch(base + CT, min(CT, qlen - base - CT));
-        if (a.g_col0 >= 0 && ot < n) {
-            const bf16* g = proj + (int64_t)(t0 + base + ot) * a.ld + a.g_col0 + h * dv;
+        if (n_next > 0) fetch(base + CT, n_next);
+        if (a.g_col0 >= 0 && st_t < n) {
+            const bf16* g = proj + (int64_t)(t0 + base + st_t) * a.ld + a.g_col0 + h * dv + st_p * 8;
 #pragma unroll
-            for (int j = 0; j < VT * 2; ++j) gr[j] = j * 16 + oq * 4 < dv ? *reinterpret_cast<const bf16x4*>(g + j * 16 + oq * 4) : bf16x4{};
+            for (int u = 0; u < VH; ++u) gr[u] = u * 64 + st_p * 8 < dv ? *reinterpret_cast<const bf16x8*>(g + u * 64) : bf16x8{};
         }
-        // ---- weighted scores: waves 0, 1, 2 take the (s, t) tiles (0, 0), (0, 1), (1, 1), transposed (a lane has one t)
-        if (wave < 3) {
-            const int ts = wave >> 1, tt = (wave + 1) >> 1;
+        // ---- weighted scores: waves 4, 5, 6 take the (s, t) tiles (0, 0), (0, 1), (1, 1), transposed (a lane has one t)
+        if (wave >= 4 && wave < 7) {
+            const int ts = (wave - 4) >> 1, tt = (wave - 3) >> 1;
             f32x16 P = {};
 #pragma unroll
             for (int s = 0; s < KT * 2; ++s) {
@@ -448,12 +458,12 @@ __global__ __launch_bounds__(256) void matrix_memory_chunk_kernel(MemoryArgs a) 
                 P = mfma32(x, y, P);
             }
             const int t = tt * 32 + c;
-            const float top = sm.top[t];
+            const float top = G.top[t];
             float sum = 0.f;
 #pragma unroll
             for (int g = 0; g < 4; ++g) {
                 const int s0 = ts * 32 + g * 8 + half * 4;
-                const f32x4 as = *reinterpret_cast<const f32x4*>(sm.a + s0);
+                const f32x4 as = *reinterpret_cast<const f32x4*>(G.a + s0);
                 bf16x4 hi, lo;
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
@@ -470,14 +480,14 @@ __global__ __launch_bounds__(256) void matrix_memory_chunk_kernel(MemoryArgs a) 
             sum += __shfl_xor(sum, 32, 64);
             if (half == 0) {
                 sm.part[ts][t] = sum;
-                if (wave == 0) sm.part[1][t] = 0.f;  // no later keys for the first 32 tokens
+                if (wave == 4) sm.part[1][t] = 0.f;  // no later keys for the first 32 tokens
             }
         }
         // ---- what the state of the chunk's start gives: S_0^T q and n_0 . q
         f32x16 O[2] = {};
         if (owner) {
 #pragma unroll
-            for (int kt = 0; kt < KT; ++kt)
+            for (int kt = 0; kt < KH; ++kt)
 #pragma unroll
                 for (int x = 0; x < 2; ++x) {
                     bf16x8 hi, lo;  // rows 16 x + 8 (j / 4) + 4 half + j % 4 of the tile: the A operand follows that order
@@ -488,20 +498,23 @@ __global__ __launch_bounds__(256) void matrix_memory_chunk_kernel(MemoryArgs a) 
                         hi[j] = u;
                         lo[j] = v;
                     }
+                    bf16x8 qa[2];
 #pragma unroll
                     for (int tt = 0; tt < 2; ++tt) {
-                        const bf16* q = sm.qs + (tt * 32 + c) * QROW + kt * 32 + x * 16 + half * 4;
+                        const bf16* q = sm.qs + (tt * 32 + c) * QROW + (hw * KH + kt) * 32 + x * 16 + half * 4;
                         const bf16x4 q0 = *reinterpret_cast<const bf16x4*>(q), q1 = *reinterpret_cast<const bf16x4*>(q + 8);
-                        const bf16x8 qa = __builtin_shufflevector(q0, q1, 0, 1, 2, 3, 4, 5, 6, 7);
-                        O[tt] = mfma32(qa, hi, O[tt]);
-                        O[tt] = mfma32(qa, lo, O[tt]);
+                        qa[tt] = __builtin_shufflevector(q0, q1, 0, 1, 2, 3, 4, 5, 6, 7);
                     }
+                    O[0] = mfma32(qa[0], hi, O[0]);
+                    O[1] = mfma32(qa[1], hi, O[1]);
+                    O[0] = mfma32(qa[0], lo, O[0]);
+                    O[1] = mfma32(qa[1], lo, O[1]);
                 }
 #pragma unroll
             for (int tt = 0; tt < 2; ++tt)
 #pragma unroll
                 for (int g = 0; g < 4; ++g) {
-                    const f32x4 d = *reinterpret_cast<const f32x4*>(sm.d0 + tt * 32 + g * 8 + half * 4);
+                    const f32x4 d = *reinterpret_cast<const f32x4*>(G.d0 + tt * 32 + g * 8 + half * 4);
 #pragma unroll
                     for (int i = 0; i < 4; ++i) O[tt][g * 4 + i] *= d[i];
                 }
@@ -509,122 +522,136 @@ __global__ __launch_bounds__(256) void matrix_memory_chunk_kernel(MemoryArgs a) 
         {
             float d = 0.f;
 #pragma unroll
-            for (int u = 0; u < KT; ++u) {
-                const bf16x8 q = *reinterpret_cast<const bf16x8*>(sm.qs + ot * QROW + (u * 4 + oq) * 8);
-                const f32x4 n0 = *reinterpret_cast<const f32x4*>(sm.n + (u * 4 + oq) * 8), n1 = *reinterpret_cast<const f32x4*>(sm.n + (u * 4 + oq) * 8 + 4);
+            for (int u = 0; u < KH; ++u) {
+                const int ch = u * 64 + st_p * 8;
+                const bf16x8 q = *reinterpret_cast<const bf16x8*>(sm.qs + st_t * QROW + ch);
+                const f32x4 n0 = *reinterpret_cast<const f32x4*>(sm.n + ch), n1 = *reinterpret_cast<const f32x4*>(sm.n + ch + 4);
 #pragma unroll
                 for (int i = 0; i < 4; ++i) d += (float)q[i] * n0[i] + (float)q[4 + i] * n1[i];
             }
-            d += __shfl_xor(d, 1, 64);
-            d += __shfl_xor(d, 2, 64);
-            if (oq == 0) sm.nq[ot] = d;
+            d = sum_neighbours<8>(d);
+            if (st_p == 0) sm.nq[st_t] = d;
         }
+        if (wave == 3 && n_next > 0) make_gates(n_next, sm.gates[buf ^ 1]);
         __syncthreads();
         // ---- the chunk's own keys and values; the state of its end
-        const float keep = sm.keep;
+        const float keep = G.keep;
         if (owner) {
-            const bf16* vrow = sm.vt + col * TROW + half * 8;
+#pragma unroll
+            for (int kt = 0; kt < KH; ++kt) S[kt] *= keep;
+            // the state takes all keys; the read-outs of either half of the waves those of one half of the chunk
 #pragma unroll
             for (int kk = 0; kk < 4; ++kk) {
-                const bf16x8 v = *reinterpret_cast<const bf16x8*>(vrow + kk * 16);
-                // read-outs: tokens of the first half see keys of the first half only
+                const int g8 = kk * 2 + half;
+                const bf16x8 v = *reinterpret_cast<const bf16x8*>(sm.vt + col * TROW + token_group(col, g8));
+                bf16x8 k[KH];
 #pragma unroll
-                for (int tt = 0; tt < 2; ++tt) {
-                    if (tt == 0 && kk >= 2) continue;
-                    const int at = (tt * 32 + c) * TROW + kk * 16 + half * 8;
-                    O[tt] = mfma32(*reinterpret_cast<const bf16x8*>(sm.ph + at), v, O[tt]);
-                    O[tt] = mfma32(*reinterpret_cast<const bf16x8*>(sm.pl + at), v, O[tt]);
+                for (int kt = 0; kt < KH; ++kt) {
+                    const int row = (hw * KH + kt) * 32 + c;
+                    k[kt] = *reinterpret_cast<const bf16x8*>(sm.kt + row * TROW + token_group(row, g8));
                 }
                 // values times their write weights
-                const f32x4 w0 = *reinterpret_cast<const f32x4*>(sm.w + kk * 16 + half * 8), w1 = *reinterpret_cast<const f32x4*>(sm.w + kk * 16 + half * 8 + 4);
-                bf16x8 hi, lo;
+                const f32x4 w0 = *reinterpret_cast<const f32x4*>(G.w + kk * 16 + half * 8), w1 = *reinterpret_cast<const f32x4*>(G.w + kk * 16 + half * 8 + 4);
+                bf16x8 hl[2];
 #pragma unroll
                 for (int j = 0; j < 8; ++j) {
                     bf16 x, y;
                     split_bf16((float)v[j] * (j < 4 ? w0[j & 3] : w1[j & 3]), x, y);
-                    hi[j] = x;
-                    lo[j] = y;
+                    hl[0][j] = x;
+                    hl[1][j] = y;
                 }
 #pragma unroll
-                for (int kt = 0; kt < KT; ++kt) {
-                    if (kk == 0) S[kt] *= keep;
-                    const bf16x8 k = *reinterpret_cast<const bf16x8*>(sm.kt + (kt * 32 + c) * TROW + kk * 16 + half * 8);
-                    S[kt] = mfma32(k, hi, S[kt]);
-                    S[kt] = mfma32(k, lo, S[kt]);
+                for (int part = 0; part < 2; ++part)
+#pragma unroll
+                    for (int kt = 0; kt < KH; ++kt) S[kt] = mfma32(k[kt], hl[part], S[kt]);
+            }
+#pragma unroll
+            for (int x = 0; x < 2; ++x) {
+                const int kk = hw * 2 + x;
+                const bf16x8 v = *reinterpret_cast<const bf16x8*>(sm.vt + col * TROW + token_group(col, kk * 2 + half));
+                bf16x8 p[2][2];
+#pragma unroll
+                for (int tt = 0; tt < 2; ++tt) {
+                    const int at = (tt * 32 + c) * TROW + kk * 16 + half * 8;
+                    p[tt][0] = *reinterpret_cast<const bf16x8*>(sm.ph + at);
+                    p[tt][1] = *reinterpret_cast<const bf16x8*>(sm.pl + at);
+                }
+#pragma unroll
+                for (int part = 0; part < 2; ++part) {
+                    O[0] = mfma32(p[0][part], v, O[0]);
+                    O[1] = mfma32(p[1][part], v, O[1]);
                 }
             }
 #pragma unroll
             for (int tt = 0; tt < 2; ++tt)
 #pragma unroll
-                for (int i = 0; i < 16; ++i) sm.o[(tt * 32 + (i >> 2) * 8 + half * 4 + (i & 3)) * OROW + col] = O[tt][i];
+                for (int i = 0; i < 16; ++i) sm.o[hw][(tt * 32 + (i >> 2) * 8 + half * 4 + (i & 3)) * OROW + col] = O[tt][i];
         }
-        if (tid >= 256 - L::DKP) {  // the last waves have least else to do
-            const int i = tid - (256 - L::DKP);
-            float s = sm.n[i] * keep;
+        {
+            // rows of n: 16 / KT neighbouring lanes share one, each takes its tokens
+            constexpr int SHARE = 16 / KT;
+            const int i = tid / SHARE, part = tid % SHARE;
+            float s = 0.f;
 #pragma unroll
-            for (int p = 0; p < CT / 8; ++p) {
-                const bf16x8 k = *reinterpret_cast<const bf16x8*>(sm.kt + i * TROW + p * 8);
-                const f32x4 w0 = *reinterpret_cast<const f32x4*>(sm.w + p * 8), w1 = *reinterpret_cast<const f32x4*>(sm.w + p * 8 + 4);
+            for (int p = 0; p < KH; ++p) {
+                const int g8 = part * KH + p;
+                const bf16x8 k = *reinterpret_cast<const bf16x8*>(sm.kt + i * TROW + token_group(i, g8));
+                const f32x4 w0 = *reinterpret_cast<const f32x4*>(G.w + g8 * 8), w1 = *reinterpret_cast<const f32x4*>(G.w + g8 * 8 + 4);
 #pragma unroll
                 for (int j = 0; j < 4; ++j) s += (float)k[j] * w0[j] + (float)k[4 + j] * w1[j];
             }
-            sm.n[i] = s;
+            s = sum_neighbours<SHARE>(s);
+            if (part == 0) sm.n[i] = fmaf(sm.n[i], keep, s);
         }
         __syncthreads();
-        // ---- normaliser, norm and gate: four neighbouring lanes per token
+        // ---- normaliser, norm and gate: eight neighbouring lanes per token
         {
-            const float nq = (sm.nq[ot] * sm.d0[ot] + sm.part[0][ot] + sm.part[1][ot]) * a.q_scale;
-            const float den = fmaxf(fabsf(nq), sm.fl[ot]) + a.read_eps;
-            f32x4 v[VT * 2];
+            const float nq = (sm.nq[st_t] * G.d0[st_t] + sm.part[0][st_t] + sm.part[1][st_t]) * a.q_scale;
+            const float den = fmaxf(fabsf(nq), G.fl[st_t]) + a.read_eps;
+            f32x4 v[VH * 2];
             float ss = 0.f;
 #pragma unroll
-            for (int j = 0; j < VT * 2; ++j) {
-                v[j] = *reinterpret_cast<const f32x4*>(sm.o + ot * OROW + j * 16 + oq * 4) * a.q_scale;
+            for (int j = 0; j < VH * 2; ++j) {
+                const int at = st_t * OROW + (j >> 1) * 64 + st_p * 8 + (j & 1) * 4;
+                v[j] = (*reinterpret_cast<const f32x4*>(sm.o[0] + at) + *reinterpret_cast<const f32x4*>(sm.o[1] + at)) * a.q_scale;
 #pragma unroll
                 for (int i = 0; i < 4; ++i) ss += v[j][i] * v[j][i];  // columns past dv are zero
             }
-            ss += __shfl_xor(ss, 1, 64);
-            ss += __shfl_xor(ss, 2, 64);
-            const float rinv = 1.f / (den * sqrtf(ss / ((float)dv * den * den) + a.eps));
-            if (ot < n) {
-                bf16* orow = reinterpret_cast<bf16*>(a.out) + (int64_t)(t0 + base + ot) * a.ld_out + (int64_t)h * dv;
+            ss = sum_neighbours<8>(ss);
+            const float rinv = __builtin_amdgcn_rsqf(ss * inv_dv + a.eps * den * den);  // o / den, normed
+            bf16* orow = reinterpret_cast<bf16*>(a.out) + (int64_t)(t0 + base + st_t) * a.ld_out + (int64_t)h * dv + st_p * 8;
 #pragma unroll
-                for (int j = 0; j < VT * 2; ++j) {
-                    const int at = j * 16 + oq * 4;
-                    if (at >= dv) continue;
-                    const f32x4 gain = *reinterpret_cast<const f32x4*>(a.gain + h * dv + at);
-                    bf16x4 y;
+            for (int u = 0; u < VH; ++u) {
+                bf16x8 y;
 #pragma unroll
-                    for (int i = 0; i < 4; ++i) {
-                        const float g = a.g_col0 >= 0 ? __builtin_amdgcn_rcpf(1.f + __expf(-(float)gr[j][i])) : 1.f;
-                        y[i] = (bf16)(v[j][i] * rinv * gain[i] * g);
-                    }
-                    *reinterpret_cast<bf16x4*>(orow + at) = y;
+                for (int i = 0; i < 8; ++i) {
+                    const float g = a.g_col0 >= 0 ? __builtin_amdgcn_rcpf(1.f + __expf(-(float)gr[u][i])) : 1.f;
+                    y[i] = (bf16)(v[u * 2 + (i >> 2)][i & 3] * rinv * sm.gain[u * 64 + st_p * 8 + i] * g);
                 }
+                if (st_t < n && u * 64 + st_p * 8 < dv) *reinterpret_cast<bf16x8*>(orow + u * 64) = y;
             }
         }
-        // the next chunk's buffers: everything the last part reads (o, nq, part, fl, d0) is written behind the next barriers, except
-        // d0 and fl, which wave 0 writes in front of the first of them
-        __syncthreads();
+        // no barrier here: what this part reads (o, nq, part, n, this buffer's gates) is written again only behind the barrier after the
+        // next chunk's staging, and that staging touches only what the part before this one read (in front of the last barrier)
     }
     if (owner) {
 #pragma unroll
-        for (int kt = 0; kt < KT; ++kt)
+        for (int kt = 0; kt < KH; ++kt)
 #pragma unroll
             for (int i = 0; i < 16; ++i) {
-                const int r = kt * 32 + (i >> 2) * 8 + half * 4 + (i & 3);
+                const int r = (hw * KH + kt) * 32 + (i >> 2) * 8 + half * 4 + (i & 3);
                 if (r < dk && col < dv) Sg[(int64_t)r * dv + col] = S[kt][i];
             }
     }
     if (tid < dk) Ng[tid] = sm.n[tid];
-    if (tid == 0) Ng[dk] = m_run;
+    if (tid == 192) Ng[dk] = m_run;  // the gates' wave
 }
 
 template <int KT, int VT> void launch_chunks(const MemoryArgs& a, int64_t B, hipStream_t st) {
     constexpr size_t lds = sizeof(ChunkLds<KT, VT>);
     static_assert(lds <= 160 * 1024, "a chunk's operands fit the LDS of a compute unit");
     (void)hipFuncSetAttribute((const void*)matrix_memory_chunk_kernel<KT, VT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-    hipLaunchKernelGGL((matrix_memory_chunk_kernel<KT, VT>), dim3((unsigned)B, (unsigned)a.H), dim3(256), lds, st, a);
+    hipLaunchKernelGGL((matrix_memory_chunk_kernel<KT, VT>), dim3((unsigned)B, (unsigned)a.H), dim3(512), lds, st, a);
 }
 
 // runs from this length on are worth a chunk of 64 (a single token costs a whole one)
@@ -633,7 +660,7 @@ constexpr int64_t CHUNKS_FROM = 12;
 bool chunks_ok(const MemoryArgs& a, int dtype) {
     auto al = [](const void* p, size_t n) { return ((uintptr_t)p % n) == 0; };
     return dtype == TGIS_BF16 && a.dk <= 128 && a.dv <= 128 && a.dk % 8 == 0 && a.dv % 8 == 0 && a.ld % 8 == 0 && a.q_col0 % 8 == 0 && a.k_col0 % 8 == 0 &&
-           a.v_col0 % 8 == 0 && (a.g_col0 < 0 || a.g_col0 % 4 == 0) && a.ld_out % 4 == 0 && al(a.proj, 16) && al(a.out, 8) && al(a.gain, 16);
+           a.v_col0 % 8 == 0 && (a.g_col0 < 0 || a.g_col0 % 8 == 0) && a.ld_out % 8 == 0 && al(a.proj, 16) && al(a.out, 16);
 }
 
 }  // namespace

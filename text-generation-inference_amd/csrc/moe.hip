@@ -12,6 +12,7 @@
 //
 // The number of tiles is data dependent; the grid is sized for the worst case (T k + E * (tile rows - 1) rows) and tiles past
 // n_tiles leave at once.
+#include <type_traits>
 #include "common.h"
 #include "mfma_frag.h"
 #include "route_top.h"
@@ -265,24 +266,37 @@ __global__ __launch_bounds__(KW > 4 ? 512 : 256) void moe_gemm_kernel(const T* _
     // this wave's k range, in whole steps
     const int64_t steps = (K + F::KSTEP - 1) / F::KSTEP;
     const int64_t s0 = KSPLIT ? steps * wave / KW : 0, s1 = KSPLIT ? steps * (wave + 1) / KW : steps;
-#pragma unroll(KSPLIT ? 4 : 2)
-    for (int64_t st = s0; st < s1; ++st) {
-        const int64_t kk = st * F::KSTEP;
-        // K is a multiple of PER: a fragment is whole or absent.  Padding rows are not fetched: a decode step has a few live rows
-        // per tile, and their lines are as many as the weights' otherwise
-        const bool in = live && kk + half * F::PER + F::PER <= K;
-        V a = in ? *reinterpret_cast<const V*>(ap + kk) : F::zero();
-        if (pair_scale) a = F::scaled(a, scale);
+    // U steps' fragments are asked for before the first product of them: a wave streams several KiB of weights at a time
+    constexpr int U = KSPLIT ? 4 : 2;
+    auto steps_of = [&](auto count, int64_t st) {
+        constexpr int N_ = decltype(count)::value;
+        V a[N_], bw[N_][NB], bw2[N_][NB];
 #pragma unroll
-        for (int nb = 0; nb < NB; ++nb) {
-            const V b = *reinterpret_cast<const V*>(bp[nb] + st * (64 * F::PER));
-            F::mma(a, b, acc[nb]);
-            if (GLU) {
-                const V b2 = *reinterpret_cast<const V*>(bp2[nb] + st * (64 * F::PER));
-                F::mma(a, b2, acc2[nb]);
+        for (int u = 0; u < N_; ++u) {
+            const int64_t kk = (st + u) * F::KSTEP;
+            // K is a multiple of PER: a fragment is whole or absent.  Padding rows are not fetched: a decode step has a few live rows
+            // per tile, and their lines are as many as the weights' otherwise
+            const bool in = live && kk + half * F::PER + F::PER <= K;
+            a[u] = in ? *reinterpret_cast<const V*>(ap + kk) : F::zero();
+#pragma unroll
+            for (int nb = 0; nb < NB; ++nb) {
+                bw[u][nb] = *reinterpret_cast<const V*>(bp[nb] + (st + u) * (64 * F::PER));
+                if (GLU) bw2[u][nb] = *reinterpret_cast<const V*>(bp2[nb] + (st + u) * (64 * F::PER));
             }
         }
-    }
+#pragma unroll
+        for (int u = 0; u < N_; ++u) {
+            if (pair_scale) a[u] = F::scaled(a[u], scale);
+#pragma unroll
+            for (int nb = 0; nb < NB; ++nb) {
+                F::mma(a[u], bw[u][nb], acc[nb]);
+                if (GLU) F::mma(a[u], bw2[u][nb], acc2[nb]);
+            }
+        }
+    };
+    int64_t st = s0;
+    for (; st + U <= s1; st += U) steps_of(std::integral_constant<int, U>{}, st);
+    for (; st < s1; ++st) steps_of(std::integral_constant<int, 1>{}, st);
     // accumulator i of lane l: A row (i / 4) * 8 + (l / 32) * 4 + i % 4, B row (= output column) l % 32
     if (KSPLIT) {
         constexpr int NA = GLU ? 2 : 1;

@@ -12,13 +12,14 @@
 #include "common.h"
 #include "route_top.h"
 #include "sublayer_result.h"
+#include "wave_dpp.h"
 
 namespace {
 
 // Products the next sublayer wants of the row (w null: none).  idx null: they are the result (out [tokens][R]); else they are the
 // logits of a grouped sigmoid router.
 struct RowProducts {
-    const float* w;  // [R][W]
+    const void* w;   // [R][W] of the activation dtype
     int R;
     float* out;
     int32_t* idx;    // [tokens][k]
@@ -26,6 +27,71 @@ struct RowProducts {
     int k, groups, keep;
     float scale;
 };
+
+// the sum over a workgroup of up to eight waves, in every thread
+__device__ __forceinline__ float group_sum(float v, float* red) {
+    v = wave_total(v);
+    const int wave = threadIdx.x >> 6, nw = (blockDim.x + 63) >> 6;
+    __syncthreads();  // red may still be read from the call before
+    if ((threadIdx.x & 63) == 0) red[wave] = v;
+    __syncthreads();
+    float s = 0.f;
+    for (int i = 0; i < nw; ++i) s += red[i];
+    return s;
+}
+
+// eight consecutive elements of a row of products' weights
+__device__ __forceinline__ void load8(const float* p, f32x4& a, f32x4& b) {
+    a = Vec4<float>::ld(p);
+    b = Vec4<float>::ld(p + 4);
+}
+template <typename T> __device__ __forceinline__ void load8(const T* p, f32x4& a, f32x4& b) {
+    const typename VecT<T>::x8 v = *reinterpret_cast<const typename VecT<T>::x8*>(p);
+    a = f32x4{(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
+    b = f32x4{(float)v[4], (float)v[5], (float)v[6], (float)v[7]};
+}
+__device__ __forceinline__ float dot4(f32x4 a, f32x4 b) { return a[0] * b[0] + a[1] * b[1] + a[2] * b[2] + a[3] * b[3]; }
+
+// The products of the row in LDS, two rows of weights per wave at a time; then the choice of a router by wave 0.
+template <typename T, bool VEC>
+__device__ __forceinline__ void row_products(const float* urow, float* dots, int64_t row, int64_t W, const RowProducts& rp) {
+    __syncthreads();
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, nw = blockDim.x >> 6;
+    const T* w = reinterpret_cast<const T*>(rp.w);
+    for (int e = wave; e < rp.R; e += 2 * nw) {
+        const bool two = e + nw < rp.R;
+        const T* w0 = w + (int64_t)e * W;
+        const T* w1 = two ? w0 + (int64_t)nw * W : w0;
+        float s0 = 0.f, s1 = 0.f;
+        if (VEC && (W & 7) == 0) {
+#pragma unroll 4
+            for (int64_t c = lane * 8; c < W; c += 512) {
+                f32x4 a0, b0, a1, b1;
+                load8(w0 + c, a0, b0);
+                load8(w1 + c, a1, b1);
+                const f32x4 x = Vec4<float>::ld(urow + c), y = Vec4<float>::ld(urow + c + 4);
+                s0 += dot4(a0, x) + dot4(b0, y);
+                s1 += dot4(a1, x) + dot4(b1, y);
+            }
+        } else {
+            for (int64_t c = lane; c < W; c += 64) {
+                s0 += Elem<T>::ld(w0 + c) * urow[c];
+                s1 += Elem<T>::ld(w1 + c) * urow[c];
+            }
+        }
+        s0 = wave_total(s0);
+        s1 = wave_total(s1);
+        if (lane == 0) {
+            float* out = rp.idx ? dots : rp.out + row * rp.R;
+            out[e] = s0;
+            if (two) out[e + nw] = s1;
+        }
+    }
+    if (!rp.idx) return;
+    __syncthreads();
+    if (wave != 0) return;
+    route_grouped_sigmoid_wave(dots, dots + rp.R, rp.R, rp.k, rp.groups, rp.keep, rp.scale, rp.idx + row * rp.k, rp.weight + row * rp.k);
+}
 
 template <typename T, int V>
 __global__ __launch_bounds__(512) void post_norm_kernel(const float* x, const int64_t* __restrict__ ids, const T* __restrict__ table,
@@ -49,7 +115,7 @@ __global__ __launch_bounds__(512) void post_norm_kernel(const float* x, const in
     }
     // from here on a thread reads back what it wrote itself
     if (w) {
-        ss = block_sum(ss, red);
+        ss = group_sum(ss, red);
         const float rinv = 1.f / sqrtf(ss / (float)W + eps);
         ss = 0.f;
         for (int64_t c = (int64_t)threadIdx.x * V; c < W; c += step) {
@@ -64,7 +130,7 @@ __global__ __launch_bounds__(512) void post_norm_kernel(const float* x, const in
     }
     float rinv2 = 1.f;
     if (w2) {
-        ss = block_sum(ss, red);
+        ss = group_sum(ss, red);
         rinv2 = 1.f / sqrtf(ss / (float)W + eps);
     }
     for (int64_t c = (int64_t)threadIdx.x * V; c < W; c += step) {
@@ -82,35 +148,70 @@ __global__ __launch_bounds__(512) void post_norm_kernel(const float* x, const in
             for (int i = 0; i < V; ++i) urow[c + i] = (float)(T)v[i];
         }
     }
-    if (!rp.w) return;
-    __syncthreads();
-    float* dots = urow + W;
-    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, nw = blockDim.x >> 6;
-    for (int e = wave; e < rp.R; e += nw) {
-        const float* we = rp.w + (int64_t)e * W;
-        float s = 0.f;
-        if (V == 4) {
-#pragma unroll 4
-            for (int64_t c = lane * 4; c < W; c += 256) {
-                const f32x4 wv = *reinterpret_cast<const f32x4*>(we + c);
-                const f32x4 hv = *reinterpret_cast<const f32x4*>(urow + c);
-                s += wv[0] * hv[0] + wv[1] * hv[1] + wv[2] * hv[2] + wv[3] * hv[3];
-            }
-        } else {
-            for (int64_t c = lane; c < W; c += 64) s += we[c] * urow[c];
-        }
-        s = wave_sum(s);
-        if (lane == 0) {
-            if (rp.idx)
-                dots[e] = s;
-            else
-                rp.out[row * rp.R + e] = s;
+    if (rp.w) row_products<T, V == 4>(urow, urow + W, row, W, rp);
+}
+
+// The same for W % 4 == 0 up to 512 * 4 * NV: a thread keeps NV groups of four consecutive elements in registers, and everything the
+// row needs is asked for in front of the first sum — a decode step is a few rows, so the launch is a chain of trips to memory.
+template <typename T, int NV>
+__global__ __launch_bounds__(512) void post_norm_held_kernel(const float* x, const int64_t* __restrict__ ids, const T* __restrict__ table,
+                                                             float emb_scale, int64_t vocab, float alpha, float* x_out, SublayerResult r,
+                                                             const float* __restrict__ w, const float* __restrict__ w2, T* __restrict__ h,
+                                                             int64_t W, float eps, RowProducts rp) {
+    extern __shared__ __attribute__((aligned(16))) float urow[];  // products: [W] + products and group ranks
+    __shared__ float red[8];
+    const int64_t row = blockIdx.x;
+    const int64_t tok = ids ? min(max(ids[row], (int64_t)0), vocab - 1) : 0;
+    f32x4 v[NV], g[NV], g2[NV];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int64_t c = ((int64_t)threadIdx.x + blockDim.x * i) * 4;
+        v[i] = g[i] = g2[i] = f32x4{};
+        if (c < W) {
+            v[i] = ids ? Vec4<T>::ld(table + tok * W + c) * emb_scale : Vec4<float>::ld(x + row * W + c);
+            if (w) g[i] = Vec4<float>::ld(w + c);
+            if (w2) g2[i] = Vec4<float>::ld(w2 + c);
         }
     }
-    if (!rp.idx) return;
-    __syncthreads();
-    if (wave != 0) return;
-    route_grouped_sigmoid_wave(dots, dots + rp.R, rp.R, rp.k, rp.groups, rp.keep, rp.scale, rp.idx + row * rp.k, rp.weight + row * rp.k);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int64_t c = ((int64_t)threadIdx.x + blockDim.x * i) * 4;
+        if (r.kind && c < W) v[i] = v[i] * alpha + result_at<T, 4>(r, row, c);
+        ss += dot4(v[i], v[i]);
+    }
+    if (w) {
+        ss = group_sum(ss, red);
+        const float rinv = 1.f / sqrtf(ss / (float)W + eps);
+        ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            v[i] = v[i] * rinv * g[i];
+            ss += dot4(v[i], v[i]);
+        }
+    }
+    if (x_out) {
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int64_t c = ((int64_t)threadIdx.x + blockDim.x * i) * 4;
+            if (c < W) Vec4<float>::st(x_out + row * W + c, v[i]);
+        }
+    }
+    if (w2) {
+        ss = group_sum(ss, red);
+        const float rinv = 1.f / sqrtf(ss / (float)W + eps);
+#pragma unroll
+        for (int i = 0; i < NV; ++i) v[i] = v[i] * rinv * g2[i];
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int64_t c = ((int64_t)threadIdx.x + blockDim.x * i) * 4;
+        if (c < W) {
+            Vec4<T>::st(h + row * W + c, v[i]);
+            if (rp.w) Vec4<float>::st(urow + c, f32x4{(float)(T)v[i][0], (float)(T)v[i][1], (float)(T)v[i][2], (float)(T)v[i][3]});
+        }
+    }
+    if (rp.w) row_products<T, true>(urow, urow + W, row, W, rp);
 }
 
 template <typename T>
@@ -118,15 +219,23 @@ void launch_post_norm(bool vec, const float* x, const int64_t* ids, const void* 
                       const SublayerResult& r, const float* w, const float* w2, void* h, int64_t rows, int64_t W, float eps, const RowProducts& rp,
                       hipStream_t st) {
     const int64_t lanes = vec ? W / 4 : W;
-    const size_t lds = ((size_t)W + (rp.w ? rp.R + (rp.idx ? rp.groups : 0) : 0)) * 4;
+    const size_t products = rp.w ? ((size_t)rp.R + (rp.idx ? rp.groups : 0)) * 4 : 0;
     // products of the row keep eight waves busy whatever the width
     const int nt = rp.w ? 512 : (int)(lanes >= 512 ? 512 : (lanes + 63) / 64 * 64);
-    if (vec)
-        hipLaunchKernelGGL((post_norm_kernel<T, 4>), dim3((unsigned)rows), dim3(nt), lds, st, x, ids, (const T*)table, emb_scale, vocab, alpha,
-                           x_out, r, w, w2, (T*)h, W, eps, rp);
+#define TGIS_POST_NORM(KERNEL, LDS)                                                                                                          \
+    hipLaunchKernelGGL(KERNEL, dim3((unsigned)rows), dim3(nt), LDS, st, x, ids, (const T*)table, emb_scale, vocab, alpha, x_out, r, w, w2,   \
+                       (T*)h, W, eps, rp)
+    if (vec && W <= 512 * 4)
+        TGIS_POST_NORM((post_norm_held_kernel<T, 1>), (rp.w ? (size_t)W * 4 : 0) + products);
+    else if (vec && W <= 512 * 8)
+        TGIS_POST_NORM((post_norm_held_kernel<T, 2>), (rp.w ? (size_t)W * 4 : 0) + products);
+    else if (vec && W <= 512 * 16)
+        TGIS_POST_NORM((post_norm_held_kernel<T, 4>), (rp.w ? (size_t)W * 4 : 0) + products);
+    else if (vec)
+        TGIS_POST_NORM((post_norm_kernel<T, 4>), (size_t)W * 4 + products);
     else
-        hipLaunchKernelGGL((post_norm_kernel<T, 1>), dim3((unsigned)rows), dim3(nt), lds, st, x, ids, (const T*)table, emb_scale, vocab, alpha,
-                           x_out, r, w, w2, (T*)h, W, eps, rp);
+        TGIS_POST_NORM((post_norm_kernel<T, 1>), (size_t)W * 4 + products);
+#undef TGIS_POST_NORM
 }
 
 // ---- out[t][n] = sum_c h[t][c] w[n][c] in fp32 for few outputs and many tokens (two-byte h and w, fp32 sums) --------------------
@@ -191,7 +300,7 @@ __global__ __launch_bounds__(256) void narrow_product_kernel(const T* __restrict
 extern "C" int tgis_post_norm_update(const float* x, const int64_t* ids, const void* table, int64_t vocab, float emb_scale, float alpha,
                                      float* x_out, int kind, const void* y, int64_t ld_y, int slabs, const int32_t* pos,
                                      const float* pair_weight, int pairs, const float* w, const float* w2, void* h, int64_t rows, int64_t W,
-                                     float eps, const float* dot_w, int R, float* dot_out, int32_t* idx, float* route_weight, int top,
+                                     float eps, const void* dot_w, int R, float* dot_out, int32_t* idx, float* route_weight, int top,
                                      int groups, int keep, float route_scale, int dtype, void* stream) {
     TGIS_CHECK_ARG(dtype == TGIS_F16 || dtype == TGIS_BF16 || dtype == TGIS_F32, "tgis_post_norm_update: bad dtype");
     TGIS_CHECK_ARG((x != nullptr) != (ids != nullptr) && h && (!ids || (table && vocab >= 1)), "tgis_post_norm_update: a stream, or token ids and their table");

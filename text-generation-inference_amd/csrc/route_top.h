@@ -1,6 +1,7 @@
 // The choice of a router for one token, by one wave.  k passes over E numbers in LDS (consumed), ties go to the lower index; k <= 64.
 #pragma once
 #include "common.h"
+#include "wave_dpp.h"
 
 namespace {
 
@@ -19,10 +20,16 @@ __device__ __forceinline__ void take_top_wave(float* score, int E, int k, int32_
                 best = e;
             }
         }
-        const float m = wave_max(bv);
-        int cand = (bv == m && best != 0x7fffffff) ? best : 0x7fffffff;
+        const float m = lane_value(scan_max(bv), 63);
+        const uint64_t hit = __ballot(bv == m && best != 0x7fffffff);
+        int cand = 0x7fffffff;
+        if (E <= 64) {  // a lane has one number: the lowest lane that holds the maximum
+            if (hit) cand = __ffsll((unsigned long long)hit) - 1;
+        } else {
+            cand = (hit >> lane & 1) ? best : 0x7fffffff;
 #pragma unroll
-        for (int o = 32; o > 0; o >>= 1) cand = min(cand, __shfl_xor(cand, o, 64));
+            for (int o = 32; o > 0; o >>= 1) cand = min(cand, __shfl_xor(cand, o, 64));
+        }
         const int chosen = cand == 0x7fffffff ? 0 : cand;  // NaN: still a valid index
         if (j == 0) top = m;
         if (lane == j) {

@@ -478,3 +478,51 @@ def gopetar_tensors(config, seed: int, device="cpu", dtype=torch.bfloat16) -> Di
     t["final.norm"] = torch.ones((), device=device).to(dtype)
     lin("head", config.vocab, W)
     return t
+
+
+def fidatar_tensors(config, seed: int, device="cpu", dtype=torch.bfloat16) -> Dict[str, torch.Tensor]:
+    """Seeded full Fidatar checkpoint in the family's tensor naming for a `FidatarConfig`: N(0, 1 / fan_in) projections, gains around
+    one, forget gates that keep for tens of tokens."""
+    g = torch.Generator(device=device).manual_seed(seed)
+    W = config.width
+    t: Dict[str, torch.Tensor] = {}
+
+    def lin(name, n, k):
+        t[name] = (torch.randn(n, k, generator=g, device=device) * k ** -0.5).to(dtype)
+
+    def vec(name, n, mean=0.0, std=0.05):
+        t[name] = (mean + torch.randn(n, generator=g, device=device) * std).to(dtype)
+
+    t["embed"] = torch.randn(config.vocab, W, generator=g, device=device).to(dtype)
+    for i, lay in enumerate(config.layers):
+        m, p = lay["mixer"], f"l{i}.mix"
+        H, dk = m["heads"], m["dim"]
+        dv = m.get("vdim", dk)
+        vec(f"l{i}.norm1", W, 1.0)
+        if lay["type"] == "attention":
+            G = m.get("kv_heads", H)
+            for n_, rows in (("q", H * dk), ("k", G * dk), ("v", G * dv)):
+                lin(f"{p}.{n_}", rows, W)
+                vec(f"{p}.{n_}.b", rows, 0.0, 0.1)
+            vec(f"{p}.q.norm", dk, 1.0)
+            vec(f"{p}.k.norm", dk, 1.0)
+        else:
+            for n_, rows in (("q", H * dk), ("k", H * dk), ("v", H * dv), ("g", H * dv), ("i", H), ("f", H)):
+                lin(f"{p}.{n_}", rows, W)
+            vec(f"{p}.norm", H * dv, 1.0)
+            vec(f"{p}.i.b", H, -1.0, 1.0)
+            vec(f"{p}.f.b", H, 4.0, 1.0)
+        lin(f"{p}.o", W, H * dv)
+        f = lay.get("mlp")
+        if f:
+            vec(f"l{i}.norm2", W, 1.0)
+            q = f"l{i}.mlp"
+            units = [(q, f["ff"])] if f["kind"] == "dense" else [(f"{q}.e{e}", f["expert"]["ff"]) for e in range(f["router"]["experts"])]
+            for name, n_ in units:
+                lin(f"{name}.up", n_, W)
+                lin(f"{name}.down", W, n_)
+            if f["kind"] == "moe":
+                lin(f"{q}.router", f["router"]["experts"], W)
+    vec("final.norm", W, 1.0)
+    lin("head", config.vocab, W)
+    return t

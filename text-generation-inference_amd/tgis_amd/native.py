@@ -1662,7 +1662,7 @@ def post_norm_update(x, y, alpha: float, w, eps: float, y_dtype, ids=None, table
                      dots=None, router=None):
     """x [T, W] fp32 (in place): x <- rms_norm(alpha x + y) * w, h = x rounded to y_dtype (or rms_norm(x) * w2).  y: a tensor of
     y_dtype, split-K slabs (`Partial`), `MixtureRows` without a shared row, or None; ids + table instead of x: the scaled embedding
-    rows begin the stream.  dots [R, W] fp32: products of the row h; router = (top, groups, keep, scale): they are logits to choose
+    rows begin the stream.  dots [R, W] of y_dtype: fp32 products of the row h; router = (top, groups, keep, scale): they are logits to choose
     from.  Returns (x or None, h, products [T, R] / (idx, weight) / None)."""
     if ids is not None:
         assert x is None and y is None and ids.dtype == torch.int64 and table.is_contiguous() and table.dtype == y_dtype
@@ -1688,7 +1688,7 @@ def post_norm_update(x, y, alpha: float, w, eps: float, y_dtype, ids=None, table
     R, extra, out, idx, wt, (top, groups, keep, scale) = 0, None, None, None, None, (0, 1, 1, 1.0)
     if dots is not None:
         R = dots.shape[0]
-        assert dots.shape[1] == W
+        assert dots.shape[1] == W and dots.dtype == y_dtype and dots.is_contiguous()
         if router is not None:
             top, groups, keep, scale = router
             extra = idx, wt = (torch.empty((T, top), dtype=torch.int32, device=dev), torch.empty((T, top), dtype=torch.float32, device=dev))
@@ -1696,7 +1696,7 @@ def post_norm_update(x, y, alpha: float, w, eps: float, y_dtype, ids=None, table
             extra = out = torch.empty((T, R), dtype=torch.float32, device=dev)
     _check(load_library().tgis_post_norm_update(
         _ptr(x), _ptr(ids), _ptr(table), table.shape[0] if table is not None else 0, float(emb_scale), float(alpha), _ptr(x_out), kind, p, ld,
-        slabs, pos, weight, k, _f32(w, "w"), _f32(w2, "w2"), _ptr(h), T, W, float(eps), _f32(dots, "dots"), R, _ptr(out), _ptr(idx), _ptr(wt),
+        slabs, pos, weight, k, _f32(w, "w"), _f32(w2, "w2"), _ptr(h), T, W, float(eps), _ptr(dots), R, _ptr(out), _ptr(idx), _ptr(wt),
         int(top), int(groups), int(keep), float(scale), dtype_code3(y_dtype), _stream()), "tgis_post_norm_update")
     return x_out, h, extra
 

@@ -210,7 +210,7 @@ class RoutedExperts:
             if top > 64 or top > self.keep_groups * (experts // self.groups):
                 raise ValueError(f"{prefix}: {top} of {experts} experts in the best {self.keep_groups} of {self.groups} groups")
             self.products = RowProducts(weights.get_tensor(f"{prefix}.router"), router=(top, self.groups, self.keep_groups, float(grouped_sigmoid)))
-        self.router = _f32(weights.get_tensor(f"{prefix}.router")) if self.products is None else self.products.w32
+        self.router = _f32(weights.get_tensor(f"{prefix}.router")) if self.products is None else None
         self.router_b = _f32(weights.get_tensor(f"{prefix}.router.b")) if router_bias else None
         pad8 = lambda n: (n + 7) // 8 * 8
         gate = [weights.get_tensor(f"{prefix}.e{e}.gate") for e in range(experts)] if not self.relu2 else None
@@ -955,7 +955,6 @@ class RowProducts:
     (router = (top, groups, kept groups, scale): experts are chosen from them) or the gates of a recurrence."""
 
     def __init__(self, weight: torch.Tensor, router=None):
-        self.w32 = _f32(weight)
         self.w = weight.contiguous()
         self.router = router
 
@@ -964,7 +963,10 @@ class RowProducts:
         return rows <= ROW_PRODUCTS_FUSED_MAX_ROWS or self.w.dtype == torch.float32 or self.w.shape[1] % 8 != 0
 
     def of(self, h: torch.Tensor):
-        z = native.narrow_product(h, self.w) if h.dtype != torch.float32 and h.shape[1] % 8 == 0 else torch.nn.functional.linear(h.float(), self.w32)
+        if h.dtype != torch.float32 and h.shape[1] % 8 == 0:
+            z = native.narrow_product(h, self.w)
+        else:
+            z = torch.nn.functional.linear(h.float(), self.w.float())
         return native.moe_choose(z, *self.router) if self.router is not None else z
 
 
@@ -980,7 +982,7 @@ class PostNormResidual:
 
     def _update(self, rows: int, products: Optional[RowProducts], **kw):
         ride = products is not None and products.rides(rows)
-        x, h, extra = native.post_norm_update(alpha=self.alpha, eps=self.eps, dots=products.w32 if ride else None,
+        x, h, extra = native.post_norm_update(alpha=self.alpha, eps=self.eps, dots=products.w if ride else None,
                                               router=products.router if ride else None, **kw)
         if products is not None and not ride:
             extra = products.of(h)
