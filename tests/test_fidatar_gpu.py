@@ -392,16 +392,13 @@ def chunks_ok(dtype, dk, dv):
     return dtype == torch.bfloat16 and dk <= 128 and dv <= 128 and dk % 8 == 0 and dv % 8 == 0
 
 
-@pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("H,dk,dv", MEMORY_SIZES)
-@pytest.mark.parametrize("impl", [0, 1, 2])
+@pytest.mark.parametrize("dtype,H,dk,dv,impl", [(t, *s, i) for t in DTYPES for s in MEMORY_SIZES for i in (0, 1, 2) if i < 2 or chunks_ok(t, *s[1:])])
 def test_matrix_memory_and_its_state(gpu_device, dtype, H, dk, dv, impl):
     """Two sequences in one launch, in portions of 1, 2 and more tokens, in slots with stale contents, gates of every size; the final
-    state; nothing outside the two slots is written.  impl: the launcher's choice, token by token, chunks."""
+    state; nothing outside the two slots is written.  impl: the launcher's choice, token by token, chunks (bfloat16, head widths that
+    are multiples of 8 up to 128)."""
     from tgis_amd import native
 
-    if impl == 2 and not chunks_ok(dtype, dk, dv):
-        pytest.skip("the chunked form takes bfloat16 and head widths that are multiples of 8 up to 128")
     g = torch.Generator().manual_seed(H * dk + dv)
     dev, eps, cap = gpu_device, 1e-6, 9.0
     widths = (H * dk, H * dk, H * dv, H * dv)

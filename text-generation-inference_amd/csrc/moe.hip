@@ -296,7 +296,11 @@ __global__ __launch_bounds__(KW > 4 ? 512 : 256) void moe_gemm_kernel(const T* _
     };
     int64_t st = s0;
     for (; st + U <= s1; st += U) steps_of(std::integral_constant<int, U>{}, st);
-    for (; st < s1; ++st) steps_of(std::integral_constant<int, 1>{}, st);
+    if (U >= 4 && st + 2 <= s1) {
+        steps_of(std::integral_constant<int, 2>{}, st);
+        st += 2;
+    }
+    if (st < s1) steps_of(std::integral_constant<int, 1>{}, st);
     // accumulator i of lane l: A row (i / 4) * 8 + (l / 32) * 4 + i % 4, B row (= output column) l % 32
     if (KSPLIT) {
         constexpr int NA = GLU ? 2 : 1;
