@@ -472,6 +472,11 @@ def test_matrix_memory_keeps_a_far_write(gpu_device, dtype, impl):
         got = torch.cat(outs)
         tol = 1e-4 if dtype == torch.float32 else 0.01
         assert max_err(got, want) <= tol and max_err(got[503], want[503]) <= tol and max_err(got[:3], want[:3]) <= 2 * tol, cuts
+    # without an output gate at all (the gates above are open)
+    st = _Step([0], [n], [0], dev)
+    bare = native.matrix_memory(proj.to(dev), *cols[:3], -1, gates.to(dev), None, None, cap, one.to(dev), torch.zeros(1, 1, dk, dv, device=dev),
+                                torch.zeros(1, 1, dk + 1, device=dev), st.slots, st.cu, st.pos, 1, dk, dv, dk ** -0.5, eps, 1e-6, max_q_len=n, impl=impl)
+    assert max_err(bare, want) <= tol
 
 
 GEOMETRIES = [(6, 3, 32, 24), (8, 2, 80, 64), (4, 4, 16, 32), (2, 1, 128, 128), (3, 1, 10, 6), (16, 1, 64, 96)]
